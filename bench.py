@@ -301,7 +301,7 @@ def parse_args(argv=None):
                          "96, the row limit of its weight-streaming kernel)")
     ap.add_argument("--no-other-configs", action="store_true",
                     help="N = 1, default workload only: skip the short legs of BASELINE configs 3 / 4 / 5 (`other_configs` of the line)")
-    ap.add_argument("--design", default=None, choices=["runevik"],
+    ap.add_argument("--design", default=None, choices=["runevik", "dolurax"],
                     help="instead of the headline workload: prefill and decode of this layer-list design beside a llama stack of "
                          "equal size (random weights), one JSON line with every leg and its kernel times")
     ap.add_argument("--design-sizes", default="1024x8,2048x8,4096x4", help="--design: comma-separated WIDTHxLAYERS")
@@ -437,9 +437,18 @@ def mixed_leg(engine, cfg, args, sample, dist, world):
     return out
 
 
-# ---- --design runevik: the layer-list design beside a llama stack of equal width, depth, vocabulary and parameter count ----
-def design_configs(width, layers):
+# ---- --design NAME: a layer-list design beside a llama stack of equal width, depth, vocabulary and parameter count (dolurax: of
+# ---- as many parameters per token: four experts of width / 2 and a shared one of width against one layer of 3 x width) ----
+def design_configs(design, width, layers):
     heads, vocab = width // 128, 32000
+    if design == "dolurax":
+        mixer = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "mask": {"size": 2048}, "scale": 128 ** -0.5,
+                 "softcap": 50.0, "v_mix": True}
+        mlp = {"kind": "moe", "expert": {"ff": width // 2}, "shared": {"ff": width},
+               "router": {"experts": 32, "top": 4, "groups": {"count": 4, "keep": 2}}}
+        run = {"model_type": "dolurax", "architecture": "Dolurax", "width": width, "vocab": vocab, "norm": {"eps": 1e-5},
+               "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp}] * layers, "logit_scale": 0.25, "logit_softcap": 30.0}
+        return run, llama_like(width, layers, heads, vocab)
     one = []
     for i in range(layers):
         if i % 4 == 3:
@@ -450,10 +459,36 @@ def design_configs(width, layers):
                         "mixer": {"heads": heads, "kv_heads": heads // 2, "dim": 128, "vdim": 128, "conv": 4}})
     run = {"model_type": "runevik", "architecture": "Runevik", "width": width, "vocab": vocab, "layers": one, "norm": {"eps": 1e-5},
            "token_side": {"dim": 64}}
-    lla = dict(model_type="llama", hidden_size=width, num_hidden_layers=layers, num_attention_heads=heads,
-               num_key_value_heads=max(1, heads // 4), intermediate_size=3 * width, vocab_size=vocab, rms_norm_eps=1e-5,
-               rope_theta=10000.0, tie_word_embeddings=False, max_position_embeddings=16384)
-    return run, lla
+    return run, llama_like(width, layers, heads, vocab)
+
+
+def llama_like(width, layers, heads, vocab):
+    return dict(model_type="llama", hidden_size=width, num_hidden_layers=layers, num_attention_heads=heads,
+                num_key_value_heads=max(1, heads // 4), intermediate_size=3 * width, vocab_size=vocab, rms_norm_eps=1e-5,
+                rope_theta=10000.0, tie_word_embeddings=False, max_position_embeddings=16384)
+
+
+def dolurax_specs(cfg):
+    W, V = cfg["width"], cfg["vocab"]
+    yield "embed", (V, W)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer["mlp"]
+        for t in ("norm1", "norm1.b", "norm2", "norm2.b"):
+            yield p + t, (W,)
+        for t, n in (("q", m["heads"] * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"]), ("g", m["heads"] * m["vdim"])):
+            yield p + "mix." + t, (n, W)
+        yield p + "mix.q.norm", (m["dim"],)
+        yield p + "mix.k.norm", (m["dim"],)
+        yield p + "mix.vmix", ()
+        yield p + "mix.o", (W, m["heads"] * m["vdim"])
+        yield p + "mlp.router", (mlp["router"]["experts"], W)
+        for e, ff in [(f"e{e}", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])] + [("shared", mlp["shared"]["ff"])]:
+            yield p + f"mlp.{e}.gate", (ff, W)
+            yield p + f"mlp.{e}.up", (ff, W)
+            yield p + f"mlp.{e}.down", (W, ff)
+    yield "final.norm", (W,)
+    yield "final.norm.b", (W,)
+    yield "head", (V, W)
 
 
 def runevik_specs(cfg):
@@ -505,12 +540,12 @@ def design_engine(cfg, seed, max_positions):
         params = sum(int(__import__("math").prod(sh)) for _n, sh, _k in tensor_specs(cfg))
         return eng, params
     gen = torch.Generator(device="cuda")
-    for i, (name, shape) in enumerate(runevik_specs(cfg)):
+    for i, (name, shape) in enumerate({"runevik": runevik_specs, "dolurax": dolurax_specs}[cfg["model_type"]](cfg)):
         gen.manual_seed(seed * 1000003 + i)
         if len(shape) == 2:
             t = torch.randn(shape, generator=gen, device="cuda") * (0.02 if "conv" not in name else 0.5)
         else:
-            t = torch.full(shape, 0.5 if name.endswith("act") else 1.0, device="cuda")
+            t = torch.full(shape, 0.5 if name.endswith(("act", "vmix")) else (0.0 if name.endswith(".b") and "norm" in name else 1.0), device="cuda")
         eng.set_tensor(name, t.to(torch.bfloat16))
         params += t.numel()
     torch.cuda.synchronize()
@@ -527,9 +562,10 @@ def design_leg(args):
     rng = np.random.default_rng(args.seed)
     legs = []
     fams = {"runevik": ["gemv_in", "gemv_out", "delta", "latent_pre", "latent_decode", "latent_gather", "latent_kv", "latent_prefill", "side", "embed", "gemv_head", "sample"],
+            "dolurax": ["gemv_in", "gqa_pre", "gqa_decode", "gqa_prefill", "gemv_out", "post_norm", "moe_route", "moe_plan", "moe_up", "moe_down", "post_norm2", "embed", "gemv_head", "logit_cap", "sample"],
             "llama": ["gemv_qkv", "attn", "gemv_o", "gemv_gate_up", "gemv_down", "rope_append", "embed", "gemv_head", "sample"]}
     for width, layers in [tuple(map(int, x.split("x"))) for x in args.design_sizes.split(",")]:
-        for name, cfg in zip(("runevik", "llama"), design_configs(width, layers)):
+        for name, cfg in zip((args.design, "llama"), design_configs(args.design, width, layers)):
             eng, params = design_engine(cfg, args.seed, 16384)
             V = 32000
             leg = {"design": name, "width": width, "layers": layers, "params": params, "prefill": {}, "decode": {}, "kernel_us": {}}

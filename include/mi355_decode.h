@@ -35,7 +35,7 @@ extern "C" {
  * `struct_size`, which the caller sets to sizeof() of ITS definition -- a binding generated from another version of this
  * header (a shorter mi_sample_params would make the library read pointers past its end) is refused with MI_ERR_INVALID
  * by mi_engine_create / mi_decode_sample / mi_step_enqueue(_rows) / mi_score_tokens instead of being read. */
-#define MI_ABI_VERSION 3
+#define MI_ABI_VERSION 4
 
 #define MI_OK 0
 #define MI_ERR_INVALID (-1)
@@ -58,13 +58,20 @@ extern "C" {
 #define MI_POS_NONE 0
 #define MI_POS_SINUSOIDAL 1 /* added to the embeddings: entry 2i sin(p 10000^(-2i/width)), entry 2i+1 the cosine */
 #define MI_BLOCK_PARALLEL 0 /* x += mixer(norm(x)) + ff(norm(x)), one norm */
+#define MI_BLOCK_POST_NORM 1 /* x += norm1(mixer(x)), then x += norm2(ff(x)): the sublayers read x itself */
 #define MI_NORM_VECTOR 0    /* RMS norm, a weight per coordinate */
 #define MI_NORM_SCALAR 1    /* RMS norm, one weight for all coordinates */
+#define MI_NORM_LAYER 2     /* layer norm (mean taken off), weight and bias per coordinate; MI_BLOCK_POST_NORM only */
 /* mixers */
 #define MI_MIXER_DELTA 0    /* gated delta rule with short convolutions (recurrent state per cache row) */
 #define MI_MIXER_LATENT 1   /* latent attention without positions (the cache holds one latent per token) */
-/* feed-forward activations */
+#define MI_MIXER_GQA 2      /* grouped-query attention without rotation: normed q / k, soft cap, distance bias, chunks of
+                             * positions, values mixed with an earlier layer's, sigmoid gate on the output (MI_BLOCK_POST_NORM) */
+/* feed-forward kinds and activations */
+#define MI_FF_DENSE 0
+#define MI_FF_MOE 1         /* routed experts and at most one shared expert (MI_BLOCK_POST_NORM) */
 #define MI_ACT_POLYNORM 0   /* a N(z) + b N(z^2) + c N(z^3) + e, N = division by the root mean square over the row */
+#define MI_ACT_SWIGLU 1     /* silu(gate) * up */
 
 /* KV-cache element type selector for mi_kv_create */
 #define MI_KV_MODEL (-1) /* BatchedKVCache semantics: KV in the model dtype (models/base.py:66-85) */
@@ -98,23 +105,37 @@ typedef struct mi_model_desc {
   int32_t block_form;        /* MI_BLOCK_* */
   int32_t norm_kind;         /* MI_NORM_* */
   int32_t side_dim;          /* width of the per-layer token input added after each layer; 0 = none */
+  float logit_scale;         /* logits = softcap(logit_scale * head x); 0 = 1 */
+  float logit_softcap;       /* c tanh(z / c); 0 = none */
 } mi_model_desc;
 
 /* one layer of a MI_ARCH_LAYERS model (num_heads, num_kv_heads, head_dim, intermediate_size of mi_model_desc are unused) */
 typedef struct mi_layer_desc {
   uint32_t struct_size;      /* = sizeof(mi_layer_desc) of the caller's header (ABI guard) */
   int32_t mixer;             /* MI_MIXER_* */
-  int32_t heads;             /* value heads (delta) / query heads (latent) */
-  int32_t kv_heads;          /* delta: q/k heads, heads is a multiple of it */
+  int32_t heads;             /* value heads (delta) / query heads (latent, gqa) */
+  int32_t kv_heads;          /* delta: q/k heads, gqa: k/v heads; heads is a multiple of it */
   int32_t dim;               /* query / key size per head */
   int32_t vdim;              /* value size per head */
   int32_t conv;              /* delta: taps of the short convolutions (>= 1) */
   int32_t kv_rank;           /* latent: size of the latent */
   int32_t kv_from;           /* latent: earlier layer whose latents are read, -1 = this layer's own */
-  float scale;               /* latent: score scale; delta: factor on the unit query */
+  float scale;               /* latent, gqa: score scale; delta: factor on the unit query */
   float unit_eps;            /* delta: eps of the unit vectors x / sqrt(sum x^2 + eps) */
-  int32_t ff;                /* feed-forward width, 0 = none */
+  int32_t ff;                /* feed-forward width (of one expert for MI_FF_MOE), 0 = none */
   int32_t act;               /* MI_ACT_* */
+  /* gqa */
+  float softcap;             /* scores c tanh(s / c), 0 = none */
+  float slope_exp;           /* distance bias -2^(-slope_exp (h + 1) / heads) (i - j) of head h, 0 = none */
+  int32_t chunk;             /* i sees j <= i only if i / chunk = j / chunk (positions of the sequence), 0 = causal only */
+  int32_t v_mix;             /* 1: v = (1 - w) v + w v_first, v_first = the values of the first such layer (which mixes nothing) */
+  /* mixture of experts: softmax router, `top` experts among the `keep` best of `groups` equal groups, weights normalised */
+  int32_t ff_kind;           /* MI_FF_* */
+  int32_t experts;
+  int32_t top;
+  int32_t groups;
+  int32_t keep;
+  int32_t shared_ff;         /* width of the shared expert, 0 = none */
 } mi_layer_desc;
 
 /* arguments of the `sample` closure (utils.py:345-364) + top_p_sampling (sample_utils.py:3-38) */

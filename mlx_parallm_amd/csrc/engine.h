@@ -51,7 +51,7 @@ struct PackedLinear {
 };
 
 // A small tensor kept in float32 whatever the model dtype (norm weights, decay parameters, convolution taps)
-struct Vec32 { std::string name; int n = 0; float* p = nullptr; bool seen = false; };
+struct Vec32 { std::string name; int n = 0; float* p = nullptr; bool seen = false; bool optional = false; };
 
 // One layer of a layer-list model
 struct ListLayer {
@@ -73,12 +73,28 @@ struct ListLayer {
   bool uk_seen = false, uv_seen = false;
   int kdp = 0, vdp = 0, rp = 0;  // padded key / value / latent sizes
   int src = -1;                  // the layer whose latents this layer reads (itself or kv_from)
-  int lat_index = -1;            // which latent arena of the cache (own latents only)
+  int lat_index = -1;            // which arena of the cache holds the latents (own latents only)
   // per-layer token input
   void* side_gate = nullptr; void* side_proj_t = nullptr; void* side_proj_p = nullptr;   // [dim][width], transposed [dim][width], padded [width][dim]
   bool side_gate_seen = false, side_proj_seen = false;
   Vec32 side_norm;
+  // grouped-query attention
+  Vec32 q_norm, k_norm, vmix;
+  float* slopes = nullptr;       // [heads] distance bias
+  bool v_first = false;          // the first layer whose values are mixed: the later ones read its values
+  bool gqa_fast = false;         // matrix-core forms
+  // post-norm blocks: norm of the mixer's output (`norm` is in front of the parallel block), of the feed-forward's output
+  Vec32 norm_b, norm2, norm2_b;
+  // mixture of experts
+  PackedLinear gu, dn, sgu, sdn; // all routed experts' gate | up and down matrices, stacked; the shared expert's
+  int ffp = 0, sffp = 0;         // padded widths
+  void* router = nullptr;        // [experts][padded width] row-major
+  bool router_seen = false;
+  int arena_k = -1, arena_v = -1;
 };
+
+// one slab of the cache of a layer-list model: [place][heads][width] elements per token from element offset `off`
+struct KvArena { size_t off; int heads, width; };
 
 constexpr int NSLOT = 4;
 struct Slot {
@@ -157,9 +173,17 @@ struct mi_engine {
   // ---- layer-list models (engine_layers.hip)
   bool layered = false;
   std::vector<ListLayer> list;
-  int n_latent = 0, n_state = 0;
+  int n_arena = 0, n_state = 0;
   PackedLinear list_head;
-  Vec32 list_final_norm;
+  Vec32 list_final_norm, list_final_norm_b;
+  float* y32 = nullptr;          // [rows][wp] a sublayer's output in front of its norm
+  int n_vfirst = 0;
+  void* v_first = nullptr;       // [rows][n_vfirst] values of the first mixing layer
+  int32_t* moe_ids = nullptr; float* moe_wts = nullptr;       // [rows][max top]
+  void* moe_mid = nullptr; void* moe_out = nullptr;           // [slots][max ff], [slots][wp]
+  int32_t* moe_plan = nullptr;
+  float* gqa_part = nullptr; size_t gqa_part_cap = 0;         // split-KV partials of the decode attention
+  int* gqa_ctr = nullptr; size_t gqa_ctr_cap = 0;             // its arrival tickets (zero between launches)
   void* tok_embed = nullptr; bool tok_embed_seen = false;     // [vocab][width] row-major
   void* side_embed = nullptr; bool side_embed_seen = false;   // [vocab][layers * side_dim]
   double* d_freq = nullptr;      // [ceil(width / 2)] angular frequencies of the sinusoidal positions
@@ -216,10 +240,9 @@ struct mi_kv {
   std::unordered_map<uint64_t, PrefixEntry> prefix;
   std::list<uint64_t> lru;       // front = most recently used
   int64_t stat_hit_tokens = 0, stat_lookup_tokens = 0, stat_evictions = 0;
-  // ---- layer-list models: latents live in k (one arena per layer that has its own, element offset lat_off[i], lat_rp[i]
-  // elements per token; the same block table for all), recurrent layers in `state` (one slot per cache row)
-  std::vector<size_t> lat_off;
-  std::vector<int> lat_rp;
+  // ---- layer-list models: latents, keys and values live in k (one arena per layer that has its own latents, two per
+  // grouped-query layer; the same block table for all), recurrent layers in `state` (one slot per cache row)
+  std::vector<KvArena> arenas;
   char* state = nullptr;
   size_t list_bytes = 0, state_bytes = 0;
   std::vector<size_t> state_off, ring_off;   // bytes: [row][heads][dim][vdim] float32, [row][taps][channels] model dtype

@@ -1399,8 +1399,8 @@ int mi_kv_reserve(mi_kv* kv, int capacity_tokens) {
   if (capacity_tokens > e->d.max_positions) return fail(MI_ERR_INVALID, "capacity exceeds desc.max_positions");
   MI_HIP(hipSetDevice(e->device));
   const size_t es = dtype_size(kv->dtype);
-  if (e->layered) {              // latents move to the wider rows; the recurrent state does not depend on the capacity
-    const std::vector<size_t> old_off = kv->lat_off;
+  if (e->layered) {              // latents, keys and values move to the wider rows; the recurrent state does not depend on the capacity
+    const std::vector<KvArena> old = kv->arenas;
     const int old_cap = kv->cap;
     kv->cap = capacity_tokens;
     layers_kv_plan(e, kv);
@@ -1409,10 +1409,11 @@ int mi_kv_reserve(mi_kv* kv, int capacity_tokens) {
       kv->cap = old_cap; layers_kv_plan(e, kv);
       return fail(MI_ERR_RUNTIME, "out of device memory growing the KV cache");
     }
-    for (size_t i = 0; i < old_off.size(); ++i) {
-      const size_t rb = (size_t)kv->lat_rp[i] * es;
-      MI_HIP(hipMemcpy2DAsync((char*)nk + kv->lat_off[i] * es, rb * capacity_tokens, (char*)kv->k + old_off[i] * es, rb * old_cap, rb * old_cap,
-                              kv->B, hipMemcpyDeviceToDevice, e->stream));
+    MI_HIP(hipMemsetAsync(nk, 0, kv->list_bytes, e->stream));
+    for (size_t i = 0; i < old.size(); ++i) {
+      const size_t rb = (size_t)old[i].width * es;
+      MI_HIP(hipMemcpy2DAsync((char*)nk + kv->arenas[i].off * es, rb * capacity_tokens, (char*)kv->k + old[i].off * es, rb * old_cap, rb * old_cap,
+                              (size_t)kv->B * old[i].heads, hipMemcpyDeviceToDevice, e->stream));
     }
     MI_HIP(hipStreamSynchronize(e->stream));
     hipFree(kv->k);

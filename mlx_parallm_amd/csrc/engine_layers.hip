@@ -1,10 +1,17 @@
 // engine_layers.hip -- layer-list models (MI_ARCH_LAYERS): a stack whose layers differ in mixer and sizes.
 //
-// What a layer launches, in order:
+// What a layer launches, in order -- parallel block, x += mixer(norm(x)) + ff(norm(x)):
 //   in        every projection of the normed input as ONE matrix (q | k | v | gates | feed-forward up)
 //   mixer     delta.hip or latent.hip; the feed-forward activation rides in one of its launches
 //   out       [mixer output | activation] times [W_o | W_down] side by side: ONE matrix, added to the float32 residual stream
 //   rows      per-layer token input, residual update and the norm in front of the next layer (layer_rows.hip)
+// post-norm block, x += norm1(mixer(x)), x += norm2(ff(x)):
+//   in        every projection of x as ONE matrix (q | k | v | gate)
+//   mixer     gqa.hip, delta.hip or latent.hip
+//   out       W_o, float32
+//   rows      norm1, residual update, router of the experts (layer_rows.hip; many rows: the router in moe.hip)
+//   experts   gate | up of all routed experts and the shared one in one launch, down in another (moe.hip)
+//   rows      weighted sum over the experts, norm2, residual update
 // The matrices go through gemv_rows like every other linear of the engine.  A call is a list of segments (tokens of one
 // cache row each), so prefill, decode and mixed steps are the same pass.
 #include <cmath>
@@ -121,7 +128,9 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
   e->layered = true;
   e->wp = up(d.hidden_size, 64);
   e->list.resize(d.num_layers);
-  const bool mfma16 = d.act_dtype != MI_F32;
+  const bool mfma16 = d.act_dtype != MI_F32, post = d.block_form == MI_BLOCK_POST_NORM;
+  const int n_norm = d.norm_kind == MI_NORM_SCALAR ? 1 : d.hidden_size;
+  int first_mix = -1;            // first layer whose values are mixed into the later ones
   for (int i = 0; i < d.num_layers; ++i) {
     ListLayer& l = e->list[i];
     l.d = layers[i];
@@ -129,7 +138,8 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
     const std::string p = "l" + std::to_string(i) + ".", bad = "layer " + std::to_string(i) + ": ";
     if (m.struct_size != sizeof(mi_layer_desc)) return fail(MI_ERR_INVALID, "mi_layer_desc.struct_size does not match this library");
     if (m.heads < 1 || m.dim < 1 || m.vdim < 1 || m.ff < 0) return fail(MI_ERR_INVALID, bad + "sizes must be positive");
-    if (m.ff > 0 && m.act != MI_ACT_POLYNORM) return fail(MI_ERR_UNSUPPORTED, bad + "unknown activation");
+    if (m.ff > 0 && (m.act != (post ? MI_ACT_SWIGLU : MI_ACT_POLYNORM) || m.ff_kind != (post ? MI_FF_MOE : MI_FF_DENSE)))
+      return fail(MI_ERR_UNSUPPORTED, bad + "feed-forward kind / activation not supported in this block form");
     l.in.K = e->wp;
     if (m.mixer == MI_MIXER_DELTA) {
       if (m.kv_heads < 1 || m.heads % m.kv_heads != 0) return fail(MI_ERR_INVALID, bad + "heads must be a multiple of kv_heads");
@@ -164,17 +174,64 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       if (m.kv_from < 0) {
         l.o_c = part_below(l.in, p + "mix.dkv", m.kv_rank);
         name_vec(l.c_norm, p + "mix.dkv.norm", m.kv_rank);
-        l.lat_index = e->n_latent++;
+        l.lat_index = e->n_arena++;
       }
       if (mfma16 && m.scale > 0.f && latent_mfma_supported(d.act_dtype, m.dim, m.vdim, l.rp)) {
         l.kdp = latent_pad(m.dim); l.vdp = latent_pad(m.vdim);
         l.ukv.K = l.rp; l.ukv.N = m.heads * (l.kdp + l.vdp);
       }
+    } else if (m.mixer == MI_MIXER_GQA) {
+      if (!post) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention is a mixer of post-norm blocks");
+      if (m.kv_heads < 1 || m.heads % m.kv_heads != 0) return fail(MI_ERR_INVALID, bad + "heads must be a multiple of kv_heads");
+      if (!gqa_supported(m.dim, m.vdim)) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention: head sizes not supported");
+      if (m.chunk < 0 || m.softcap < 0.f) return fail(MI_ERR_INVALID, bad + "chunk and softcap must not be negative");
+      l.kdp = gqa_pad(m.dim); l.vdp = gqa_pad(m.vdim);
+      l.gqa_fast = gqa_mfma_supported(d.act_dtype, m.dim, m.vdim);
+      l.o_q = part_below(l.in, p + "mix.q", m.heads * m.dim);
+      l.o_k = part_below(l.in, p + "mix.k", m.kv_heads * m.dim);
+      l.o_v = part_below(l.in, p + "mix.v", m.kv_heads * m.vdim);
+      l.o_g = part_below(l.in, p + "mix.g", m.heads * m.vdim);
+      name_vec(l.q_norm, p + "mix.q.norm", m.dim);
+      name_vec(l.k_norm, p + "mix.k.norm", m.dim);
+      if (m.v_mix) {
+        name_vec(l.vmix, p + "mix.vmix", 1);
+        if (first_mix < 0) { first_mix = i; l.v_first = true; l.vmix.optional = true; }
+        else if (layers[first_mix].kv_heads * layers[first_mix].vdim != m.kv_heads * m.vdim)
+          return fail(MI_ERR_INVALID, bad + "mixed values must have the size of the first such layer's");
+        e->n_vfirst = m.kv_heads * m.vdim;
+      }
+      std::vector<float> slopes(m.heads, 0.f);
+      if (m.slope_exp > 0.f) for (int h = 0; h < m.heads; ++h) slopes[h] = (float)std::pow(2.0, -(double)m.slope_exp * (h + 1) / m.heads);
+      MI_HIP(hipMalloc(&l.slopes, m.heads * sizeof(float)));
+      MI_TRY(copy_in(l.slopes, slopes.data(), m.heads * sizeof(float), 0, e->stream));
+      MI_HIP(hipStreamSynchronize(e->stream));
+      l.arena_k = e->n_arena++;
+      l.arena_v = e->n_arena++;
     } else return fail(MI_ERR_UNSUPPORTED, bad + "unknown mixer");
     const int hv = m.heads * m.vdim;
     part(l.out, p + "mix.o", 0, 0, d.hidden_size, hv);
     l.n_cat = up(hv, 64);
-    if (m.ff > 0) {
+    if (m.ff > 0 && post) {
+      if (m.experts < 1 || m.experts > MOE_MAX_EXPERTS || m.top < 1 || m.top > MOE_MAX_TOP || m.groups < 1 || m.experts % m.groups != 0 ||
+          m.keep < 1 || m.keep > m.groups || m.top > m.keep * (m.experts / m.groups) || m.shared_ff < 0)
+        return fail(MI_ERR_INVALID, bad + "experts, top, groups and keep do not fit each other (at most 512 experts, 64 of them per token)");
+      l.ffp = up(m.ff, 64); l.sffp = up(m.shared_ff, 64);
+      l.gu.K = l.sgu.K = e->wp;
+      l.dn.K = l.ffp; l.sdn.K = l.sffp;
+      for (int x = 0; x < m.experts; ++x) {
+        const std::string pe = p + "mlp.e" + std::to_string(x) + ".";
+        part(l.gu, pe + "gate", x * 2 * l.ffp, 0, m.ff, d.hidden_size);
+        part(l.gu, pe + "up", x * 2 * l.ffp + l.ffp, 0, m.ff, d.hidden_size);
+        part(l.dn, pe + "down", x * e->wp, 0, d.hidden_size, m.ff);
+      }
+      l.gu.N = m.experts * 2 * l.ffp; l.dn.N = m.experts * e->wp;
+      if (m.shared_ff > 0) {
+        part(l.sgu, p + "mlp.shared.gate", 0, 0, m.shared_ff, d.hidden_size);
+        part(l.sgu, p + "mlp.shared.up", l.sffp, 0, m.shared_ff, d.hidden_size);
+        part(l.sdn, p + "mlp.shared.down", 0, 0, d.hidden_size, m.shared_ff);
+        l.sgu.N = 2 * l.sffp; l.sdn.N = e->wp;
+      }
+    } else if (m.ff > 0) {
       l.o_up = part_below(l.in, p + "mlp.up", m.ff);
       l.o_ff = l.n_cat;
       part(l.out, p + "mlp.down", 0, l.o_ff, d.hidden_size, m.ff);
@@ -183,10 +240,16 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
     }
     for (auto& q : l.in.parts) if (q.cols < 0) q.cols = d.hidden_size;
     l.out.N = e->wp; l.out.K = l.n_cat;
-    name_vec(l.norm, p + "norm1", d.norm_kind == MI_NORM_SCALAR ? 1 : d.hidden_size);
+    name_vec(l.norm, p + "norm1", n_norm);
+    if (post && m.ff > 0) name_vec(l.norm2, p + "norm2", n_norm);
+    if (d.norm_kind == MI_NORM_LAYER) {
+      name_vec(l.norm_b, p + "norm1.b", n_norm);
+      if (m.ff > 0) name_vec(l.norm2_b, p + "norm2.b", n_norm);
+    }
     if (d.side_dim > 0) name_vec(l.side_norm, p + "side.norm", d.hidden_size);
   }
-  name_vec(e->list_final_norm, "final.norm", d.norm_kind == MI_NORM_SCALAR ? 1 : d.hidden_size);
+  name_vec(e->list_final_norm, "final.norm", n_norm);
+  if (d.norm_kind == MI_NORM_LAYER) name_vec(e->list_final_norm_b, "final.norm.b", n_norm);
   e->list_head.K = e->wp; e->list_head.N = d.vocab_size;
   part(e->list_head, "head", 0, 0, d.vocab_size, d.hidden_size);
   const int nf = (d.hidden_size + 1) / 2;
@@ -202,8 +265,10 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
 template <typename F>
 void each_vec(mi_engine* e, F f) {
   for (auto& l : e->list)
-    for (Vec32* v : {&l.norm, &l.act, &l.conv_q, &l.conv_k, &l.conv_v, &l.A_log, &l.dt_bias, &l.head_norm, &l.c_norm, &l.side_norm}) f(*v);
+    for (Vec32* v : {&l.norm, &l.act, &l.conv_q, &l.conv_k, &l.conv_v, &l.A_log, &l.dt_bias, &l.head_norm, &l.c_norm, &l.side_norm,
+                     &l.q_norm, &l.k_norm, &l.vmix, &l.norm_b, &l.norm2, &l.norm2_b}) f(*v);
   f(e->list_final_norm);
+  f(e->list_final_norm_b);
 }
 
 int finalize_packed(mi_engine* e, PackedLinear& L) {
@@ -282,6 +347,67 @@ int latent_nsplit(const mi_kv* kv, const int32_t* rows, const int32_t* lens, int
   return std::max(1, std::min(ns, 32));
 }
 
+// key splits of a decode launch: enough workgroups for the chip, at least two 32-key blocks per wave
+int gqa_nsplit(const mi_kv* kv, const ListLayer& l, const int32_t* rows, const int32_t* lens, int n, int nd) {
+  int mx = 0;
+  for (int i = 0; i < n; ++i)
+    if (lens[i] == 1) { const int pos = kv->h_off[rows[i]]; mx = std::max(mx, l.d.chunk > 0 ? pos % l.d.chunk : pos); }
+  const int ns = std::max(1, 512 / std::max(1, nd * l.d.kv_heads * gqa_head_tiles(l.d.heads, l.d.kv_heads)));
+  return std::max(1, std::min({ns, (mx + 127) / 128, 32}));
+}
+
+int run_gqa(mi_engine* e, mi_kv* kv, ListLayer& l, const Tables& tb, const int32_t* rows, const int32_t* lens, int n) {
+  const mi_model_desc& d = e->d;
+  const mi_layer_desc& m = l.d;
+  hipStream_t st = e->stream;
+  const size_t es = dtype_size(kv->dtype);
+  GqaCall c{};
+  c.t = tb.t;
+  c.sk = AttnShape{1, 1, m.heads, m.kv_heads, l.kdp, d.act_dtype, kv->dtype, RND_NONE, kv->cap, nullptr, nullptr, 0, 0};
+  kv_shape(kv, c.sk);
+  c.sv = c.sk;
+  c.sv.D = l.vdp;
+  c.H = m.heads; c.G = m.kv_heads; c.dim = m.dim; c.vdim = m.vdim; c.kdp = l.kdp; c.vdp = l.vdp;
+  c.proj = e->proj; c.ldp = l.in.N; c.o_q = l.o_q; c.o_k = l.o_k; c.o_v = l.o_v; c.o_g = l.o_g;
+  c.q_norm = l.q_norm.p; c.k_norm = l.k_norm.p; c.eps = d.rms_norm_eps;
+  c.scale = m.scale; c.softcap = m.softcap; c.slopes = l.slopes; c.chunk = m.chunk;
+  if (m.v_mix && l.v_first) c.v_first_out = e->v_first;
+  else if (m.v_mix) { c.v_mix = l.vmix.p; c.v_first_in = e->v_first; }
+  c.kcache = (char*)kv->k + kv->arenas[l.arena_k].off * es;
+  c.vcache = (char*)kv->k + kv->arenas[l.arena_v].off * es;
+  c.q = e->lq; c.nsplit = 1;
+  c.cat = e->cat; c.ldc = l.n_cat; c.act = d.act_dtype;
+  c.all_tokens = l.gqa_fast ? 0 : 1;
+  if (!l.gqa_fast || c.t.nc > 0) { Prof pr(e, "gqa_pre"); MI_TRY(launch_gqa_pre(c, st)); }
+  if (!l.gqa_fast) { Prof pr(e, "gqa_generic"); return launch_gqa_generic(c, st); }
+  if (c.t.nd > 0) {
+    c.nsplit = gqa_nsplit(kv, l, rows, lens, n, c.t.nd);
+    if (c.nsplit > 1) {
+      MI_TRY(grow(e, (void**)&e->gqa_part, &e->gqa_part_cap, (size_t)c.t.nd * m.heads * c.nsplit * (l.vdp + 2) * sizeof(float)));
+      const size_t ctr = (size_t)c.t.nd * m.kv_heads * gqa_head_tiles(m.heads, m.kv_heads) * sizeof(int), had = e->gqa_ctr_cap;
+      MI_TRY(grow(e, (void**)&e->gqa_ctr, &e->gqa_ctr_cap, ctr));
+      if (e->gqa_ctr_cap != had) MI_HIP(hipMemsetAsync(e->gqa_ctr, 0, e->gqa_ctr_cap, st));
+      c.partial = e->gqa_part; c.counters = e->gqa_ctr;
+    }
+    Prof pr(e, "gqa_decode");
+    MI_TRY(launch_gqa_decode(c, st));
+  }
+  if (c.t.nc > 0) { Prof pr(e, "gqa_prefill"); MI_TRY(launch_gqa_prefill(c, st)); }
+  return MI_OK;
+}
+
+// the second half of a post-norm layer: experts behind the row kernel that made their input
+MoeCall moe_call(mi_engine* e, const ListLayer& l, int R) {
+  MoeCall c{};
+  c.R = R; c.width = e->d.hidden_size; c.ld = e->wp;
+  c.r = RouteArgs{l.d.experts, l.d.top, l.d.groups, l.d.keep};
+  c.x = e->x32; c.h = e->hn; c.router = l.router; c.ids = e->moe_ids; c.wts = e->moe_wts;
+  c.gu = l.gu.f.W; c.dn = l.dn.f.W; c.sgu = l.sgu.f.W; c.sdn = l.sdn.f.W;
+  c.ffp = l.ffp; c.sffp = l.sffp; c.lda = std::max(l.ffp, l.sffp);
+  c.mid = e->moe_mid; c.out = e->moe_out; c.plan = e->moe_plan; c.act = e->d.act_dtype;
+  return c;
+}
+
 int run_latent(mi_engine* e, mi_kv* kv, ListLayer& l, const Tables& tb, const int32_t* rows, const int32_t* lens, int n, LatentCall c) {
   hipStream_t st = e->stream;
   { Prof pr(e, "latent_pre"); MI_TRY(launch_latent_pre(c, st)); }
@@ -342,7 +468,8 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
   };
   bool found = false;
   MI_TRY(try_packed(e->list_head, found));
-  for (auto& l : e->list) { MI_TRY(try_packed(l.in, found)); MI_TRY(try_packed(l.out, found)); }
+  for (auto& l : e->list)
+    for (PackedLinear* L : {&l.in, &l.out, &l.gu, &l.dn, &l.sgu, &l.sdn}) MI_TRY(try_packed(*L, found));
   if (found) return MI_OK;
   const int W = d.hidden_size;
   if (name == "embed") {
@@ -383,6 +510,13 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
       l.side_proj_seen = true;
       return MI_OK;
     }
+    if (m.ff_kind == MI_FF_MOE && m.ff > 0 && name == p + "mlp.router") {
+      MI_TRY(dense());
+      MI_TRY(check_matrix(name, shape, ndim, m.experts, W));
+      MI_TRY(put_raw(e, l.router, m.experts, W, e->wp, data, on_device));
+      l.router_seen = true;
+      return MI_OK;
+    }
     if (m.mixer != MI_MIXER_LATENT) continue;
     const bool uk = name == p + "mix.uk", uv = name == p + "mix.uv";
     if (!uk && !uv) continue;
@@ -412,7 +546,7 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
 int layers_finalize(mi_engine* e) {
   const mi_model_desc& d = e->d;
   std::string missing;
-  each_vec(e, [&](Vec32& v) { if (v.n > 0 && !v.seen && missing.empty()) missing = v.name; });
+  each_vec(e, [&](Vec32& v) { if (v.n > 0 && !v.seen && !v.optional && missing.empty()) missing = v.name; });
   if (!missing.empty()) return fail(MI_ERR_NOTFOUND, missing + ": not set");
   if (!e->tok_embed_seen) return fail(MI_ERR_NOTFOUND, "embed: not set");
   if (d.side_dim > 0 && !e->side_embed_seen) return fail(MI_ERR_NOTFOUND, "side.embed: not set");
@@ -423,7 +557,13 @@ int layers_finalize(mi_engine* e) {
     if (l.d.mixer == MI_MIXER_LATENT && (!l.uk_seen || !l.uv_seen)) return fail(MI_ERR_NOTFOUND, p + "mix.uk / mix.uv: not set");
     MI_TRY(finalize_packed(e, l.in));
     MI_TRY(finalize_packed(e, l.out));
-    if (l.kdp > 0) MI_TRY(finalize_packed(e, l.ukv));
+    if (l.d.mixer == MI_MIXER_LATENT && l.kdp > 0) MI_TRY(finalize_packed(e, l.ukv));
+    if (l.d.ff_kind == MI_FF_MOE && l.d.ff > 0) {
+      if (!l.router_seen) return fail(MI_ERR_NOTFOUND, p + "mlp.router: not set");
+      MI_TRY(finalize_packed(e, l.gu));
+      MI_TRY(finalize_packed(e, l.dn));
+      if (l.sffp > 0) { MI_TRY(finalize_packed(e, l.sgu)); MI_TRY(finalize_packed(e, l.sdn)); }
+    }
   }
   MI_TRY(finalize_packed(e, e->list_head));
   MI_HIP(hipStreamSynchronize(e->stream));
@@ -434,22 +574,26 @@ void layers_free(mi_engine* e) {
   if (!e->layered) return;
   each_vec(e, [](Vec32& v) { hipFree(v.p); v.p = nullptr; });
   for (auto& l : e->list) {
-    free_packed(l.in); free_packed(l.out); free_packed(l.ukv);
+    for (PackedLinear* L : {&l.in, &l.out, &l.ukv, &l.gu, &l.dn, &l.sgu, &l.sdn}) free_packed(*L);
+    hipFree(l.slopes); hipFree(l.router);
     hipFree(l.uk); hipFree(l.uv); hipFree(l.uk_t); hipFree(l.uv_p); hipFree(l.side_gate); hipFree(l.side_proj_t); hipFree(l.side_proj_p);
   }
   free_packed(e->list_head);
   for (void* p : {e->tok_embed, e->side_embed, (void*)e->d_freq, (void*)e->x32, e->hn, e->proj, e->cat, (void*)e->scan32, (void*)e->gate32,
-                  e->lq, (void*)e->lat_part, e->lat_m, e->lat_x, e->lat_kv, (void*)e->dl_w, (void*)e->dl_p, (void*)e->dl_k, (void*)e->dl_f, (void*)e->d_meta, (void*)e->d_gather_list, e->head_x}) hipFree(p);
+                  e->lq, (void*)e->lat_part, e->lat_m, e->lat_x, e->lat_kv, (void*)e->dl_w, (void*)e->dl_p, (void*)e->dl_k, (void*)e->dl_f, (void*)e->d_meta, (void*)e->d_gather_list, e->head_x,
+                  (void*)e->y32, e->v_first, (void*)e->moe_ids, (void*)e->moe_wts, e->moe_mid, e->moe_out, (void*)e->moe_plan, (void*)e->gqa_part, (void*)e->gqa_ctr}) hipFree(p);
 }
 
-// element offsets of the latent arenas for `tokens` token places, byte offsets of the recurrent state for kv->B rows
+// element offsets of the arenas (latents, keys, values) for `tokens` token places, byte offsets of the recurrent state for kv->B rows
 int layers_kv_plan(mi_engine* e, mi_kv* kv) {
   const size_t es = dtype_size(kv->dtype);
-  kv->lat_off.clear(); kv->lat_rp.clear(); kv->state_off.clear(); kv->ring_off.clear();
+  kv->arenas.clear(); kv->state_off.clear(); kv->ring_off.clear();
   const size_t tokens = kv->paged ? ((size_t)kv->nblocks << kv->bs_shift) : (size_t)kv->B * kv->cap;
   size_t at = 0, sb = 0;
   for (auto& l : e->list) {
-    if (l.lat_index >= 0) { kv->lat_off.push_back(at); kv->lat_rp.push_back(l.rp); at += tokens * l.rp; }
+    auto arena = [&](int heads, int width) { kv->arenas.push_back(KvArena{at, heads, width}); at += tokens * heads * width; };
+    if (l.lat_index >= 0) arena(1, l.rp);
+    if (l.arena_k >= 0) { arena(l.d.kv_heads, l.kdp); arena(l.d.kv_heads, l.vdp); }
     if (l.state_index >= 0) {
       const mi_layer_desc& m = l.d;
       kv->state_off.push_back(sb);
@@ -466,25 +610,37 @@ int layers_kv_plan(mi_engine* e, mi_kv* kv) {
 int layers_ensure_workspace(mi_engine* e, size_t rows) {
   if (rows <= e->lw_rows) return MI_OK;
   MI_HIP(hipStreamSynchronize(e->stream));
-  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4;
+  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4, n_pick = 0, n_mid = 0, n_out = 0, n_plan = 0;
   for (auto& l : e->list) {
     n_in = std::max(n_in, (size_t)l.in.N);
     n_cat = std::max(n_cat, (size_t)l.n_cat);
     if (l.d.mixer == MI_MIXER_DELTA) {
       n_scan = std::max(n_scan, (size_t)2 * l.d.kv_heads * l.d.dim + (size_t)l.d.heads * l.d.vdim);
       n_heads = std::max(n_heads, (size_t)l.d.heads);
-    } else n_lq = std::max(n_lq, (size_t)l.d.heads * l.rp);
+    } else n_lq = std::max(n_lq, (size_t)l.d.heads * (l.d.mixer == MI_MIXER_GQA ? l.kdp : l.rp));
+    if (l.d.ff_kind == MI_FF_MOE && l.d.ff > 0) {
+      const size_t slots = (size_t)l.d.top + (l.sffp > 0 ? 1 : 0);
+      n_pick = std::max(n_pick, (size_t)l.d.top);
+      n_mid = std::max(n_mid, slots * std::max(l.ffp, l.sffp));
+      n_out = std::max(n_out, slots * e->wp);
+      n_plan = std::max(n_plan, moe_plan_ints((int)rows, RouteArgs{l.d.experts, l.d.top, l.d.groups, l.d.keep}, l.sffp > 0 ? 1 : 0));
+    }
   }
+  const size_t n_y = e->d.block_form == MI_BLOCK_POST_NORM ? e->wp : 0;
   n_scan = up((int)n_scan, 4);
   e->scan_ld = (int)n_scan; e->gate_ld = (int)(4 * n_heads);
   const size_t es = act_size(e);
   struct B { void** p; size_t n; } bufs[] = {
       {(void**)&e->x32, rows * e->wp * sizeof(float)}, {&e->hn, rows * e->wp * es}, {&e->proj, rows * n_in * es}, {&e->cat, rows * n_cat * es},
       {(void**)&e->scan32, rows * n_scan * sizeof(float)}, {(void**)&e->gate32, rows * 4 * n_heads * sizeof(float)},
-      {&e->lq, rows * n_lq * sizeof(float)}};
+      {&e->lq, rows * n_lq * sizeof(float)},
+      {(void**)&e->y32, rows * n_y * sizeof(float)}, {&e->v_first, rows * (size_t)e->n_vfirst * es}, {(void**)&e->moe_ids, rows * n_pick * sizeof(int32_t)},
+      {(void**)&e->moe_wts, rows * n_pick * sizeof(float)}, {&e->moe_mid, rows * n_mid * es}, {&e->moe_out, rows * n_out * es},
+      {(void**)&e->moe_plan, n_plan * sizeof(int32_t)}};
   e->lw_rows = 0;
   for (auto& b : bufs) {
     hipFree(*b.p); *b.p = nullptr;
+    if (b.n == 0) continue;
     MI_HIP(hipMalloc(b.p, b.n));
     MI_HIP(hipMemsetAsync(*b.p, 0, b.n, e->stream));      // (padding columns are multiplied by zero weights: they must be finite)
   }
@@ -512,7 +668,9 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
   e->sq_valid = false;
   const int nstride = d.norm_kind == MI_NORM_SCALAR ? 0 : 1;
   const int32_t* tok = e->tok_src ? e->tok_src : e->d_tokens;
+  const bool post = d.block_form == MI_BLOCK_POST_NORM;
   auto norm_of = [&](int li) {
+    if (post) return RowNormW{nullptr, 0, 0.f};                // (the sublayers read the residual stream itself)
     const Vec32& v = li < d.num_layers ? e->list[li].norm : e->list_final_norm;
     return RowNormW{v.p, nstride, d.rms_norm_eps};
   };
@@ -524,7 +682,7 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
     const mi_layer_desc& m = l.d;
     GemvCall ci; ci.x = e->hn; ci.ldx = e->wp; ci.act = act; ci.epi = EPI_STORE; ci.out = e->proj; ci.ldo = l.in.N;
     MI_TRY(gemv_rows(e, l.in.f, ci, R, es, es, "gemv_in"));
-    const PolyNormArgs ff{m.ff, l.o_up, l.o_ff, l.act.p, d.rms_norm_eps};
+    const PolyNormArgs ff{post ? 0 : m.ff, l.o_up, l.o_ff, l.act.p, d.rms_norm_eps};
     if (m.mixer == MI_MIXER_DELTA) {
       DeltaCall c{};
       c.t = t; c.H = m.heads; c.G = m.kv_heads; c.d = m.dim; c.e = m.vdim; c.taps = m.conv;
@@ -547,6 +705,8 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
       }
       Prof pr(e, "delta");
       MI_TRY(launch_delta(c, st));
+    } else if (m.mixer == MI_MIXER_GQA) {
+      MI_TRY(run_gqa(e, kv, l, tb, rows, lens, n));
     } else {
       LatentCall c{};
       const int li_src = e->list[l.src].lat_index;
@@ -556,15 +716,38 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
       c.H = m.heads; c.dim = m.dim; c.vdim = m.vdim; c.rank = m.kv_rank; c.rp = l.rp; c.kdp = l.kdp; c.vdp = l.vdp;
       c.proj = e->proj; c.ldp = l.in.N; c.o_q = l.o_q; c.o_g = l.o_g; c.o_c = l.o_c;
       c.c_norm = l.c_norm.p; c.eps = d.rms_norm_eps;
-      c.cache = (char*)kv->k + kv->lat_off[li_src] * dtype_size(kv->dtype);
+      c.cache = (char*)kv->k + kv->arenas[li_src].off * dtype_size(kv->dtype);
       c.uk = l.uk; c.uv = l.uv; c.uk_t = l.uk_t; c.uv_p = l.uv_p; c.scale = m.scale;
       c.lq = e->lq; c.nsplit = 1;
       c.cat = e->cat; c.ldc = l.n_cat; c.ff = ff; c.act = act;
       MI_TRY(run_latent(e, kv, l, tb, rows, lens, n, c));
     }
     GemvCall co; co.x = e->cat; co.ldx = l.n_cat; co.act = act; co.epi = EPI_RESID; co.out32 = 1; co.resid = e->x32; co.ldo = e->wp;
+    if (post) { co.epi = EPI_STORE; co.resid = nullptr; co.out = e->y32; }
     MI_TRY(gemv_rows(e, l.out.f, co, R, es, sizeof(float), "gemv_out"));
-    { Prof pr(e, "side");
+    if (post) {
+      PostNormCall pn{};
+      pn.rows = R; pn.y = e->y32; pn.kind = d.norm_kind; pn.eps = d.rms_norm_eps; pn.norm = PostNormW{l.norm.p, l.norm_b.p, nstride};
+      pn.width = d.hidden_size; pn.ld = e->wp; pn.x = e->x32; pn.h = e->hn; pn.act = act;
+      const PostNormW last{e->list_final_norm.p, e->list_final_norm_b.p, nstride};
+      const bool end = li + 1 == d.num_layers;
+      if (m.ff > 0) {
+        const MoeCall mc = moe_call(e, l, R);
+        const bool fused = route_fused(act, R, m.experts);
+        pn.r = mc.r; pn.ids = mc.ids; pn.wts = mc.wts;
+        pn.router = fused ? l.router : nullptr;
+        { Prof pr(e, "post_norm"); MI_TRY(launch_post_norm(pn, st)); }
+        if (!fused) { Prof pr(e, "moe_route"); MI_TRY(launch_route(mc, st)); }
+        { Prof pr(e, "moe_plan"); MI_TRY(launch_moe_plan(mc, st)); }
+        { Prof pr(e, "moe_up"); MI_TRY(launch_moe_up(mc, st)); }
+        { Prof pr(e, "moe_down"); MI_TRY(launch_moe_down(mc, st)); }
+        pn.y = nullptr; pn.parts = mc.out; pn.part_w = mc.wts; pn.top = m.top; pn.shared = l.sffp > 0 ? 1 : 0; pn.router = nullptr;
+        pn.norm = PostNormW{l.norm2.p, l.norm2_b.p, nstride};
+      }
+      if (end) pn.next = last;
+      Prof pr(e, m.ff > 0 ? "post_norm2" : "post_norm");
+      MI_TRY(launch_post_norm(pn, st));
+    } else { Prof pr(e, "side");
       SideNormCall c{R, tok, e->side_embed, d.num_layers * d.side_dim, li * d.side_dim, d.vocab_size, l.side_gate, l.side_proj_t, l.side_proj_p,
                      l.side_norm.p, d.rms_norm_eps, d.side_dim, d.hidden_size, e->wp, norm_of(li + 1), e->x32, e->hn, act};
       MI_TRY(launch_side_norm(c, st)); }
@@ -591,6 +774,8 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
     const int rc = gemv_rows(e, e->list_head.f, c, n_out, es, sizeof(float), "gemv_head");
     e->cur_L = keep;
     MI_TRY(rc);
+    Prof pr(e, "logit_cap");
+    MI_TRY(launch_logit_cap(e->logits, (size_t)n_out * d.vocab_size, d.logit_scale == 0.f ? 1.0f : d.logit_scale, d.logit_softcap, st));
   }
   MI_TRY(launch_advance_segments(t, kv->d_off, st));
   for (int i = 0; i < n; ++i) kv->h_off[rows[i]] += lens[i];
@@ -611,8 +796,10 @@ int mi_engine_create_layers(const mi_model_desc* desc, const mi_layer_desc* laye
   if (d.act_dtype != MI_F32 && d.act_dtype != MI_BF16 && d.act_dtype != MI_F16) return fail(MI_ERR_INVALID, "bad act_dtype");
   if (d.quant_bits != 0) return fail(MI_ERR_UNSUPPORTED, "layer-list models: no quantised weights");
   if (d.position != MI_POS_NONE && d.position != MI_POS_SINUSOIDAL) return fail(MI_ERR_UNSUPPORTED, "unknown position encoding");
-  if (d.block_form != MI_BLOCK_PARALLEL) return fail(MI_ERR_UNSUPPORTED, "unknown block form");
-  if (d.norm_kind != MI_NORM_VECTOR && d.norm_kind != MI_NORM_SCALAR) return fail(MI_ERR_UNSUPPORTED, "unknown norm");
+  if (d.block_form != MI_BLOCK_PARALLEL && d.block_form != MI_BLOCK_POST_NORM) return fail(MI_ERR_UNSUPPORTED, "unknown block form");
+  const bool post = d.block_form == MI_BLOCK_POST_NORM;
+  if (d.norm_kind != MI_NORM_VECTOR && d.norm_kind != MI_NORM_SCALAR && !(post && d.norm_kind == MI_NORM_LAYER)) return fail(MI_ERR_UNSUPPORTED, "unknown norm");
+  if (post && d.side_dim > 0) return fail(MI_ERR_UNSUPPORTED, "post-norm blocks: no per-layer token input");
   int ndev = 0;
   if (hipGetDeviceCount(&ndev) != hipSuccess || ndev <= 0)
     return fail(MI_ERR_RUNTIME, "no HIP device available (this library has no CPU backend)");

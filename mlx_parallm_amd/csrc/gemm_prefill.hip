@@ -60,6 +60,9 @@ struct GemmParams {
   // few hundred tokens against N = 4096: 32 x 2..8 blocks); slice z leaves its float32 partial tile in ws[z][M][N] and
   // splitk_epilogue_kernel adds the slices in order and applies the epilogue
   int ksplit; float* ws;
+  // grouped form (GroupedGemm, kernels.h)
+  const int32_t* tiles; const int32_t* x_rows; const int32_t* out_rows; int groups;
+  const void* w_last; int N_last, K_last;
 };
 
 // the epilogues in float32 storage (PagedKVCache mode after layer 0: every op produces a float32 array)
@@ -74,7 +77,8 @@ __device__ __forceinline__ void epi32_plain(const GemmParams& p, int m, int n, f
 }
 
 // grid: (n blocks, m blocks).  SWIGLU: a block covers 64 gate columns + the 64 matching up columns.
-template <typename AT, bool SWIGLU>
+// GROUPED: blockIdx.x = tile of the device-resident table; every group of rows has its own matrix (GroupedGemm, kernels.h)
+template <typename AT, bool SWIGLU, bool GROUPED = false>
 __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   __shared__ __attribute__((aligned(16))) AT As[2][BM][LDA];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -83,7 +87,17 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   // blockIdx.x = M block (fastest): the blocks that run together share one N block, i.e. the same
   // W tiles, which then stay in the XCD's L2 instead of being re-fetched per block
   const int bm = blockIdx.x, bn = blockIdx.y;
-  const int m0 = bm * BM;
+  int m0 = bm * BM, place0 = 0;
+  if constexpr (GROUPED) {
+    if (bm >= p.tiles[0]) return;
+    const int32_t* t = p.tiles + 8 + 4 * bm;
+    const int grp = t[0];
+    place0 = t[1]; m0 = 0; p.M = t[2];
+    if (grp == p.groups) { p.w = p.w_last; p.N = p.N_last; p.K = p.ka = p.kw = p.K_last; }
+    else p.w = (const char*)p.w + (size_t)grp * p.N * p.K * sizeof(AT);
+    if constexpr (SWIGLU) p.pair_offset = p.N / 2;
+    if (bn * (SWIGLU ? 64 : BN) >= (SWIGLU ? p.pair_offset : p.N)) return;
+  }
   const int nk_all = p.K / BK, nkw = p.kw / BK;
   const int ks0 = (int)(((long)blockIdx.z * nk_all) / p.ksplit), ks1 = (int)(((long)(blockIdx.z + 1) * nk_all) / p.ksplit);
   const int nk = ks1;                               // (the loop runs over [ks0, ks1); "nk" bounds the prefetches)
@@ -113,7 +127,9 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   for (int i = 0; i < 4; ++i) {
     const int c = tid + 256 * i, row = c >> 3, kq = c & 7;
     aok[i] = m0 + row < p.M;
-    arow[i] = x + (size_t)min(m0 + row, p.M - 1) * p.ldx + kq * 8;
+    int xr = min(m0 + row, p.M - 1);
+    if constexpr (GROUPED) { xr += place0; if (p.x_rows != nullptr) xr = p.x_rows[xr]; }
+    arow[i] = x + (size_t)xr * p.ldx + kq * 8;
   }
   auto load_a = [&](int ks) {
     const int ka = (ks * BK) % p.ka;
@@ -198,13 +214,19 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   for (int mt = 0; mt < 4; ++mt)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int m = m0 + wm * 64 + mt * 16 + 4 * g + r;
+      int m = m0 + wm * 64 + mt * 16 + 4 * g + r;
       if (m >= p.M) continue;
+      if constexpr (GROUPED) { m += place0; if (p.out_rows != nullptr) m = p.out_rows[m]; }
       if constexpr (SWIGLU) {
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
           const int n = bn * 64 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
+          if constexpr (GROUPED) {
+            const float gt = acc[mt][j][r];
+            out[(size_t)m * p.ldo + n] = (AT)(gt / (1.0f + expf(-gt)) * acc[mt][j + 2][r]);
+            continue;
+          }
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
           const float gt = (float)(AT)acc[mt][j][r], up = (float)(AT)acc[mt][j + 2][r];
           const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
@@ -1255,6 +1277,31 @@ int launch_gemm_prefill(const LinearW& W, const GemvCall& c, size_t rows, hipStr
     else hipLaunchKernelGGL(splitk_epilogue_kernel<bf16>, rg, dim3(256), 0, st, p);
     MI_HIP(hipGetLastError());
   }
+  return MI_OK;
+}
+
+int launch_gemm_grouped(const GroupedGemm& g, hipStream_t st) {
+  const bool dense = (g.W.wk == WK_BF16 && g.act == MI_BF16) || (g.W.wk == WK_F16 && g.act == MI_F16);
+  const bool last = g.last.w != nullptr;
+  if (!dense || g.W.layout != 1 || g.W.K % BK != 0 || g.ldx % 8 != 0 || g.rows % 32 != 0 || g.W.N != g.rows * g.groups ||
+      (last && (g.last.wk != g.W.wk || g.last.layout != 1 || g.last.K % BK != 0 || g.last.N % 32 != 0)))
+    return fail(MI_ERR_UNSUPPORTED, "gemm_grouped: shape / layout not supported");
+  GemmParams p{};
+  p.ksplit = 1;
+  p.x = g.x; p.ldx = g.ldx; p.w = g.W.w; p.N = g.rows; p.K = p.ka = p.kw = g.W.K;
+  p.epi = EPI_STORE; p.out = g.out; p.ldo = g.ldo;
+  p.tiles = g.tiles; p.x_rows = g.x_rows; p.out_rows = g.out_rows; p.groups = g.groups;
+  p.w_last = g.last.w; p.N_last = last ? g.last.N : 0; p.K_last = last ? g.last.K : 0;
+  const int cols = std::max(g.rows, p.N_last) / (g.swiglu ? 2 : 1);
+  const dim3 grid(g.max_tiles, (cols + (g.swiglu ? 64 : BN) - 1) / (g.swiglu ? 64 : BN)), block(256);
+  if (g.act == MI_BF16) {
+    if (g.swiglu) hipLaunchKernelGGL((gemm_tile_kernel<bf16, true, true>), grid, block, 0, st, p);
+    else hipLaunchKernelGGL((gemm_tile_kernel<bf16, false, true>), grid, block, 0, st, p);
+  } else {
+    if (g.swiglu) hipLaunchKernelGGL((gemm_tile_kernel<f16, true, true>), grid, block, 0, st, p);
+    else hipLaunchKernelGGL((gemm_tile_kernel<f16, false, true>), grid, block, 0, st, p);
+  }
+  MI_HIP(hipGetLastError());
   return MI_OK;
 }
 

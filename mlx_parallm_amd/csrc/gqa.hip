@@ -1,0 +1,726 @@
+// gqa.hip -- grouped-query attention without rotation (layer-list models).  q and k are divided by their root mean square,
+// head h scores  softcap tanh(q.k scale / softcap) - slope_h (i - j)  over the keys j <= i of i's own chunk of positions, the
+// values are mixed with an earlier layer's of the same token before they are cached, and the output is multiplied element by
+// element with sigmoid(gate).
+//
+//   gqa_pre        norms, value mix and append of every token of the longer segments (generic form: of all tokens)
+//   gqa_generic    any size and dtype: one workgroup per (token, query head), float32 arithmetic
+//   gqa_decode     16-bit caches, one-token segments: norms, append, split-KV attention, combine and gate in ONE launch; the query
+//                  heads of a group are the columns of the MFMAs and share every key and value that is read
+//   gqa_prefill    16-bit caches, longer segments: flash attention over the paged cache, tiles of 64 or 128 queries of one head
+// Only the key blocks that a tile's chunks reach are walked.
+#include <algorithm>
+#include <type_traits>
+
+#include "layer_rows.h"
+
+namespace mi {
+
+namespace {
+
+using namespace rows;
+
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+constexpr float LOG2E = 1.4426950408889634f;
+
+__device__ __forceinline__ size_t cache_at(const AttnShape& s, int row, int head, int key) {
+  return s.btab ? kv_elem<true>(s, row, head, key) : kv_elem<false>(s, row, head, key);
+}
+__device__ __forceinline__ int chunk_start(int pos, int chunk) { return chunk > 0 ? pos / chunk * chunk : 0; }
+
+// ---- norms, value mix, append ----------------------------------------------------------------------------------------
+// grid R.  VEC: head sizes are multiples of 8 up to 128, 16 lanes per head; otherwise a wave per head.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
+  const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const TokenAt at = token_at(c.t, r);
+  if (!c.all_tokens && c.t.len[at.seg] == 1) return;           // (gqa_decode does its own)
+  const T* pr = (const T*)c.proj + (size_t)r * c.ldp;
+  const float lam = c.v_mix != nullptr ? *c.v_mix : 0.f;
+  const int nh = c.H + 2 * c.G;
+  if constexpr (VEC) {
+    const int g = lane >> 4, l = lane & 15;
+    for (int h0 = wave * 4; h0 < nh; h0 += 16) {
+      const int h = h0 + g;
+      if (h >= nh) continue;                                    // (whole groups of 16 lanes)
+      const int kind = h < c.H ? 0 : (h < c.H + c.G ? 1 : 2), hh = kind == 0 ? h : (kind == 1 ? h - c.H : h - c.H - c.G);
+      const int n = kind == 2 ? c.vdim : c.dim, np = kind == 2 ? c.vdp : c.kdp, k = 8 * l;
+      const T* src = pr + (kind == 0 ? c.o_q : (kind == 1 ? c.o_k : c.o_v)) + hh * n;
+      float v[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] = 0.f;
+      if (k < n) load8f<T>(src + k, v);
+      if (kind < 2) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
+        const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)n + c.eps);
+        const float* w = kind == 0 ? c.q_norm : c.k_norm;
+        if (k < n) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) v[i] *= rs * w[k + i];
+        }
+      } else {
+        const size_t fo = (size_t)r * c.G * c.vdim + hh * c.vdim + k;
+        if (k < n && c.v_first_out != nullptr) store8f<T>((T*)c.v_first_out + fo, v);
+        if (k < n && c.v_mix != nullptr) {
+          float f[8];
+          load8f<T>((const T*)c.v_first_in + fo, f);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) v[i] = (1.0f - lam) * v[i] + lam * f[i];
+        }
+      }
+      if (k < np) {
+        T* dst = kind == 0 ? (T*)c.q + ((size_t)r * c.H + hh) * c.kdp
+                           : (kind == 1 ? (T*)c.kcache + cache_at(c.sk, at.row, hh, at.pos) : (T*)c.vcache + cache_at(c.sv, at.row, hh, at.pos));
+        store8f<T>(dst + k, v);
+      }
+    }
+  } else {
+    for (int h = wave; h < nh; h += 4) {
+      const int kind = h < c.H ? 0 : (h < c.H + c.G ? 1 : 2), hh = kind == 0 ? h : (kind == 1 ? h - c.H : h - c.H - c.G);
+      const int n = kind == 2 ? c.vdim : c.dim, np = kind == 2 ? c.vdp : c.kdp;
+      const T* src = pr + (kind == 0 ? c.o_q : (kind == 1 ? c.o_k : c.o_v)) + hh * n;
+      T* dst = kind == 0 ? (T*)c.q + ((size_t)r * c.H + hh) * c.kdp
+                         : (kind == 1 ? (T*)c.kcache + cache_at(c.sk, at.row, hh, at.pos) : (T*)c.vcache + cache_at(c.sv, at.row, hh, at.pos));
+      float rs = 1.0f;
+      const float* w = kind == 0 ? c.q_norm : c.k_norm;
+      if (kind < 2) {
+        float ss = 0.f;
+        for (int k = lane; k < n; k += 64) { const float v = to_f32(src[k]); ss += v * v; }
+        rs = 1.0f / sqrtf(wave_sum(ss) / (float)n + c.eps);
+      }
+      for (int k = lane; k < np; k += 64) {
+        float v = k < n ? to_f32(src[k]) : 0.f;
+        if (kind < 2) { if (k < n) v *= rs * w[k]; }
+        else if (k < n) {
+          const size_t fo = (size_t)r * c.G * c.vdim + hh * c.vdim + k;
+          if (c.v_first_out != nullptr) ((T*)c.v_first_out)[fo] = from_f32<T>(v);
+          if (c.v_mix != nullptr) v = (1.0f - lam) * v + lam * to_f32(((const T*)c.v_first_in)[fo]);
+        }
+        dst[k] = from_f32<T>(v);
+      }
+    }
+  }
+}
+
+// ---- generic form ----------------------------------------------------------------------------------------------------
+// grid (R, H), 4 waves: wave w takes keys w, w + 4, .. of the token's chunk; NR key / value elements per lane
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
+  extern __shared__ float sm[];                      // [4][vdp] sums
+  __shared__ float ml[8];
+  const int r = blockIdx.x, h = blockIdx.y, g = h / (c.H / c.G), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const TokenAt at = token_at(c.t, r);
+  const int lo = chunk_start(at.pos, c.chunk);
+  const T* qp = (const T*)c.q + ((size_t)r * c.H + h) * c.kdp;
+  const float slope = c.slopes[h];
+  float q[NR], o[NR], m = -INFINITY, l = 0.f;
+#pragma unroll
+  for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; q[i] = k < c.dim ? to_f32(qp[k]) : 0.f; o[i] = 0.f; }
+  constexpr int U = NR <= 2 ? 4 : 2;                 // keys in flight
+  for (int key = lo + wave; key <= at.pos; key += 4 * U) {
+    float x[U][NR], sc[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const T* p = (const T*)c.kcache + cache_at(c.sk, at.row, g, min(key + 4 * u, at.pos));
+      float a = 0.f;
+#pragma unroll
+      for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; if (k < c.dim) a = fmaf(q[i], to_f32(p[k]), a); }
+      sc[u] = a;
+      const T* pv = (const T*)c.vcache + cache_at(c.sv, at.row, g, min(key + 4 * u, at.pos));
+#pragma unroll
+      for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; x[u][i] = k < c.vdim ? to_f32(pv[k]) : 0.f; }
+    }
+    float mx = m;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      float s = wave_sum(sc[u]) * c.scale;
+      if (c.softcap > 0.f) s = c.softcap * tanhf(s / c.softcap);
+      sc[u] = s - slope * (float)(at.pos - (key + 4 * u));
+      if (key + 4 * u <= at.pos) mx = fmaxf(mx, sc[u]);
+    }
+    const float corr = expf(m - mx);                 // (the first key of the loop is visible: mx is finite)
+    m = mx; l *= corr;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) o[i] *= corr;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const float p = key + 4 * u <= at.pos ? expf(sc[u] - m) : 0.f;
+      l += p;
+#pragma unroll
+      for (int i = 0; i < NR; ++i) o[i] = fmaf(p, x[u][i], o[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; if (k < c.vdim) sm[wave * c.vdp + k] = o[i]; }
+  if (lane == 0) { ml[wave] = m; ml[4 + wave] = l; }
+  __syncthreads();
+  const float mx = fmaxf(fmaxf(ml[0], ml[1]), fmaxf(ml[2], ml[3]));
+  float w[4], lt = 0.f;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) { w[i] = expf(ml[i] - mx); lt += w[i] * ml[4 + i]; }
+  const T* gate = (const T*)c.proj + (size_t)r * c.ldp + c.o_g + h * c.vdim;
+  T* cat = (T*)c.cat + (size_t)r * c.ldc + h * c.vdim;
+  for (int k = threadIdx.x; k < c.vdim; k += 256) {
+    const float v = (w[0] * sm[k] + w[1] * sm[c.vdp + k] + w[2] * sm[2 * c.vdp + k] + w[3] * sm[3 * c.vdp + k]) / lt;
+    cat[k] = from_f32<T>(v * sigmoid_f(to_f32(gate[k])));
+  }
+}
+
+// ---- matrix-core forms ------------------------------------------------------------------------------------------------
+template <typename T>
+__device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
+  if constexpr (std::is_same<T, bf16>::value)
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+  else
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
+}
+
+// two float32 values as hi + lo pairs of 16-bit values (softmax weights keep 32-bit accuracy through two MFMAs)
+template <typename T>
+__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
+  const T ha = (T)a, hb = (T)b;
+  T h[2] = {ha, hb};
+  T l[2] = {(T)(a - (float)ha), (T)(b - (float)hb)};
+  hi = __builtin_bit_cast(uint32_t, h);
+  lo = __builtin_bit_cast(uint32_t, l);
+}
+
+// A score in the exp2 domain: LOG2E (softcap tanh(s scale / softcap) + bias); bias in the exp2 domain, with the cap's constant
+// folded in:  softcap tanh(u) = softcap - 2 softcap / (e^(2u) + 1)
+struct ScoreScale { float a, b, c0; };
+__device__ __forceinline__ ScoreScale score_scale(const GqaCall& c) {
+  if (c.softcap > 0.f) return ScoreScale{2.0f * LOG2E * c.scale / c.softcap, -2.0f * c.softcap * LOG2E, c.softcap * LOG2E};
+  return ScoreScale{c.scale * LOG2E, 0.f, 0.f};
+}
+template <bool CAP>
+__device__ __forceinline__ float score2(const ScoreScale& k, float s, float bias) {
+  if constexpr (CAP) return fmaf(k.b, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * k.a) + 1.0f), bias);
+  else return fmaf(s, k.a, bias);
+}
+
+// grid (nsplit, G x head tiles, nd), 4 waves; a wave walks its 32-key blocks on its own, the next block's loads in flight during
+// the current one.  The token's own key and value are added by the last split from LDS, which also appends them.
+template <typename T, int KD, int VD, bool PAGED, bool CAP>
+__global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
+  constexpr int KK = KD / 32, DT = VD / 16, KB = 32, IMG = KB * VD * 2, NV = KB * VD / 8 / 64, LQ = KD + 8;
+  static_assert(IMG == 16 * VD * 4, "a wave's value image holds its 16 output rows");
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];      // 4 value images; later [5][16][VD] outputs
+  __shared__ __attribute__((aligned(16))) T qs[16 * LQ];
+  __shared__ __attribute__((aligned(16))) T kn[KD];
+  __shared__ float vn[VD];
+  __shared__ float st_m[5 * 16], st_l[5 * 16];
+  __shared__ int last_sh;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int rep = c.H / c.G, ht_n = (rep + 15) / 16;
+  const int split = blockIdx.x, kh = blockIdx.y / ht_n, ht = blockIdx.y % ht_n, m = blockIdx.z;
+  const int seg = c.t.dec[m], row = c.t.row[seg], tok = c.t.tok0[seg], pos = c.t.off[row];
+  const int h0 = kh * rep + ht * 16, nh = min(16, rep - ht * 16);
+  const int lo = chunk_start(pos, c.chunk);          // cached keys [lo, pos)
+  const int blk0 = lo / KB, nblk = pos > lo ? (pos + KB - 1) / KB - blk0 : 0, per = (nblk + c.nsplit - 1) / c.nsplit;
+  const int b0 = blk0 + split * per, b1 = min(b0 + per, blk0 + nblk);
+  const T* kc = (const T*)c.kcache;
+  const T* vc = (const T*)c.vcache;
+  unsigned char* img = smem + wave * IMG;
+  u32x4 kf[2][KK], vr[NV];
+  auto load_k = [&](int blk) {
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      const T* p = kc + kv_elem<PAGED>(c.sk, row, kh, max(0, min(blk * KB + 16 * t + c16, pos - 1))) + 8 * g4;
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) kf[t][kk] = *(const u32x4*)(p + 32 * kk);
+    }
+  };
+  auto load_v = [&](int blk) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int piece = i * 64 + lane;
+      vr[i] = *(const u32x4*)(vc + kv_elem<PAGED>(c.sv, row, kh, max(0, min(blk * KB + piece / (VD / 8), pos - 1))) + 8 * (piece % (VD / 8)));
+    }
+  };
+  if (b0 + wave < b1) { load_k(b0 + wave); load_v(b0 + wave); }
+
+  // queries (and, in the last split, the token's own key and value): 16 lanes per head
+  const T* pr = (const T*)c.proj + (size_t)tok * c.ldp;
+  const bool own = split == c.nsplit - 1;
+  {
+    const int hh = tid >> 4, l = tid & 15;
+    constexpr int PL = KD / 16;                      // elements per lane: l PL ..
+    float v[PL], ss = 0.f;
+    auto head = [&](const T* src, bool there, const float* w, T* dst) {
+      ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < PL; ++i) { const int k = l * PL + i; v[i] = there && k < c.dim ? to_f32(src[k]) : 0.f; ss += v[i] * v[i]; }
+      const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)c.dim + c.eps);
+#pragma unroll
+      for (int i = 0; i < PL; ++i) { const int k = l * PL + i; dst[k] = from_f32<T>(k < c.dim ? v[i] * rs * w[k] : 0.f); }
+    };
+    head(pr + c.o_q + (h0 + min(hh, nh - 1)) * c.dim, hh < nh, c.q_norm, qs + hh * LQ);
+    if (own && wave == 0 && hh == 0) head(pr + c.o_k + kh * c.dim, true, c.k_norm, kn);
+    if (own && tid >= 64 && tid < 64 + VD) {
+      const int k = tid - 64;
+      float x = 0.f;
+      if (k < c.vdim) {
+        x = to_f32(pr[c.o_v + kh * c.vdim + k]);
+        const size_t fo = (size_t)tok * c.G * c.vdim + kh * c.vdim + k;
+        if (c.v_first_out != nullptr && ht == 0) ((T*)c.v_first_out)[fo] = from_f32<T>(x);
+        if (c.v_mix != nullptr) { const float lam = *c.v_mix; x = (1.0f - lam) * x + lam * to_f32(((const T*)c.v_first_in)[fo]); }
+      }
+      const T xt = from_f32<T>(x);
+      vn[k] = to_f32(xt);
+      if (ht == 0) ((T*)c.vcache)[kv_elem<PAGED>(c.sv, row, kh, pos) + k] = xt;
+    }
+  }
+  __syncthreads();
+  if (own && ht == 0 && tid < KD) ((T*)c.kcache)[kv_elem<PAGED>(c.sk, row, kh, pos) + tid] = kn[tid];
+  u32x4 qf[KK];
+#pragma unroll
+  for (int kk = 0; kk < KK; ++kk) qf[kk] = *(const u32x4*)(qs + c16 * LQ + 32 * kk + 8 * g4);
+  const ScoreScale ks = score_scale(c);
+  const float slope2 = c.slopes[h0 + min(c16, nh - 1)] * LOG2E;
+  float m_run = -1e30f, l_run = 0.f;
+  f32x4 acc[DT];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) acc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int tq4 = c16 >> 2, tp = c16 & 3;
+
+  for (int blk = b0 + wave; blk < b1; blk += 4) {
+    f32x4 sc[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      sc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) sc[t] = mfma16<T>(kf[t][kk], qf[kk], sc[t]);
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int piece = i * 64 + lane, key = piece / (VD / 8), dc = piece % (VD / 8);
+      *(u32x4*)(img + (size_t)(dc >> 1) * (KB * 32) + key * 32 + (dc & 1) * 16) = vr[i];
+    }
+    if (blk + 4 < b1) { load_k(blk + 4); load_v(blk + 4); }
+    float mx = -INFINITY;
+    const float bias0 = fmaf(slope2, (float)(blk * KB + 4 * g4 - pos), ks.c0);
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = blk * KB + 16 * t + 4 * g4 + r;
+        const float s = score2<CAP>(ks, sc[t][r], fmaf(slope2, (float)(16 * t + r), bias0));
+        sc[t][r] = key >= lo && key < pos ? s : -INFINITY;
+        mx = fmaxf(mx, sc[t][r]);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m_run, mx);
+    if (__builtin_amdgcn_ballot_w64(mn != m_run) != 0) {
+      const float corr = __builtin_amdgcn_exp2f(m_run - mn);
+      m_run = mn;
+      l_run *= corr;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) acc[dt] *= corr;
+    }
+    uint32_t ph[4], pw[4];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      float p[4];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(sc[t][r] - mn); l_run += p[r]; }
+      split2<T>(p[0], p[1], ph[2 * t], pw[2 * t]);
+      split2<T>(p[2], p[3], ph[2 * t + 1], pw[2 * t + 1]);
+    }
+    const u32x4 pf = {ph[0], ph[1], ph[2], ph[3]}, pl = {pw[0], pw[1], pw[2], pw[3]};
+    asm volatile("" ::: "memory");                   // (a wave's LDS operations complete in order)
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const unsigned char* a0 = img + (size_t)dt * (KB * 32) + (4 * g4 + tq4) * 32 + tp * 8;
+      const s16x4 v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a0);
+      const s16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a0 + 16 * 32));
+      const uint32_t* w0 = (const uint32_t*)&v0;
+      const uint32_t* w1 = (const uint32_t*)&v1;
+      const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
+      acc[dt] = mfma16<T>(vf, pf, acc[dt]);
+      acc[dt] = mfma16<T>(vf, pl, acc[dt]);
+    }
+    asm volatile("" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+  }
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  // this wave's maximum, weight sum and outputs of the heads in columns c16 (its own image is free)
+  float* of = (float*)smem;                          // [5][16][VD]
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt) *(f32x4*)(of + (size_t)(wave * 16 + c16) * VD + 16 * dt + 4 * g4) = acc[dt];
+  if (g4 == 0) { st_m[wave * 16 + c16] = m_run; st_l[wave * 16 + c16] = l_run; }
+  {                                                  // entry 4: the token's own key and value
+    const int hh = tid >> 4, l = tid & 15;
+    float s = 0.f;
+    if (own) {
+#pragma unroll
+      for (int i = 0; i < KD / 16; ++i) s = fmaf(to_f32(qs[hh * LQ + l * (KD / 16) + i]), to_f32(kn[l * (KD / 16) + i]), s);
+    }
+    s = row16_sum(s);
+    if (l == 0) { st_m[64 + hh] = own ? score2<CAP>(ks, s, ks.c0) : -1e30f; st_l[64 + hh] = own ? 1.0f : 0.f; }
+    for (int i = tid; i < 16 * VD; i += 256) of[64 * VD + i] = own ? vn[i % VD] : 0.f;
+  }
+  __syncthreads();
+  T* cat = (T*)c.cat + (size_t)tok * c.ldc;
+  const T* gate = pr + c.o_g;
+  float* pp0 = c.partial + (size_t)m * c.H * c.nsplit * (VD + 2);
+  for (int idx = tid; idx < nh * VD; idx += 256) {
+    const int hh = idx / VD, d = idx % VD;
+    float mn = -1e30f;
+#pragma unroll
+    for (int w = 0; w < 5; ++w) mn = fmaxf(mn, st_m[w * 16 + hh]);
+    float L = 0.f, O = 0.f;
+#pragma unroll
+    for (int w = 0; w < 5; ++w) {
+      const float cw = __builtin_amdgcn_exp2f(st_m[w * 16 + hh] - mn);
+      L = fmaf(st_l[w * 16 + hh], cw, L);
+      O = fmaf(of[(size_t)(w * 16 + hh) * VD + d], cw, O);
+    }
+    const int h = h0 + hh;
+    if (c.nsplit == 1) {
+      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * sigmoid_f(to_f32(gate[h * c.vdim + d])));
+    } else {
+      float* pp = pp0 + ((size_t)h * c.nsplit + split) * (VD + 2);
+      __hip_atomic_store(&pp[2 + d], O, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      if (d == 0) {
+        __hip_atomic_store(&pp[0], mn, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        __hip_atomic_store(&pp[1], L, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      }
+    }
+  }
+  if (c.nsplit == 1) return;
+  // the last split to arrive combines (nobody waits): partials are at agent scope, the ticket follows them
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  if (tid == 0) {
+    int* ctr = &c.counters[m * gridDim.y + blockIdx.y];
+    const int ticket = __hip_atomic_fetch_add(ctr, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    last_sh = ticket == c.nsplit - 1;
+    if (last_sh) __hip_atomic_store(ctr, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!last_sh) return;
+  for (int idx = tid; idx < nh * VD; idx += 256) {
+    const int hh = idx / VD, d = idx % VD, h = h0 + hh;
+    const float* pp = pp0 + (size_t)h * c.nsplit * (VD + 2);
+    float mn = -1e30f, L = 0.f, O = 0.f;
+    for (int i0 = 0; i0 < c.nsplit; i0 += 4) {       // four splits' loads in flight, merged in split order
+      float mv[4], lv[4], ov[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float* q = pp + (size_t)min(i0 + j, c.nsplit - 1) * (VD + 2);
+        mv[j] = __hip_atomic_load(&q[0], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        lv[j] = __hip_atomic_load(&q[1], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        ov[j] = __hip_atomic_load(&q[2 + d], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (i0 + j < c.nsplit) {
+          const float bm = fmaxf(mn, mv[j]), cs = __builtin_amdgcn_exp2f(mn - bm), cw = __builtin_amdgcn_exp2f(mv[j] - bm);
+          L = fmaf(lv[j], cw, L * cs);
+          O = fmaf(ov[j], cw, O * cs);
+          mn = bm;
+        }
+    }
+    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * sigmoid_f(to_f32(gate[h * c.vdim + d])));
+  }
+}
+
+// grid (query tiles, H), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys, two LDS
+// buffers, the next block's global loads in flight during the current block's MFMAs.
+// PG: 0 contiguous cache, 1 pages of 64 tokens and more (one page per block of keys), 2 smaller pages
+template <typename T, int KD, int VD, int QG, int PG, bool CAP>
+__global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
+  constexpr int KB = 64, KK = KD / 32, DT = VD / 16, KT = KB / 16, KIMG = KB * KD * 2, VIMG = KB * VD * 2;
+  constexpr int NKP = KB * KD / 8 / 256, NVP = KB * VD / 8 / 256;      // 16-byte pieces per thread
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];  // K[2], V[2]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int seg = c.t.tile[2 * blockIdx.x], t0 = c.t.tile[2 * blockIdx.x + 1], h = blockIdx.y, kh = h / (c.H / c.G);
+  const int row = c.t.row[seg], len = c.t.len[seg], off = c.t.off[row], tok0 = c.t.tok0[seg];
+  const int nk = off + min(t0 + 64 * QG, len);       // keys any query of the tile may see: [chunk of the first query, nk)
+  const int nb = (nk + KB - 1) / KB, j0 = chunk_start(off + t0, c.chunk) / KB;
+  const T* kc = (const T*)c.kcache;
+  const T* vc = (const T*)c.vcache;
+  auto kimg = [&](int b) { return smem + b * KIMG; };
+  auto vimg = [&](int b) { return smem + 2 * KIMG + b * VIMG; };
+
+  // page of key block j (PG 1): looked up one block ahead of its loads
+  const int32_t* btab = PG ? c.sk.btab + (size_t)row * c.sk.bt_stride : nullptr;
+  int page = 0;
+  auto find_page = [&](int j) { if constexpr (PG == 1) page = btab[min(j * KB, nk - 1) >> c.sk.bs_shift]; };
+  u32x4 kreg[NKP], vreg[NVP];
+  auto elem = [&](const AttnShape& s, int key) -> size_t {
+    if constexpr (PG == 1) return (((((size_t)page * s.Hkv + kh) << s.bs_shift) + (size_t)(key & ((1 << s.bs_shift) - 1))) * s.D);
+    else return kv_elem<PG != 0>(s, row, kh, key);
+  };
+  auto load_block = [&](int j) {
+#pragma unroll
+    for (int i = 0; i < NKP; ++i) {
+      const int piece = i * 256 + tid;
+      kreg[i] = *(const u32x4*)(kc + elem(c.sk, min(j * KB + piece / (KD / 8), nk - 1)) + 8 * (piece % (KD / 8)));
+    }
+#pragma unroll
+    for (int i = 0; i < NVP; ++i) {
+      const int piece = i * 256 + tid;
+      vreg[i] = *(const u32x4*)(vc + elem(c.sv, min(j * KB + piece / (VD / 8), nk - 1)) + 8 * (piece % (VD / 8)));
+    }
+  };
+  auto store_block = [&](int buf) {
+#pragma unroll
+    for (int i = 0; i < NKP; ++i) {
+      const int piece = i * 256 + tid, key = piece / (KD / 8), dc = piece % (KD / 8);
+      *(u32x4*)(kimg(buf) + ((((key >> 4) * KK + (dc >> 2)) * 4 + (dc & 3)) * 16 + (key & 15)) * 16) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NVP; ++i) {
+      const int piece = i * 256 + tid, key = piece / (VD / 8), dc = piece % (VD / 8);
+      *(u32x4*)(vimg(buf) + (size_t)((key >> 5) * DT + (dc >> 1)) * (32 * 32) + (key & 31) * 32 + (dc & 1) * 16) = vreg[i];
+    }
+  };
+  find_page(j0);
+  load_block(j0);
+  find_page(j0 + 1);
+  u32x4 qf[QG][KK];
+  int tq[QG], lo[QG];                                // this lane's query of group u and the first key of its chunk
+#pragma unroll
+  for (int u = 0; u < QG; ++u) {
+    tq[u] = t0 + (wave * QG + u) * 16 + c16;
+    lo[u] = chunk_start(off + tq[u], c.chunk);
+    const T* q = (const T*)c.q + ((size_t)(tok0 + min(tq[u], len - 1)) * c.H + h) * KD;
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) qf[u][kk] = *(const u32x4*)(q + 32 * kk + 8 * g4);
+  }
+  store_block(0);
+#pragma unroll
+  for (int u = 0; u < QG; ++u)
+#pragma unroll
+    for (int kk = 0; kk < KK; ++kk) asm volatile("" :: "v"(qf[u][kk]));      // (loaded from here on: no wait carried round the loop)
+  __syncthreads();
+  const ScoreScale ks = score_scale(c);
+  const float slope2 = c.slopes[h] * LOG2E;
+  float m_run[QG], l_run[QG];
+  f32x4 acc[QG][DT];
+#pragma unroll
+  for (int u = 0; u < QG; ++u) {
+    m_run[u] = -1e30f; l_run[u] = 0.f;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) acc[u][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const int tq4 = c16 >> 2, tp = c16 & 3;
+  for (int j = j0; j < nb; ++j) {
+    const int buf = (j - j0) & 1;
+    if (j + 1 < nb) { load_block(j + 1); find_page(j + 2); }
+    f32x4 sc[QG][KT];
+#pragma unroll
+    for (int t = 0; t < KT; ++t) {
+#pragma unroll
+      for (int u = 0; u < QG; ++u) sc[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < KK; ++kk) {
+        const u32x4 kf = *(const u32x4*)(kimg(buf) + (((t * KK + kk) * 4 + g4) * 16 + c16) * 16);
+#pragma unroll
+        for (int u = 0; u < QG; ++u) sc[u][t] = mfma16<T>(kf, qf[u][kk], sc[u][t]);
+      }
+    }
+    u32x4 pf[QG][2], pl[QG][2];
+#pragma unroll
+    for (int u = 0; u < QG; ++u) {
+      const int q0 = off + t0 + (wave * QG + u) * 16;    // position of the group's first query
+      const float bias0 = fmaf(slope2, (float)(j * KB + 4 * g4 - (q0 + c16)), ks.c0);
+      float mx = -INFINITY;
+#pragma unroll
+      for (int t = 0; t < KT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[u][t][r] = score2<CAP>(ks, sc[u][t][r], fmaf(slope2, (float)(16 * t + r), bias0));
+      // a block that reaches past the first query, or in front of the last query's chunk (uniform)
+      if (j * KB + KB - 1 > q0 || (c.chunk > 0 && j * KB < chunk_start(q0 + 15, c.chunk))) {
+#pragma unroll
+        for (int t = 0; t < KT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int key = j * KB + 16 * t + 4 * g4 + r;
+            sc[u][t][r] = key <= q0 + c16 && key >= lo[u] ? sc[u][t][r] : -INFINITY;
+          }
+      }
+#pragma unroll
+      for (int t = 0; t < KT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mx = fmaxf(mx, sc[u][t][r]);
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m_run[u], mx);
+      if (__builtin_amdgcn_ballot_w64(mn != m_run[u]) != 0) {
+        const float corr = __builtin_amdgcn_exp2f(m_run[u] - mn);
+        m_run[u] = mn;
+        l_run[u] *= corr;
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt) acc[u][dt] *= corr;
+      }
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf) {
+        uint32_t ph[4], pw[4];
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+          float p[4];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(sc[u][2 * hf + t][r] - mn); l_run[u] += p[r]; }
+          split2<T>(p[0], p[1], ph[2 * t], pw[2 * t]);
+          split2<T>(p[2], p[3], ph[2 * t + 1], pw[2 * t + 1]);
+        }
+        pf[u][hf] = u32x4{ph[0], ph[1], ph[2], ph[3]};
+        pl[u][hf] = u32x4{pw[0], pw[1], pw[2], pw[3]};
+      }
+    }
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        const unsigned char* a0 = vimg(buf) + (size_t)(hf * DT + dt) * (32 * 32) + (4 * g4 + tq4) * 32 + tp * 8;
+        const s16x4 v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a0);
+        const s16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a0 + 16 * 32));
+        const uint32_t* w0 = (const uint32_t*)&v0;
+        const uint32_t* w1 = (const uint32_t*)&v1;
+        const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
+#pragma unroll
+        for (int u = 0; u < QG; ++u) {
+          acc[u][dt] = mfma16<T>(vf, pf[u][hf], acc[u][dt]);
+          acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
+        }
+      }
+    if (j + 1 < nb) store_block(buf ^ 1);                // the other buffer: nobody reads it during this block
+    __syncthreads();
+  }
+#pragma unroll
+  for (int u = 0; u < QG; ++u) {
+    float l = l_run[u];
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (tq[u] >= len) continue;
+    const int tok = tok0 + tq[u];
+    const float inv = 1.0f / l;
+    const T* gate = (const T*)c.proj + (size_t)tok * c.ldp + c.o_g + h * c.vdim;
+    T* o = (T*)c.cat + (size_t)tok * c.ldc + h * c.vdim;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const int k = 16 * dt + 4 * g4;
+      if (c.vdim % 4 == 0) {
+        if (k < c.vdim) {
+          const float4 gt = load4f<T>(gate + k);
+          T v[4] = {(T)(acc[u][dt][0] * inv * sigmoid_f(gt.x)), (T)(acc[u][dt][1] * inv * sigmoid_f(gt.y)),
+                    (T)(acc[u][dt][2] * inv * sigmoid_f(gt.z)), (T)(acc[u][dt][3] * inv * sigmoid_f(gt.w))};
+          *(uint2*)(o + k) = __builtin_bit_cast(uint2, v);
+        }
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) if (k + r < c.vdim) o[k + r] = (T)(acc[u][dt][r] * inv * sigmoid_f(to_f32(gate[k + r])));
+      }
+    }
+  }
+}
+
+template <typename T>
+int pre_at(const GqaCall& c, hipStream_t st) {
+  if (c.dim % 8 == 0 && c.vdim % 8 == 0 && c.kdp <= 128 && c.vdp <= 128)
+    hipLaunchKernelGGL((gqa_pre_kernel<T, true>), dim3(c.t.R), dim3(256), 0, st, c);
+  else hipLaunchKernelGGL((gqa_pre_kernel<T, false>), dim3(c.t.R), dim3(256), 0, st, c);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+template <typename T>
+int generic_at(const GqaCall& c, hipStream_t st) {
+  const dim3 grid(c.t.R, c.H), block(256);
+  const size_t lds = (size_t)4 * c.vdp * sizeof(float);
+  const int nr = (std::max(c.dim, c.vdim) + 63) / 64;
+#define GO(N) hipLaunchKernelGGL((gqa_generic_kernel<T, N>), grid, block, lds, st, c)
+  if (nr <= 1) GO(1); else if (nr <= 2) GO(2); else if (nr <= 4) GO(4); else if (nr <= 8) GO(8);
+  else return fail(MI_ERR_UNSUPPORTED, "gqa: head sizes above 512");
+#undef GO
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+template <typename T, int KD, int VD>
+int decode_kv(const GqaCall& c, hipStream_t st) {
+  constexpr int lds = 5 * 16 * VD * 4;
+  const dim3 grid(c.nsplit, c.G * gqa_head_tiles(c.H, c.G), c.t.nd);
+  auto go = [&](auto kern) -> int {
+    hipLaunchKernelGGL(kern, grid, dim3(256), lds, st, c);
+    MI_HIP(hipGetLastError());
+    return MI_OK;
+  };
+  if (c.softcap > 0.f) return c.sk.btab ? go(gqa_decode_kernel<T, KD, VD, true, true>) : go(gqa_decode_kernel<T, KD, VD, false, true>);
+  return c.sk.btab ? go(gqa_decode_kernel<T, KD, VD, true, false>) : go(gqa_decode_kernel<T, KD, VD, false, false>);
+}
+
+template <typename T, int KD, int VD, int QG>
+int prefill_qg(const GqaCall& c, hipStream_t st) {
+  constexpr int lds = 2 * 64 * (KD + VD) * 2;
+  auto go = [&](auto kern) -> int {
+    MI_HIP(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL(kern, dim3(c.t.nt, c.H), dim3(256), lds, st, c);
+    MI_HIP(hipGetLastError());
+    return MI_OK;
+  };
+  const int pg = c.sk.btab == nullptr ? 0 : (c.sk.bs_shift >= 6 ? 1 : 2);
+#define GO(CAP) (pg == 0 ? go(gqa_prefill_kernel<T, KD, VD, QG, 0, CAP>) : (pg == 1 ? go(gqa_prefill_kernel<T, KD, VD, QG, 1, CAP>) : go(gqa_prefill_kernel<T, KD, VD, QG, 2, CAP>)))
+  return c.softcap > 0.f ? GO(true) : GO(false);
+#undef GO
+}
+
+template <typename T, int KD, int VD>
+int prefill_kv(const GqaCall& c, hipStream_t st) { return c.t.qt == 128 ? prefill_qg<T, KD, VD, 2>(c, st) : prefill_qg<T, KD, VD, 1>(c, st); }
+
+template <typename T, bool DECODE>
+int fast_at(const GqaCall& c, hipStream_t st) {
+#define V(KD, VD) if (c.kdp == KD && c.vdp == VD) { if constexpr (DECODE) return decode_kv<T, KD, VD>(c, st); else return prefill_kv<T, KD, VD>(c, st); }
+  V(32, 32) V(32, 64) V(32, 128) V(64, 32) V(64, 64) V(64, 128) V(128, 32) V(128, 64) V(128, 128)
+#undef V
+  return fail(MI_ERR_UNSUPPORTED, "gqa: head sizes");
+}
+
+#define BY_ACT(fn) \
+  switch (c.act) { \
+    case MI_F32: return fn<float>(c, st); \
+    case MI_BF16: return fn<bf16>(c, st); \
+    case MI_F16: return fn<f16>(c, st); \
+  } \
+  return fail(MI_ERR_INVALID, "gqa: bad dtype")
+
+int check_call(const GqaCall& c) {
+  if (c.G < 1 || c.H % c.G != 0 || c.sk.D != c.kdp || c.sv.D != c.vdp || c.sk.Hkv != c.G || c.sv.Hkv != c.G || c.kdp < c.dim || c.vdp < c.vdim)
+    return fail(MI_ERR_INVALID, "gqa: cache shape does not match the layer");
+  return MI_OK;
+}
+
+}  // namespace
+
+int gqa_pad(int n) { return n <= 32 ? 32 : (n <= 64 ? 64 : (n <= 128 ? 128 : (n + 31) / 32 * 32)); }
+bool gqa_supported(int dim, int vdim) { return dim >= 1 && vdim >= 1 && dim <= 512 && vdim <= 512; }
+bool gqa_mfma_supported(int act, int dim, int vdim) { return (act == MI_BF16 || act == MI_F16) && dim <= 128 && vdim <= 128; }
+
+int launch_gqa_pre(const GqaCall& c, hipStream_t st) { MI_TRY(check_call(c)); BY_ACT(pre_at); }
+int launch_gqa_generic(const GqaCall& c, hipStream_t st) { MI_TRY(check_call(c)); BY_ACT(generic_at); }
+int launch_gqa_decode(const GqaCall& c, hipStream_t st) {
+  MI_TRY(check_call(c));
+  if (c.nsplit < 1 || (c.nsplit > 1 && (c.partial == nullptr || c.counters == nullptr))) return fail(MI_ERR_INVALID, "gqa_decode: bad split configuration");
+  if (c.act == MI_BF16) return fast_at<bf16, true>(c, st);
+  if (c.act == MI_F16) return fast_at<f16, true>(c, st);
+  return fail(MI_ERR_UNSUPPORTED, "gqa_decode: 16-bit caches only");
+}
+int launch_gqa_prefill(const GqaCall& c, hipStream_t st) {
+  MI_TRY(check_call(c));
+  if (c.act == MI_BF16) return fast_at<bf16, false>(c, st);
+  if (c.act == MI_F16) return fast_at<f16, false>(c, st);
+  return fail(MI_ERR_UNSUPPORTED, "gqa_prefill: 16-bit caches only");
+}
+
+}  // namespace mi

@@ -26,7 +26,8 @@ struct SegTables {               // device tables of one call (engine_layers.hip
 
 struct RowNormW { const float* w; int stride; float eps; };     // stride 1: a weight per coordinate, 0: one number for all
 
-// x = table[token] (+ sinusoidal position), h = norm(x) in the activation dtype; columns [width, ld) are zero (layer_rows.hip)
+// x = table[token] (+ sinusoidal position), h = norm(x) (norm.w null: h = x) in the activation dtype; columns [width, ld) are
+// zero (layer_rows.hip)
 struct EmbedPosCall {
   SegTables t;
   const int32_t* tokens;
@@ -112,6 +113,87 @@ int launch_latent_decode(const LatentCall& c, hipStream_t st);         // one-to
 int launch_latent_gather(const LatentCall& c, void* dst, hipStream_t st);   // cached + new latents of the chunks, contiguous
 int launch_latent_prefill(const LatentCall& c, hipStream_t st);        // segments of two tokens and more
 constexpr int LATENT_GT = 64;    // keys per gather tile
+
+// Grouped-query attention without rotation (gqa.hip): q and k divided by their root mean square, scores
+//   softcap tanh(q.k scale / softcap) - slope_h (i - j),  j <= i in i's own chunk of positions,
+// values mixed with an earlier layer's of the same token, the output times sigmoid(gate) element by element.
+// K and V arenas of the layer: [place][G][..][kdp] / [vdp] as AttnShape sk / sv address them.
+struct GqaCall {
+  SegTables t;
+  AttnShape sk, sv;              // cache addressing of the keys (D = kdp) and of the values (D = vdp)
+  int H, G, dim, vdim, kdp, vdp;
+  const void* proj; int ldp;     // [R][ldp] outputs of the fused input projection
+  int o_q, o_k, o_v, o_g;
+  const float* q_norm; const float* k_norm; float eps;
+  float scale, softcap;          // softcap 0: none
+  const float* slopes;           // [H]
+  int chunk;                     // 0: causal only
+  const float* v_mix;            // weight of v_first, or null
+  const void* v_first_in;        // [R][G vdim] values of the first mixing layer (v_mix non-null)
+  void* v_first_out;             // this layer IS the first mixing layer: its values go here; or null
+  void* kcache; void* vcache;
+  void* q;                       // [R][H][kdp] normed queries (prefill, generic form)
+  int all_tokens;                // gqa_pre: also the one-token segments (generic form)
+  float* partial; int* counters; int nsplit;      // decode: [nd][H][nsplit][vdp + 2], [nd][G head tiles] zero between launches
+  void* cat; int ldc;
+  int act;
+};
+int gqa_pad(int n);                                         // padded head size in the cache
+bool gqa_mfma_supported(int act, int dim, int vdim);
+bool gqa_supported(int dim, int vdim);
+int launch_gqa_pre(const GqaCall& c, hipStream_t st);       // norms, value mix, append to the cache
+int launch_gqa_generic(const GqaCall& c, hipStream_t st);   // any size and dtype, all tokens (after gqa_pre)
+int launch_gqa_prefill(const GqaCall& c, hipStream_t st);   // segments of two tokens and more (after gqa_pre)
+int launch_gqa_decode(const GqaCall& c, hipStream_t st);    // one-token segments, norms and append included
+inline int gqa_head_tiles(int H, int G) { return (H / G + 15) / 16; }
+
+// Norm of a sublayer's output + residual update + operand of what follows (layer_rows.hip):
+//   x += norm(y) ;  h = next.w ? norm'(x) : x            kind: MI_NORM_*
+// y comes from `y` or is the weighted sum of the experts' outputs; `router` non-null: the routing of the row as well.
+struct PostNormW { const float* w; const float* b; int stride; };     // b: layer norm only
+struct RouteArgs { int experts, top, groups, keep; };
+struct PostNormCall {
+  int rows;
+  const float* y;                // [rows][ld], or null: parts
+  const void* parts;             // [rows * top (+ rows)][ld]: routed outputs of row r at r * top + j, shared ones behind them
+  const float* part_w;           // [rows][top]
+  int top, shared;
+  int kind; float eps;
+  PostNormW norm, next;
+  int width, ld;
+  float* x; void* h;
+  RouteArgs r; const void* router; int32_t* ids; float* wts;          // router [experts][ld] in the activation dtype
+  int act;
+};
+int launch_post_norm(const PostNormCall& c, hipStream_t st);
+// logits = softcap(scale * logits) in place
+int launch_logit_cap(float* logits, size_t n, float scale, float softcap, hipStream_t st);
+
+// Mixture of experts (moe.hip).  A slot is one (token, expert) pair: r * top + j for the routed ones, R * top + r for the shared.
+constexpr int MOE_MAX_EXPERTS = 512, MOE_MAX_TOP = 64;
+constexpr int MOE_STREAM_ROWS = 64;      // calls of up to so many tokens stream the weights, longer ones go through the tile GEMM
+struct MoeCall {
+  int R, width, ld;              // ld: padded width
+  RouteArgs r;
+  const float* x;                // [R][ld] residual stream (router)
+  const void* h;                 // [R][ld] the same in the activation dtype
+  const void* router;            // [experts][ld]
+  int32_t* ids; float* wts;      // [R][top]
+  LinearW gu, dn;                // routed: [experts][gate ffp | up ffp][ld], [experts][ld][ffp]
+  LinearW sgu, sdn;              // shared: [gate sffp | up sffp][ld], [ld][sffp] (sffp = 0: none)
+  int ffp, sffp, lda;            // lda: row stride of `mid`
+  void* mid;                     // [slots][lda] activations
+  void* out;                     // [slots][ld]
+  int32_t* plan;                 // moe_plan_ints() words: sorted slots, their tokens, tile table
+  int act;
+};
+size_t moe_plan_ints(int R, const RouteArgs& r, int shared);
+bool moe_mfma_supported(const MoeCall& c);
+int launch_route(const MoeCall& c, hipStream_t st);         // many rows of 16-bit models (few: launch_post_norm)
+bool route_fused(int act, int rows, int experts);           // launch_post_norm does the routing
+int launch_moe_plan(const MoeCall& c, hipStream_t st);      // many rows: order of the slots (nothing otherwise)
+int launch_moe_up(const MoeCall& c, hipStream_t st);        // mid[slot] = silu(W_gate h) * W_up h
+int launch_moe_down(const MoeCall& c, hipStream_t st);      // out[slot] = W_down mid[slot]
 
 // dst[b * db + i * di + j * dj] = src[b * sb + i * si + j * sj] for an [nb][ni][nj] box of es-byte elements
 struct PlaceCall { const void* src; void* dst; int nb, ni, nj, es; size_t sb, si, sj, db, di, dj; };

@@ -105,5 +105,56 @@ __device__ __forceinline__ void polynorm_row(const PolyNormArgs& f, const T* z, 
   if (tail < f.ff) { const float v = to_f32(z[tail]); out[tail] = from_f32<T>(((cc * v + cb) * v + ca) * v + ce); }
 }
 
+// Routing of one token by one wave: z [E] logits in LDS -> the `top` experts with the largest softmax scores among the `keep`
+// groups with the largest best score, in falling order, and their weights (scores over their sum).  `sel` / `sw`: [top] in LDS.
+// Ranks by counting: no expert or group is taken twice, ties go to the lower number.
+__device__ __forceinline__ void route_wave(const float* z, const RouteArgs& r, int* sel, float* sw, int32_t* ids, float* wts) {
+  const int lane = threadIdx.x & 63, E = r.experts, gs = E / r.groups;
+  for (int j = lane; j < r.top; j += 64) { sel[j] = j; sw[j] = 0.f; }
+  float zm = -INFINITY;
+  for (int e = lane; e < E; e += 64) zm = fmaxf(zm, z[e]);
+  zm = wave_max(zm);
+  float tot = 0.f;
+  for (int e = lane; e < E; e += 64) tot += expf(z[e] - zm);
+  tot = wave_sum(tot);
+  float chosen = 0.f;
+  for (int e0 = 0; e0 < E; e0 += 64) {                 // (uniform: the sums at the end take every lane)
+    const int e = min(e0 + lane, E - 1), g = e / gs;
+    const float ze = z[e];
+    // rank of the expert's group: groups with a larger best score, or an equal one and a lower number
+    int ahead = 0;
+    if (r.keep < r.groups) {
+      float best = -INFINITY;
+      for (int i = 0; i < gs; ++i) best = fmaxf(best, z[g * gs + i]);
+      for (int o = 0; o < r.groups; ++o) {
+        float b = -INFINITY;
+        for (int i = 0; i < gs; ++i) b = fmaxf(b, z[o * gs + i]);
+        ahead += b > best || (b == best && o < g) ? 1 : 0;
+      }
+    }
+    const bool ok = e0 + lane < E && ahead < r.keep;
+    // rank among the experts of the kept groups: a lane cannot know the others' groups cheaply, so they are marked in two steps
+    const unsigned long long m = __builtin_amdgcn_ballot_w64(ok);
+    if (lane == 0) ((unsigned long long*)(sw + r.top + (r.top & 1)))[e0 >> 6] = m;
+  }
+  const unsigned long long* kept = (const unsigned long long*)(sw + r.top + (r.top & 1));
+  for (int e0 = 0; e0 < E; e0 += 64) {
+    const int e = min(e0 + lane, E - 1);
+    const float ze = z[e];
+    int rank = e0 + lane < E && (kept[e0 >> 6] >> lane & 1) ? 0 : E;
+    for (int o = 0; o < E; ++o)
+      rank += (kept[o >> 6] >> (o & 63) & 1) && (z[o] > ze || (z[o] == ze && o < e)) ? 1 : 0;
+    if (rank < r.top) {
+      const float s = expf(ze - zm) / tot;
+      sel[rank] = e; sw[rank] = s;
+      chosen += s;
+    }
+  }
+  chosen = wave_sum(chosen) + 1e-20f;
+  for (int j = lane; j < r.top; j += 64) { ids[j] = sel[j]; wts[j] = sw[j] / chosen; }
+}
+// floats of LDS that route_wave needs behind `sel`: weights, then a bit per expert
+__host__ __device__ constexpr int route_lds_floats(int experts, int top) { return top + (top & 1) + 2 * ((experts + 63) / 64); }
+
 }  // namespace rows
 }  // namespace mi

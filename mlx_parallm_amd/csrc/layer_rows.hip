@@ -37,9 +37,15 @@ __global__ __launch_bounds__(NT) void embed_pos_kernel(EmbedPosCall c) {
     }
     *(float2*)(x + k) = v;
   }
+  T* h = (T*)c.h + (size_t)r * c.ld;
+  if (c.norm.w == nullptr) {
+    for (int k = 2 * threadIdx.x; k < c.ld; k += 2 * NT)
+#pragma unroll
+      for (int j = k; j < k + 2; ++j) h[j] = from_f32<T>(x[j]);
+    return;
+  }
   block_sum<NT, 1>(ss, red);
   const float rs = 1.0f / sqrtf(ss[0] / (float)c.width + c.norm.eps);
-  T* h = (T*)c.h + (size_t)r * c.ld;
   for (int k = 2 * threadIdx.x; k < c.ld; k += 2 * NT)          // (each thread reads what it wrote)
 #pragma unroll
     for (int j = k; j < k + 2; ++j)
@@ -345,6 +351,152 @@ int side_norm_at(const SideNormCall& c, hipStream_t st) {
   return MI_OK;
 }
 
+// ---- norm of a sublayer's output, residual update, operand of what follows: one workgroup per row ------------------------
+template <typename T>
+__device__ __forceinline__ f32x4 load4v(const T* p) {
+  const float4 v = load4f<T>(p);
+  return f32x4{v.x, v.y, v.z, v.w};
+}
+// NQ: pieces of four columns of the row per thread, held in registers (ld <= 4 NT NQ)
+template <typename T, int NT, int NQ, bool ROUTE>
+__global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
+  extern __shared__ __attribute__((aligned(16))) float smem[];      // ROUTE: [ld] the row, [experts (even)] logits, weights | marks, [top] choices
+  __shared__ float red[NT / 64];
+  const int r = blockIdx.x, tid = threadIdx.x, n4 = c.ld / 4;
+  const float inv_n = 1.0f / (float)c.width;
+  f32x4 y[NQ], x[NQ];
+  float* xg = c.x + (size_t)r * c.ld;
+#pragma unroll
+  for (int q = 0; q < NQ; ++q) {
+    const int i = min(q * NT + tid, n4 - 1);
+    x[q] = ((const f32x4*)xg)[i];
+    if (c.y != nullptr) y[q] = ((const f32x4*)(c.y + (size_t)r * c.ld))[i];
+    else {
+      const T* p = (const T*)c.parts + (size_t)r * c.top * c.ld + 4 * i;
+      const float* pw = c.part_w + (size_t)r * c.top;
+      f32x4 a = {0.f, 0.f, 0.f, 0.f};
+      if (c.shared) a = load4v<T>((const T*)c.parts + ((size_t)c.rows * c.top + r) * c.ld + 4 * i);
+#pragma unroll 4
+      for (int j = 0; j < c.top; ++j) {
+        const f32x4 v = load4v<T>(p + (size_t)j * c.ld);
+        const float w = pw[j];
+#pragma unroll
+        for (int i4 = 0; i4 < 4; ++i4) a[i4] = fmaf(w, v[i4], a[i4]);
+      }
+      y[q] = a;
+    }
+  }
+  // element k = 4 (q NT + tid) + j of the row counts when k < width
+  auto each = [&](auto f) {
+#pragma unroll
+    for (int q = 0; q < NQ; ++q)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int k = 4 * (q * NT + tid) + j;
+        if (k < c.width) f(q, j, k);
+      }
+  };
+  // v <- norm of the row: mean taken off for a layer norm, weight w, bias b
+  auto normed = [&](f32x4 (&v)[NQ], const PostNormW& n) {
+    float mean = 0.f, s[1] = {0.f};
+    if (c.kind == MI_NORM_LAYER) {
+      each([&](int q, int j, int k) { s[0] += v[q][j]; });
+      block_sum<NT, 1>(s, red);
+      mean = s[0] * inv_n;
+    }
+    s[0] = 0.f;
+    each([&](int q, int j, int k) { const float d = v[q][j] - mean; s[0] += d * d; });
+    block_sum<NT, 1>(s, red);
+    const float rs = 1.0f / sqrtf(s[0] * inv_n + c.eps);
+    each([&](int q, int j, int k) {
+      float e = (v[q][j] - mean) * rs * n.w[(size_t)k * n.stride];
+      if (n.b != nullptr) e += n.b[k];
+      v[q][j] = e;
+    });
+  };
+  normed(y, c.norm);
+  each([&](int q, int j, int k) { x[q][j] += y[q][j]; });
+#pragma unroll
+  for (int q = 0; q < NQ; ++q) {
+    const int i = q * NT + tid;
+    if (i >= n4) continue;
+    ((f32x4*)xg)[i] = x[q];
+    if constexpr (ROUTE) ((f32x4*)smem)[i] = x[q];
+  }
+  if (c.next.w != nullptr) normed(x, c.next);
+  T* h = (T*)c.h + (size_t)r * c.ld;
+#pragma unroll
+  for (int q = 0; q < NQ; ++q) {
+    const int i = q * NT + tid;
+    if (i >= n4) continue;
+    T o[4] = {from_f32<T>(x[q][0]), from_f32<T>(x[q][1]), from_f32<T>(x[q][2]), from_f32<T>(x[q][3])};
+    if constexpr (sizeof(T) == 2) *(uint2*)(h + 4 * i) = __builtin_bit_cast(uint2, o);
+    else *(f32x4*)(h + 4 * i) = x[q];
+  }
+  if constexpr (ROUTE) {
+    float* z = smem + c.ld;
+    float* sw = z + ((c.r.experts + 1) & ~1);
+    int* sel = (int*)(sw + route_lds_floats(c.r.experts, c.r.top));
+    const int lane = tid & 63, wave = tid >> 6;
+    constexpr int JB = 2;
+    __syncthreads();
+    for (int e0 = wave * JB; e0 < c.r.experts; e0 += NT / 64 * JB) {
+      float acc[JB] = {0.f, 0.f};
+      for (int k = lane * 8; k < c.ld; k += 512) {
+        float xv[8];
+        load8f<float>(smem + k, xv);
+#pragma unroll
+        for (int j = 0; j < JB; ++j) {
+          float w[8];
+          load8f<T>((const T*)c.router + (size_t)min(e0 + j, c.r.experts - 1) * c.ld + k, w);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) acc[j] = fmaf(w[i], xv[i], acc[j]);
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < JB; ++j) {
+        const float v = wave_sum(acc[j]);
+        if (lane == 0 && e0 + j < c.r.experts) z[e0 + j] = v;
+      }
+    }
+    __syncthreads();
+    if (wave == 0) route_wave(z, c.r, sel, sw, c.ids + (size_t)r * c.r.top, c.wts + (size_t)r * c.r.top);
+  }
+}
+
+template <typename T>
+int post_norm_at(const PostNormCall& c, hipStream_t st) {
+  const bool route = c.router != nullptr;
+  const size_t lds = !route ? 0 : ((size_t)c.ld + c.r.experts + 1 + route_lds_floats(c.r.experts, c.r.top) + c.r.top) * sizeof(float);
+  if (lds > 128 * 1024) return fail(MI_ERR_UNSUPPORTED, "post_norm: row too wide for the LDS");
+  auto go = [&](auto k, int nt) -> int {
+    if (lds > 65536) MI_HIP(hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+    hipLaunchKernelGGL(k, dim3(c.rows), dim3(nt), lds, st, c);
+    MI_HIP(hipGetLastError());
+    return MI_OK;
+  };
+#define PN(NT, NQ) return route ? go(post_norm_kernel<T, NT, NQ, true>, NT) : go(post_norm_kernel<T, NT, NQ, false>, NT)
+  if (c.rows < 256) {                                  // few rows: more threads for each
+    if (c.ld <= 4096) PN(1024, 1);
+    if (c.ld <= 8192) PN(1024, 2);
+    if (c.ld <= 16384) PN(1024, 4);
+  }
+  if (c.ld <= 1024) PN(256, 1);
+  if (c.ld <= 2048) PN(256, 2);
+  if (c.ld <= 4096) PN(512, 2);
+  if (c.ld <= 8192) PN(1024, 2);
+  if (c.ld <= 16384) PN(1024, 4);
+#undef PN
+  return fail(MI_ERR_UNSUPPORTED, "post_norm: rows of more than 16384 columns");
+}
+
+__global__ __launch_bounds__(256) void logit_cap_kernel(float* z, size_t n, float scale, float cap) {
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (size_t)gridDim.x * 256) {
+    const float v = z[i] * scale;
+    z[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
+  }
+}
+
 __global__ void advance_segments_kernel(SegTables t, int32_t* off) {
   const int i = blockIdx.x * 256 + threadIdx.x;
   if (i < t.n) off[t.row[i]] += t.len[i];            // (distinct rows)
@@ -386,6 +538,23 @@ int launch_side_norm(const SideNormCall& c, hipStream_t st) {
     case MI_F16: return side_norm_at<f16>(c, st);
   }
   return fail(MI_ERR_INVALID, "side_norm: bad dtype");
+}
+
+int launch_post_norm(const PostNormCall& c, hipStream_t st) {
+  if (c.ld % 8 != 0) return fail(MI_ERR_INVALID, "post_norm: row stride must be a multiple of 8");
+  switch (c.act) {
+    case MI_F32: return post_norm_at<float>(c, st);
+    case MI_BF16: return post_norm_at<bf16>(c, st);
+    case MI_F16: return post_norm_at<f16>(c, st);
+  }
+  return fail(MI_ERR_INVALID, "post_norm: bad dtype");
+}
+
+int launch_logit_cap(float* logits, size_t n, float scale, float softcap, hipStream_t st) {
+  if (n == 0 || (scale == 1.0f && softcap <= 0.f)) return MI_OK;
+  hipLaunchKernelGGL(logit_cap_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 8192)), dim3(256), 0, st, logits, n, scale, softcap);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
 }
 
 int launch_advance_segments(const SegTables& t, int32_t* off, hipStream_t st) {

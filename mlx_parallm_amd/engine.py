@@ -15,7 +15,7 @@ import numpy as np
 
 from . import _lib as L
 
-LAYER_LIST_MODELS = ("runevik",)     # described layer by layer (models/<name>.py: layer_list)
+LAYER_LIST_MODELS = ("runevik", "dolurax")     # described layer by layer (models/<name>.py: layer_list)
 _DT_NAMES = {"float32": L.MI_F32, "bfloat16": L.MI_BF16, "float16": L.MI_F16}
 
 
@@ -287,9 +287,15 @@ class Engine:
         """Bytes one block of a paged cache takes over all layers."""
         esz = 4 if kv_dtype == "float32" or self.act_dtype == "float32" else 2
         d = self.desc
-        if d.arch == L.MI_ARCH_LAYERS:           # one latent per token and layer that keeps its own (padded to 64 elements)
-            return max(1, sum((x.kv_rank + 63) // 64 * 64 for x in self.layer_descs
-                              if x.mixer == L.MI_MIXER_LATENT and x.kv_from < 0) * block_tokens * esz)
+        if d.arch == L.MI_ARCH_LAYERS:
+            def head(n):                         # padded head size of a key / value (engine_layers.hip: gqa_pad)
+                return next((p for p in (32, 64, 128) if n <= p), (n + 31) // 32 * 32)
+
+            def elements(x):                     # one latent per token (padded to 64), or the keys and values of every head
+                if x.mixer == L.MI_MIXER_LATENT:
+                    return (x.kv_rank + 63) // 64 * 64 if x.kv_from < 0 else 0
+                return x.kv_heads * (head(x.dim) + head(x.vdim)) if x.mixer == L.MI_MIXER_GQA else 0
+            return max(1, sum(map(elements, self.layer_descs)) * block_tokens * esz)
         return 2 * d.num_layers * d.num_kv_heads * block_tokens * d.head_dim * esz
 
     # -- loading
