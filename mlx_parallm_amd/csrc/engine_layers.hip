@@ -205,6 +205,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       MI_HIP(hipMalloc(&l.slopes, m.heads * sizeof(float)));
       MI_TRY(copy_in(l.slopes, slopes.data(), m.heads * sizeof(float), 0, e->stream));
       MI_HIP(hipStreamSynchronize(e->stream));
+      if (e->gqa_chunk < 0) e->gqa_chunk = m.chunk;
       l.arena_k = e->n_arena++;
       l.arena_v = e->n_arena++;
     } else return fail(MI_ERR_UNSUPPORTED, bad + "unknown mixer");
@@ -298,12 +299,20 @@ int build_tables(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t* le
     cbase[i] = (int)ct.size() / 2;
     for (int k = 0; k < lens[i]; k += DELTA_CHUNK) { ct.push_back(i); ct.push_back(k); }
   }
-  // the heaviest query tiles (latest queries) first
   int longest = 0;
   for (int i : chunk) longest = std::max(longest, lens[i]);
   t.qt = longest >= 256 ? 128 : 64;
+  if (e->gqa_chunk >= 0) t.qt = 64;              // (gqa.hip has the small tile only)
+  // the tiles with the most keys in front of them first (attention over chunks of positions: within the chunk)
+  struct Tile { int keys, seg, q; };
+  std::vector<Tile> order;
   for (int i : chunk)
-    for (int q = (lens[i] - 1) / t.qt * t.qt; q >= 0; q -= t.qt) { tile.push_back(i); tile.push_back(q); }
+    for (int q = (lens[i] - 1) / t.qt * t.qt; q >= 0; q -= t.qt) {
+      const int p0 = kv->h_off[rows[i]] + q, p1 = kv->h_off[rows[i]] + std::min(q + t.qt, lens[i]);
+      order.push_back(Tile{e->gqa_chunk > 0 ? p1 - p0 / e->gqa_chunk * e->gqa_chunk : p1, i, q});
+    }
+  std::stable_sort(order.begin(), order.end(), [](const Tile& a, const Tile& b) { return a.keys > b.keys; });
+  for (const Tile& x : order) { tile.push_back(x.seg); tile.push_back(x.q); }
   std::vector<int32_t> m;
   auto add = [&](const int32_t* p, size_t k) { const size_t at = m.size(); m.insert(m.end(), p, p + k); while (m.size() % 4) m.push_back(0); return at; };
   const size_t a_row = add(rows, n), a_t0 = add(tok0.data(), n), a_len = add(lens, n), a_kb = add(kbase.data(), n), a_cb = add(cbase.data(), n),

@@ -77,6 +77,21 @@ __device__ __forceinline__ void epi32_plain(const GemmParams& p, int m, int n, f
 }
 
 // grid: (n blocks, m blocks).  SWIGLU: a block covers 64 gate columns + the 64 matching up columns.
+__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.0f + expf(-g)) * u; }
+
+// grouped form: the matrix and the rows of tile bm of the device-resident table; false: no such tile, or no columns from n0 on
+template <typename AT, bool SWIGLU>
+__device__ __forceinline__ bool group_of_tile(GemmParams& p, int bm, int n0, int& place0) {
+  if (bm >= p.tiles[0]) return false;
+  const int32_t* t = p.tiles + 8 + 4 * bm;
+  const int grp = t[0];
+  place0 = t[1]; p.M = t[2];
+  if (grp == p.groups) { p.w = p.w_last; p.N = p.N_last; p.K = p.ka = p.kw = p.K_last; }
+  else p.w = (const char*)p.w + (size_t)grp * p.N * p.K * sizeof(AT);
+  if constexpr (SWIGLU) p.pair_offset = p.N / 2;
+  return n0 < (SWIGLU ? p.pair_offset : p.N);
+}
+
 // GROUPED: blockIdx.x = tile of the device-resident table; every group of rows has its own matrix (GroupedGemm, kernels.h)
 template <typename AT, bool SWIGLU, bool GROUPED = false>
 __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
@@ -89,14 +104,8 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   const int bm = blockIdx.x, bn = blockIdx.y;
   int m0 = bm * BM, place0 = 0;
   if constexpr (GROUPED) {
-    if (bm >= p.tiles[0]) return;
-    const int32_t* t = p.tiles + 8 + 4 * bm;
-    const int grp = t[0];
-    place0 = t[1]; m0 = 0; p.M = t[2];
-    if (grp == p.groups) { p.w = p.w_last; p.N = p.N_last; p.K = p.ka = p.kw = p.K_last; }
-    else p.w = (const char*)p.w + (size_t)grp * p.N * p.K * sizeof(AT);
-    if constexpr (SWIGLU) p.pair_offset = p.N / 2;
-    if (bn * (SWIGLU ? 64 : BN) >= (SWIGLU ? p.pair_offset : p.N)) return;
+    if (!group_of_tile<AT, SWIGLU>(p, bm, bn * (SWIGLU ? 64 : BN), place0)) return;
+    m0 = 0;
   }
   const int nk_all = p.K / BK, nkw = p.kw / BK;
   const int ks0 = (int)(((long)blockIdx.z * nk_all) / p.ksplit), ks1 = (int)(((long)(blockIdx.z + 1) * nk_all) / p.ksplit);
@@ -143,6 +152,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
       *(u32x4*)&As[buf][row][kq * 8] = aok[i] ? areg[i] : u32x4{0u, 0u, 0u, 0u};
     }
   };
+  const bool live = !GROUPED || wm * 64 < p.M;     // (grouped: a short tile leaves half of the waves without rows)
   u32x4 breg[3][4][2];     // [set][n tile][k block]; W fragments are fetched two K steps ahead
   auto load_b = [&](int set, int ks) {
 #pragma unroll
@@ -166,8 +176,9 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
     constexpr int SET = decltype(set_tag)::value;
     const int cur = (ks - ks0) & 1;
     load_a(min(ks + 1, nk - 1));
-    load_b((SET + 2) % 3, min(ks + 2, nk - 1));
+    if (live) load_b((SET + 2) % 3, min(ks + 2, nk - 1));
     __builtin_amdgcn_sched_barrier(0);           // the loads stay ahead of this step's MFMAs
+    if (live)
 #pragma unroll
     for (int kb = 0; kb < 2; ++kb) {
       u32x4 af[4];
@@ -222,11 +233,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
         for (int j = 0; j < 2; ++j) {
           const int n = bn * 64 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
-          if constexpr (GROUPED) {
-            const float gt = acc[mt][j][r];
-            out[(size_t)m * p.ldo + n] = (AT)(gt / (1.0f + expf(-gt)) * acc[mt][j + 2][r]);
-            continue;
-          }
+          if constexpr (GROUPED) { out[(size_t)m * p.ldo + n] = (AT)silu_mul(acc[mt][j][r], acc[mt][j + 2][r]); continue; }
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
           const float gt = (float)(AT)acc[mt][j][r], up = (float)(AT)acc[mt][j + 2][r];
           const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
@@ -308,6 +315,44 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
         }
       }
     }
+}
+
+// Grouped form: whole rows.  A wave's tile goes through its own strip of LDS, 64 rows at a time, and leaves it as 16-byte pieces of
+// rows (out_rows may scatter them): 16 stores per wave instead of 128.  The LDS must be free (every DMA landed, every read done).
+template <typename AT, bool SWIGLU>
+__device__ __forceinline__ void tile256_epilogue_rows(const GemmParams& p, f32x4 (&acc)[8][4], unsigned char* lds, int bn, int wave, int lane, int place0) {
+  constexpr int WC = SWIGLU ? 32 : 64, LDW = WC + 8, NP = WC / 8;
+  const int wm = wave >> 2, wn = wave & 3, c16 = lane & 15, g = lane >> 4;
+  AT* strip = (AT*)lds + (size_t)wave * 64 * LDW;
+  const int n0 = bn * 4 * WC + wn * WC, cols = SWIGLU ? p.pair_offset : p.N;
+#pragma unroll
+  for (int hf = 0; hf < 2; ++hf) {
+#pragma unroll
+    for (int mt = 0; mt < 4; ++mt)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        AT* row = strip + (mt * 16 + 4 * g + r) * LDW + c16;
+        const f32x4 (&a)[4] = acc[hf * 4 + mt];
+        if constexpr (SWIGLU) {
+#pragma unroll
+          for (int j = 0; j < 2; ++j) row[j * 16] = (AT)silu_mul(a[j][r], a[j + 2][r]);
+        } else {
+#pragma unroll
+          for (int nt = 0; nt < 4; ++nt) row[nt * 16] = (AT)a[nt][r];
+        }
+      }
+    asm volatile("" ::: "memory");                     // (a wave's LDS operations complete in order)
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int piece = i * 64 + lane, row = piece / NP, c8 = piece % NP, m = wm * 128 + hf * 64 + row, n = n0 + c8 * 8;
+      if (m >= p.M || n >= cols) continue;
+      const int orow = p.out_rows != nullptr ? p.out_rows[place0 + m] : place0 + m;
+      *(u32x4*)((AT*)p.out + (size_t)orow * p.ldo + n) = *(const u32x4*)(strip + row * LDW + c8 * 8);
+    }
+    asm volatile("" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+  }
 }
 
 // The residual epilogue (h += y in place) with the loads of h batched: written as in tile256_epilogue every load of
@@ -582,14 +627,19 @@ __device__ __forceinline__ void dma_kib(const void* gsrc, unsigned lds_dst) {
 }
 typedef __attribute__((address_space(3))) u32x4 lds_u32x4_t;
 
-template <typename AT, bool SWIGLU>
+// GROUPED: as in gemm_tile_kernel
+template <typename AT, bool SWIGLU, bool GROUPED = false>
 __global__ __launch_bounds__(512) void gemm_dma256_kernel(GemmParams p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem2[];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int wm = wave >> 2, wn = wave & 3;              // 2 x 4 waves
   const int c16 = lane & 15, g = lane >> 4;
   const int bm = blockIdx.x, bn = blockIdx.y;
-  const int m0 = bm * BM2;
+  int m0 = bm * BM2, place0 = 0;
+  if constexpr (GROUPED) {
+    if (!group_of_tile<AT, SWIGLU>(p, bm, bn * (SWIGLU ? 128 : BN2), place0)) return;
+    m0 = 0;
+  }
   // K split over gridDim.z workgroups (a prompt of 256..4095 rows against N = 4096: the (M, N) grid alone leaves most CUs
   // idle): slice z multiplies the K tiles [tb, tb + nk) and leaves its float32 partial tile in ws[z][M][N];
   // splitk_epilogue_kernel adds the slices in order and applies the epilogue (host: >= 2 tiles per slice)
@@ -618,7 +668,9 @@ __global__ __launch_bounds__(512) void gemm_dma256_kernel(GemmParams p) {
       const int ir = (2 * wave + i) * 8 + 2 * rl + (col >> 3);            // image row of the unit: wm' * 64 + r
       const int q = (col & 7) ^ (4 * i + rl);
       const int row = (ir >> 6) * 128 + h * 64 + (ir & 63);                 // row of the 256-row tile
-      asrc[h][i] = (const char*)p.x + ((size_t)min(m0 + row, p.M - 1) * p.ldx + q * 8) * sizeof(AT);
+      int xr = min(m0 + row, p.M - 1);
+      if constexpr (GROUPED) { xr += place0; if (p.x_rows != nullptr) xr = p.x_rows[xr]; }
+      asrc[h][i] = (const char*)p.x + ((size_t)xr * p.ldx + q * 8) * sizeof(AT);
     }
   const char* bsrc[2];                                                     // B unit: fragment slots 2 wave, 2 wave + 1
 #pragma unroll
@@ -733,7 +785,10 @@ __global__ __launch_bounds__(512) void gemm_dma256_kernel(GemmParams p) {
       return;
     }
   }
-  tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  if constexpr (GROUPED) {
+    __syncthreads();
+    tile256_epilogue_rows<AT, SWIGLU>(p, acc, smem2, bn, wave, lane, place0);
+  } else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
 }
 
 
@@ -1283,7 +1338,7 @@ int launch_gemm_prefill(const LinearW& W, const GemvCall& c, size_t rows, hipStr
 int launch_gemm_grouped(const GroupedGemm& g, hipStream_t st) {
   const bool dense = (g.W.wk == WK_BF16 && g.act == MI_BF16) || (g.W.wk == WK_F16 && g.act == MI_F16);
   const bool last = g.last.w != nullptr;
-  if (!dense || g.W.layout != 1 || g.W.K % BK != 0 || g.ldx % 8 != 0 || g.rows % 32 != 0 || g.W.N != g.rows * g.groups ||
+  if (!dense || g.W.layout != 1 || g.W.K % BK != 0 || g.ldx % 8 != 0 || g.ldo % 8 != 0 || g.rows % 32 != 0 || g.W.N != g.rows * g.groups ||
       (last && (g.last.wk != g.W.wk || g.last.layout != 1 || g.last.K % BK != 0 || g.last.N % 32 != 0)))
     return fail(MI_ERR_UNSUPPORTED, "gemm_grouped: shape / layout not supported");
   GemmParams p{};
@@ -1293,6 +1348,19 @@ int launch_gemm_grouped(const GroupedGemm& g, hipStream_t st) {
   p.tiles = g.tiles; p.x_rows = g.x_rows; p.out_rows = g.out_rows; p.groups = g.groups;
   p.w_last = g.last.w; p.N_last = last ? g.last.N : 0; p.K_last = last ? g.last.K : 0;
   const int cols = std::max(g.rows, p.N_last) / (g.swiglu ? 2 : 1);
+  if (g.tile == BM2) {
+    if (g.W.K < 2 * BK || (last && g.last.K < 2 * BK)) return fail(MI_ERR_UNSUPPORTED, "gemm_grouped: the 256 x 256 tile needs two K tiles");
+    const dim3 grid(g.max_tiles, (cols + (g.swiglu ? 128 : BN2) - 1) / (g.swiglu ? 128 : BN2)), block(512);
+    auto go = [&](auto k) -> int {
+      MI_HIP(hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, 2 * DMA_BUF));
+      hipLaunchKernelGGL(k, grid, block, 2 * DMA_BUF, st, p);
+      MI_HIP(hipGetLastError());
+      return MI_OK;
+    };
+    if (g.act == MI_BF16) return g.swiglu ? go(gemm_dma256_kernel<bf16, true, true>) : go(gemm_dma256_kernel<bf16, false, true>);
+    return g.swiglu ? go(gemm_dma256_kernel<f16, true, true>) : go(gemm_dma256_kernel<f16, false, true>);
+  }
+  if (g.tile != BM) return fail(MI_ERR_INVALID, "gemm_grouped: tiles of 128 or 256 places");
   const dim3 grid(g.max_tiles, (cols + (g.swiglu ? 64 : BN) - 1) / (g.swiglu ? 64 : BN)), block(256);
   if (g.act == MI_BF16) {
     if (g.swiglu) hipLaunchKernelGGL((gemm_tile_kernel<bf16, true, true>), grid, block, 0, st, p);

@@ -184,11 +184,12 @@ __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
 // two float32 values as hi + lo pairs of 16-bit values (softmax weights keep 32-bit accuracy through two MFMAs)
 template <typename T>
 __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  const T ha = (T)a, hb = (T)b;
-  T h[2] = {ha, hb};
-  T l[2] = {(T)(a - (float)ha), (T)(b - (float)hb)};
+  typedef float f32x2 __attribute__((ext_vector_type(2)));
+  typedef T tx2 __attribute__((ext_vector_type(2)));
+  const tx2 h = __builtin_convertvector((f32x2{a, b}), tx2);
+  const f32x2 back = __builtin_convertvector(h, f32x2);
   hi = __builtin_bit_cast(uint32_t, h);
-  lo = __builtin_bit_cast(uint32_t, l);
+  lo = __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2{a - back[0], b - back[1]}), tx2));
 }
 
 // A score in the exp2 domain: LOG2E (softcap tanh(s scale / softcap) + bias); bias in the exp2 domain, with the cap's constant
@@ -202,6 +203,35 @@ template <bool CAP>
 __device__ __forceinline__ float score2(const ScoreScale& k, float s, float bias) {
   if constexpr (CAP) return fmaf(k.b, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * k.a) + 1.0f), bias);
   else return fmaf(s, k.a, bias);
+}
+
+// 1 / (1 + e^-z) on the hardware's exponential and reciprocal (a last bit each)
+__device__ __forceinline__ float gate_f(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-LOG2E * z)); }
+
+// How many keys back the distance bias leaves anything: a capped score is at most softcap and the token's own at least -softcap, so
+// a key further away than this has a weight below 2^-40 of the token's own -- nothing in a float32 sum
+__device__ __forceinline__ int key_reach(const GqaCall& c, float slope2) {
+  if (c.softcap <= 0.f || slope2 <= 0.f) return 1 << 30;
+  return (int)fminf((2.0f * LOG2E * c.softcap + 40.0f) / slope2, 1e9f) + 1;
+}
+
+// The same for a block whose scores all stay below 0.6 softcap / scale: softcap tanh(s scale / softcap) = s P(s^2), P a polynomial
+// (least-squares fit of tanh(u) / u at Chebyshev points, |u| <= 0.6: relative error 1.6e-7) -- no transcendentals
+struct CapPoly { float c[5], lim; };
+__device__ __forceinline__ CapPoly cap_poly(const GqaCall& c) {
+  const float f = c.scale / c.softcap, f2 = f * f;
+  CapPoly k;
+  k.c[0] = c.scale * LOG2E;
+  k.c[1] = -0.33332324028015137f * f2 * k.c[0];
+  k.c[2] = 0.13310357928276062f * f2 * f2 * k.c[0];
+  k.c[3] = -0.052109625190496445f * f2 * f2 * f2 * k.c[0];
+  k.c[4] = 0.01548669021576643f * f2 * f2 * f2 * f2 * k.c[0];
+  k.lim = 0.6f / fabsf(f);
+  return k;
+}
+__device__ __forceinline__ float score_poly(const CapPoly& k, float s, float bias) {
+  const float w = s * s;
+  return fmaf(s, fmaf(fmaf(fmaf(fmaf(k.c[4], w, k.c[3]), w, k.c[2]), w, k.c[1]), w, k.c[0]), bias);
 }
 
 // grid (nsplit, G x head tiles, nd), 4 waves; a wave walks its 32-key blocks on its own, the next block's loads in flight during
@@ -221,7 +251,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   const int split = blockIdx.x, kh = blockIdx.y / ht_n, ht = blockIdx.y % ht_n, m = blockIdx.z;
   const int seg = c.t.dec[m], row = c.t.row[seg], tok = c.t.tok0[seg], pos = c.t.off[row];
   const int h0 = kh * rep + ht * 16, nh = min(16, rep - ht * 16);
-  const int lo = chunk_start(pos, c.chunk);          // cached keys [lo, pos)
+  const int lo = max(chunk_start(pos, c.chunk), pos - key_reach(c, c.slopes[h0 + nh - 1] * LOG2E));     // cached keys [lo, pos) (the slopes fall)
   const int blk0 = lo / KB, nblk = pos > lo ? (pos + KB - 1) / KB - blk0 : 0, per = (nblk + c.nsplit - 1) / c.nsplit;
   const int b0 = blk0 + split * per, b1 = min(b0 + per, blk0 + nblk);
   const T* kc = (const T*)c.kcache;
@@ -386,7 +416,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
     }
     const int h = h0 + hh;
     if (c.nsplit == 1) {
-      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * sigmoid_f(to_f32(gate[h * c.vdim + d])));
+      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(to_f32(gate[h * c.vdim + d])));
     } else {
       float* pp = pp0 + ((size_t)h * c.nsplit + split) * (VD + 2);
       __hip_atomic_store(&pp[2 + d], O, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -430,64 +460,88 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
           mn = bm;
         }
     }
-    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * sigmoid_f(to_f32(gate[h * c.vdim + d])));
+    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(to_f32(gate[h * c.vdim + d])));
   }
 }
 
-// grid (query tiles, H), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys, two LDS
-// buffers, the next block's global loads in flight during the current block's MFMAs.
+// grid (H, query tiles), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys from the
+// tile's last one downwards, two LDS buffers, the next block's global loads in flight during the current block's MFMAs.
+// Downwards because of the distance bias: the running maximum is found in the first block and seldom moves.  It lags: a block's
+// weights are taken relative to the maximum of the blocks before it, and only a score more than 8 (a factor 256) above that makes
+// the wave find the new maximum and rescale -- no cross-lane step in most blocks.
+// LDS images, XOR-ed so that the 16-byte writes of consecutive lanes hit different banks:
+//   K [16-key tile][kk][g][key ^ (4 kk + g)] x 16 B     V [32 keys][16-value tile dt][key ^ (dt & 7)] x 32 B
 // PG: 0 contiguous cache, 1 pages of 64 tokens and more (one page per block of keys), 2 smaller pages
 template <typename T, int KD, int VD, int QG, int PG, bool CAP>
 __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
   constexpr int KB = 64, KK = KD / 32, DT = VD / 16, KT = KB / 16, KIMG = KB * KD * 2, VIMG = KB * VD * 2;
   constexpr int NKP = KB * KD / 8 / 256, NVP = KB * VD / 8 / 256;      // 16-byte pieces per thread
+  constexpr float UNSET = -1e30f, LAG = 8.0f;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];  // K[2], V[2]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
-  const int seg = c.t.tile[2 * blockIdx.x], t0 = c.t.tile[2 * blockIdx.x + 1], h = blockIdx.y, kh = h / (c.H / c.G);
+  const int seg = c.t.tile[2 * blockIdx.y], t0 = c.t.tile[2 * blockIdx.y + 1], h = blockIdx.x, kh = h / (c.H / c.G);
   const int row = c.t.row[seg], len = c.t.len[seg], off = c.t.off[row], tok0 = c.t.tok0[seg];
-  const int nk = off + min(t0 + 64 * QG, len);       // keys any query of the tile may see: [chunk of the first query, nk)
-  const int nb = (nk + KB - 1) / KB, j0 = chunk_start(off + t0, c.chunk) / KB;
+  const float slope2 = c.slopes[h] * LOG2E;
+  const int nk = off + min(t0 + 64 * QG, len);       // keys any query of the tile may see: [first, nk)
+  const int first = max(chunk_start(off + t0, c.chunk), off + t0 - key_reach(c, slope2));
+  const int jlast = (nk - 1) / KB, jfirst = first / KB;
   const T* kc = (const T*)c.kcache;
   const T* vc = (const T*)c.vcache;
   auto kimg = [&](int b) { return smem + b * KIMG; };
   auto vimg = [&](int b) { return smem + 2 * KIMG + b * VIMG; };
 
-  // page of key block j (PG 1): looked up one block ahead of its loads
+  // key block j of the cache: element of its first key (PG 0, 1); `page` is looked up one block ahead of its use
   const int32_t* btab = PG ? c.sk.btab + (size_t)row * c.sk.bt_stride : nullptr;
   int page = 0;
-  auto find_page = [&](int j) { if constexpr (PG == 1) page = btab[min(j * KB, nk - 1) >> c.sk.bs_shift]; };
-  u32x4 kreg[NKP], vreg[NVP];
-  auto elem = [&](const AttnShape& s, int key) -> size_t {
-    if constexpr (PG == 1) return (((((size_t)page * s.Hkv + kh) << s.bs_shift) + (size_t)(key & ((1 << s.bs_shift) - 1))) * s.D);
-    else return kv_elem<PG != 0>(s, row, kh, key);
+  auto find_page = [&](int j) { if constexpr (PG == 1) page = __builtin_amdgcn_readfirstlane(btab[(max(j, jfirst) * KB) >> c.sk.bs_shift]); };
+  auto block_at = [&](const AttnShape& s, int j) -> size_t {
+    if constexpr (PG == 0) return (((size_t)row * s.Hkv + kh) * s.cap + (size_t)j * KB) * s.D;
+    else return ((((size_t)page * s.Hkv + kh) << s.bs_shift) + (size_t)((j * KB) & ((1 << s.bs_shift) - 1))) * s.D;
   };
-  auto load_block = [&](int j) {
+  u32x4 kreg[NKP], vreg[NVP];
+  auto load_block = [&](int j) {                     // (keys beyond nk are read as the last one: the cache may end there)
+    const int top = min(nk - 1 - j * KB, KB - 1);
+    if constexpr (PG == 2) {
 #pragma unroll
-    for (int i = 0; i < NKP; ++i) {
-      const int piece = i * 256 + tid;
-      kreg[i] = *(const u32x4*)(kc + elem(c.sk, min(j * KB + piece / (KD / 8), nk - 1)) + 8 * (piece % (KD / 8)));
-    }
+      for (int i = 0; i < NKP; ++i) {
+        const int piece = i * 256 + tid;
+        kreg[i] = *(const u32x4*)(kc + kv_elem<true>(c.sk, row, kh, j * KB + min(piece / (KD / 8), top)) + 8 * (piece % (KD / 8)));
+      }
 #pragma unroll
-    for (int i = 0; i < NVP; ++i) {
-      const int piece = i * 256 + tid;
-      vreg[i] = *(const u32x4*)(vc + elem(c.sv, min(j * KB + piece / (VD / 8), nk - 1)) + 8 * (piece % (VD / 8)));
+      for (int i = 0; i < NVP; ++i) {
+        const int piece = i * 256 + tid;
+        vreg[i] = *(const u32x4*)(vc + kv_elem<true>(c.sv, row, kh, j * KB + min(piece / (VD / 8), top)) + 8 * (piece % (VD / 8)));
+      }
+    } else {
+      const T* kb = kc + block_at(c.sk, j);
+      const T* vb = vc + block_at(c.sv, j);
+#pragma unroll
+      for (int i = 0; i < NKP; ++i) {
+        const int piece = i * 256 + tid, key = min(piece / (KD / 8), top);
+        kreg[i] = *(const u32x4*)(kb + key * KD + 8 * (piece % (KD / 8)));
+      }
+#pragma unroll
+      for (int i = 0; i < NVP; ++i) {
+        const int piece = i * 256 + tid, key = min(piece / (VD / 8), top);
+        vreg[i] = *(const u32x4*)(vb + key * VD + 8 * (piece % (VD / 8)));
+      }
     }
   };
   auto store_block = [&](int buf) {
 #pragma unroll
     for (int i = 0; i < NKP; ++i) {
       const int piece = i * 256 + tid, key = piece / (KD / 8), dc = piece % (KD / 8);
-      *(u32x4*)(kimg(buf) + ((((key >> 4) * KK + (dc >> 2)) * 4 + (dc & 3)) * 16 + (key & 15)) * 16) = kreg[i];
+      *(u32x4*)(kimg(buf) + (((key >> 4) * KK * 4 + dc) * 16 + ((key ^ dc) & 15)) * 16) = kreg[i];
     }
 #pragma unroll
     for (int i = 0; i < NVP; ++i) {
       const int piece = i * 256 + tid, key = piece / (VD / 8), dc = piece % (VD / 8);
-      *(u32x4*)(vimg(buf) + (size_t)((key >> 5) * DT + (dc >> 1)) * (32 * 32) + (key & 31) * 32 + (dc & 1) * 16) = vreg[i];
+      *(u32x4*)(vimg(buf) + (size_t)((key >> 5) * DT + (dc >> 1)) * (32 * 32) + ((key & 31) ^ ((dc >> 1) & 7)) * 32 + (dc & 1) * 16) = vreg[i];
     }
   };
-  find_page(j0);
-  load_block(j0);
-  find_page(j0 + 1);
+  find_page(jlast);
+  load_block(jlast);
+  find_page(jlast - 1);
   u32x4 qf[QG][KK];
   int tq[QG], lo[QG];                                // this lane's query of group u and the first key of its chunk
 #pragma unroll
@@ -505,19 +559,21 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
     for (int kk = 0; kk < KK; ++kk) asm volatile("" :: "v"(qf[u][kk]));      // (loaded from here on: no wait carried round the loop)
   __syncthreads();
   const ScoreScale ks = score_scale(c);
-  const float slope2 = c.slopes[h] * LOG2E;
+  CapPoly kp{};
+  if constexpr (CAP) kp = cap_poly(c);
   float m_run[QG], l_run[QG];
   f32x4 acc[QG][DT];
 #pragma unroll
   for (int u = 0; u < QG; ++u) {
-    m_run[u] = -1e30f; l_run[u] = 0.f;
+    m_run[u] = UNSET; l_run[u] = 0.f;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc[u][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const int tq4 = c16 >> 2, tp = c16 & 3;
-  for (int j = j0; j < nb; ++j) {
-    const int buf = (j - j0) & 1;
-    if (j + 1 < nb) { load_block(j + 1); find_page(j + 2); }
+  for (int j = jlast; j >= jfirst; --j) {
+    const int buf = (jlast - j) & 1;
+    load_block(max(j - 1, jfirst));               // straight-line (in front of the first block: that block again, not stored): a
+    find_page(j - 2);                                    // conditional load would make the compiler wait for all loads at the loop's head
     f32x4 sc[QG][KT];
 #pragma unroll
     for (int t = 0; t < KT; ++t) {
@@ -525,7 +581,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
       for (int u = 0; u < QG; ++u) sc[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < KK; ++kk) {
-        const u32x4 kf = *(const u32x4*)(kimg(buf) + (((t * KK + kk) * 4 + g4) * 16 + c16) * 16);
+        const u32x4 kf = *(const u32x4*)(kimg(buf) + (((t * KK + kk) * 4 + g4) * 16 + (c16 ^ ((4 * kk + g4) & 15))) * 16);
 #pragma unroll
         for (int u = 0; u < QG; ++u) sc[u][t] = mfma16<T>(kf, qf[u][kk], sc[u][t]);
       }
@@ -534,12 +590,29 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 #pragma unroll
     for (int u = 0; u < QG; ++u) {
       const int q0 = off + t0 + (wave * QG + u) * 16;    // position of the group's first query
-      const float bias0 = fmaf(slope2, (float)(j * KB + 4 * g4 - (q0 + c16)), ks.c0);
-      float mx = -INFINITY;
+      // scores relative to the running maximum
+      const float ref = m_run[u] == UNSET ? 0.f : m_run[u];
+      const float bias0 = fmaf(slope2, (float)(j * KB + 4 * g4 - (q0 + c16)), -ref);
+      bool small = CAP;
+      if constexpr (CAP) {
+        float am = 0.f;
 #pragma unroll
-      for (int t = 0; t < KT; ++t)
+        for (int t = 0; t < KT; ++t)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) sc[u][t][r] = score2<CAP>(ks, sc[u][t][r], fmaf(slope2, (float)(16 * t + r), bias0));
+          for (int r = 0; r < 4; ++r) am = fmaxf(am, fabsf(sc[u][t][r]));
+        small = __builtin_amdgcn_ballot_w64(am > kp.lim) == 0;
+      }
+      if (small) {
+#pragma unroll
+        for (int t = 0; t < KT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sc[u][t][r] = score_poly(kp, sc[u][t][r], fmaf(slope2, (float)(16 * t + r), bias0));
+      } else {
+#pragma unroll
+        for (int t = 0; t < KT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sc[u][t][r] = score2<CAP>(ks, sc[u][t][r], fmaf(slope2, (float)(16 * t + r), bias0 + ks.c0));
+      }
       // a block that reaches past the first query, or in front of the last query's chunk (uniform)
       if (j * KB + KB - 1 > q0 || (c.chunk > 0 && j * KB < chunk_start(q0 + 15, c.chunk))) {
 #pragma unroll
@@ -550,19 +623,24 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
             sc[u][t][r] = key <= q0 + c16 && key >= lo[u] ? sc[u][t][r] : -INFINITY;
           }
       }
+      float mx = -INFINITY;
 #pragma unroll
       for (int t = 0; t < KT; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) mx = fmaxf(mx, sc[u][t][r]);
-      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m_run[u], mx);
-      if (__builtin_amdgcn_ballot_w64(mn != m_run[u]) != 0) {
-        const float corr = __builtin_amdgcn_exp2f(m_run[u] - mn);
+      if (__builtin_amdgcn_ballot_w64(mx > LAG || m_run[u] == UNSET) != 0) {
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float mn = fmaxf(m_run[u], ref + mx);                    // (UNSET while the query has seen no key)
+        const float corr = __builtin_amdgcn_exp2f(m_run[u] - mn), d = (mn == UNSET ? 0.f : mn) - ref;
         m_run[u] = mn;
         l_run[u] *= corr;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) acc[u][dt] *= corr;
+#pragma unroll
+        for (int t = 0; t < KT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sc[u][t][r] -= d;
       }
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf) {
@@ -571,7 +649,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
         for (int t = 0; t < 2; ++t) {
           float p[4];
 #pragma unroll
-          for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(sc[u][2 * hf + t][r] - mn); l_run[u] += p[r]; }
+          for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(sc[u][2 * hf + t][r]); l_run[u] += p[r]; }
           split2<T>(p[0], p[1], ph[2 * t], pw[2 * t]);
           split2<T>(p[2], p[3], ph[2 * t + 1], pw[2 * t + 1]);
         }
@@ -583,45 +661,52 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
     for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
-        const unsigned char* a0 = vimg(buf) + (size_t)(hf * DT + dt) * (32 * 32) + (4 * g4 + tq4) * 32 + tp * 8;
+        const unsigned char* a0 = vimg(buf) + (size_t)(hf * DT + dt) * (32 * 32) + ((4 * g4 + tq4) ^ (dt & 7)) * 32 + tp * 8;
         const s16x4 v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a0);
         const s16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a0 + 16 * 32));
         const uint32_t* w0 = (const uint32_t*)&v0;
         const uint32_t* w1 = (const uint32_t*)&v1;
         const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
 #pragma unroll
-        for (int u = 0; u < QG; ++u) {
-          acc[u][dt] = mfma16<T>(vf, pf[u][hf], acc[u][dt]);
-          acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
-        }
+        for (int u = 0; u < QG; ++u) acc[u][dt] = mfma16<T>(vf, pf[u][hf], acc[u][dt]);
+#pragma unroll
+        for (int u = 0; u < QG; ++u) acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
       }
-    if (j + 1 < nb) store_block(buf ^ 1);                // the other buffer: nobody reads it during this block
+    if (j > jfirst) store_block(buf ^ 1);                // the other buffer: nobody reads it during this block
     __syncthreads();
   }
+  // output: the gates of a query are fetched in one round trip
 #pragma unroll
   for (int u = 0; u < QG; ++u) {
     float l = l_run[u];
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
-    if (tq[u] >= len) continue;
-    const int tok = tok0 + tq[u];
+    const int tok = tok0 + min(tq[u], len - 1);
     const float inv = 1.0f / l;
     const T* gate = (const T*)c.proj + (size_t)tok * c.ldp + c.o_g + h * c.vdim;
     T* o = (T*)c.cat + (size_t)tok * c.ldc + h * c.vdim;
+    if (c.vdim % 4 == 0) {
+      uint2 gt[DT];
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      const int k = 16 * dt + 4 * g4;
-      if (c.vdim % 4 == 0) {
-        if (k < c.vdim) {
-          const float4 gt = load4f<T>(gate + k);
-          T v[4] = {(T)(acc[u][dt][0] * inv * sigmoid_f(gt.x)), (T)(acc[u][dt][1] * inv * sigmoid_f(gt.y)),
-                    (T)(acc[u][dt][2] * inv * sigmoid_f(gt.z)), (T)(acc[u][dt][3] * inv * sigmoid_f(gt.w))};
-          *(uint2*)(o + k) = __builtin_bit_cast(uint2, v);
-        }
-      } else {
+      for (int dt = 0; dt < DT; ++dt) gt[dt] = *(const uint2*)(gate + min(16 * dt + 4 * g4, c.vdim - 4));
+      if (tq[u] >= len) continue;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) if (k + r < c.vdim) o[k + r] = (T)(acc[u][dt][r] * inv * sigmoid_f(to_f32(gate[k + r])));
+      for (int dt = 0; dt < DT; ++dt) {
+        const int k = 16 * dt + 4 * g4;
+        const T* ge = (const T*)&gt[dt];
+        T v[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = (T)(acc[u][dt][r] * inv * gate_f(to_f32(ge[r])));
+        if (k < c.vdim) *(uint2*)(o + k) = __builtin_bit_cast(uint2, v);
       }
+    } else if (tq[u] < len) {
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int k = 16 * dt + 4 * g4 + r;
+          if (k < c.vdim) o[k] = (T)(acc[u][dt][r] * inv * gate_f(to_f32(gate[k])));
+        }
     }
   }
 }
@@ -661,23 +746,20 @@ int decode_kv(const GqaCall& c, hipStream_t st) {
   return c.sk.btab ? go(gqa_decode_kernel<T, KD, VD, true, false>) : go(gqa_decode_kernel<T, KD, VD, false, false>);
 }
 
-template <typename T, int KD, int VD, int QG>
-int prefill_qg(const GqaCall& c, hipStream_t st) {
+template <typename T, int KD, int VD>
+int prefill_kv(const GqaCall& c, hipStream_t st) {
   constexpr int lds = 2 * 64 * (KD + VD) * 2;
   auto go = [&](auto kern) -> int {
     MI_HIP(hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-    hipLaunchKernelGGL(kern, dim3(c.t.nt, c.H), dim3(256), lds, st, c);
+    hipLaunchKernelGGL(kern, dim3(c.H, c.t.nt), dim3(256), lds, st, c);
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
   const int pg = c.sk.btab == nullptr ? 0 : (c.sk.bs_shift >= 6 ? 1 : 2);
-#define GO(CAP) (pg == 0 ? go(gqa_prefill_kernel<T, KD, VD, QG, 0, CAP>) : (pg == 1 ? go(gqa_prefill_kernel<T, KD, VD, QG, 1, CAP>) : go(gqa_prefill_kernel<T, KD, VD, QG, 2, CAP>)))
+#define GO(CAP) (pg == 0 ? go(gqa_prefill_kernel<T, KD, VD, 1, 0, CAP>) : (pg == 1 ? go(gqa_prefill_kernel<T, KD, VD, 1, 1, CAP>) : go(gqa_prefill_kernel<T, KD, VD, 1, 2, CAP>)))
   return c.softcap > 0.f ? GO(true) : GO(false);
 #undef GO
 }
-
-template <typename T, int KD, int VD>
-int prefill_kv(const GqaCall& c, hipStream_t st) { return c.t.qt == 128 ? prefill_qg<T, KD, VD, 2>(c, st) : prefill_qg<T, KD, VD, 1>(c, st); }
 
 template <typename T, bool DECODE>
 int fast_at(const GqaCall& c, hipStream_t st) {
@@ -718,6 +800,7 @@ int launch_gqa_decode(const GqaCall& c, hipStream_t st) {
 }
 int launch_gqa_prefill(const GqaCall& c, hipStream_t st) {
   MI_TRY(check_call(c));
+  if (c.t.qt != 64) return fail(MI_ERR_INVALID, "gqa_prefill: tiles of 64 queries");
   if (c.act == MI_BF16) return fast_at<bf16, false>(c, st);
   if (c.act == MI_F16) return fast_at<f16, false>(c, st);
   return fail(MI_ERR_UNSUPPORTED, "gqa_prefill: 16-bit caches only");

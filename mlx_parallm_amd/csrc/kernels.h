@@ -85,17 +85,17 @@ bool gemm_prefill_supported(const LinearW& W, const GemvCall& c, size_t rows);
 // matrix); null = never split
 int launch_gemm_prefill(const LinearW& W, const GemvCall& c, size_t rows, hipStream_t st, void* scratch = nullptr,
                         void* splitk_ws = nullptr, size_t splitk_cap = 0);
-// The 128 x 128 tile over groups of rows, each with a matrix of its own (mixture of experts): group g of `groups` multiplies by
+// The tile GEMM over groups of rows, each with a matrix of its own (mixture of experts): group g of `groups` multiplies by
 // rows [g rows, (g + 1) rows) of W, group `groups` by the whole of `last`.  The tile table lives on the device: tiles[0] = number
-// of tiles (at most max_tiles), then from word 8 four words each: group, first place, places (<= MOE_TILE), 0.  Place p reads
+// of tiles (at most max_tiles), then from word 8 four words each: group, first place, places (<= tile), 0.  Place p reads
 // row x_rows[p] of x (null: p) and writes row out_rows[p] of out (null: p).  Tile-major 16-bit weights, K a multiple of 64.
-constexpr int MOE_TILE = 128;
 struct GroupedGemm {
   LinearW W, last;
   int rows, groups;
   const void* x; int ldx; const int32_t* x_rows;
   void* out; int ldo; const int32_t* out_rows;
   const int32_t* tiles; int max_tiles;
+  int tile;                   // 128 or 256 places per tile: the 128 x 128 kernel, or the 256 x 256 LDS-DMA kernel
   bool swiglu;                // rows = gate rows, then as many up rows: out = silu(gate) * up, in float32 before the store
   int act;
 };

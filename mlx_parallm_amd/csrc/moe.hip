@@ -4,7 +4,7 @@
 //
 //   route       many rows: router logits on the matrix cores (x as hi + lo, so they keep 32-bit accuracy), softmax, groups, choice
 //               (few rows and float32: inside post_norm_kernel)
-//   plan        many rows: slots sorted by expert, table of 128-slot tiles, for the grouped tile GEMM (gemm_prefill.hip)
+//   plan        many rows: slots sorted by expert, table of tiles, for the grouped tile GEMM (gemm_prefill.hip)
 //   stream      up to MOE_STREAM_ROWS tokens: one workgroup per (expert, strip of weight rows) collects the expert's slots and
 //               streams its weights once per 16 or 32 of them
 //   generic     any dtype, row-major weights: one workgroup per (slot, strip of rows), float32 arithmetic
@@ -103,10 +103,16 @@ constexpr int ROUTE_MFMA_EXPERTS = 256;
 
 // ---- plan: one workgroup sorts the slots by expert ------------------------------------------------------------------------
 // words: [0] tiles, [8 ..) tiles of four words (expert, first place, places, 0), then slot and token of every place
-__host__ __device__ inline int plan_tiles(int R, int experts, int top, int shared) {
-  return R * top / MOE_TILE + experts + (shared ? (R + MOE_TILE - 1) / MOE_TILE : 0);
+inline int plan_tiles(int R, int experts, int top, int shared, int tile) {
+  return R * top / tile + experts + (shared ? (R + tile - 1) / tile : 0);
 }
-__global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles) {
+// places per tile: the large tile where an expert fills at least most of one on average
+constexpr int MOE_LARGE = 160;
+inline int tile_of(const MoeCall& c) {
+  const bool deep = c.ld >= 128 && c.ffp >= 128 && (c.sffp == 0 || c.sffp >= 128);
+  return deep && (size_t)c.R * c.r.top >= (size_t)MOE_LARGE * c.r.experts ? 256 : 128;
+}
+__global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles, int tile) {
   __shared__ int cnt[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], at[MOE_MAX_EXPERTS], tile0[MOE_MAX_EXPERTS + 1];
   const int tid = threadIdx.x, E = c.r.experts, n = c.R * c.r.top, shared = c.sffp > 0;
   int32_t* tiles = c.plan + 8;
@@ -119,7 +125,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles
   if (tid < 64) {                                      // running sums of places and tiles, 64 experts at a time
     int p0 = 0, t0 = 0;
     for (int b = 0; b < E; b += 64) {
-      const int e = b + tid, k = e < E ? cnt[e] : 0, t = (k + MOE_TILE - 1) / MOE_TILE;
+      const int e = b + tid, k = e < E ? cnt[e] : 0, t = (k + tile - 1) / tile;
       int p = k, q = t;
       for (int o = 1; o < 64; o *= 2) {
         const int pu = __shfl_up(p, o, 64), qu = __shfl_up(q, o, 64);
@@ -132,15 +138,15 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles
     if (tid == 0) tile0[E] = t0;
   }
   __syncthreads();
-  const int ns = shared ? (c.R + MOE_TILE - 1) / MOE_TILE : 0;
+  const int ns = shared ? (c.R + tile - 1) / tile : 0;
   for (int e = tid; e < E; e += 1024)
-    for (int i = 0, k = 0; k < cnt[e]; ++i, k += MOE_TILE) {
-      int32_t* t = tiles + 4 * (tile0[e] + i);
-      t[0] = e; t[1] = start[e] + k; t[2] = min(MOE_TILE, cnt[e] - k); t[3] = 0;
+    for (int i = 0, k = 0; k < cnt[e]; ++i, k += tile) {
+      int32_t* t = tiles + 4 * (ns + tile0[e] + i);
+      t[0] = e; t[1] = start[e] + k; t[2] = min(tile, cnt[e] - k); t[3] = 0;
     }
   for (int i = tid; i < ns; i += 1024) {
-    int32_t* t = tiles + 4 * (tile0[E] + i);
-    t[0] = E; t[1] = n + i * MOE_TILE; t[2] = min(MOE_TILE, c.R - i * MOE_TILE); t[3] = 0;
+    int32_t* t = tiles + 4 * i;                        // (first: the shared expert is usually the widest)
+    t[0] = E; t[1] = n + i * tile; t[2] = min(tile, c.R - i * tile); t[3] = 0;
   }
   if (tid == 0) c.plan[0] = tile0[E] + ns;
   for (int i = tid; i < n; i += 1024) {
@@ -346,7 +352,7 @@ int generic_at(const MoeCall& c, hipStream_t st) {
 }  // namespace
 
 size_t moe_plan_ints(int R, const RouteArgs& r, int shared) {
-  return 8 + 4 * (size_t)plan_tiles(R, r.experts, r.top, shared) + 2 * ((size_t)R * r.top + (shared ? R : 0));
+  return 8 + 4 * (size_t)plan_tiles(R, r.experts, r.top, shared, 128) + 2 * ((size_t)R * r.top + (shared ? R : 0));
 }
 
 // the matrix-core forms read tile-major 16-bit weights
@@ -384,11 +390,11 @@ int experts_at(const MoeCall& c, hipStream_t st) {
   MI_TRY(form_of(c, form));
   if (form == FORM_GENERIC) return c.act == MI_F32 ? generic_at<float, UP>(c, st) : (c.act == MI_BF16 ? generic_at<bf16, UP>(c, st) : generic_at<f16, UP>(c, st));
   if (form == FORM_STREAM) return c.act == MI_BF16 ? stream_at<bf16, UP>(c, st) : stream_at<f16, UP>(c, st);
-  const int shared = c.sffp > 0 ? 1 : 0, n = c.R * c.r.top, max_tiles = plan_tiles(c.R, c.r.experts, c.r.top, shared);
+  const int shared = c.sffp > 0 ? 1 : 0, n = c.R * c.r.top, tile = tile_of(c), max_tiles = plan_tiles(c.R, c.r.experts, c.r.top, shared, tile);
   const int32_t* slot = c.plan + 8 + 4 * max_tiles;
   const int32_t* token = slot + n + (shared ? c.R : 0);
   GroupedGemm g{};
-  g.tiles = c.plan; g.max_tiles = max_tiles; g.groups = c.r.experts; g.act = c.act; g.swiglu = UP;
+  g.tiles = c.plan; g.max_tiles = max_tiles; g.tile = tile; g.groups = c.r.experts; g.act = c.act; g.swiglu = UP;
   if (UP) {
     g.x = c.h; g.ldx = c.ld; g.x_rows = token; g.out = c.mid; g.ldo = c.lda;
     g.W = c.gu; g.rows = 2 * c.ffp; g.last = shared ? c.sgu : LinearW{};
@@ -405,7 +411,7 @@ int launch_moe_plan(const MoeCall& c, hipStream_t st) {
   int form = FORM_GENERIC;
   MI_TRY(form_of(c, form));
   if (form != FORM_TILES) return MI_OK;
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, st, c, plan_tiles(c.R, c.r.experts, c.r.top, c.sffp > 0 ? 1 : 0));
+  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, st, c, plan_tiles(c.R, c.r.experts, c.r.top, c.sffp > 0 ? 1 : 0, tile_of(c)), tile_of(c));
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

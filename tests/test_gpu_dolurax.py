@@ -149,14 +149,15 @@ def test_each_attention_mechanism_alone(bank, name, dtype):
 
 
 ROUTERS = {"top1": (8, 1, 1, 1, 0), "all": (6, 6, 1, 1, 0), "one_group": (12, 3, 4, 1, 0), "all_groups": (12, 3, 4, 4, 0), "groups_of_one": (8, 2, 8, 3, 0),
-           "shared": (8, 2, 2, 1, 50), "uneven": (90, 7, 9, 4, 20)}
+           "shared": (8, 2, 2, 1, 50), "uneven": (90, 7, 9, 4, 20), "large_tiles": (4, 2, 2, 2, 200, 136),
+           "large_tiles_no_shared": (3, 2, 1, 1, 0, 128)}
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", list(ROUTERS))
 def test_each_router_form_alone(bank, name, dtype):
-    E, top, groups, keep, shared = ROUTERS[name]
-    cfg = config(64, 96, [layer(attn(2, 1, 16, 16, 40), moe(E, top, 48, groups, keep, shared))])
+    E, top, groups, keep, shared, ff, width = (*ROUTERS[name], 48, 64)[:7] if len(ROUTERS[name]) == 5 else (*ROUTERS[name], 150)
+    cfg = config(width, 96, [layer(attn(2, 1, 16, 16, 40), moe(E, top, ff, groups, keep, shared))])
     cfg, w, m = bank(f"router_{name}", dtype, cfg)
     t = tokens(cfg, 333, 5)
     want, clear = plain(cfg, w, t)
