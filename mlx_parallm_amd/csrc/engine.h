@@ -181,7 +181,7 @@ struct mi_engine {
   void* v_first = nullptr;       // [rows][n_vfirst] values of the first mixing layer
   int32_t* moe_ids = nullptr; float* moe_wts = nullptr;       // [rows][max top]
   void* moe_mid = nullptr; void* moe_out = nullptr;           // [slots][max ff], [slots][wp]
-  int32_t* moe_plan = nullptr;
+  int32_t* moe_plan = nullptr; int32_t* moe_counts = nullptr;
   int gqa_chunk = -1;            // chunk of the first grouped-query layer (order of the query tiles), -1: no such layer
   float* gqa_part = nullptr; size_t gqa_part_cap = 0;         // split-KV partials of the decode attention
   int* gqa_ctr = nullptr; size_t gqa_ctr_cap = 0;             // its arrival tickets (zero between launches)

@@ -413,7 +413,7 @@ MoeCall moe_call(mi_engine* e, const ListLayer& l, int R) {
   c.x = e->x32; c.h = e->hn; c.router = l.router; c.ids = e->moe_ids; c.wts = e->moe_wts;
   c.gu = l.gu.f.W; c.dn = l.dn.f.W; c.sgu = l.sgu.f.W; c.sdn = l.sdn.f.W;
   c.ffp = l.ffp; c.sffp = l.sffp; c.lda = std::max(l.ffp, l.sffp);
-  c.mid = e->moe_mid; c.out = e->moe_out; c.plan = e->moe_plan; c.act = e->d.act_dtype;
+  c.mid = e->moe_mid; c.out = e->moe_out; c.plan = e->moe_plan; c.counts = e->moe_counts; c.act = e->d.act_dtype;
   return c;
 }
 
@@ -590,7 +590,7 @@ void layers_free(mi_engine* e) {
   free_packed(e->list_head);
   for (void* p : {e->tok_embed, e->side_embed, (void*)e->d_freq, (void*)e->x32, e->hn, e->proj, e->cat, (void*)e->scan32, (void*)e->gate32,
                   e->lq, (void*)e->lat_part, e->lat_m, e->lat_x, e->lat_kv, (void*)e->dl_w, (void*)e->dl_p, (void*)e->dl_k, (void*)e->dl_f, (void*)e->d_meta, (void*)e->d_gather_list, e->head_x,
-                  (void*)e->y32, e->v_first, (void*)e->moe_ids, (void*)e->moe_wts, e->moe_mid, e->moe_out, (void*)e->moe_plan, (void*)e->gqa_part, (void*)e->gqa_ctr}) hipFree(p);
+                  (void*)e->y32, e->v_first, (void*)e->moe_ids, (void*)e->moe_wts, e->moe_mid, e->moe_out, (void*)e->moe_plan, (void*)e->moe_counts, (void*)e->gqa_part, (void*)e->gqa_ctr}) hipFree(p);
 }
 
 // element offsets of the arenas (latents, keys, values) for `tokens` token places, byte offsets of the recurrent state for kv->B rows
@@ -619,7 +619,7 @@ int layers_kv_plan(mi_engine* e, mi_kv* kv) {
 int layers_ensure_workspace(mi_engine* e, size_t rows) {
   if (rows <= e->lw_rows) return MI_OK;
   MI_HIP(hipStreamSynchronize(e->stream));
-  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4, n_pick = 0, n_mid = 0, n_out = 0, n_plan = 0;
+  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4, n_pick = 0, n_mid = 0, n_out = 0, n_plan = 0, n_count = 0;
   for (auto& l : e->list) {
     n_in = std::max(n_in, (size_t)l.in.N);
     n_cat = std::max(n_cat, (size_t)l.n_cat);
@@ -632,7 +632,9 @@ int layers_ensure_workspace(mi_engine* e, size_t rows) {
       n_pick = std::max(n_pick, (size_t)l.d.top);
       n_mid = std::max(n_mid, slots * std::max(l.ffp, l.sffp));
       n_out = std::max(n_out, slots * e->wp);
-      n_plan = std::max(n_plan, moe_plan_ints((int)rows, RouteArgs{l.d.experts, l.d.top, l.d.groups, l.d.keep}, l.sffp > 0 ? 1 : 0));
+      const RouteArgs r{l.d.experts, l.d.top, l.d.groups, l.d.keep};
+      n_plan = std::max(n_plan, moe_plan_ints((int)rows, r, l.sffp > 0 ? 1 : 0));
+      n_count = std::max(n_count, moe_count_ints((int)rows, r));
     }
   }
   const size_t n_y = e->d.block_form == MI_BLOCK_POST_NORM ? e->wp : 0;
@@ -645,7 +647,7 @@ int layers_ensure_workspace(mi_engine* e, size_t rows) {
       {&e->lq, rows * n_lq * sizeof(float)},
       {(void**)&e->y32, rows * n_y * sizeof(float)}, {&e->v_first, rows * (size_t)e->n_vfirst * es}, {(void**)&e->moe_ids, rows * n_pick * sizeof(int32_t)},
       {(void**)&e->moe_wts, rows * n_pick * sizeof(float)}, {&e->moe_mid, rows * n_mid * es}, {&e->moe_out, rows * n_out * es},
-      {(void**)&e->moe_plan, n_plan * sizeof(int32_t)}};
+      {(void**)&e->moe_plan, n_plan * sizeof(int32_t)}, {(void**)&e->moe_counts, n_count * sizeof(int32_t)}};
   e->lw_rows = 0;
   for (auto& b : bufs) {
     hipFree(*b.p); *b.p = nullptr;
@@ -745,12 +747,13 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
         const bool fused = route_fused(act, R, m.experts);
         pn.r = mc.r; pn.ids = mc.ids; pn.wts = mc.wts;
         pn.router = fused ? l.router : nullptr;
+        if (!fused) { pn.clear = mc.counts; pn.n_clear = m.experts; }
         { Prof pr(e, "post_norm"); MI_TRY(launch_post_norm(pn, st)); }
         if (!fused) { Prof pr(e, "moe_route"); MI_TRY(launch_route(mc, st)); }
         { Prof pr(e, "moe_plan"); MI_TRY(launch_moe_plan(mc, st)); }
         { Prof pr(e, "moe_up"); MI_TRY(launch_moe_up(mc, st)); }
         { Prof pr(e, "moe_down"); MI_TRY(launch_moe_down(mc, st)); }
-        pn.y = nullptr; pn.parts = mc.out; pn.part_w = mc.wts; pn.top = m.top; pn.shared = l.sffp > 0 ? 1 : 0; pn.router = nullptr;
+        pn.y = nullptr; pn.parts = mc.out; pn.part_w = mc.wts; pn.top = m.top; pn.shared = l.sffp > 0 ? 1 : 0; pn.router = nullptr; pn.clear = nullptr;
         pn.norm = PostNormW{l.norm2.p, l.norm2_b.p, nstride};
       }
       if (end) pn.next = last;

@@ -234,6 +234,20 @@ __device__ __forceinline__ float score_poly(const CapPoly& k, float s, float bia
   return fmaf(s, fmaf(fmaf(fmaf(fmaf(k.c[4], w, k.c[3]), w, k.c[2]), w, k.c[1]), w, k.c[0]), bias);
 }
 
+// N consecutive elements, n of them there (the rest zero): one load where N divides n
+template <typename T, int N>
+__device__ __forceinline__ void load_upto(const T* p, int k, int n, float (&v)[N]) {
+  typedef T tv __attribute__((ext_vector_type(N)));
+  if (n % N == 0 && ((uintptr_t)p & (N * sizeof(T) - 1)) == 0) {
+    const tv x = *(const tv*)(p + min(k, n - N));
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = k < n ? to_f32(x[i]) : 0.f;
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) v[i] = k + i < n ? to_f32(p[k + i]) : 0.f;
+  }
+}
+
 // grid (nsplit, G x head tiles, nd), 4 waves; a wave walks its 32-key blocks on its own, the next block's loads in flight during
 // the current one.  The token's own key and value are added by the last split from LDS, which also appends them.
 template <typename T, int KD, int VD, bool PAGED, bool CAP>
@@ -273,25 +287,32 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
       vr[i] = *(const u32x4*)(vc + kv_elem<PAGED>(c.sv, row, kh, max(0, min(blk * KB + piece / (VD / 8), pos - 1))) + 8 * (piece % (VD / 8)));
     }
   };
-  if (b0 + wave < b1) { load_k(b0 + wave); load_v(b0 + wave); }
 
-  // queries (and, in the last split, the token's own key and value): 16 lanes per head
+  // queries (and, in the last split, the token's own key and value): 16 lanes per head.  Their loads go first: memory answers in order
   const T* pr = (const T*)c.proj + (size_t)tok * c.ldp;
   const bool own = split == c.nsplit - 1;
   {
     const int hh = tid >> 4, l = tid & 15;
     constexpr int PL = KD / 16;                      // elements per lane: l PL ..
-    float v[PL], ss = 0.f;
-    auto head = [&](const T* src, bool there, const float* w, T* dst) {
-      ss = 0.f;
+    float vq[PL], wq[PL], vk[PL], wk[PL];
+    const bool key_lanes = own && tid < 16;
+    load_upto<T, PL>(pr + c.o_q + (h0 + min(hh, nh - 1)) * c.dim, l * PL, c.dim, vq);
+    load_upto<float, PL>(c.q_norm, l * PL, c.dim, wq);
+    if (key_lanes) {
+      load_upto<T, PL>(pr + c.o_k + kh * c.dim, l * PL, c.dim, vk);
+      load_upto<float, PL>(c.k_norm, l * PL, c.dim, wk);
+    }
+    if (b0 + wave < b1) { load_k(b0 + wave); load_v(b0 + wave); }
+    auto head = [&](const float (&v)[PL], const float (&w)[PL], bool there, T* dst) {
+      float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < PL; ++i) { const int k = l * PL + i; v[i] = there && k < c.dim ? to_f32(src[k]) : 0.f; ss += v[i] * v[i]; }
+      for (int i = 0; i < PL; ++i) ss += v[i] * v[i];
       const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)c.dim + c.eps);
 #pragma unroll
-      for (int i = 0; i < PL; ++i) { const int k = l * PL + i; dst[k] = from_f32<T>(k < c.dim ? v[i] * rs * w[k] : 0.f); }
+      for (int i = 0; i < PL; ++i) dst[l * PL + i] = from_f32<T>(there ? v[i] * rs * w[i] : 0.f);
     };
-    head(pr + c.o_q + (h0 + min(hh, nh - 1)) * c.dim, hh < nh, c.q_norm, qs + hh * LQ);
-    if (own && wave == 0 && hh == 0) head(pr + c.o_k + kh * c.dim, true, c.k_norm, kn);
+    head(vq, wq, hh < nh, qs + hh * LQ);
+    if (key_lanes) head(vk, wk, true, kn);
     if (own && tid >= 64 && tid < 64 + VD) {
       const int k = tid - 64;
       float x = 0.f;
@@ -441,26 +462,31 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   for (int idx = tid; idx < nh * VD; idx += 256) {
     const int hh = idx / VD, d = idx % VD, h = h0 + hh;
     const float* pp = pp0 + (size_t)h * c.nsplit * (VD + 2);
+    const float gv = to_f32(gate[h * c.vdim + min(d, c.vdim - 1)]);
     float mn = -1e30f, L = 0.f, O = 0.f;
-    for (int i0 = 0; i0 < c.nsplit; i0 += 4) {       // four splits' loads in flight, merged in split order
-      float mv[4], lv[4], ov[4];
+    for (int i0 = 0; i0 < c.nsplit; i0 += 8) {       // eight splits' loads in flight, merged in split order
+      float mv[8], lv[8], ov[8];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
+      for (int j = 0; j < 8; ++j) {
         const float* q = pp + (size_t)min(i0 + j, c.nsplit - 1) * (VD + 2);
         mv[j] = __hip_atomic_load(&q[0], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         lv[j] = __hip_atomic_load(&q[1], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         ov[j] = __hip_atomic_load(&q[2 + d], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
       }
+      float bm = mn;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
+      for (int j = 0; j < 8; ++j) if (i0 + j < c.nsplit) bm = fmaxf(bm, mv[j]);
+      const float cs = __builtin_amdgcn_exp2f(mn - bm);
+      L *= cs; O *= cs; mn = bm;
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
         if (i0 + j < c.nsplit) {
-          const float bm = fmaxf(mn, mv[j]), cs = __builtin_amdgcn_exp2f(mn - bm), cw = __builtin_amdgcn_exp2f(mv[j] - bm);
-          L = fmaf(lv[j], cw, L * cs);
-          O = fmaf(ov[j], cw, O * cs);
-          mn = bm;
+          const float cw = __builtin_amdgcn_exp2f(mv[j] - bm);
+          L = fmaf(lv[j], cw, L);
+          O = fmaf(ov[j], cw, O);
         }
     }
-    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(to_f32(gate[h * c.vdim + d])));
+    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(gv));
   }
 }
 

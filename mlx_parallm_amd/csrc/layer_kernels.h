@@ -162,6 +162,7 @@ struct PostNormCall {
   PostNormW norm, next;
   int width, ld;
   float* x; void* h;
+  int32_t* clear; int n_clear;   // words set to zero, or null
   RouteArgs r; const void* router; int32_t* ids; float* wts;          // router [experts][ld] in the activation dtype
   int act;
 };
@@ -184,10 +185,13 @@ struct MoeCall {
   int ffp, sffp, lda;            // lda: row stride of `mid`
   void* mid;                     // [slots][lda] activations
   void* out;                     // [slots][ld]
-  int32_t* plan;                 // moe_plan_ints() words: sorted slots, their tokens, tile table
+  int32_t* plan;                 // moe_plan_ints() words: tile table, sorted slots, their tokens
+  int32_t* counts;               // [experts] slots per expert, [R][top] a slot's place among its expert's: left by launch_route, whose
+                                 // caller clears the counts first (launch_post_norm: `clear`)
   int act;
 };
 size_t moe_plan_ints(int R, const RouteArgs& r, int shared);
+inline size_t moe_count_ints(int R, const RouteArgs& r) { return (size_t)r.experts + (size_t)R * r.top; }
 bool moe_mfma_supported(const MoeCall& c);
 int launch_route(const MoeCall& c, hipStream_t st);         // many rows of 16-bit models (few: launch_post_norm)
 bool route_fused(int act, int rows, int experts);           // launch_post_norm does the routing

@@ -106,55 +106,77 @@ __device__ __forceinline__ void polynorm_row(const PolyNormArgs& f, const T* z, 
 }
 
 // Routing of one token by one wave: z [E] logits in LDS -> the `top` experts with the largest softmax scores among the `keep`
-// groups with the largest best score, in falling order, and their weights (scores over their sum).  `sel` / `sw`: [top] in LDS.
-// Ranks by counting: no expert or group is taken twice, ties go to the lower number.
+// groups with the largest best score, in falling order, and their weights (scores over their sum).  `sel`: [top] in LDS, `sw`:
+// route_lds_floats() floats of LDS, 8-byte aligned.  Ranks by counting, the others' values broadcast from their lanes: no expert or
+// group is taken twice, ties go to the lower number.
+__device__ __forceinline__ float lane_value(float v, int lane) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), lane));
+}
+// how many of the n values v(i) come before (mine, me) in falling order
+template <typename F>
+__device__ __forceinline__ int rank_of(float mine, int me, int n, F v) {
+  const int lane = threadIdx.x & 63;
+  int rank = 0;
+  for (int b = 0; b < n; b += 64) {
+    const float vb = v(min(b + lane, n - 1));
+    const int k = min(64, n - b);
+#pragma unroll 8
+    for (int o = 0; o < k; ++o) {
+      const float x = lane_value(vb, o);
+      rank += x > mine || (x == mine && b + o < me) ? 1 : 0;
+    }
+  }
+  return rank;
+}
 __device__ __forceinline__ void route_wave(const float* z, const RouteArgs& r, int* sel, float* sw, int32_t* ids, float* wts) {
   const int lane = threadIdx.x & 63, E = r.experts, gs = E / r.groups;
-  for (int j = lane; j < r.top; j += 64) { sel[j] = j; sw[j] = 0.f; }
+  unsigned long long* marks = (unsigned long long*)sw;                 // a bit per kept group
+  float* gbest = sw + 2 * ((r.groups + 63) / 64);                      // [groups] best logit of a group
+  float* wsel = gbest + r.groups;                                      // [top]
+  for (int j = lane; j < r.top; j += 64) { sel[j] = j; wsel[j] = 0.f; }
   float zm = -INFINITY;
   for (int e = lane; e < E; e += 64) zm = fmaxf(zm, z[e]);
   zm = wave_max(zm);
   float tot = 0.f;
   for (int e = lane; e < E; e += 64) tot += expf(z[e] - zm);
   tot = wave_sum(tot);
-  float chosen = 0.f;
-  for (int e0 = 0; e0 < E; e0 += 64) {                 // (uniform: the sums at the end take every lane)
-    const int e = min(e0 + lane, E - 1), g = e / gs;
-    const float ze = z[e];
-    // rank of the expert's group: groups with a larger best score, or an equal one and a lower number
-    int ahead = 0;
-    if (r.keep < r.groups) {
+  const bool grouped = r.keep < r.groups;
+  if (grouped) {
+    for (int g = lane; g < r.groups; g += 64) {
       float best = -INFINITY;
+#pragma unroll 8
       for (int i = 0; i < gs; ++i) best = fmaxf(best, z[g * gs + i]);
-      for (int o = 0; o < r.groups; ++o) {
-        float b = -INFINITY;
-        for (int i = 0; i < gs; ++i) b = fmaxf(b, z[o * gs + i]);
-        ahead += b > best || (b == best && o < g) ? 1 : 0;
-      }
+      gbest[g] = best;
     }
-    const bool ok = e0 + lane < E && ahead < r.keep;
-    // rank among the experts of the kept groups: a lane cannot know the others' groups cheaply, so they are marked in two steps
-    const unsigned long long m = __builtin_amdgcn_ballot_w64(ok);
-    if (lane == 0) ((unsigned long long*)(sw + r.top + (r.top & 1)))[e0 >> 6] = m;
+    for (int g0 = 0; g0 < r.groups; g0 += 64) {
+      const int g = min(g0 + lane, r.groups - 1);
+      const int ahead = rank_of(gbest[g], g, r.groups, [&](int o) { return gbest[o]; });
+      const unsigned long long m = __builtin_amdgcn_ballot_w64(g0 + lane < r.groups && ahead < r.keep);
+      if (lane == 0) marks[g0 >> 6] = m;
+    }
   }
-  const unsigned long long* kept = (const unsigned long long*)(sw + r.top + (r.top & 1));
+  auto kept = [&](int e) {                             // the expert's logit, -inf outside the kept groups
+    const float v = z[e];
+    if (!grouped) return v;
+    const int g = e / gs;
+    return marks[g >> 6] >> (g & 63) & 1 ? v : -INFINITY;
+  };
+  float chosen = 0.f;
   for (int e0 = 0; e0 < E; e0 += 64) {
     const int e = min(e0 + lane, E - 1);
-    const float ze = z[e];
-    int rank = e0 + lane < E && (kept[e0 >> 6] >> lane & 1) ? 0 : E;
-    for (int o = 0; o < E; ++o)
-      rank += (kept[o >> 6] >> (o & 63) & 1) && (z[o] > ze || (z[o] == ze && o < e)) ? 1 : 0;
-    if (rank < r.top) {
+    const float ze = kept(e);
+    const int rank = rank_of(ze, e, E, kept);
+    if (e0 + lane < E && ze > -INFINITY && rank < r.top) {
       const float s = expf(ze - zm) / tot;
-      sel[rank] = e; sw[rank] = s;
+      sel[rank] = e; wsel[rank] = s;
       chosen += s;
     }
   }
   chosen = wave_sum(chosen) + 1e-20f;
-  for (int j = lane; j < r.top; j += 64) { ids[j] = sel[j]; wts[j] = sw[j] / chosen; }
+  for (int j = lane; j < r.top; j += 64) { ids[j] = sel[j]; wts[j] = wsel[j] / chosen; }
 }
-// floats of LDS that route_wave needs behind `sel`: weights, then a bit per expert
-__host__ __device__ constexpr int route_lds_floats(int experts, int top) { return top + (top & 1) + 2 * ((experts + 63) / 64); }
+// floats of LDS behind `sw`, an even number: marks, groups, weights
+__host__ __device__ constexpr int route_lds_floats(const RouteArgs& r) { return (2 * ((r.groups + 63) / 64) + r.groups + r.top + 1) & ~1; }
 
 }  // namespace rows
 }  // namespace mi

@@ -364,6 +364,19 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
   __shared__ float red[NT / 64];
   const int r = blockIdx.x, tid = threadIdx.x, n4 = c.ld / 4;
   const float inv_n = 1.0f / (float)c.width;
+  if (c.clear != nullptr && r == 0)
+    for (int i = tid; i < c.n_clear; i += NT) c.clear[i] = 0;
+  // the first router rows of this wave (columns below 512 PRE) are on their way while the norm runs
+  constexpr int JB = 2, PRE = ROUTE && sizeof(T) == 2 ? 4 : 0;
+  const int lane = tid & 63, wave = tid >> 6;
+  u32x4 wpre[JB][PRE > 0 ? PRE : 1];
+  if constexpr (PRE > 0) {
+#pragma unroll
+    for (int j = 0; j < JB; ++j)
+#pragma unroll
+      for (int i = 0; i < PRE; ++i)
+        wpre[j][i] = *(const u32x4*)((const T*)c.router + (size_t)min(wave * JB + j, c.r.experts - 1) * c.ld + min(lane * 8 + 512 * i, c.ld - 8));
+  }
   f32x4 y[NQ], x[NQ];
   float* xg = c.x + (size_t)r * c.ld;
 #pragma unroll
@@ -436,22 +449,41 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
   if constexpr (ROUTE) {
     float* z = smem + c.ld;
     float* sw = z + ((c.r.experts + 1) & ~1);
-    int* sel = (int*)(sw + route_lds_floats(c.r.experts, c.r.top));
-    const int lane = tid & 63, wave = tid >> 6;
-    constexpr int JB = 2;
+    int* sel = (int*)(sw + route_lds_floats(c.r));
     __syncthreads();
     for (int e0 = wave * JB; e0 < c.r.experts; e0 += NT / 64 * JB) {
       float acc[JB] = {0.f, 0.f};
-      for (int k = lane * 8; k < c.ld; k += 512) {
+      auto add = [&](int k, const float (&w)[JB][8]) {
         float xv[8];
         load8f<float>(smem + k, xv);
 #pragma unroll
-        for (int j = 0; j < JB; ++j) {
-          float w[8];
-          load8f<T>((const T*)c.router + (size_t)min(e0 + j, c.r.experts - 1) * c.ld + k, w);
+        for (int j = 0; j < JB; ++j)
 #pragma unroll
-          for (int i = 0; i < 8; ++i) acc[j] = fmaf(w[i], xv[i], acc[j]);
+          for (int i = 0; i < 8; ++i) acc[j] = fmaf(w[j][i], xv[i], acc[j]);
+      };
+      int k0 = lane * 8;
+      if constexpr (PRE > 0) {
+        if (e0 == wave * JB) {
+#pragma unroll
+          for (int q = 0; q < PRE; ++q, k0 += 512)
+            if (k0 < c.ld) {
+              float w[JB][8];
+#pragma unroll
+              for (int j = 0; j < JB; ++j) {
+                const T* e = (const T*)&wpre[j][q];
+#pragma unroll
+                for (int i = 0; i < 8; ++i) w[j][i] = to_f32(e[i]);
+              }
+              add(k0, w);
+            }
         }
+      }
+#pragma unroll 2
+      for (int k = k0; k < c.ld; k += 512) {
+        float w[JB][8];
+#pragma unroll
+        for (int j = 0; j < JB; ++j) load8f<T>((const T*)c.router + (size_t)min(e0 + j, c.r.experts - 1) * c.ld + k, w[j]);
+        add(k, w);
       }
 #pragma unroll
       for (int j = 0; j < JB; ++j) {
@@ -467,7 +499,7 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
 template <typename T>
 int post_norm_at(const PostNormCall& c, hipStream_t st) {
   const bool route = c.router != nullptr;
-  const size_t lds = !route ? 0 : ((size_t)c.ld + c.r.experts + 1 + route_lds_floats(c.r.experts, c.r.top) + c.r.top) * sizeof(float);
+  const size_t lds = !route ? 0 : ((size_t)c.ld + c.r.experts + 1 + route_lds_floats(c.r) + c.r.top) * sizeof(float);
   if (lds > 128 * 1024) return fail(MI_ERR_UNSUPPORTED, "post_norm: row too wide for the LDS");
   auto go = [&](auto k, int nt) -> int {
     if (lds > 65536) MI_HIP(hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));

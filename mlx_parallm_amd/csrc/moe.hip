@@ -43,6 +43,7 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
   f32x4 acc[NE];
 #pragma unroll
   for (int t = 0; t < NE; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
   for (int k = wave * 32; k < c.ld; k += RTW * 32) {
     float v[8];
     load8f<float>(x + k, v);
@@ -75,10 +76,23 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
 #pragma unroll
   for (int i = 0; i < PER; ++i) { const int idx = i * RTW * 64 + tid; if (idx < 16 * EP) sm[idx] = z[i]; }
   __syncthreads();
-  const int per_wave = (route_lds_floats(E, c.r.top) + 1) & ~1;
-  float* sw = sm + 16 * EP + wave * (per_wave + ((c.r.top + 1) & ~1));
-  int* sel = (int*)(sw + per_wave);
-  for (int m = wave; m < nr; m += RTW) route_wave(sm + m * EP, c.r, sel, sw, c.ids + (size_t)(r0 + m) * c.r.top, c.wts + (size_t)(r0 + m) * c.r.top);
+  const int top = c.r.top;
+  float* sw = sm + 16 * EP + wave * route_lds_floats(c.r);
+  int* sel = (int*)(sm + 16 * EP + RTW * route_lds_floats(c.r));       // [16][top]
+  int* cnt = sel + 16 * top;                                          // [E] of this workgroup, then the places in front of them
+  for (int e = tid; e < E; e += RTW * 64) cnt[e] = 0;
+  for (int m = wave; m < nr; m += RTW) route_wave(sm + m * EP, c.r, sel + m * top, sw, c.ids + (size_t)(r0 + m) * top, c.wts + (size_t)(r0 + m) * top);
+  __syncthreads();
+  // places among the expert's slots (their order does not matter): one global addition per expert and workgroup
+  constexpr int NI = (16 * MOE_MAX_TOP + RTW * 64 - 1) / (RTW * 64);
+  int at[NI];
+#pragma unroll
+  for (int i = 0; i < NI; ++i) { const int idx = i * RTW * 64 + tid; at[i] = idx < nr * top ? atomicAdd(&cnt[sel[idx]], 1) : 0; }
+  __syncthreads();
+  for (int e = tid; e < E; e += RTW * 64) cnt[e] = cnt[e] > 0 ? atomicAdd(&c.counts[e], cnt[e]) : 0;
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < NI; ++i) { const int idx = i * RTW * 64 + tid; if (idx < nr * top) c.counts[E + (size_t)r0 * top + idx] = cnt[sel[idx]] + at[i]; }
 }
 
 template <typename T>
@@ -86,7 +100,7 @@ int route_at(const MoeCall& c, hipStream_t st) {
   const int ne = (c.r.experts + 15) / 16;
   auto go = [&](auto k, int NE) -> int {
     const size_t part = (size_t)RTW * NE * 1024,
-                 pick = ((size_t)16 * 16 * NE + RTW * (((route_lds_floats(c.r.experts, c.r.top) + 1) & ~1) + ((c.r.top + 1) & ~1))) * sizeof(float);
+                 pick = ((size_t)16 * 16 * NE + RTW * route_lds_floats(c.r) + 16 * c.r.top + c.r.experts) * sizeof(float);
     const size_t lds = std::max(part, pick);
     if (lds > 65536) MI_HIP(hipFuncSetAttribute((const void*)k, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     hipLaunchKernelGGL(k, dim3((c.R + 15) / 16), dim3(RTW * 64), lds, st, c);
@@ -101,7 +115,7 @@ int route_at(const MoeCall& c, hipStream_t st) {
 }
 constexpr int ROUTE_MFMA_EXPERTS = 256;
 
-// ---- plan: one workgroup sorts the slots by expert ------------------------------------------------------------------------
+// ---- plan: the slots sorted by expert, and the tile table ------------------------------------------------------------------
 // words: [0] tiles, [8 ..) tiles of four words (expert, first place, places, 0), then slot and token of every place
 inline int plan_tiles(int R, int experts, int top, int shared, int tile) {
   return R * top / tile + experts + (shared ? (R + tile - 1) / tile : 0);
@@ -112,18 +126,29 @@ inline int tile_of(const MoeCall& c) {
   const bool deep = c.ld >= 128 && c.ffp >= 128 && (c.sffp == 0 || c.sffp >= 128);
   return deep && (size_t)c.R * c.r.top >= (size_t)MOE_LARGE * c.r.experts ? 256 : 128;
 }
+// counts of a router that does not count (launch_post_norm's): one workgroup
+__global__ __launch_bounds__(1024) void moe_count_kernel(MoeCall c) {
+  __shared__ int cnt[MOE_MAX_EXPERTS];
+  const int tid = threadIdx.x, E = c.r.experts, n = c.R * c.r.top;
+  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  for (int i = tid; i < n; i += 1024) c.counts[E + i] = atomicAdd(&cnt[min(max(c.ids[i], 0), E - 1)], 1);
+  __syncthreads();
+  for (int e = tid; e < E; e += 1024) c.counts[e] = cnt[e];
+}
+
+// grid: PLAN_SLOTS slots per workgroup (every one makes the running sums for itself); the first also writes the table
+constexpr int PLAN_SLOTS = 4096;
 __global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles, int tile) {
-  __shared__ int cnt[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], at[MOE_MAX_EXPERTS], tile0[MOE_MAX_EXPERTS + 1];
-  const int tid = threadIdx.x, E = c.r.experts, n = c.R * c.r.top, shared = c.sffp > 0;
+  __shared__ int cnt[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], tile0[MOE_MAX_EXPERTS + 1];
+  const int tid = threadIdx.x, E = c.r.experts, n = c.R * c.r.top, shared = c.sffp > 0, ns = shared ? (c.R + tile - 1) / tile : 0;
   int32_t* tiles = c.plan + 8;
   int32_t* slot = tiles + 4 * max_tiles;
   int32_t* token = slot + n + (shared ? c.R : 0);
-  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
-  __syncthreads();
-  for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[min(max(c.ids[i], 0), E - 1)], 1);
+  for (int e = tid; e < E; e += 1024) cnt[e] = c.counts[e];
   __syncthreads();
   if (tid < 64) {                                      // running sums of places and tiles, 64 experts at a time
-    int p0 = 0, t0 = 0;
+    int p0 = 0, t0 = ns;                               // (the shared expert's tiles first: it is usually the widest)
     for (int b = 0; b < E; b += 64) {
       const int e = b + tid, k = e < E ? cnt[e] : 0, t = (k + tile - 1) / tile;
       int p = k, q = t;
@@ -131,29 +156,31 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(MoeCall c, int max_tiles
         const int pu = __shfl_up(p, o, 64), qu = __shfl_up(q, o, 64);
         if (tid >= o) { p += pu; q += qu; }
       }
-      if (e < E) { start[e] = at[e] = p0 + p - k; tile0[e] = t0 + q - t; }
+      if (e < E) { start[e] = p0 + p - k; tile0[e] = t0 + q - t; }
       p0 += __shfl(p, 63, 64);
       t0 += __shfl(q, 63, 64);
     }
     if (tid == 0) tile0[E] = t0;
   }
   __syncthreads();
-  const int ns = shared ? (c.R + tile - 1) / tile : 0;
-  for (int e = tid; e < E; e += 1024)
-    for (int i = 0, k = 0; k < cnt[e]; ++i, k += tile) {
-      int32_t* t = tiles + 4 * (ns + tile0[e] + i);
-      t[0] = e; t[1] = start[e] + k; t[2] = min(tile, cnt[e] - k); t[3] = 0;
+  if (blockIdx.x == 0) {
+    for (int e = tid; e < E; e += 1024)
+      for (int i = 0, k = 0; k < cnt[e]; ++i, k += tile) {
+        int32_t* t = tiles + 4 * (tile0[e] + i);
+        t[0] = e; t[1] = start[e] + k; t[2] = min(tile, cnt[e] - k); t[3] = 0;
+      }
+    for (int i = tid; i < ns; i += 1024) {
+      int32_t* t = tiles + 4 * i;
+      t[0] = E; t[1] = n + i * tile; t[2] = min(tile, c.R - i * tile); t[3] = 0;
     }
-  for (int i = tid; i < ns; i += 1024) {
-    int32_t* t = tiles + 4 * i;                        // (first: the shared expert is usually the widest)
-    t[0] = E; t[1] = n + i * tile; t[2] = min(tile, c.R - i * tile); t[3] = 0;
+    if (tid == 0) c.plan[0] = tile0[E];
   }
-  if (tid == 0) c.plan[0] = tile0[E] + ns;
-  for (int i = tid; i < n; i += 1024) {
-    const int p = atomicAdd(&at[min(max(c.ids[i], 0), E - 1)], 1);
-    slot[p] = i; token[p] = i / c.r.top;
+  const int end = min(n + (shared ? c.R : 0), (int)(blockIdx.x + 1) * PLAN_SLOTS);
+  for (int i = blockIdx.x * PLAN_SLOTS + tid; i < end; i += 1024) {
+    const int p = i < n ? start[min(max(c.ids[i], 0), E - 1)] + c.counts[E + i] : i;
+    slot[p] = i;
+    token[p] = i < n ? i / c.r.top : i - n;
   }
-  if (shared) for (int i = tid; i < c.R; i += 1024) { slot[n + i] = n + i; token[n + i] = i; }
 }
 
 // ---- streaming form -------------------------------------------------------------------------------------------------------
@@ -411,7 +438,13 @@ int launch_moe_plan(const MoeCall& c, hipStream_t st) {
   int form = FORM_GENERIC;
   MI_TRY(form_of(c, form));
   if (form != FORM_TILES) return MI_OK;
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(1024), 0, st, c, plan_tiles(c.R, c.r.experts, c.r.top, c.sffp > 0 ? 1 : 0, tile_of(c)), tile_of(c));
+  if (route_fused(c.act, c.R, c.r.experts)) {
+    hipLaunchKernelGGL(moe_count_kernel, dim3(1), dim3(1024), 0, st, c);
+    MI_HIP(hipGetLastError());
+  }
+  const int shared = c.sffp > 0 ? 1 : 0, slots = c.R * (c.r.top + shared);
+  hipLaunchKernelGGL(moe_plan_kernel, dim3((slots + PLAN_SLOTS - 1) / PLAN_SLOTS), dim3(1024), 0, st, c,
+                     plan_tiles(c.R, c.r.experts, c.r.top, shared, tile_of(c)), tile_of(c));
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
