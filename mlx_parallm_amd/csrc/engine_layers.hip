@@ -362,7 +362,7 @@ int gqa_nsplit(const mi_kv* kv, const ListLayer& l, const int32_t* rows, const i
   for (int i = 0; i < n; ++i)
     if (lens[i] == 1) { const int pos = kv->h_off[rows[i]]; mx = std::max(mx, l.d.chunk > 0 ? pos % l.d.chunk : pos); }
   const int ns = std::max(1, 512 / std::max(1, nd * l.d.kv_heads * gqa_head_tiles(l.d.heads, l.d.kv_heads)));
-  return std::max(1, std::min({ns, (mx + 127) / 128, 32}));
+  return std::max(1, std::min({ns, (mx + 255) / 256, 32}));
 }
 
 int run_gqa(mi_engine* e, mi_kv* kv, ListLayer& l, const Tables& tb, const int32_t* rows, const int32_t* lens, int n) {

@@ -32,9 +32,8 @@ __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
 }
 
-// ---- router of many rows: 16 rows per workgroup, 8 waves split K ---------------------------------------------------------
-constexpr int RTW = 8;
-template <typename T, int NE>                          // NE: 16-expert tiles
+// ---- router of many rows: 16 rows per workgroup, RTW waves split K ---------------------------------------------------------
+template <typename T, int NE, int RTW>                 // NE: 16-expert tiles
 __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
   extern __shared__ __attribute__((aligned(16))) float sm[];      // partial tiles [RTW][NE][64][4]; then logits [16][16 NE], per wave weights | marks, choices
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
@@ -43,20 +42,31 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
   f32x4 acc[NE];
 #pragma unroll
   for (int t = 0; t < NE; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = wave * 32; k < c.ld; k += RTW * 32) {
-    float v[8];
-    load8f<float>(x + k, v);
-    T hi[8], lo[8];
+  constexpr int KU = NE <= 2 ? 4 : (NE <= 4 ? 2 : 1);               // k steps whose loads are in flight together
+  for (int k0 = wave * 32; k0 < c.ld; k0 += KU * RTW * 32) {
+    float v[KU][8];
+    u32x4 b[KU][NE];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) { hi[i] = (T)v[i]; lo[i] = (T)(v[i] - (float)hi[i]); }
-    const u32x4 ah = __builtin_bit_cast(u32x4, hi), al = __builtin_bit_cast(u32x4, lo);
+    for (int u = 0; u < KU; ++u) {
+      const int k = min(k0 + u * RTW * 32, c.ld - 32);               // (steps beyond the row: loaded, not used)
+      load8f<float>(x + k, v[u]);
 #pragma unroll
-    for (int t = 0; t < NE; ++t) {
-      const u32x4 b = *(const u32x4*)((const T*)c.router + (size_t)min(t * 16 + c16, E - 1) * c.ld + k + 8 * g4);
-      acc[t] = mfma16<T>(ah, b, acc[t]);
-      acc[t] = mfma16<T>(al, b, acc[t]);
+      for (int t = 0; t < NE; ++t) b[u][t] = *(const u32x4*)((const T*)c.router + (size_t)min(t * 16 + c16, E - 1) * c.ld + k + 8 * g4);
     }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int u = 0; u < KU; ++u)
+      if (k0 + u * RTW * 32 < c.ld) {
+        T hi[8], lo[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) { hi[i] = (T)v[u][i]; lo[i] = (T)(v[u][i] - (float)hi[i]); }
+        const u32x4 ah = __builtin_bit_cast(u32x4, hi), al = __builtin_bit_cast(u32x4, lo);
+#pragma unroll
+        for (int t = 0; t < NE; ++t) {
+          acc[t] = mfma16<T>(ah, b[u][t], acc[t]);
+          acc[t] = mfma16<T>(al, b[u][t], acc[t]);
+        }
+      }
   }
 #pragma unroll
   for (int t = 0; t < NE; ++t) *(f32x4*)(sm + ((wave * NE + t) * 64 + lane) * 4) = acc[t];
@@ -98,7 +108,7 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
 template <typename T>
 int route_at(const MoeCall& c, hipStream_t st) {
   const int ne = (c.r.experts + 15) / 16;
-  auto go = [&](auto k, int NE) -> int {
+  auto go = [&](auto k, int NE, int RTW) -> int {
     const size_t part = (size_t)RTW * NE * 1024,
                  pick = ((size_t)16 * 16 * NE + RTW * route_lds_floats(c.r) + 16 * c.r.top + c.r.experts) * sizeof(float);
     const size_t lds = std::max(part, pick);
@@ -107,11 +117,11 @@ int route_at(const MoeCall& c, hipStream_t st) {
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
-  if (ne <= 1) return go(route_kernel<T, 1>, 1);
-  if (ne <= 2) return go(route_kernel<T, 2>, 2);
-  if (ne <= 4) return go(route_kernel<T, 4>, 4);
-  if (ne <= 8) return go(route_kernel<T, 8>, 8);
-  return go(route_kernel<T, 16>, 16);                  // (route_fused: at most ROUTE_MFMA_EXPERTS)
+  if (ne <= 1) return go(route_kernel<T, 1, 16>, 1, 16);
+  if (ne <= 2) return go(route_kernel<T, 2, 16>, 2, 16);
+  if (ne <= 4) return go(route_kernel<T, 4, 16>, 4, 16);
+  if (ne <= 8) return go(route_kernel<T, 8, 16>, 8, 16);
+  return go(route_kernel<T, 16, 8>, 16, 8);                  // (route_fused: at most ROUTE_MFMA_EXPERTS)
 }
 constexpr int ROUTE_MFMA_EXPERTS = 256;
 
