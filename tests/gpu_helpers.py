@@ -130,3 +130,64 @@ def gemm_prefill(ol: L.OpLinear, x, M, act, *, epi=0, out=None, ldo=0, resid=Non
     ms = C.c_float(0.0)
     L.check(L.lib().mi_op_gemm_prefill(C.byref(ol), C.byref(a), int(iters), C.byref(ms)))
     return ms.value if iters >= 1 else None
+
+
+def serve_and_compare(model_dir, scheduler, oracle, cfg, greedy):
+    """``python -m mlx_parallm_amd.cli`` on a checkpoint of this design: concurrent completions of unequal prompts are the plain
+    implementation's greedy tokens, a streamed chat ends."""
+    import concurrent.futures
+    import os
+    import signal
+    import subprocess
+    import sys
+    import time
+    from pathlib import Path
+
+    import requests
+
+    from mlx_parallm_amd.tokenizer_utils import load_tokenizer
+    from tests.test_gpu_server import _free_port
+
+    root = Path(__file__).resolve().parent.parent
+
+    w = oracle.random_model(cfg, 6)
+    oracle.save_model(model_dir, cfg, w, "float32")
+    w, tok, port = oracle.as_f64(w), load_tokenizer(str(model_dir)), _free_port()
+    env = dict(os.environ, PYTHONPATH=str(root) + os.pathsep + os.environ.get("PYTHONPATH", ""))
+    log = model_dir / "server.log"
+    with open(log, "w") as lf:
+        proc = subprocess.Popen([sys.executable, "-m", "mlx_parallm_amd.cli", "--model-path", str(model_dir), "--port", str(port), "--host", "127.0.0.1",
+                                 "--scheduler", scheduler, "--batch-timeout", "0.2"], cwd=str(root), stdout=lf, stderr=subprocess.STDOUT, env=env)
+    base = f"http://127.0.0.1:{port}"
+    try:
+        end = time.time() + 90
+        while True:
+            try:
+                if requests.get(f"{base}/health", timeout=2).ok:
+                    break
+            except requests.RequestException:
+                pass
+            assert proc.poll() is None and time.time() < end, log.read_text()[-2000:]
+            time.sleep(0.3)
+        prompts = ["Say hello.", "A", "A somewhat longer prompt than the other two, to be cut into portions: " + 8 * "abc "]
+
+        def ask(p):
+            return requests.post(f"{base}/v1/completions", timeout=60,
+                                 json={"model": str(model_dir), "prompt": p, "max_tokens": 9, "temperature": 0.0}).json()
+        with concurrent.futures.ThreadPoolExecutor(3) as ex:
+            got = list(ex.map(ask, prompts))
+        for p, g in zip(prompts, got):
+            want = greedy(cfg, w, tok.encode(p), 9)
+            if tok.eos_token_id in want:
+                want = want[:want.index(tok.eos_token_id)]
+            assert g["choices"][0]["text"] == tok.decode(want, skip_special_tokens=True), (p, g)
+        with requests.post(f"{base}/v1/chat/completions", stream=True, timeout=60, json={
+                "model": str(model_dir), "messages": [{"role": "user", "content": "hi"}], "max_tokens": 6, "temperature": 0.7, "stream": True}) as r:
+            lines = [x for x in r.iter_lines(decode_unicode=True) if x]
+        assert r.status_code == 200 and lines[-1].strip() == "data: [DONE]" and "error" not in lines[0], lines[:2]
+    finally:
+        proc.send_signal(signal.SIGTERM)
+        try:
+            proc.wait(timeout=20)
+        except subprocess.TimeoutExpired:
+            proc.kill()

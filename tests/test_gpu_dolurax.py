@@ -9,6 +9,7 @@ import pytest
 
 from oracle import ref_dolurax as R
 from tests.dolurax_models import CONFIGS, attn, config, layer, moe
+from tests.gpu_helpers import serve_and_compare
 
 pytestmark = pytest.mark.gpu
 ROOT = Path(__file__).resolve().parent.parent
@@ -298,6 +299,27 @@ def test_long_decoding_behind_a_long_prompt(bank):
         assert worst(e, clear, "bfloat16") < TOL["bfloat16"] and (e[clear] > TOL["bfloat16"]).mean() < 0.02
 
 
+@pytest.mark.parametrize("dtype", ["bfloat16", "float16"])
+@pytest.mark.parametrize("cap", [1.0, 6.0, None])
+def test_keys_beyond_the_reach_of_the_distance_bias(bank, cap, dtype):
+    """Steep slopes and small caps: the kernels leave out keys whose capped score cannot matter any more, nothing else.  Large norms:
+    scores run into the cap, where its polynomial does not hold."""
+    mix = attn(6, 2, 32, 48, 0, 0.4, cap, False)
+    cfg = config(64, 96, [layer(mix), layer({**mix, "mask": {"size": 300}})], logit_scale=1.0, logit_softcap=None)
+
+    def edit(w):
+        for k in w:
+            if k.endswith(("q.norm", "k.norm")):
+                w[k] = w[k] * (1.5 if k.startswith("l1") else 0.5)
+    cfg, w, m = bank(f"reach_{cap}", dtype, cfg, edit)
+    t = tokens(cfg, 700, 8)
+    want = R.forward(cfg, w, t)
+    for sizes in ([700], [299, 2, 1, 1, 1, 96, 300], [600] + [1] * 100):
+        kv = m.engine.new_paged_kv(1, block_tokens=64, n_blocks=12, max_tokens_per_row=704)
+        assert np.quantile(err(run_portions(m.engine, kv, 0, t, sizes), want), 0.99) < TOL[dtype], sizes[:2]
+        kv.close()
+
+
 def test_growth_of_a_contiguous_cache_keeps_keys_and_values(bank):
     cfg, w, m = bank("odd")
     t = tokens(cfg, 120, 9)
@@ -418,3 +440,12 @@ def test_trace_replay_program(bank, tmp_path):
     for step, want in ((0, wa[[59, 3]]), (1, wa[[60]]), (2, np.stack([wa[69], wb[8]]))):
         got = np.fromfile(tmp_path / f"{step}.f32", "<f4").reshape(want.shape)
         assert err(got, want).max() < TOL["float32"]
+
+
+@pytest.mark.parametrize("scheduler", ["default", "continuous"])
+def test_server_program_completes_and_streams(tmp_path, scheduler):
+    from mlx_parallm_amd.tiny_model import build_byte_tokenizer
+
+    cfg = config(72, build_byte_tokenizer(tmp_path), [layer(attn(4, 2, 20, 24, 33), moe(6, 2, 40, 3, 2, 24)), layer(attn(3, 3, 16, 16, 50)),
+                                                     layer(attn(2, 1, 32, 48, 0), moe(5, 3, 24))])
+    serve_and_compare(tmp_path, scheduler, R, cfg, greedy)

@@ -2,13 +2,13 @@
 reused rows and blocks, each mechanism alone, greedy generation through the framework's own entry points."""
 import json
 import subprocess
-import sys
 from pathlib import Path
 
 import numpy as np
 import pytest
 
 from oracle import ref_runevik as R
+from tests.gpu_helpers import serve_and_compare
 from tests.runevik_models import CONFIGS, config, delta, latent
 
 pytestmark = pytest.mark.gpu
@@ -366,58 +366,7 @@ def test_trace_replay_program(bank, tmp_path):
 
 @pytest.mark.parametrize("scheduler", ["default", "continuous"])
 def test_server_program_completes_and_streams(tmp_path, scheduler):
-    """``python -m mlx_parallm_amd.cli`` on a checkpoint of this design: concurrent completions of unequal prompts are the plain
-    implementation's greedy tokens, a streamed chat ends."""
-    import concurrent.futures
-    import os
-    import signal
-    import time
-
-    import requests
-
     from mlx_parallm_amd.tiny_model import build_byte_tokenizer
-    from mlx_parallm_amd.tokenizer_utils import load_tokenizer
-    from tests.test_gpu_server import _free_port
 
     cfg = config(72, build_byte_tokenizer(tmp_path), [delta(4, 2, 20, 24, 3, 80), latent(3, 16, 24, 40, 0.4, 72), latent(2, 24, 16, 40, 0.3, 0, 1)], 8)
-    w = R.random_model(cfg, 6)
-    R.save_model(tmp_path, cfg, w, "float32")
-    w, tok, port = R.as_f64(w), load_tokenizer(str(tmp_path)), _free_port()
-    env = dict(os.environ, PYTHONPATH=str(ROOT) + os.pathsep + os.environ.get("PYTHONPATH", ""))
-    log = tmp_path / "server.log"
-    with open(log, "w") as lf:
-        proc = subprocess.Popen([sys.executable, "-m", "mlx_parallm_amd.cli", "--model-path", str(tmp_path), "--port", str(port), "--host", "127.0.0.1",
-                                 "--scheduler", scheduler, "--batch-timeout", "0.2"], cwd=str(ROOT), stdout=lf, stderr=subprocess.STDOUT, env=env)
-    base = f"http://127.0.0.1:{port}"
-    try:
-        end = time.time() + 90
-        while True:
-            try:
-                if requests.get(f"{base}/health", timeout=2).ok:
-                    break
-            except requests.RequestException:
-                pass
-            assert proc.poll() is None and time.time() < end, log.read_text()[-2000:]
-            time.sleep(0.3)
-        prompts = ["Say hello.", "A", "A somewhat longer prompt than the other two, to be cut into portions: " + 8 * "abc "]
-
-        def ask(p):
-            return requests.post(f"{base}/v1/completions", timeout=60,
-                                 json={"model": str(tmp_path), "prompt": p, "max_tokens": 9, "temperature": 0.0}).json()
-        with concurrent.futures.ThreadPoolExecutor(3) as ex:
-            got = list(ex.map(ask, prompts))
-        for p, g in zip(prompts, got):
-            want = greedy(cfg, w, tok.encode(p), 9)
-            if tok.eos_token_id in want:
-                want = want[:want.index(tok.eos_token_id)]
-            assert g["choices"][0]["text"] == tok.decode(want, skip_special_tokens=True), (p, g)
-        with requests.post(f"{base}/v1/chat/completions", stream=True, timeout=60, json={
-                "model": str(tmp_path), "messages": [{"role": "user", "content": "hi"}], "max_tokens": 6, "temperature": 0.7, "stream": True}) as r:
-            lines = [x for x in r.iter_lines(decode_unicode=True) if x]
-        assert r.status_code == 200 and lines[-1].strip() == "data: [DONE]" and "error" not in lines[0], lines[:2]
-    finally:
-        proc.send_signal(signal.SIGTERM)
-        try:
-            proc.wait(timeout=20)
-        except subprocess.TimeoutExpired:
-            proc.kill()
+    serve_and_compare(tmp_path, scheduler, R, cfg, greedy)
