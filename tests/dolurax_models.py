@@ -40,6 +40,9 @@ CONFIGS = {
     # head sizes beyond the matrix-core kernels, more experts than the matrix-core router takes, no logit transformation
     "generic": config(128, 160, [layer(attn(2, 1, 144, 200, 45, 0.08), moe(300, 2, 8)), layer(attn(2, 2, 136, 100, 33, 0.1), moe(3, 1, 700))],
                       1e-5, 1.0, None),
+    # matrix-core and generic attention in one stack, mixed values between them
+    "both_forms": config(80, 120, [layer(attn(2, 1, 144, 64, 30, 0.08), moe(4, 2, 24)), layer(attn(4, 2, 48, 32, 41, 0.15)),
+                                   layer(attn(1, 1, 200, 64, 0, 0.07, None), moe(4, 1, 16, 4, 2, 8)), layer(attn(2, 1, 96, 64, 25, 0.1))]),
     # a wide row (several pieces per thread in the row kernels)
     "wide_row": config(2304, 96, [layer(attn(3, 1, 48, 64, 40), moe(4, 2, 64, 2, 2, 96)), layer(attn(2, 2, 64, 32, 25))]),
 }
