@@ -58,7 +58,7 @@ extern "C" {
 #define MI_POS_NONE 0
 #define MI_POS_SINUSOIDAL 1 /* added to the embeddings: entry 2i sin(p 10000^(-2i/width)), entry 2i+1 the cosine */
 #define MI_BLOCK_PARALLEL 0 /* x += mixer(norm(x)) + ff(norm(x)), one norm */
-#define MI_BLOCK_POST_NORM 1 /* x += norm1(mixer(x)), then x += norm2(ff(x)): the sublayers read x itself */
+#define MI_BLOCK_POST_NORM 1 /* x += norm1(mixer(x)), then x += norm2(ff(x)); nothing in front of mixer and ff */
 #define MI_NORM_VECTOR 0    /* RMS norm, a weight per coordinate */
 #define MI_NORM_SCALAR 1    /* RMS norm, one weight for all coordinates */
 #define MI_NORM_LAYER 2     /* layer norm (mean taken off), weight and bias per coordinate; MI_BLOCK_POST_NORM only */

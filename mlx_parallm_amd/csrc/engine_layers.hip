@@ -681,7 +681,7 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
   const int32_t* tok = e->tok_src ? e->tok_src : e->d_tokens;
   const bool post = d.block_form == MI_BLOCK_POST_NORM;
   auto norm_of = [&](int li) {
-    if (post) return RowNormW{nullptr, 0, 0.f};                // (the sublayers read the residual stream itself)
+    if (post) return RowNormW{nullptr, 0, 0.f};                // (no norm in front of a sublayer)
     const Vec32& v = li < d.num_layers ? e->list[li].norm : e->list_final_norm;
     return RowNormW{v.p, nstride, d.rms_norm_eps};
   };

@@ -1,5 +1,5 @@
 // moe.hip -- mixture of experts (layer-list models): a softmax router picks `top` experts per token among the `keep` best of
-// `groups` equal groups; an expert is W_down (silu(W_gate h) * W_up h); a shared expert runs for every token.  The weighted sum
+// `groups` equal groups; an expert is W_down (silu(W_gate h) * W_up h); the shared expert takes all tokens.  The weighted sum
 // over a token's slots is taken by the row kernel behind (layer_rows.hip: post_norm_kernel).
 //
 //   route       many rows: router logits on the matrix cores (x as hi + lo, so they keep 32-bit accuracy), softmax, groups, choice

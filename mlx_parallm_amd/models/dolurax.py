@@ -1,7 +1,7 @@
 """Dolurax model handle: chunked grouped-query attention and a mixture of experts, layer norms behind the sublayers
 (``config["architecture"] = "Dolurax"``).
 
-A layer is ``x += norm1(attention(x))``, then ``x += norm2(experts(x))``; the sublayers read the residual stream itself.  The
+A layer is ``x += norm1(attention(x))``, then ``x += norm2(experts(x))``, without a norm in front of either.  The
 configuration lists the layers with their own sizes, so the engine gets one ``mi_layer_desc`` per layer (``layer_list``); the
 handle around it is the one of the llama family.
 """
