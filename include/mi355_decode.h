@@ -35,7 +35,7 @@ extern "C" {
  * `struct_size`, which the caller sets to sizeof() of ITS definition -- a binding generated from another version of this
  * header (a shorter mi_sample_params would make the library read pointers past its end) is refused with MI_ERR_INVALID
  * by mi_engine_create / mi_decode_sample / mi_step_enqueue(_rows) / mi_score_tokens instead of being read. */
-#define MI_ABI_VERSION 4
+#define MI_ABI_VERSION 5
 
 #define MI_OK 0
 #define MI_ERR_INVALID (-1)
@@ -59,19 +59,27 @@ extern "C" {
 #define MI_POS_SINUSOIDAL 1 /* added to the embeddings: entry 2i sin(p 10000^(-2i/width)), entry 2i+1 the cosine */
 #define MI_BLOCK_PARALLEL 0 /* x += mixer(norm(x)) + ff(norm(x)), one norm */
 #define MI_BLOCK_POST_NORM 1 /* x += norm1(mixer(x)), then x += norm2(ff(x)); nothing in front of mixer and ff */
+#define MI_BLOCK_PRE_NORM 2 /* x += m mixer(norm1(x)), then x += m ff(norm2(x)); with `streams` copies of x (hyper-connections): a sublayer
+                             * reads u = sum_s in[s] x_s and writes x_t <- sum_s mix[s][t] x_s + m out[t] y, per layer and sublayer */
 #define MI_NORM_VECTOR 0    /* RMS norm, a weight per coordinate */
 #define MI_NORM_SCALAR 1    /* RMS norm, one weight for all coordinates */
 #define MI_NORM_LAYER 2     /* layer norm (mean taken off), weight and bias per coordinate; MI_BLOCK_POST_NORM only */
 /* mixers */
-#define MI_MIXER_DELTA 0    /* gated delta rule with short convolutions (recurrent state per cache row) */
+#define MI_MIXER_DELTA 0    /* gated delta rule with short convolutions (recurrent state per cache row); the decay is one number per
+                             * head, or one per head and key channel through a low-rank map (decay_rank) */
 #define MI_MIXER_LATENT 1   /* latent attention without positions (the cache holds one latent per token) */
-#define MI_MIXER_GQA 2      /* grouped-query attention without rotation: normed q / k, soft cap, distance bias, chunks of
-                             * positions, values mixed with an earlier layer's, sigmoid gate on the output (MI_BLOCK_POST_NORM) */
+#define MI_MIXER_GQA 2      /* grouped-query attention with normed q / k (post- and pre-norm blocks).  Each of: rotation, soft cap,
+                             * distance bias, chunks of positions or a sliding window with kept first tokens, sink, values mixed with
+                             * an earlier layer's, sigmoid gate on the output */
 /* feed-forward kinds and activations */
 #define MI_FF_DENSE 0
 #define MI_FF_MOE 1         /* routed experts and at most one shared expert (MI_BLOCK_POST_NORM) */
 #define MI_ACT_POLYNORM 0   /* a N(z) + b N(z^2) + c N(z^3) + e, N = division by the root mean square over the row */
 #define MI_ACT_SWIGLU 1     /* silu(gate) * up */
+/* gate on a mixer's output, element by element */
+#define MI_GATE_NONE 0
+#define MI_GATE_SILU 1
+#define MI_GATE_SIGMOID 2
 
 /* KV-cache element type selector for mi_kv_create */
 #define MI_KV_MODEL (-1) /* BatchedKVCache semantics: KV in the model dtype (models/base.py:66-85) */
@@ -107,6 +115,17 @@ typedef struct mi_model_desc {
   int32_t side_dim;          /* width of the per-layer token input added after each layer; 0 = none */
   float logit_scale;         /* logits = softcap(logit_scale * head x); 0 = 1 */
   float logit_softcap;       /* c tanh(z / c); 0 = none */
+  int32_t norm_offset;       /* 1: the weights of norm1, norm2 and the final norm are stored as their distance from one */
+  float embed_scale;         /* factor on the token embedding; 0 = 1 */
+  int32_t pair_buckets;      /* > 0: row (previous token * pair_mul_prev + token * pair_mul_cur) mod pair_buckets of the table "bigram" is
+                              * added to the embedding; a sequence's first token takes row pair_buckets */
+  int32_t pair_mul_prev;     /* both in [0, pair_buckets) */
+  int32_t pair_mul_cur;
+  float residual_mult;       /* MI_BLOCK_PRE_NORM: factor on a sublayer's output; 0 = 1 */
+  int32_t streams;           /* MI_BLOCK_PRE_NORM: copies of the residual stream (hyper-connections, at most 16); 0 = one, plain sums */
+  int32_t loop_start;        /* layers loop_start .. loop_stop - 1 run loop_times times in a row, every pass with a cache or state of */
+  int32_t loop_stop;         /* its own; loop_stop = 0: no loop */
+  int32_t loop_times;
 } mi_model_desc;
 
 /* one layer of a MI_ARCH_LAYERS model (num_heads, num_kv_heads, head_dim, intermediate_size of mi_model_desc are unused) */
@@ -136,6 +155,16 @@ typedef struct mi_layer_desc {
   int32_t groups;
   int32_t keep;
   int32_t shared_ff;         /* width of the shared expert, 0 = none */
+  int32_t out_gate;          /* delta, gqa: MI_GATE_* */
+  /* gqa */
+  int32_t rot_dims;          /* the first rot_dims (even) coordinates of a query or key head are rotated, coordinate i with i + rot_dims / 2 */
+  float rot_base;            /* by position * rot_base^(-2i / rot_dims); rot_dims = 0: none */
+  int32_t window;            /* i sees j <= i only if i - j < window or j < keep_first; 0 = all (not together with chunk) */
+  int32_t keep_first;
+  int32_t sink;              /* 1: the softmax denominator has the term exp(sink_h) as well */
+  /* delta */
+  int32_t decay_rank;        /* > 0: one decay per head and key channel, a = W_a2 (W_a1 h) with this inner size; 0: one per head, a = W_a h */
+  int32_t gate_rank;         /* > 0: gate = W_g2 (W_g1 h) with this inner size; 0: W_g h */
 } mi_layer_desc;
 
 /* arguments of the `sample` closure (utils.py:345-364) + top_p_sampling (sample_utils.py:3-38) */
@@ -274,7 +303,7 @@ int mi_step_enqueue_mixed(mi_engine* e, mi_kv* kv, const int32_t* rows, const in
 int mi_forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t* lens, int n, const int32_t* tokens,
                         const int32_t* out_idx, int n_out, float* logits_out);
 /* Tests: while `out` is set, every pass of a layer-list model copies the residual stream after each layer into it, as
- * [num_layers][tokens of the pass][width] floats (a pass that needs more than capacity_floats fails).  NULL = off. */
+ * [layer runs][tokens of the pass][width] floats (a looped layer counts once per pass; the sum of the streams, if there are several) (a pass that needs more than capacity_floats fails).  NULL = off. */
 int mi_debug_residual(mi_engine* e, float* out, int64_t capacity_floats);
 /* Forget the contents of one row (its length becomes 0); ordered behind the steps already enqueued. */
 int mi_kv_reset_row(mi_kv* kv, int row);

@@ -18,13 +18,14 @@ MI_F32, MI_BF16, MI_F16, MI_U32 = 0, 1, 2, 3
 MI_KV_MODEL = -1
 MI_ARCH_LLAMA, MI_ARCH_QWEN3, MI_ARCH_LAYERS = 0, 1, 2
 MI_POS_NONE, MI_POS_SINUSOIDAL = 0, 1
-MI_BLOCK_PARALLEL, MI_BLOCK_POST_NORM = 0, 1
+MI_BLOCK_PARALLEL, MI_BLOCK_POST_NORM, MI_BLOCK_PRE_NORM = 0, 1, 2
 MI_NORM_VECTOR, MI_NORM_SCALAR, MI_NORM_LAYER = 0, 1, 2
 MI_MIXER_DELTA, MI_MIXER_LATENT, MI_MIXER_GQA = 0, 1, 2
 MI_FF_DENSE, MI_FF_MOE = 0, 1
 MI_ACT_POLYNORM, MI_ACT_SWIGLU = 0, 1
+MI_GATE_NONE, MI_GATE_SILU, MI_GATE_SIGMOID = 0, 1, 2
 MI_MAX_TOP_LOGPROBS = 20
-MI_ABI_VERSION = 4
+MI_ABI_VERSION = 5
 WK = {"f32": 0, "bf16": 1, "f16": 2, "q4_f32": 3, "q4_bf16": 4, "q4_f16": 5, "q8_f32": 6, "q8_bf16": 7, "q8_f16": 8}
 RND_NONE, RND_BF16, RND_F16 = 0, 1, 2
 PRO_NONE, PRO_NORM = 0, 1
@@ -43,6 +44,9 @@ class ModelDesc(C.Structure):
         ("quant_bits", C.c_int32), ("quant_group_size", C.c_int32), ("max_positions", C.c_int32),
         ("position", C.c_int32), ("block_form", C.c_int32), ("norm_kind", C.c_int32), ("side_dim", C.c_int32),
         ("logit_scale", C.c_float), ("logit_softcap", C.c_float),
+        ("norm_offset", C.c_int32), ("embed_scale", C.c_float), ("pair_buckets", C.c_int32), ("pair_mul_prev", C.c_int32),
+        ("pair_mul_cur", C.c_int32), ("residual_mult", C.c_float), ("streams", C.c_int32), ("loop_start", C.c_int32),
+        ("loop_stop", C.c_int32), ("loop_times", C.c_int32),
     ]
 
 
@@ -53,6 +57,8 @@ class LayerDesc(C.Structure):
         ("unit_eps", C.c_float), ("ff", C.c_int32), ("act", C.c_int32),
         ("softcap", C.c_float), ("slope_exp", C.c_float), ("chunk", C.c_int32), ("v_mix", C.c_int32), ("ff_kind", C.c_int32),
         ("experts", C.c_int32), ("top", C.c_int32), ("groups", C.c_int32), ("keep", C.c_int32), ("shared_ff", C.c_int32),
+        ("out_gate", C.c_int32), ("rot_dims", C.c_int32), ("rot_base", C.c_float), ("window", C.c_int32), ("keep_first", C.c_int32),
+        ("sink", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32),
     ]
 
 

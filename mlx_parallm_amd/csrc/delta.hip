@@ -3,7 +3,8 @@
 //   q, k, v  = silu(short causal convolution of the projections);  q, k unit vectors per head, q scaled
 //   beta     = sigmoid(b),  g = exp(-exp(A_log) softplus(a + dt_bias))                      per value head
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q                            S: [d][e] float32
-//   out      = rms(o) * w * silu(gate)
+//   out      = rms(o) * w * silu(gate)       (or sigmoid)
+// The second form (channel) has a decay g_c per value head and key channel: row c of S is multiplied by g_c.
 //
 // State per cache row: S, and the last inputs of the convolutions in a ring (the input of position p lies in slot p mod taps:
 // a step reads the slots of p-1 .. p-taps+1 and writes the one of p, so the workgroups that share a q/k head may read while
@@ -17,6 +18,10 @@
 //                k_i . k_j (j < i), T = (I + A)^-1:  W = T diag(beta e^G) K,  U = T diag(beta) V,  P_ij = e^(G_i - G_j) q_i . k_j (j <= i)
 //   delta_carry  the chunks of a segment in order, a workgroup per 16 columns of S:
 //                X = U - W S,  O = diag(e^G) Q S + P X,  S <- e^(G_last) S + K^T diag(e^(G_last - G)) X
+// With a decay per channel the factors belong to elements of Q and K instead of rows: delta_chunk_channel makes
+//                A_ij = beta_i sum_c k_ic k_jc D_ijc,  P_ij = sum_c q_ic k_jc D_ijc,  D_ijc = product of g_c over the tokens j + 1 .. i
+// without ever dividing by a decay: between blocks of 16 tokens D is (start of i's block .. i) x (blocks between) x (j + 1 .. end of j's
+// block), each at most one, so those tiles are matrix products of scaled rows; inside a block D is a running product.
 // Short portions, and sizes the chunk kernels do not take: delta_prep (convolutions, norms, gates, all tokens in parallel) ->
 // delta_scan (token by token; columns of S are independent, so a wave owns four columns and keeps them in registers, 16 lanes
 // per column).  Both end in delta_out.
@@ -52,8 +57,14 @@ __device__ __forceinline__ Chan channel(const DeltaCall& c, int ch) {
   return {c.o_v + ch - 2 * gd, c.conv_v + (size_t)(ch - 2 * gd) * c.taps};
 }
 
-__device__ __forceinline__ float decay_of(const DeltaCall& c, int h, float a) {
-  return expf(-expf(c.A_log[h]) * softplus_f(a + c.dt_bias[h]));
+// i: the head, or (channel) head * d + channel
+__device__ __forceinline__ float decay_of(const DeltaCall& c, int h, int i, float a) {
+  return expf(-expf(c.A_log[h]) * softplus_f(a + c.dt_bias[i]));
+}
+template <typename T>
+__device__ __forceinline__ float out_gate(const DeltaCall& c, int r, int i) {
+  const float z = to_f32(((const T*)c.gp)[(size_t)r * c.ldgp + c.o_g + i]);
+  return c.gate_act == MI_GATE_SIGMOID ? sigmoid_f(z) : silu_f(z);
 }
 
 template <int VEC> struct Vec;
@@ -61,14 +72,14 @@ template <> struct Vec<1> { float v[1]; };
 template <> struct alignas(16) Vec<4> { float v[4]; };
 
 // grid (one-token segments, H + (ff ? 1 : 0)).  MAXR > 0: the thread's rows of S stay in registers between the two passes.
+// CHAN: a decay per channel.
 constexpr int DNT = 512;
-template <typename T, int VEC, int MAXR>
+template <typename T, int VEC, int MAXR, bool CHAN>
 __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
   __shared__ float red[DNT / 64 * 3];
   __shared__ Vec<VEC> part[2][DNT];
-  __shared__ float ks[512], qs[512];
+  __shared__ float ks[512], qs[512], gs[CHAN ? 512 : 1];
   __shared__ float vs[DNT * VEC];
-  __shared__ float sh[2];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int seg = c.t.dec[blockIdx.x], r = c.t.tok0[seg], row = c.t.row[seg], pos = c.t.off[row];
   const T* proj = (const T*)c.proj;
@@ -108,13 +119,21 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
     if (i < d) qs[i] = y; else if (i < 2 * d) ks[i - d] = y; else vs[i - 2 * d] = y;
     if (i >= 2 * d || h % hg == 0) ring[(size_t)(pos % K) * C + ch] = pr[cn.col];
   }
+  const T* ar = (const T*)c.ap + (size_t)r * c.ldap + c.o_a;
+  if constexpr (CHAN) {
+    for (int i = tid; i < d; i += DNT) gs[i] = decay_of(c, h, h * d + i, to_f32(ar[h * d + i]));
+  }
   __syncthreads();
   float n3[3] = {0.f, 0.f, 0.f};
   for (int i = tid; i < d; i += DNT) { n3[0] += qs[i] * qs[i]; n3[1] += ks[i] * ks[i]; n3[2] += qs[i] * ks[i]; }
   block_sum<DNT, 3>(n3, red);
   const float iq = c.scale / sqrtf(n3[0] + c.unit_eps), ik = 1.0f / sqrtf(n3[1] + c.unit_eps);
   const float kq = n3[2] * iq * ik;
-  const float g = decay_of(c, h, to_f32(pr[c.o_a + h])), beta = sigmoid_f(to_f32(pr[c.o_b + h]));
+  const float beta = sigmoid_f(to_f32(pr[c.o_b + h]));
+  float g = 1.f;
+  if constexpr (!CHAN) g = decay_of(c, h, h, to_f32(ar[h]));
+  auto row_decay = [&](int dr) { if constexpr (CHAN) return gs[dr]; else return g; };      // of row dr of S
+  auto in_row = [&](const float* x, int dr) { if constexpr (CHAN) return x[dr] * gs[dr]; else return x[dr]; };   // (one decay: applied to the sums)
 
   Vec<VEC> pa, pb;
 #pragma unroll
@@ -124,7 +143,7 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
 #pragma unroll
       for (int i = 0; i < MAXR; ++i) {
         const int dr = sl + i * slices;
-        const float kk = dr < d ? ks[dr] : 0.f, qq = dr < d ? qs[dr] : 0.f;
+        const float kk = dr < d ? in_row(ks, dr) : 0.f, qq = dr < d ? in_row(qs, dr) : 0.f;
 #pragma unroll
         for (int j = 0; j < VEC; ++j) { pa.v[j] = fmaf(s[i].v[j], kk, pa.v[j]); pb.v[j] = fmaf(s[i].v[j], qq, pb.v[j]); }
       }
@@ -132,7 +151,7 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
       for (int dr = sl; dr < d; dr += slices) {
         const Vec<VEC> x = *(const Vec<VEC>*)(S + (size_t)dr * e + col * VEC);
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) { pa.v[j] = fmaf(x.v[j], ks[dr], pa.v[j]); pb.v[j] = fmaf(x.v[j], qs[dr], pb.v[j]); }
+        for (int j = 0; j < VEC; ++j) { pa.v[j] = fmaf(x.v[j], in_row(ks, dr), pa.v[j]); pb.v[j] = fmaf(x.v[j], in_row(qs, dr), pb.v[j]); }
       }
     }
     part[0][tid] = pa; part[1][tid] = pb;
@@ -161,10 +180,10 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
       for (int i = 0; i < MAXR; ++i) {
         const int dr = sl + i * slices;
         if (dr < d) {
-          const float kk = ks[dr] * ik;
+          const float kk = ks[dr] * ik, gr = row_decay(dr);
           Vec<VEC> x;
 #pragma unroll
-          for (int j = 0; j < VEC; ++j) x.v[j] = fmaf(kk, u.v[j], g * s[i].v[j]);
+          for (int j = 0; j < VEC; ++j) x.v[j] = fmaf(kk, u.v[j], gr * s[i].v[j]);
           *(Vec<VEC>*)(S + (size_t)dr * e + col * VEC) = x;
         }
       }
@@ -176,7 +195,7 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
         for (int j = 0; j < VEC; ++j) x.v[j] = 0.f;
         if (pos > 0) x = *p;
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) x.v[j] = fmaf(ks[dr] * ik, u.v[j], g * x.v[j]);
+        for (int j = 0; j < VEC; ++j) x.v[j] = fmaf(ks[dr] * ik, u.v[j], row_decay(dr) * x.v[j]);
         *p = x;
       }
     }
@@ -187,10 +206,10 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
       const int k = col * VEC + j;
-      cat[h * e + k] = from_f32<T>(o.v[j] * rs * c.head_norm[k] * silu_f(to_f32(pr[c.o_g + h * e + k])));
+      cat[h * e + k] = from_f32<T>(o.v[j] * rs * c.head_norm[k] * out_gate<T>(c, r, h * e + k));
     }
   }
-  (void)lane; (void)wave; (void)sh;
+  (void)lane; (void)wave;
 }
 
 // ---- longer segments -----------------------------------------------------------------------------------------------
@@ -205,6 +224,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaCall c) {
   const T* ring = (const T*)c.ring + (size_t)at.row * K * C;
   float* out = c.scan + (size_t)r * c.lds;
   const T* pr = proj + (size_t)r * c.ldp;
+  const T* ar = (const T*)c.ap + (size_t)r * c.ldap + c.o_a;
   const int hg = c.H / c.G;
   // q and k: a wave per q/k head, which also leaves the gates of its value heads
   for (int hh = wave; hh < c.G; hh += 4) {
@@ -223,13 +243,15 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(DeltaCall c) {
     for (int j = lane; j < hg; j += 64) {
       const int h = hh * hg + j;
       float* ga = c.gate + (size_t)r * c.ldg + 4 * h;
-      *(float4*)ga = float4{decay_of(c, h, to_f32(pr[c.o_a + h])), sigmoid_f(to_f32(pr[c.o_b + h])), qk, 0.f};
+      *(float4*)ga = float4{c.channel ? 1.f : decay_of(c, h, h, to_f32(ar[h])), sigmoid_f(to_f32(pr[c.o_b + h])), qk, 0.f};
     }
   }
   for (int i = tid; i < c.H * c.e; i += 256) {
     const Chan cn = channel(c, 2 * gd + i);
     out[2 * gd + i] = silu_f(conv_at<T>(proj, c.ldp, cn.col, r, at.t, at.pos, ring, C, 2 * gd + i, cn.taps, K));
   }
+  if (c.channel)
+    for (int i = tid; i < c.H * c.d; i += 256) out[C + i] = decay_of(c, i / c.d, i, to_f32(ar[i]));
 }
 
 // the last inputs of a segment's convolutions into the ring (whoever reads it in this call ran in an earlier launch);
@@ -255,12 +277,13 @@ __device__ __forceinline__ void put_ring(const DeltaCall& c, int h, int gq, int 
 // The operands of TC tokens at a time are staged in LDS (two buffers; the next ones travel in registers during the current
 // ones' arithmetic): q and k of the head, v of the workgroup's 16 columns, decay, step size and k . q.  Per token, with
 // a = S^T k and b = S^T q of the state BEFORE the token:  u = beta (v - g a),  o = g b + (k . q) u,  S <- g S + k u^T.
-template <typename T, int DPL>
+// CHAN: the head's decays are staged beside q and k, and S is multiplied by them before the two products.
+template <typename T, int DPL, bool CHAN>
 __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaCall c) {
   constexpr int DP = 16 * DPL;                        // padded state rows
-  constexpr int TC = DPL <= 16 ? 16 : 8;
-  constexpr int NQK = (TC * 2 * DP + 255) / 256;      // staged q / k floats per thread
-  __shared__ float qk[2][TC][2][DP];
+  constexpr int TC = DPL <= 12 || (DPL <= 16 && !CHAN) ? 16 : 8, NR = CHAN ? 3 : 2;
+  constexpr int NQK = (TC * NR * DP + 255) / 256;     // staged q / k (/ decay) floats per thread
+  __shared__ float qk[2][TC][NR][DP];
   __shared__ float vb[2][TC][16];
   __shared__ float ga[2][TC][4];
   __shared__ float ob[TC][16];
@@ -284,8 +307,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaCall c) {
   auto load = [&](int t0) {
 #pragma unroll
     for (int i = 0; i < NQK; ++i) {
-      const int x = i * 256 + tid, t = min(t0 + x / (2 * DP), n - 1), w = (x / DP) & 1, dd = x % DP;
-      const float v = base[(size_t)t * c.lds + w * gd + gq * d + min(dd, d - 1)];
+      const int x = i * 256 + tid, t = min(t0 + x / (NR * DP), n - 1), w = x / DP % NR, dd = x % DP;
+      const float v = base[(size_t)t * c.lds + (w < 2 ? w * gd + gq * d : 2 * gd + c.H * e + h * d) + min(dd, d - 1)];
       rqk[i] = dd < d ? v : 0.f;
     }
     rv = base[(size_t)min(t0 + min(vt, TC - 1), n - 1) * c.lds + 2 * gd + h * e + min((int)blockIdx.x * 16 + vc, e - 1)];
@@ -295,7 +318,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaCall c) {
 #pragma unroll
     for (int i = 0; i < NQK; ++i) {
       const int x = i * 256 + tid;
-      if (x < TC * 2 * DP) (&qk[buf][0][0][0])[x] = rqk[i];
+      if (x < TC * NR * DP) (&qk[buf][0][0][0])[x] = rqk[i];
     }
     if (vt < TC) vb[buf][vt][vc] = rv;
     if (tid < 4 * TC) ga[buf][gt][gi] = rg;
@@ -314,6 +337,10 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaCall c) {
       float k[DPL], q[DPL];
 #pragma unroll
       for (int i = 0; i < DPL; ++i) { k[i] = kp[i]; q[i] = qp[i]; }
+      if constexpr (CHAN) {
+#pragma unroll
+        for (int i = 0; i < DPL; ++i) s[i] *= qk[buf][t][NR - 1][d0 + i];
+      }
       float a[2] = {0.f, 0.f}, b[2] = {0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < DPL; ++i) { a[i & 1] = fmaf(s[i], k[i], a[i & 1]); b[i & 1] = fmaf(s[i], q[i], b[i & 1]); }
@@ -433,7 +460,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(DeltaCall c) {
     const T* pr = (const T*)c.proj + (size_t)(r0 + min(lane, n - 1)) * c.ldp;
     const bool on = lane < n;
     const float beta = on ? sigmoid_f(to_f32(pr[c.o_b + h])) : 0.f;
-    double g = on ? -(double)expf(c.A_log[h]) * (double)softplus_f(to_f32(pr[c.o_a + h]) + c.dt_bias[h]) : 0.0;
+    const T* ar = (const T*)c.ap + (size_t)(r0 + min(lane, n - 1)) * c.ldap + c.o_a;
+    double g = on ? -(double)expf(c.A_log[h]) * (double)softplus_f(to_f32(ar[h]) + c.dt_bias[h]) : 0.0;
 #pragma unroll
     for (int s = 1; s < 64; s *= 2) {
       const double o = __shfl_up(g, s, 64);
@@ -563,6 +591,252 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(DeltaCall c) {
   }
 }
 
+// ---- a decay per channel: grid (chunks, H), 8 waves ----------------------------------------------------------------------
+// T = (I + A)^-1 in place of A by the first four waves (all waves of the workgroup call this): block (i, j) of T ends up at block (j, i)
+__device__ __forceinline__ void invert_chunk(float* am, int LA, int wave, int c16, int g4) {
+  f32x4 tb[4];
+  const int o = 16 * wave;
+  if (wave < 4) {
+    float tc[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == c16 ? 1.f : 0.f;
+#pragma unroll
+      for (int l = 0; l < i; ++l) v = fmaf(-am[(o + i) * LA + o + l], tc[l], v);
+      tc[i] = v;
+    }
+    f32x4 t;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) t[r] = g4 == 0 ? tc[r] : (g4 == 1 ? tc[4 + r] : (g4 == 2 ? tc[8 + r] : tc[12 + r]));
+#pragma unroll
+    for (int i = 0; i < 4; ++i) tb[i] = t;
+  }
+  __syncthreads();
+  if (wave < 4) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) am[(o + 4 * g4 + r) * LA + o + c16] = tb[0][r];
+  }
+  __syncthreads();
+  if (wave < 4) {
+#pragma unroll
+    for (int i = 1; i < 4; ++i) {
+      if (i <= wave) continue;
+      f32x4 m = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int l = 0; l < i; ++l)
+        if (l >= wave) m = mfma_slice(*(const f32x4*)(am + (16 * i + c16) * LA + 16 * l + 4 * g4), tb[l], m);
+      const f32x4 z = {0.f, 0.f, 0.f, 0.f};
+      tb[i] = -mfma_slice(*(const f32x4*)(am + (16 * i + c16) * LA + 16 * i + 4 * g4), m, z);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) am[(16 * wave + 4 * g4 + r) * LA + 16 * i + c16] = tb[i][r];
+    }
+  }
+  __syncthreads();
+}
+
+template <typename T, int DP>
+__global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c) {
+  constexpr int LK = DP + 4, LA = CH + 4, NS = DP / 16;
+  extern __shared__ __attribute__((aligned(16))) float csm[];
+  float* ks = csm;                                    // [CH][LK] unit keys
+  float* qs = ks + CH * LK;                           // unit queries; from step 3 on times the decay from their block's start
+  float* gs = qs + CH * LK;                           // decays of the tokens; from step 3 on the decay from the block's start to the token
+  float* kr = gs + CH * LK;                           // step 2: partial sums; from step 3 on the keys times the decay to their block's end
+  float* am = kr + CH * LK;                           // [CH][LA] as in delta_chunk_kernel
+  float* tot = am + CH * LA;                          // [4][DP] a block's whole decay
+  __shared__ float be[CH];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int h = blockIdx.y, seg = c.t.ctile[2 * blockIdx.x], t0 = c.t.ctile[2 * blockIdx.x + 1];
+  const int r0 = c.t.tok0[seg] + t0, n = min(CH, c.t.len[seg] - t0);
+  const int d = c.d, e = c.e, gd = c.G * d, gq = h / (c.H / c.G);
+  const float* qb = c.scan + (size_t)r0 * c.lds + gq * d;
+  const float* kb = qb + gd;
+  float* vb = c.scan + (size_t)r0 * c.lds + 2 * gd + (size_t)h * e;
+
+  // 1. unit keys and queries (eight threads per token), decays; tokens beyond the end: zero vectors, decay one
+  {
+    const int t = tid >> 3, p = tid & 7;
+    constexpr int NV = (DP + 31) / 32;
+    float sk = 0.f, sq = 0.f;
+    f32x4 kv[NV], qv[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int k = 32 * i + 4 * p;
+      kv[i] = qv[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (t < n && k < d) {
+        kv[i] = *(const f32x4*)(kb + (size_t)t * c.lds + k);
+        qv[i] = *(const f32x4*)(qb + (size_t)t * c.lds + k);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { sk += kv[i][j] * kv[i][j]; sq += qv[i][j] * qv[i][j]; }
+      }
+    }
+#pragma unroll
+    for (int s = 1; s < 8; s *= 2) { sk += __shfl_xor(sk, s, 64); sq += __shfl_xor(sq, s, 64); }
+    const float ik = 1.0f / sqrtf(sk + c.unit_eps), iq = c.scale / sqrtf(sq + c.unit_eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      *(f32x4*)(ks + t * LK + 32 * i + 4 * p) = kv[i] * ik;
+      *(f32x4*)(qs + t * LK + 32 * i + 4 * p) = qv[i] * iq;
+    }
+    const T* ar = (const T*)c.ap + (size_t)r0 * c.ldap + c.o_a + h * d;
+    const float ea = expf(c.A_log[h]);
+    for (int i = tid; i < CH * DP; i += 512) {
+      const int tt = i / DP, ch = i % DP;
+      float g = 1.f;
+      if (tt < n && ch < d) g = expf(-ea * softplus_f(to_f32(ar[(size_t)tt * c.ldap + ch]) + c.dt_bias[h * d + ch]));
+      gs[tt * LK + ch] = g;
+    }
+    if (tid < CH) be[tid] = tid < n ? sigmoid_f(to_f32(((const T*)c.proj)[(size_t)(r0 + tid) * c.ldp + c.o_b + h])) : 0.f;
+  }
+  __syncthreads();
+
+  // 2. the blocks on the diagonal: wave w has block w mod 4 and every second 16-channel slice, lane (c16, g4) column c16 and four
+  // channels of a slice.  p runs down the column: k_j at token j, times a token's decay from there on (above the diagonal zero).
+  float sa[16], sp[16];
+  {
+    const int b = wave & 3;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) sa[i] = sp[i] = 0.f;
+    for (int s = wave >> 2; s < NS; s += 2) {
+      const int k = 16 * s + 4 * g4;
+      const f32x4 kj = *(const f32x4*)(ks + (16 * b + c16) * LK + k);
+      f32x4 p = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int at = (16 * b + i) * LK + k;
+        const f32x4 g = *(const f32x4*)(gs + at), ki = *(const f32x4*)(ks + at), qi = *(const f32x4*)(qs + at);
+        p *= g;
+        if (i == c16) p = kj;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) { sa[i] = fmaf(p[j], ki[j], sa[i]); sp[i] = fmaf(p[j], qi[j], sp[i]); }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      sa[i] += __shfl_xor(sa[i], 16, 64); sa[i] += __shfl_xor(sa[i], 32, 64);
+      sp[i] += __shfl_xor(sp[i], 16, 64); sp[i] += __shfl_xor(sp[i], 32, 64);
+    }
+    if (wave >= 4 && g4 == 0) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) { kr[(b * 32 + i) * 16 + c16] = sa[i]; kr[(b * 32 + 16 + i) * 16 + c16] = sp[i]; }
+    }
+  }
+  __syncthreads();
+  if (wave < 4) {                                     // lane (c16, g4): rows 4 g4 .. 4 g4 + 3 of column c16
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      if (i / 4 != g4) continue;
+      const float a = sa[i] + kr[(wave * 32 + i) * 16 + c16], p = sp[i] + kr[(wave * 32 + 16 + i) * 16 + c16];
+      const int row = 16 * wave + i, col = 16 * wave + c16;
+      am[row * LA + col] = i > c16 ? be[row] * a : 0.f;
+      if (row < n) c.pm[((size_t)(r0 + row) * c.H + h) * CH + col] = i >= c16 ? p : 0.f;
+    }
+  }
+  __syncthreads();
+
+  // 3. decays inside the blocks: a thread per channel and block
+  if (tid < 4 * DP) {
+    const int b = tid / DP, ch = tid % DP, at = 16 * b * LK + ch;
+    float g[16], suf = 1.f, pre = 1.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) g[i] = gs[at + i * LK];
+#pragma unroll
+    for (int i = 15; i >= 0; --i) { kr[at + i * LK] = ks[at + i * LK] * suf; suf *= g[i]; }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) { pre *= g[i]; gs[at + i * LK] = pre; qs[at + i * LK] *= pre; }
+    tot[b * DP + ch] = suf;
+  }
+  __syncthreads();
+
+  // 4. the six tiles below the diagonal, of A and of P
+  for (int job = wave; job < 12; job += 8) {
+    const bool isq = job & 1;
+    const int pr = job >> 1, ti = pr < 1 ? 1 : (pr < 3 ? 2 : 3), tj = pr - ti * (ti - 1) / 2;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      const int k = 16 * s + 4 * g4, at = (16 * ti + c16) * LK + k;
+      const f32x4 a = isq ? *(const f32x4*)(qs + at) : *(const f32x4*)(ks + at) * *(const f32x4*)(gs + at);
+      f32x4 b = *(const f32x4*)(kr + (16 * tj + c16) * LK + k);
+      for (int m = tj + 1; m < ti; ++m) b *= *(const f32x4*)(tot + m * DP + k);
+      acc = mfma_slice(a, b, acc);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 16 * ti + 4 * g4 + r, j = 16 * tj + c16;
+      if (isq) { if (i < n) c.pm[((size_t)(r0 + i) * c.H + h) * CH + j] = acc[r]; }
+      else am[i * LA + j] = be[i] * acc[r];
+    }
+  }
+  // what delta_carry reads besides: queries from the chunk's start, keys to the chunk's end (transposed), the chunk's decay
+  for (int i = tid; i < CH * (DP / 4); i += 512) {
+    const int t = i / (DP / 4), k = i % (DP / 4) * 4;
+    if (t >= n) break;
+    f32x4 q = *(const f32x4*)(qs + t * LK + k);
+    for (int m = 0; m < t / 16; ++m) q *= *(const f32x4*)(tot + m * DP + k);
+    *(f32x4*)(c.qm + ((size_t)(r0 + t) * c.H + h) * DP + k) = q;
+  }
+  float* kt = c.kt + ((size_t)blockIdx.x * c.H + h) * DP * CH;
+  for (int i = tid; i < DP * (CH / 4); i += 512) {
+    const int k = i / (CH / 4), t = i % (CH / 4) * 4;
+    float f = 1.f;
+    for (int m = t / 16 + 1; m < 4; ++m) f *= tot[m * DP + k];
+    *(f32x4*)(kt + (size_t)k * CH + t) = f32x4{kr[t * LK + k], kr[(t + 1) * LK + k], kr[(t + 2) * LK + k], kr[(t + 3) * LK + k]} * f;
+  }
+  if (tid < DP) c.fac[((size_t)blockIdx.x * c.H + h) * DP + tid] = tot[tid] * tot[DP + tid] * tot[2 * DP + tid] * tot[3 * DP + tid];
+  __syncthreads();
+
+  // 5. T = (I + A)^-1, W = T diag(beta) (K with the decay from the chunk's start), U = T diag(beta) V
+  invert_chunk(am, LA, wave, c16, g4);
+  auto t_block = [&](int i, int l) { return *(const f32x4*)(am + (16 * l + c16) * LA + 16 * i + 4 * g4); };
+  for (int ct = wave; ct < NS; ct += 8) {
+    const int col = 16 * ct + c16;
+    f32x4 acc[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    float start = 1.f;
+#pragma unroll
+    for (int l = 0; l < 4; ++l) {
+      f32x4 b;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { const int t = 16 * l + 4 * g4 + j; b[j] = ks[t * LK + col] * gs[t * LK + col] * start * be[t]; }
+      start *= tot[l * DP + col];
+#pragma unroll
+      for (int i = l; i < 4; ++i) acc[i] = mfma_slice(t_block(i, l), b, acc[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * i + 4 * g4 + r;
+        if (t < n) c.wm[((size_t)(r0 + t) * c.H + h) * DP + col] = acc[i][r];
+      }
+  }
+  for (int ct = wave; ct * 16 < e; ct += 8) {
+    const int col = min(16 * ct + c16, e - 1);
+    f32x4 acc[4], b[4];
+#pragma unroll
+    for (int l = 0; l < 4; ++l) {
+      acc[l] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { const int t = 16 * l + 4 * g4 + j; b[l][j] = vb[(size_t)min(t, n - 1) * c.lds + col] * be[t]; }
+    }
+#pragma unroll
+    for (int l = 0; l < 4; ++l)
+#pragma unroll
+      for (int i = l; i < 4; ++i) acc[i] = mfma_slice(t_block(i, l), b[l], acc[i]);
+    if (16 * ct + c16 < e) {                          // (U replaces v: this wave alone reads and writes these columns)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 16 * i + 4 * g4 + r;
+          if (t < n) vb[(size_t)t * c.lds + col] = acc[i][r];
+        }
+    }
+  }
+}
+
 // a barrier for data in LDS alone: loads from memory stay in flight across it
 __device__ __forceinline__ void lds_barrier() {
   asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
@@ -575,7 +849,8 @@ __device__ __forceinline__ V from_base(const float* base, uint32_t at) { return 
 // grid (H, ceil(e / 16), chunk segments) -- the column groups of a head share an XCD where H is a multiple of 8 --, 8 waves on
 // 16 columns of S.  Waves 0..3 carry the state (wave w: tokens 16 w .. of X, NT 16-row tiles of S), waves 4..7 make the
 // outputs (tokens 16 (w - 4) ..); each SIMD has one of either, whose matrix products fill each other's waits.
-template <typename T, int DP>
+// CHAN: queries and keys come with their decays, the state's decay is a number per row of S.
+template <typename T, int DP, bool CHAN>
 __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
   constexpr int NS = DP / 16, NT = (NS + 3) / 4, LS = DP + 4, LX = CH + 4;
   __shared__ __attribute__((aligned(16))) float st[16 * LS];     // S, [column][state row]
@@ -586,8 +861,9 @@ __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
   const int d = c.d, e = c.e, gd = c.G * d, gq = h / (c.H / c.G);
   const int col = blockIdx.y * 16 + c16, colc = min(col, e - 1);
   const float* scan = c.scan + (size_t)r0 * c.lds;
-  const float* fb = c.fac + ((size_t)c.t.cbase[seg] * c.H + h) * DELTA_FAC;
-  const uint32_t lds = c.lds, ldf = c.H * DELTA_FAC, last_chunk = (n - 1) / CH;
+  constexpr int NF = CHAN ? DP : DELTA_FAC;
+  const float* fb = c.fac + ((size_t)c.t.cbase[seg] * c.H + h) * NF;
+  const uint32_t lds = c.lds, ldf = c.H * NF, last_chunk = (n - 1) / CH;
   auto chunk_of = [&](int t0) { return min((uint32_t)t0 / CH, last_chunk); };
   auto row_of = [&](int t0) { return (uint32_t)min(t0 + 16 * wave + c16, n - 1); };   // the token whose row of a left operand this lane feeds
   // right operand i of a step: 16 state rows / tokens of this lane's column
@@ -608,19 +884,24 @@ __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
       }
       if (owner) *(f32x4*)(st + c16 * LS + 16 * (wave * NT + t) + 4 * g4) = s[t];
     }
-    struct Ops { f32x4 w[NS], kk[NT][4], fk; float u[4], last; } A, B;
+    struct Ops { f32x4 w[NS], kk[NT][4], fk, lr[NT]; float u[4], last; } A, B;
     const float* wb = c.wm + ((size_t)r0 * c.H + h) * DP;
     const float* ub = scan + 2 * gd + (size_t)h * e;
-    const float* kb = c.kt + ((size_t)c.t.cbase[seg] * c.G + gq) * DP * CH;
-    const uint32_t ldw = c.H * DP, ldk = c.G * DP * CH;
+    const float* kb = c.kt + ((size_t)c.t.cbase[seg] * (CHAN ? c.H : c.G) + (CHAN ? h : gq)) * DP * CH;
+    const uint32_t ldw = c.H * DP, ldk = (CHAN ? c.H : c.G) * DP * CH;
     auto load_first = [&](Ops& o, int t0) {
       const uint32_t at = row_of(t0) * ldw + 4 * g4, ck = chunk_of(t0) * ldf;
 #pragma unroll
       for (int i = 0; i < NS; ++i) o.w[i] = from_base<f32x4>(wb, at + 16 * i);
 #pragma unroll
       for (int r = 0; r < 4; ++r) o.u[r] = from_base<float>(ub, (uint32_t)min(t0 + 16 * wave + 4 * g4 + r, n - 1) * lds + colc);
-      o.fk = from_base<f32x4>(fb, ck + CH + 16 * wave + 4 * g4);
-      o.last = from_base<float>(fb, ck + 2 * CH);
+      if constexpr (CHAN) {
+#pragma unroll
+        for (int t = 0; t < NT; ++t) o.lr[t] = from_base<f32x4>(fb, ck + min(16 * (wave * NT + t) + 4 * g4, DP - 4));
+      } else {
+        o.fk = from_base<f32x4>(fb, ck + CH + 16 * wave + 4 * g4);
+        o.last = from_base<float>(fb, ck + 2 * CH);
+      }
     };
     auto load_second = [&](Ops& o, int t0) {
       const uint32_t ck = chunk_of(t0) * ldk + 4 * g4;
@@ -640,18 +921,26 @@ __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) { x[0] = mfma4(op.w[i][j], b[i][j], x[0]); x[1] = mfma4(op.w[i + 1][j], b[i + 1][j], x[1]); }
       const bool any = t0 < n;
-      const float last = any ? op.last : 1.f;
       f32x4 xs;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         x[0][r] = op.u[r] - (x[0][r] + x[1][r]);
-        xs[r] = any ? x[0][r] * op.fk[r] : 0.f;       // (tokens beyond the end: their keys are zero)
+        if constexpr (CHAN) xs[r] = any ? x[0][r] : 0.f;
+        else xs[r] = any ? x[0][r] * op.fk[r] : 0.f;  // (tokens beyond the end: their keys are zero)
       }
       *(f32x4*)(xt[0] + c16 * LX + 16 * wave + 4 * g4) = x[0];
       *(f32x4*)(xt[1] + c16 * LX + 16 * wave + 4 * g4) = xs;
-      load_first(op, t0 + 2 * CH);
+      if constexpr (CHAN) {
 #pragma unroll
-      for (int t = 0; t < NT; ++t) s[t] *= last;
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) s[t][r] *= any ? op.lr[t][r] : 1.f;
+      } else {
+        const float last = any ? op.last : 1.f;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) s[t] *= last;
+      }
+      load_first(op, t0 + 2 * CH);
       lds_barrier();                                  // X is complete, everybody has read S
       if (owner) {
         f32x4 xb[4];
@@ -692,14 +981,15 @@ __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
     put_ring<T>(c, h, gq, blockIdx.y, row, off, r0, n);
   } else {
     struct Ops { f32x4 q[NS], p[4], fq; } A, B;
-    const float* qb = scan + gq * d;
+    const float* qb = CHAN ? c.qm + ((size_t)r0 * c.H + h) * DP : scan + gq * d;
+    const uint32_t ldq = CHAN ? c.H * DP : lds;
     const float* pb = c.pm + ((size_t)r0 * c.H + h) * CH;
     const uint32_t ldp = c.H * CH;
     auto load_first = [&](Ops& o, int t0) {
-      const uint32_t at = row_of(t0) * lds;
+      const uint32_t at = row_of(t0) * ldq;
 #pragma unroll
-      for (int i = 0; i < NS; ++i) o.q[i] = from_base<f32x4>(qb, at + min(16 * i + 4 * g4, d - 4));   // (rows of S beyond d are zero)
-      o.fq = from_base<f32x4>(fb, chunk_of(t0) * ldf + 16 * wave + 4 * g4);
+      for (int i = 0; i < NS; ++i) o.q[i] = from_base<f32x4>(qb, at + (CHAN ? 16 * i + 4 * g4 : min(16 * i + 4 * g4, d - 4)));   // (rows of S beyond d are zero)
+      if constexpr (!CHAN) o.fq = from_base<f32x4>(fb, chunk_of(t0) * ldf + 16 * wave + 4 * g4);
     };
     auto load_second = [&](Ops& o, int t0) {
       const uint32_t at = row_of(t0) * ldp + 4 * g4;
@@ -717,7 +1007,8 @@ __global__ __launch_bounds__(512, 2) void delta_carry_kernel(DeltaCall c) {
       for (int i = 0; i < NS; i += 2)
 #pragma unroll
         for (int j = 0; j < 4; ++j) { o[0] = mfma4(op.q[i][j], b[i][j], o[0]); o[1] = mfma4(op.q[i + 1][j], b[i + 1][j], o[1]); }
-      o[0] = (o[0] + o[1]) * op.fq;
+      o[0] += o[1];
+      if constexpr (!CHAN) o[0] *= op.fq;
       load_first(op, t0 + 2 * CH);
       lds_barrier();
       f32x4 xb[4];
@@ -763,7 +1054,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaCall c) {
     for (int k = lane; k < e; k += 64) { const float v = o[h * e + k]; ss += v * v; }
     const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)e + c.eps);
     for (int k = lane; k < e; k += 64)
-      cat[h * e + k] = from_f32<T>(o[h * e + k] * rs * c.head_norm[k] * silu_f(to_f32(pr[c.o_g + h * e + k])));
+      cat[h * e + k] = from_f32<T>(o[h * e + k] * rs * c.head_norm[k] * out_gate<T>(c, r, h * e + k));
   }
   if (c.ff.ff > 0) polynorm_row<T, 256>(c.ff, pr + c.ff.in_off, cat + c.ff.out_off, red);
 }
@@ -774,7 +1065,8 @@ int scanned_at(const DeltaCall& c, hipStream_t st) {
   MI_HIP(hipGetLastError());
   const dim3 grid((c.e + 15) / 16, c.H, c.t.nc), block(256);
   const int dpl = (c.d + 15) / 16;
-#define GO(D) hipLaunchKernelGGL((delta_scan_kernel<T, D>), grid, block, 0, st, c)
+#define GO(D) do { if (c.channel) hipLaunchKernelGGL((delta_scan_kernel<T, D, true>), grid, block, 0, st, c); \
+    else hipLaunchKernelGGL((delta_scan_kernel<T, D, false>), grid, block, 0, st, c); } while (0)
   if (dpl <= 1) GO(1); else if (dpl <= 2) GO(2); else if (dpl <= 4) GO(4); else if (dpl <= 6) GO(6); else if (dpl <= 8) GO(8);
   else if (dpl <= 12) GO(12); else if (dpl <= 16) GO(16); else GO(32);
 #undef GO
@@ -784,18 +1076,27 @@ int scanned_at(const DeltaCall& c, hipStream_t st) {
 
 template <typename T, int DP>
 int chunked_dp(const DeltaCall& c, hipStream_t st) {
-  const int lds = (CH * (DP + 4) + CH * (CH + 4)) * (int)sizeof(float);
-  MI_HIP(hipFuncSetAttribute((const void*)delta_chunk_kernel<T, DP>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-  hipLaunchKernelGGL((delta_chunk_kernel<T, DP>), dim3(c.t.nct, c.H), dim3(256), lds, st, c);
-  MI_HIP(hipGetLastError());
-  hipLaunchKernelGGL((delta_carry_kernel<T, DP>), dim3(c.H, (c.e + 15) / 16, c.t.nc), dim3(512), 0, st, c);
+  const dim3 carry_grid(c.H, (c.e + 15) / 16, c.t.nc);
+  if (c.channel) {
+    const int lds = (4 * CH * (DP + 4) + CH * (CH + 4) + 4 * DP) * (int)sizeof(float);
+    MI_HIP(hipFuncSetAttribute((const void*)delta_chunk_channel_kernel<T, DP>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL((delta_chunk_channel_kernel<T, DP>), dim3(c.t.nct, c.H), dim3(512), lds, st, c);
+    MI_HIP(hipGetLastError());
+    hipLaunchKernelGGL((delta_carry_kernel<T, DP, true>), carry_grid, dim3(512), 0, st, c);
+  } else {
+    const int lds = (CH * (DP + 4) + CH * (CH + 4)) * (int)sizeof(float);
+    MI_HIP(hipFuncSetAttribute((const void*)delta_chunk_kernel<T, DP>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL((delta_chunk_kernel<T, DP>), dim3(c.t.nct, c.H), dim3(256), lds, st, c);
+    MI_HIP(hipGetLastError());
+    hipLaunchKernelGGL((delta_carry_kernel<T, DP, false>), carry_grid, dim3(512), 0, st, c);
+  }
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
 template <typename T>
 int chunked_at(const DeltaCall& c, hipStream_t st) {
-  if (delta_chunk_pad(c.H, c.d, c.e, c.taps) == 0 || c.pm == nullptr || c.lds % 4 != 0 || c.t.nct < 1)
+  if (delta_chunk_pad(c.H, c.d, c.e, c.taps) == 0 || c.pm == nullptr || (c.channel && c.qm == nullptr) || c.lds % 4 != 0 || c.t.nct < 1)
     return fail(MI_ERR_INVALID, "delta: sizes not supported by the chunk kernels");
   const int C = 2 * c.G * c.d + c.H * c.e;
   const dim3 grid((C + 1023) / 1024, c.t.nct, CH / TW);
@@ -815,7 +1116,8 @@ int delta_at(const DeltaCall& c, hipStream_t st) {
   if (c.t.nd > 0) {
     const dim3 grid(c.t.nd, c.H + (c.ff.ff > 0 ? 1 : 0)), block(DNT);
     const int vec = c.e % 4 == 0 ? 4 : 1, slices = DNT / (c.e / vec), per = (c.d + slices - 1) / slices;
-#define GO(V, M) hipLaunchKernelGGL((delta_decode_kernel<T, V, M>), grid, block, 0, st, c)
+#define GO(V, M) do { if (c.channel) hipLaunchKernelGGL((delta_decode_kernel<T, V, M, true>), grid, block, 0, st, c); \
+    else hipLaunchKernelGGL((delta_decode_kernel<T, V, M, false>), grid, block, 0, st, c); } while (0)
     if (vec == 4) { if (per <= 2) GO(4, 2); else if (per <= 8) GO(4, 8); else if (per <= 16) GO(4, 16); else GO(4, 0); }
     else { if (per <= 8) GO(1, 8); else GO(1, 0); }
 #undef GO

@@ -51,7 +51,7 @@ struct PackedLinear {
 };
 
 // A small tensor kept in float32 whatever the model dtype (norm weights, decay parameters, convolution taps)
-struct Vec32 { std::string name; int n = 0; float* p = nullptr; bool seen = false; bool optional = false; };
+struct Vec32 { std::string name; int n = 0; float* p = nullptr; bool seen = false; bool optional = false; float add = 0.f; };   // add: on top of what is stored
 
 // One layer of a layer-list model
 struct ListLayer {
@@ -63,7 +63,10 @@ struct ListLayer {
   Vec32 norm, act;
   // delta rule
   Vec32 conv_q, conv_k, conv_v, A_log, dt_bias, head_norm;
-  int state_index = -1;          // which recurrent-state slot of the cache
+  // low-rank maps: the inner projections (decay | gate) lie side by side in `in`'s output from o_lr, the outer ones are one matrix
+  // over both (block-diagonal); o_a / o_g then count in a row of its output
+  PackedLinear lr;
+  int o_lr = -1;
   // latent attention
   Vec32 c_norm;
   PackedLinear ukv;              // [heads x kdp key rows | heads x vdp value rows] over the latent (padded per head)
@@ -73,25 +76,29 @@ struct ListLayer {
   bool uk_seen = false, uv_seen = false;
   int kdp = 0, vdp = 0, rp = 0;  // padded key / value / latent sizes
   int src = -1;                  // the layer whose latents this layer reads (itself or kv_from)
-  int lat_index = -1;            // which arena of the cache holds the latents (own latents only)
   // per-layer token input
   void* side_gate = nullptr; void* side_proj_t = nullptr; void* side_proj_p = nullptr;   // [dim][width], transposed [dim][width], padded [width][dim]
   bool side_gate_seen = false, side_proj_seen = false;
   Vec32 side_norm;
   // grouped-query attention
-  Vec32 q_norm, k_norm, vmix;
+  Vec32 q_norm, k_norm, vmix, sink;
+  const float2* rot_tab = nullptr;   // owned by the engine (mi_engine::rot_tabs)
   float* slopes = nullptr;       // [heads] distance bias
   bool v_first = false;          // the first layer whose values are mixed: the later ones read its values
   bool gqa_fast = false;         // matrix-core forms
-  // post-norm blocks: norm of the mixer's output (`norm` is in front of the parallel block), of the feed-forward's output
+  // `norm` is in front of a parallel block and of a pre-norm mixer, behind a post-norm one; norm2 the feed-forward's
   Vec32 norm_b, norm2, norm2_b;
-  // mixture of experts
-  PackedLinear gu, dn, sgu, sdn; // all routed experts' gate | up and down matrices, stacked; the shared expert's
+  // hyper-connections of the two sublayers: weights of the streams in what is read, [from][to], of the output in the streams
+  Vec32 hc_in[2], hc_mix[2], hc_out[2];
+  // SwiGLU feed-forward: gate | up and down matrices (gu, dn); mixture of experts: all routed experts' stacked, the shared expert's
+  PackedLinear gu, dn, sgu, sdn;
   int ffp = 0, sffp = 0;         // padded widths
   void* router = nullptr;        // [experts][padded width] row-major
   bool router_seen = false;
-  int arena_k = -1, arena_v = -1;
 };
+
+// One pass through a layer: what it keeps between calls is its own, also where a layer runs more than once
+struct LayerRun { int layer; int lat = -1, k = -1, v = -1, state = -1; };      // arenas of the latents, keys, values; recurrent-state slot
 
 // one slab of the cache of a layer-list model: [place][heads][width] elements per token from element offset `off`
 struct KvArena { size_t off; int heads, width; };
@@ -173,16 +180,23 @@ struct mi_engine {
   // ---- layer-list models (engine_layers.hip)
   bool layered = false;
   std::vector<ListLayer> list;
+  std::vector<LayerRun> runs;    // the layers in the order in which they run
   int n_arena = 0, n_state = 0;
+  struct RotTab { int dims; float base; float2* p; };
+  std::vector<RotTab> rot_tabs;  // one per (rotated coordinates, base)
+  int streams = 1;               // copies of the residual stream
+  void* pair_embed = nullptr; bool pair_embed_seen = false;   // [pair_buckets + 1][width]
+  void* low = nullptr;           // [rows][max N of `lr`]
+  float* dl_q = nullptr; size_t dl_q_cap = 0;                 // channel form: queries with their decays
   PackedLinear list_head;
   Vec32 list_final_norm, list_final_norm_b;
-  float* y32 = nullptr;          // [rows][wp] a sublayer's output in front of its norm
+  float* y32 = nullptr;          // [rows][wp] a sublayer's output in front of its norm / of the residual update
   int n_vfirst = 0;
   void* v_first = nullptr;       // [rows][n_vfirst] values of the first mixing layer
   int32_t* moe_ids = nullptr; float* moe_wts = nullptr;       // [rows][max top]
   void* moe_mid = nullptr; void* moe_out = nullptr;           // [slots][max ff], [slots][wp]
   int32_t* moe_plan = nullptr; int32_t* moe_counts = nullptr;
-  int gqa_chunk = -1;            // chunk of the first grouped-query layer (order of the query tiles), -1: no such layer
+  int gqa_chunk = -1, gqa_window = 0;      // of the first grouped-query layer (order of the query tiles); -1: no such layer
   float* gqa_part = nullptr; size_t gqa_part_cap = 0;         // split-KV partials of the decode attention
   int* gqa_ctr = nullptr; size_t gqa_ctr_cap = 0;             // its arrival tickets (zero between launches)
   void* tok_embed = nullptr; bool tok_embed_seen = false;     // [vocab][width] row-major
@@ -190,7 +204,7 @@ struct mi_engine {
   double* d_freq = nullptr;      // [ceil(width / 2)] angular frequencies of the sinusoidal positions
   int wp = 0;                    // padded width: row stride of the residual stream and of the normed input
   size_t lw_rows = 0;            // workspace rows
-  float* x32 = nullptr;          // [rows][wp] residual stream
+  float* x32 = nullptr;          // [rows][streams][wp] residual stream
   void* hn = nullptr;            // [rows][wp] normed input (model dtype)
   void* proj = nullptr;          // [rows][max N of `in`]
   void* cat = nullptr;           // [rows][max K of `out`]
@@ -247,6 +261,7 @@ struct mi_kv {
   char* state = nullptr;
   size_t list_bytes = 0, state_bytes = 0;
   std::vector<size_t> state_off, ring_off;   // bytes: [row][heads][dim][vdim] float32, [row][taps][channels] model dtype
+  int32_t* d_prev = nullptr;     // [row] last token (inside `state`; a model whose embedding looks at the previous token)
 };
 
 namespace mi {
@@ -262,6 +277,7 @@ struct Prof {
 int copy_in(void* dst, const void* src, size_t bytes, int on_device, hipStream_t st);
 int finalize_linear(mi_engine* e, FusedLinear& f, int K, const std::string& name);
 void free_linear(FusedLinear& f);
+bool ensure_gu8(mi_engine* e, FusedLinear& f, int pair_offset);
 // y = W x for `rows` rows on the kernel family that fits the call; es_in / es_out: element sizes of x and out
 int gemv_rows(mi_engine* e, const FusedLinear& f, GemvCall c, size_t rows, size_t es_in, size_t es_out, const char* prof);
 int kv_ensure_blocks(mi_kv* kv, int row, int tokens);
@@ -273,6 +289,7 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
 int layers_finalize(mi_engine* e);
 void layers_free(mi_engine* e);
 int layers_kv_plan(mi_engine* e, mi_kv* kv);                 // arena layout + recurrent-state buffers of a new cache
+void layers_kv_bind(mi_engine* e, mi_kv* kv);               // pointers into the allocated state
 int layers_ensure_workspace(mi_engine* e, size_t rows);
 // segment i = lens[i] tokens of cache row rows[i]; tokens (the concatenation) already on the device; logits of the token
 // positions out_idx[0..n_out) end up in e->logits [n_out][vocab]

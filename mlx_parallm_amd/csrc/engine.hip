@@ -1223,7 +1223,7 @@ int mi_kv_create(mi_engine* e, int batch, int capacity_tokens, int kv_dtype, mi_
   // zero-filled like the reference's mx.zeros (base.py:71-72,111-112)
   MI_HIP(hipMemsetAsync(kv->k, 0, bytes, e->stream));
   if (kv->v) MI_HIP(hipMemsetAsync(kv->v, 0, bytes, e->stream));
-  if (kv->state) MI_HIP(hipMemsetAsync(kv->state, 0, kv->state_bytes, e->stream));
+  if (kv->state) { MI_HIP(hipMemsetAsync(kv->state, 0, kv->state_bytes, e->stream)); layers_kv_bind(e, kv); }
   MI_HIP(hipMemsetAsync(kv->d_off, 0, batch * sizeof(int32_t), e->stream));
   MI_HIP(hipStreamSynchronize(e->stream));
   kv->h_off.assign(batch, 0);
@@ -1261,7 +1261,7 @@ int mi_kv_create_paged(mi_engine* e, int slots, int block_tokens, int n_blocks, 
   MI_HIP(hipMemsetAsync(kv->counters, 0, nctr * sizeof(int), e->stream));
   MI_HIP(hipMemsetAsync(kv->k, 0, bytes, e->stream));
   if (kv->v) MI_HIP(hipMemsetAsync(kv->v, 0, bytes, e->stream));
-  if (kv->state) MI_HIP(hipMemsetAsync(kv->state, 0, kv->state_bytes, e->stream));
+  if (kv->state) { MI_HIP(hipMemsetAsync(kv->state, 0, kv->state_bytes, e->stream)); layers_kv_bind(e, kv); }
   MI_HIP(hipMemsetAsync(kv->d_off, 0, slots * sizeof(int32_t), e->stream));
   MI_HIP(hipMemsetAsync(kv->d_btab, 0, ntab * sizeof(int32_t), e->stream));
   MI_HIP(hipStreamSynchronize(e->stream));
@@ -1308,6 +1308,7 @@ int mi_kv_prefix_attach(mi_kv* kv, int row, const int32_t* tokens, int n, int* n
     kv->h_off[row] = reused;
     MI_HIP(hipSetDevice(kv->e->device));
     MI_HIP(hipMemsetD32Async((hipDeviceptr_t)(kv->d_off + row), reused, 1, kv->e->stream));
+    if (kv->d_prev != nullptr) MI_HIP(hipMemsetD32Async((hipDeviceptr_t)(kv->d_prev + row), tokens[reused - 1], 1, kv->e->stream));
   }
   *n_reused = reused;
   return MI_OK;

@@ -12,6 +12,14 @@
 //   rows      norm1, residual update, router of the experts (layer_rows.hip; many rows: the router in moe.hip)
 //   experts   gate | up of all routed experts and the shared one in one launch, down in another (moe.hip)
 //   rows      weighted sum over the experts, norm2, residual update
+// pre-norm block, x += m mixer(norm1(x)), x += m ff(norm2(x)), or with several streams (hyper-connections):
+//   in        every projection of the normed input as ONE matrix (q | k | v | ..); the outer maps of a low-rank decay and gate as another
+//   mixer     gqa.hip, delta.hip or latent.hip
+//   out       W_o, float32
+//   rows      update of all streams, the next sublayer's input from them, its norm (layer_rows.hip)
+//   gate_up   gate | up with the activation in the epilogue;  down, float32
+//   rows      as above
+// A layer may run several times in a row; every run has a cache or state of its own (LayerRun).
 // The matrices go through gemv_rows like every other linear of the engine.  A call is a list of segments (tokens of one
 // cache row each), so prefill, decode and mixed steps are the same pass.
 #include <cmath>
@@ -30,10 +38,10 @@ int part(PackedLinear& L, const std::string& name, int row0, int col0, int rows,
   return row0;
 }
 // a part below the ones that are there (rows padded so that every part starts at a multiple of 16)
-int part_below(PackedLinear& L, const std::string& name, int rows) {
+int part_below(PackedLinear& L, const std::string& name, int rows, int pad = 16) {
   const int at = L.N;
   part(L, name, at, 0, rows, -1);
-  L.N += up(rows, 16);
+  L.N += up(rows, pad);
   return at;
 }
 
@@ -101,6 +109,14 @@ int set_vec(mi_engine* e, Vec32& v, const std::string& name, const void* data, c
     hipFree(tmp);
     MI_TRY(rc);
   }
+  if (v.add != 0.f) {
+    std::vector<float> host((size_t)n);
+    MI_HIP(hipMemcpyAsync(host.data(), v.p, (size_t)n * 4, hipMemcpyDeviceToHost, e->stream));
+    MI_HIP(hipStreamSynchronize(e->stream));
+    for (float& x : host) x += v.add;
+    MI_TRY(copy_in(v.p, host.data(), (size_t)n * 4, 0, e->stream));
+    MI_HIP(hipStreamSynchronize(e->stream));
+  }
   v.seen = true;
   return MI_OK;
 }
@@ -123,12 +139,25 @@ int put_placed(mi_engine* e, void*& dst, size_t dst_elems, const void* src, size
 
 void name_vec(Vec32& v, const std::string& name, int n) { v.name = name; v.n = n; }
 
+// the table of cosines and sines of a rotation, one per (coordinates, base)
+int rotation_table(mi_engine* e, int dims, float base, const float2** out) {
+  for (const auto& t : e->rot_tabs) if (t.dims == dims && t.base == base) { *out = t.p; return MI_OK; }
+  float2* p = nullptr;
+  MI_HIP(hipMalloc(&p, (size_t)e->d.max_positions * (dims / 2) * sizeof(float2)));
+  e->rot_tabs.push_back({dims, base, p});
+  MI_TRY(launch_rotation_table(p, e->d.max_positions, dims, (double)base, e->stream));
+  *out = p;
+  return MI_OK;
+}
+
 int init_layers(mi_engine* e, const mi_layer_desc* layers) {
   const mi_model_desc& d = e->d;
   e->layered = true;
   e->wp = up(d.hidden_size, 64);
   e->list.resize(d.num_layers);
-  const bool mfma16 = d.act_dtype != MI_F32, post = d.block_form == MI_BLOCK_POST_NORM;
+  const bool mfma16 = d.act_dtype != MI_F32, post = d.block_form == MI_BLOCK_POST_NORM, pre = d.block_form == MI_BLOCK_PRE_NORM;
+  const bool looped = d.loop_stop > 0;
+  e->streams = std::max(1, d.streams);
   const int n_norm = d.norm_kind == MI_NORM_SCALAR ? 1 : d.hidden_size;
   int first_mix = -1;            // first layer whose values are mixed into the later ones
   for (int i = 0; i < d.num_layers; ++i) {
@@ -138,7 +167,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
     const std::string p = "l" + std::to_string(i) + ".", bad = "layer " + std::to_string(i) + ": ";
     if (m.struct_size != sizeof(mi_layer_desc)) return fail(MI_ERR_INVALID, "mi_layer_desc.struct_size does not match this library");
     if (m.heads < 1 || m.dim < 1 || m.vdim < 1 || m.ff < 0) return fail(MI_ERR_INVALID, bad + "sizes must be positive");
-    if (m.ff > 0 && (m.act != (post ? MI_ACT_SWIGLU : MI_ACT_POLYNORM) || m.ff_kind != (post ? MI_FF_MOE : MI_FF_DENSE)))
+    if (m.ff > 0 && (m.act != (post || pre ? MI_ACT_SWIGLU : MI_ACT_POLYNORM) || m.ff_kind != (post ? MI_FF_MOE : MI_FF_DENSE)))
       return fail(MI_ERR_UNSUPPORTED, bad + "feed-forward kind / activation not supported in this block form");
     l.in.K = e->wp;
     if (m.mixer == MI_MIXER_DELTA) {
@@ -148,17 +177,29 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       const int qk = m.kv_heads * m.dim, vv = m.heads * m.vdim;
       l.o_q = part_below(l.in, p + "mix.q", qk);
       l.o_k = part_below(l.in, p + "mix.k", qk);
+      if (m.out_gate != MI_GATE_SILU && m.out_gate != MI_GATE_SIGMOID) return fail(MI_ERR_UNSUPPORTED, bad + "delta rule: unknown output gate");
+      if (m.decay_rank < 0 || m.gate_rank < 0) return fail(MI_ERR_INVALID, bad + "ranks must not be negative");
       l.o_v = part_below(l.in, p + "mix.v", vv);
-      l.o_g = part_below(l.in, p + "mix.g", vv);
+      if (m.gate_rank == 0) l.o_g = part_below(l.in, p + "mix.g", vv);
       l.o_b = part_below(l.in, p + "mix.b", m.heads);
-      l.o_a = part_below(l.in, p + "mix.a", m.heads);
+      if (m.decay_rank == 0) l.o_a = part_below(l.in, p + "mix.a", m.heads);
+      // inner projections padded to the tile GEMM's step, directly behind each other: the columns of the outer matrix
+      auto low_rank = [&](const char* name, int rank, int rows, int& out_at) {
+        if (rank == 0) return;
+        const int at = part_below(l.in, p + "mix." + name + "1", rank, 64);
+        if (l.o_lr < 0) l.o_lr = at;
+        out_at = part(l.lr, p + "mix." + name + "2", l.lr.N, at - l.o_lr, rows, rank);
+        l.lr.N += up(rows, 16);
+        l.lr.K = at - l.o_lr + up(rank, 64);
+      };
+      low_rank("a", m.decay_rank, m.heads * m.dim, l.o_a);
+      low_rank("g", m.gate_rank, vv, l.o_g);
       name_vec(l.conv_q, p + "mix.q.conv", qk * m.conv);
       name_vec(l.conv_k, p + "mix.k.conv", qk * m.conv);
       name_vec(l.conv_v, p + "mix.v.conv", vv * m.conv);
       name_vec(l.A_log, p + "mix.A_log", m.heads);
-      name_vec(l.dt_bias, p + "mix.dt_bias", m.heads);
+      name_vec(l.dt_bias, p + "mix.dt_bias", m.decay_rank > 0 ? m.heads * m.dim : m.heads);
       name_vec(l.head_norm, p + "mix.norm", m.vdim);
-      l.state_index = e->n_state++;
     } else if (m.mixer == MI_MIXER_LATENT) {
       if (m.kv_rank < 1 || m.kv_rank > 1024) return fail(MI_ERR_UNSUPPORTED, bad + "kv_rank must be in [1, 1024]");
       l.src = i;
@@ -166,6 +207,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
         if (m.kv_from >= i || layers[m.kv_from].mixer != MI_MIXER_LATENT || layers[m.kv_from].kv_from >= 0 ||
             layers[m.kv_from].kv_rank != m.kv_rank)
           return fail(MI_ERR_INVALID, bad + "kv_from must name an earlier latent-attention layer with latents of its own and the same kv_rank");
+        if (looped) return fail(MI_ERR_UNSUPPORTED, bad + "no latents of another layer in a looped stack");
         l.src = m.kv_from;
       }
       l.rp = up(m.kv_rank, 64);
@@ -174,23 +216,29 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       if (m.kv_from < 0) {
         l.o_c = part_below(l.in, p + "mix.dkv", m.kv_rank);
         name_vec(l.c_norm, p + "mix.dkv.norm", m.kv_rank);
-        l.lat_index = e->n_arena++;
       }
       if (mfma16 && m.scale > 0.f && latent_mfma_supported(d.act_dtype, m.dim, m.vdim, l.rp)) {
         l.kdp = latent_pad(m.dim); l.vdp = latent_pad(m.vdim);
         l.ukv.K = l.rp; l.ukv.N = m.heads * (l.kdp + l.vdp);
       }
     } else if (m.mixer == MI_MIXER_GQA) {
-      if (!post) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention is a mixer of post-norm blocks");
+      if (!post && !pre) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention is a mixer of post- and pre-norm blocks");
       if (m.kv_heads < 1 || m.heads % m.kv_heads != 0) return fail(MI_ERR_INVALID, bad + "heads must be a multiple of kv_heads");
       if (!gqa_supported(m.dim, m.vdim)) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention: head sizes not supported");
-      if (m.chunk < 0 || m.softcap < 0.f) return fail(MI_ERR_INVALID, bad + "chunk and softcap must not be negative");
+      if (m.chunk < 0 || m.softcap < 0.f || m.window < 0 || m.keep_first < 0) return fail(MI_ERR_INVALID, bad + "chunk, window, keep_first and softcap must not be negative");
+      if (m.chunk > 0 && m.window > 0) return fail(MI_ERR_UNSUPPORTED, bad + "chunks and a sliding window in one layer");
+      if (m.rot_dims < 0 || m.rot_dims % 2 != 0 || m.rot_dims > m.dim || (m.rot_dims > 0 && !(m.rot_base > 0.f)))
+        return fail(MI_ERR_INVALID, bad + "rot_dims must be even and at most the head size, rot_base positive");
+      if (m.out_gate != MI_GATE_NONE && m.out_gate != MI_GATE_SIGMOID) return fail(MI_ERR_UNSUPPORTED, bad + "grouped-query attention: unknown output gate");
+      if (looped && m.v_mix) return fail(MI_ERR_UNSUPPORTED, bad + "no mixed values in a looped stack");
+      if (m.rot_dims > 0) MI_TRY(rotation_table(e, m.rot_dims, m.rot_base, &l.rot_tab));
       l.kdp = gqa_pad(m.dim); l.vdp = gqa_pad(m.vdim);
       l.gqa_fast = gqa_mfma_supported(d.act_dtype, m.dim, m.vdim);
       l.o_q = part_below(l.in, p + "mix.q", m.heads * m.dim);
       l.o_k = part_below(l.in, p + "mix.k", m.kv_heads * m.dim);
       l.o_v = part_below(l.in, p + "mix.v", m.kv_heads * m.vdim);
-      l.o_g = part_below(l.in, p + "mix.g", m.heads * m.vdim);
+      if (m.out_gate != MI_GATE_NONE) l.o_g = part_below(l.in, p + "mix.g", m.heads * m.vdim);
+      if (m.sink) name_vec(l.sink, p + "mix.sink", m.heads);
       name_vec(l.q_norm, p + "mix.q.norm", m.dim);
       name_vec(l.k_norm, p + "mix.k.norm", m.dim);
       if (m.v_mix) {
@@ -205,9 +253,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       MI_HIP(hipMalloc(&l.slopes, m.heads * sizeof(float)));
       MI_TRY(copy_in(l.slopes, slopes.data(), m.heads * sizeof(float), 0, e->stream));
       MI_HIP(hipStreamSynchronize(e->stream));
-      if (e->gqa_chunk < 0) e->gqa_chunk = m.chunk;
-      l.arena_k = e->n_arena++;
-      l.arena_v = e->n_arena++;
+      if (e->gqa_chunk < 0) { e->gqa_chunk = m.chunk; e->gqa_window = m.window; }
     } else return fail(MI_ERR_UNSUPPORTED, bad + "unknown mixer");
     const int hv = m.heads * m.vdim;
     part(l.out, p + "mix.o", 0, 0, d.hidden_size, hv);
@@ -232,6 +278,13 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
         part(l.sdn, p + "mlp.shared.down", 0, 0, d.hidden_size, m.shared_ff);
         l.sgu.N = 2 * l.sffp; l.sdn.N = e->wp;
       }
+    } else if (m.ff > 0 && pre) {
+      l.ffp = up(m.ff, 64);
+      part(l.gu, p + "mlp.gate", 0, 0, m.ff, d.hidden_size);
+      part(l.gu, p + "mlp.up", l.ffp, 0, m.ff, d.hidden_size);
+      part(l.dn, p + "mlp.down", 0, 0, d.hidden_size, m.ff);
+      l.gu.N = 2 * l.ffp; l.gu.K = e->wp;
+      l.dn.N = e->wp; l.dn.K = l.ffp;
     } else if (m.ff > 0) {
       l.o_up = part_below(l.in, p + "mlp.up", m.ff);
       l.o_ff = l.n_cat;
@@ -242,14 +295,37 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
     for (auto& q : l.in.parts) if (q.cols < 0) q.cols = d.hidden_size;
     l.out.N = e->wp; l.out.K = l.n_cat;
     name_vec(l.norm, p + "norm1", n_norm);
-    if (post && m.ff > 0) name_vec(l.norm2, p + "norm2", n_norm);
+    if ((post || pre) && m.ff > 0) name_vec(l.norm2, p + "norm2", n_norm);
+    l.norm.add = l.norm2.add = d.norm_offset ? 1.f : 0.f;
+    for (int q = 0; q < 2 && d.streams > 0; ++q) {
+      if (q == 1 && m.ff == 0) break;
+      const std::string ph = p + "hc" + std::to_string(q + 1) + ".";
+      name_vec(l.hc_in[q], ph + "in", d.streams);
+      name_vec(l.hc_mix[q], ph + "mix", d.streams * d.streams);
+      name_vec(l.hc_out[q], ph + "out", d.streams);
+    }
     if (d.norm_kind == MI_NORM_LAYER) {
       name_vec(l.norm_b, p + "norm1.b", n_norm);
       if (m.ff > 0) name_vec(l.norm2_b, p + "norm2.b", n_norm);
     }
     if (d.side_dim > 0) name_vec(l.side_norm, p + "side.norm", d.hidden_size);
   }
+  for (int i = 0; i < d.num_layers; ++i) {             // the order of the runs, and what each keeps
+    const int stop = looped ? d.loop_stop : 0;
+    if (looped && i == d.loop_start) {
+      for (int pass = 0; pass < d.loop_times; ++pass)
+        for (int j = d.loop_start; j < stop; ++j) e->runs.push_back(LayerRun{j});
+      i = stop - 1;
+    } else e->runs.push_back(LayerRun{i});
+  }
+  for (LayerRun& r : e->runs) {
+    const mi_layer_desc& m = e->list[r.layer].d;
+    if (m.mixer == MI_MIXER_DELTA) r.state = e->n_state++;
+    else if (m.mixer == MI_MIXER_GQA) { r.k = e->n_arena++; r.v = e->n_arena++; }
+    else if (m.kv_from < 0) r.lat = e->n_arena++;
+  }
   name_vec(e->list_final_norm, "final.norm", n_norm);
+  e->list_final_norm.add = d.norm_offset ? 1.f : 0.f;
   if (d.norm_kind == MI_NORM_LAYER) name_vec(e->list_final_norm_b, "final.norm.b", n_norm);
   e->list_head.K = e->wp; e->list_head.N = d.vocab_size;
   part(e->list_head, "head", 0, 0, d.vocab_size, d.hidden_size);
@@ -267,7 +343,8 @@ template <typename F>
 void each_vec(mi_engine* e, F f) {
   for (auto& l : e->list)
     for (Vec32* v : {&l.norm, &l.act, &l.conv_q, &l.conv_k, &l.conv_v, &l.A_log, &l.dt_bias, &l.head_norm, &l.c_norm, &l.side_norm,
-                     &l.q_norm, &l.k_norm, &l.vmix, &l.norm_b, &l.norm2, &l.norm2_b}) f(*v);
+                     &l.q_norm, &l.k_norm, &l.vmix, &l.norm_b, &l.norm2, &l.norm2_b, &l.sink, &l.hc_in[0], &l.hc_in[1], &l.hc_mix[0], &l.hc_mix[1],
+                     &l.hc_out[0], &l.hc_out[1]}) f(*v);
   f(e->list_final_norm);
   f(e->list_final_norm_b);
 }
@@ -303,13 +380,13 @@ int build_tables(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t* le
   for (int i : chunk) longest = std::max(longest, lens[i]);
   t.qt = longest >= 256 ? 128 : 64;
   if (e->gqa_chunk >= 0) t.qt = 64;              // (gqa.hip has the small tile only)
-  // the tiles with the most keys in front of them first (attention over chunks of positions: within the chunk)
+  // the tiles with the most keys in front of them first (attention over chunks of positions: within the chunk, over a window: within it)
   struct Tile { int keys, seg, q; };
   std::vector<Tile> order;
   for (int i : chunk)
     for (int q = (lens[i] - 1) / t.qt * t.qt; q >= 0; q -= t.qt) {
       const int p0 = kv->h_off[rows[i]] + q, p1 = kv->h_off[rows[i]] + std::min(q + t.qt, lens[i]);
-      order.push_back(Tile{e->gqa_chunk > 0 ? p1 - p0 / e->gqa_chunk * e->gqa_chunk : p1, i, q});
+      order.push_back(Tile{e->gqa_chunk > 0 ? p1 - p0 / e->gqa_chunk * e->gqa_chunk : (e->gqa_window > 0 ? std::min(p1, p1 - p0 + e->gqa_window) : p1), i, q});
     }
   std::stable_sort(order.begin(), order.end(), [](const Tile& a, const Tile& b) { return a.keys > b.keys; });
   for (const Tile& x : order) { tile.push_back(x.seg); tile.push_back(x.q); }
@@ -360,12 +437,15 @@ int latent_nsplit(const mi_kv* kv, const int32_t* rows, const int32_t* lens, int
 int gqa_nsplit(const mi_kv* kv, const ListLayer& l, const int32_t* rows, const int32_t* lens, int n, int nd) {
   int mx = 0;
   for (int i = 0; i < n; ++i)
-    if (lens[i] == 1) { const int pos = kv->h_off[rows[i]]; mx = std::max(mx, l.d.chunk > 0 ? pos % l.d.chunk : pos); }
+    if (lens[i] == 1) {
+      const int pos = kv->h_off[rows[i]];
+      mx = std::max(mx, l.d.chunk > 0 ? pos % l.d.chunk : (l.d.window > 0 ? (int)std::min<int64_t>(pos, (int64_t)l.d.window + l.d.keep_first) : pos));
+    }
   const int ns = std::max(1, 512 / std::max(1, nd * l.d.kv_heads * gqa_head_tiles(l.d.heads, l.d.kv_heads)));
   return std::max(1, std::min({ns, (mx + 255) / 256, 32}));
 }
 
-int run_gqa(mi_engine* e, mi_kv* kv, ListLayer& l, const Tables& tb, const int32_t* rows, const int32_t* lens, int n) {
+int run_gqa(mi_engine* e, mi_kv* kv, ListLayer& l, const LayerRun& run, const Tables& tb, const int32_t* rows, const int32_t* lens, int n) {
   const mi_model_desc& d = e->d;
   const mi_layer_desc& m = l.d;
   hipStream_t st = e->stream;
@@ -380,10 +460,12 @@ int run_gqa(mi_engine* e, mi_kv* kv, ListLayer& l, const Tables& tb, const int32
   c.proj = e->proj; c.ldp = l.in.N; c.o_q = l.o_q; c.o_k = l.o_k; c.o_v = l.o_v; c.o_g = l.o_g;
   c.q_norm = l.q_norm.p; c.k_norm = l.k_norm.p; c.eps = d.rms_norm_eps;
   c.scale = m.scale; c.softcap = m.softcap; c.slopes = l.slopes; c.chunk = m.chunk;
+  c.rot = m.rot_dims; c.rot_tab = l.rot_tab; c.sink = l.sink.p;
+  c.window = m.window; c.keep = m.window > 0 ? m.keep_first : 0;
   if (m.v_mix && l.v_first) c.v_first_out = e->v_first;
   else if (m.v_mix) { c.v_mix = l.vmix.p; c.v_first_in = e->v_first; }
-  c.kcache = (char*)kv->k + kv->arenas[l.arena_k].off * es;
-  c.vcache = (char*)kv->k + kv->arenas[l.arena_v].off * es;
+  c.kcache = (char*)kv->k + kv->arenas[run.k].off * es;
+  c.vcache = (char*)kv->k + kv->arenas[run.v].off * es;
   c.q = e->lq; c.nsplit = 1;
   c.cat = e->cat; c.ldc = l.n_cat; c.act = d.act_dtype;
   c.all_tokens = l.gqa_fast ? 0 : 1;
@@ -478,7 +560,7 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
   bool found = false;
   MI_TRY(try_packed(e->list_head, found));
   for (auto& l : e->list)
-    for (PackedLinear* L : {&l.in, &l.out, &l.gu, &l.dn, &l.sgu, &l.sdn}) MI_TRY(try_packed(*L, found));
+    for (PackedLinear* L : {&l.in, &l.lr, &l.out, &l.gu, &l.dn, &l.sgu, &l.sdn}) MI_TRY(try_packed(*L, found));
   if (found) return MI_OK;
   const int W = d.hidden_size;
   if (name == "embed") {
@@ -486,6 +568,13 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
     MI_TRY(check_matrix(name, shape, ndim, d.vocab_size, W));
     MI_TRY(put_raw(e, e->tok_embed, d.vocab_size, W, W, data, on_device));
     e->tok_embed_seen = true;
+    return MI_OK;
+  }
+  if (name == "bigram" && d.pair_buckets > 0) {
+    MI_TRY(dense());
+    MI_TRY(check_matrix(name, shape, ndim, d.pair_buckets + 1, W));
+    MI_TRY(put_raw(e, e->pair_embed, d.pair_buckets + 1, W, W, data, on_device));
+    e->pair_embed_seen = true;
     return MI_OK;
   }
   if (name == "side.embed" && d.side_dim > 0) {
@@ -559,6 +648,7 @@ int layers_finalize(mi_engine* e) {
   if (!missing.empty()) return fail(MI_ERR_NOTFOUND, missing + ": not set");
   if (!e->tok_embed_seen) return fail(MI_ERR_NOTFOUND, "embed: not set");
   if (d.side_dim > 0 && !e->side_embed_seen) return fail(MI_ERR_NOTFOUND, "side.embed: not set");
+  if (d.pair_buckets > 0 && !e->pair_embed_seen) return fail(MI_ERR_NOTFOUND, "bigram: not set");
   for (int i = 0; i < d.num_layers; ++i) {
     ListLayer& l = e->list[i];
     const std::string p = "l" + std::to_string(i) + ".";
@@ -566,6 +656,12 @@ int layers_finalize(mi_engine* e) {
     if (l.d.mixer == MI_MIXER_LATENT && (!l.uk_seen || !l.uv_seen)) return fail(MI_ERR_NOTFOUND, p + "mix.uk / mix.uv: not set");
     MI_TRY(finalize_packed(e, l.in));
     MI_TRY(finalize_packed(e, l.out));
+    if (l.lr.N > 0) MI_TRY(finalize_packed(e, l.lr));
+    if (l.d.ff_kind == MI_FF_DENSE && l.ffp > 0) {
+      MI_TRY(finalize_packed(e, l.gu));
+      MI_TRY(finalize_packed(e, l.dn));
+      (void)ensure_gu8(e, l.gu.f, l.ffp);
+    }
     if (l.d.mixer == MI_MIXER_LATENT && l.kdp > 0) MI_TRY(finalize_packed(e, l.ukv));
     if (l.d.ff_kind == MI_FF_MOE && l.d.ff > 0) {
       if (!l.router_seen) return fail(MI_ERR_NOTFOUND, p + "mlp.router: not set");
@@ -583,12 +679,13 @@ void layers_free(mi_engine* e) {
   if (!e->layered) return;
   each_vec(e, [](Vec32& v) { hipFree(v.p); v.p = nullptr; });
   for (auto& l : e->list) {
-    for (PackedLinear* L : {&l.in, &l.out, &l.ukv, &l.gu, &l.dn, &l.sgu, &l.sdn}) free_packed(*L);
+    for (PackedLinear* L : {&l.in, &l.lr, &l.out, &l.ukv, &l.gu, &l.dn, &l.sgu, &l.sdn}) free_packed(*L);
     hipFree(l.slopes); hipFree(l.router);
     hipFree(l.uk); hipFree(l.uv); hipFree(l.uk_t); hipFree(l.uv_p); hipFree(l.side_gate); hipFree(l.side_proj_t); hipFree(l.side_proj_p);
   }
   free_packed(e->list_head);
-  for (void* p : {e->tok_embed, e->side_embed, (void*)e->d_freq, (void*)e->x32, e->hn, e->proj, e->cat, (void*)e->scan32, (void*)e->gate32,
+  for (auto& t : e->rot_tabs) hipFree(t.p);
+  for (void* p : {e->tok_embed, e->side_embed, e->pair_embed, e->low, (void*)e->dl_q, (void*)e->d_freq, (void*)e->x32, e->hn, e->proj, e->cat, (void*)e->scan32, (void*)e->gate32,
                   e->lq, (void*)e->lat_part, e->lat_m, e->lat_x, e->lat_kv, (void*)e->dl_w, (void*)e->dl_p, (void*)e->dl_k, (void*)e->dl_f, (void*)e->d_meta, (void*)e->d_gather_list, e->head_x,
                   (void*)e->y32, e->v_first, (void*)e->moe_ids, (void*)e->moe_wts, e->moe_mid, e->moe_out, (void*)e->moe_plan, (void*)e->moe_counts, (void*)e->gqa_part, (void*)e->gqa_ctr}) hipFree(p);
 }
@@ -599,11 +696,12 @@ int layers_kv_plan(mi_engine* e, mi_kv* kv) {
   kv->arenas.clear(); kv->state_off.clear(); kv->ring_off.clear();
   const size_t tokens = kv->paged ? ((size_t)kv->nblocks << kv->bs_shift) : (size_t)kv->B * kv->cap;
   size_t at = 0, sb = 0;
-  for (auto& l : e->list) {
+  for (const LayerRun& r : e->runs) {
+    const ListLayer& l = e->list[r.layer];
     auto arena = [&](int heads, int width) { kv->arenas.push_back(KvArena{at, heads, width}); at += tokens * heads * width; };
-    if (l.lat_index >= 0) arena(1, l.rp);
-    if (l.arena_k >= 0) { arena(l.d.kv_heads, l.kdp); arena(l.d.kv_heads, l.vdp); }
-    if (l.state_index >= 0) {
+    if (r.lat >= 0) arena(1, l.rp);
+    if (r.k >= 0) { arena(l.d.kv_heads, l.kdp); arena(l.d.kv_heads, l.vdp); }
+    if (r.state >= 0) {
       const mi_layer_desc& m = l.d;
       kv->state_off.push_back(sb);
       sb += ((size_t)kv->B * m.heads * m.dim * m.vdim * sizeof(float) + 255) & ~(size_t)255;
@@ -611,22 +709,29 @@ int layers_kv_plan(mi_engine* e, mi_kv* kv) {
       sb += ((size_t)kv->B * m.conv * (2 * m.kv_heads * m.dim + m.heads * m.vdim) * es + 255) & ~(size_t)255;
     }
   }
+  if (e->d.pair_buckets > 0) sb += (size_t)kv->B * sizeof(int32_t);        // (the rows' last tokens stand at the end)
   kv->list_bytes = std::max<size_t>(16, at * es);
   kv->state_bytes = std::max<size_t>(16, sb);
   return MI_OK;
 }
 
+void layers_kv_bind(mi_engine* e, mi_kv* kv) {
+  if (e->d.pair_buckets > 0) kv->d_prev = (int32_t*)(kv->state + kv->state_bytes) - kv->B;
+}
+
 int layers_ensure_workspace(mi_engine* e, size_t rows) {
   if (rows <= e->lw_rows) return MI_OK;
   MI_HIP(hipStreamSynchronize(e->stream));
-  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4, n_pick = 0, n_mid = 0, n_out = 0, n_plan = 0, n_count = 0;
+  size_t n_in = 16, n_cat = 16, n_scan = 4, n_heads = 1, n_lq = 4, n_pick = 0, n_mid = 0, n_out = 0, n_plan = 0, n_count = 0, n_low = 0;
   for (auto& l : e->list) {
     n_in = std::max(n_in, (size_t)l.in.N);
     n_cat = std::max(n_cat, (size_t)l.n_cat);
     if (l.d.mixer == MI_MIXER_DELTA) {
-      n_scan = std::max(n_scan, (size_t)2 * l.d.kv_heads * l.d.dim + (size_t)l.d.heads * l.d.vdim);
+      n_scan = std::max(n_scan, (size_t)2 * l.d.kv_heads * l.d.dim + (size_t)l.d.heads * l.d.vdim + (l.d.decay_rank > 0 ? (size_t)l.d.heads * l.d.dim : 0));
+      n_low = std::max(n_low, (size_t)l.lr.N);
       n_heads = std::max(n_heads, (size_t)l.d.heads);
     } else n_lq = std::max(n_lq, (size_t)l.d.heads * (l.d.mixer == MI_MIXER_GQA ? l.kdp : l.rp));
+    if (l.d.ff_kind == MI_FF_DENSE && l.ffp > 0) n_cat = std::max(n_cat, (size_t)l.ffp);      // (the mixer's output is done with by then)
     if (l.d.ff_kind == MI_FF_MOE && l.d.ff > 0) {
       const size_t slots = (size_t)l.d.top + (l.sffp > 0 ? 1 : 0);
       n_pick = std::max(n_pick, (size_t)l.d.top);
@@ -637,14 +742,14 @@ int layers_ensure_workspace(mi_engine* e, size_t rows) {
       n_count = std::max(n_count, moe_count_ints((int)rows, r));
     }
   }
-  const size_t n_y = e->d.block_form == MI_BLOCK_POST_NORM ? e->wp : 0;
+  const size_t n_y = e->d.block_form == MI_BLOCK_PARALLEL ? 0 : e->wp;
   n_scan = up((int)n_scan, 4);
   e->scan_ld = (int)n_scan; e->gate_ld = (int)(4 * n_heads);
   const size_t es = act_size(e);
   struct B { void** p; size_t n; } bufs[] = {
-      {(void**)&e->x32, rows * e->wp * sizeof(float)}, {&e->hn, rows * e->wp * es}, {&e->proj, rows * n_in * es}, {&e->cat, rows * n_cat * es},
+      {(void**)&e->x32, rows * e->streams * e->wp * sizeof(float)}, {&e->hn, rows * e->wp * es}, {&e->proj, rows * n_in * es}, {&e->cat, rows * n_cat * es},
       {(void**)&e->scan32, rows * n_scan * sizeof(float)}, {(void**)&e->gate32, rows * 4 * n_heads * sizeof(float)},
-      {&e->lq, rows * n_lq * sizeof(float)},
+      {&e->lq, rows * n_lq * sizeof(float)}, {&e->low, rows * n_low * es},
       {(void**)&e->y32, rows * n_y * sizeof(float)}, {&e->v_first, rows * (size_t)e->n_vfirst * es}, {(void**)&e->moe_ids, rows * n_pick * sizeof(int32_t)},
       {(void**)&e->moe_wts, rows * n_pick * sizeof(float)}, {&e->moe_mid, rows * n_mid * es}, {&e->moe_out, rows * n_out * es},
       {(void**)&e->moe_plan, n_plan * sizeof(int32_t)}, {(void**)&e->moe_counts, n_count * sizeof(int32_t)}};
@@ -673,54 +778,78 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
   MI_TRY(build_tables(e, kv, rows, lens, n, tb));
   const SegTables& t = tb.t;
   const int R = t.R;
-  if (e->resid_out != nullptr && (int64_t)R * d.hidden_size * d.num_layers > e->resid_cap)
+  if (e->resid_out != nullptr && (int64_t)R * d.hidden_size * (int64_t)e->runs.size() > e->resid_cap)
     return fail(MI_ERR_INVALID, "residual capture: buffer too small for this pass");
   e->cur_L = t.nd == n ? 1 : 2;
   e->sq_valid = false;
   const int nstride = d.norm_kind == MI_NORM_SCALAR ? 0 : 1;
   const int32_t* tok = e->tok_src ? e->tok_src : e->d_tokens;
-  const bool post = d.block_form == MI_BLOCK_POST_NORM;
-  auto norm_of = [&](int li) {
+  const bool post = d.block_form == MI_BLOCK_POST_NORM, pre = d.block_form == MI_BLOCK_PRE_NORM;
+  const int n_runs = (int)e->runs.size();
+  auto norm_of = [&](int ri) {
     if (post) return RowNormW{nullptr, 0, 0.f};                // (no norm in front of a sublayer)
-    const Vec32& v = li < d.num_layers ? e->list[li].norm : e->list_final_norm;
+    const Vec32& v = ri < n_runs ? e->list[e->runs[ri].layer].norm : e->list_final_norm;
     return RowNormW{v.p, nstride, d.rms_norm_eps};
   };
+  auto in_of = [&](int ri) { return d.streams > 0 && ri < n_runs ? e->list[e->runs[ri].layer].hc_in[0].p : nullptr; };
   { Prof pr(e, "embed");
     EmbedPosCall c{t, tok, e->tok_embed, e->d_freq, d.vocab_size, d.hidden_size, e->wp, norm_of(0), e->x32, e->hn, act};
+    c.scale = d.embed_scale == 0.f ? 1.0f : d.embed_scale;
+    c.pair = PairEmbed{e->pair_embed, d.pair_buckets, d.pair_mul_prev, d.pair_mul_cur, kv->d_prev};
+    c.streams = d.streams; c.in = in_of(0);
     MI_TRY(launch_embed_pos(c, st)); }
-  for (int li = 0; li < d.num_layers; ++li) {
+  // pre-norm blocks: sublayer q of a layer has left y32; `in` and `norm` are the next sublayer's
+  auto stream_norm = [&](const ListLayer& l, int q, const float* in, RowNormW norm, bool last) -> int {
+    StreamNormCall c{R, e->y32, d.streams, l.hc_mix[q].p, l.hc_out[q].p, in, d.residual_mult == 0.f ? 1.0f : d.residual_mult, norm,
+                     d.hidden_size, e->wp, e->x32, e->hn, last && e->resid_out == nullptr ? 0 : 1, act};
+    Prof pr(e, "stream_norm");
+    return launch_stream_norm(c, st);
+  };
+  for (int ri = 0; ri < n_runs; ++ri) {
+    const LayerRun& run = e->runs[ri];
+    const int li = run.layer;
     ListLayer& l = e->list[li];
     const mi_layer_desc& m = l.d;
     GemvCall ci; ci.x = e->hn; ci.ldx = e->wp; ci.act = act; ci.epi = EPI_STORE; ci.out = e->proj; ci.ldo = l.in.N;
     MI_TRY(gemv_rows(e, l.in.f, ci, R, es, es, "gemv_in"));
-    const PolyNormArgs ff{post ? 0 : m.ff, l.o_up, l.o_ff, l.act.p, d.rms_norm_eps};
+    const PolyNormArgs ff{post || pre ? 0 : m.ff, l.o_up, l.o_ff, l.act.p, d.rms_norm_eps};
     if (m.mixer == MI_MIXER_DELTA) {
+      const bool channel = m.decay_rank > 0;
+      if (l.lr.N > 0) {
+        GemvCall cl; cl.x = (const char*)e->proj + (size_t)l.o_lr * es; cl.ldx = l.in.N; cl.act = act; cl.epi = EPI_STORE; cl.out = e->low; cl.ldo = l.lr.N;
+        MI_TRY(gemv_rows(e, l.lr.f, cl, R, es, es, "gemv_low"));
+      }
       DeltaCall c{};
       c.t = t; c.H = m.heads; c.G = m.kv_heads; c.d = m.dim; c.e = m.vdim; c.taps = m.conv;
       c.proj = e->proj; c.ldp = l.in.N;
       c.o_q = l.o_q; c.o_k = l.o_k; c.o_v = l.o_v; c.o_g = l.o_g; c.o_b = l.o_b; c.o_a = l.o_a;
+      c.ap = channel ? e->low : e->proj; c.ldap = channel ? l.lr.N : l.in.N;
+      c.gp = m.gate_rank > 0 ? e->low : e->proj; c.ldgp = m.gate_rank > 0 ? l.lr.N : l.in.N;
+      c.channel = channel; c.gate_act = m.out_gate;
       c.conv_q = l.conv_q.p; c.conv_k = l.conv_k.p; c.conv_v = l.conv_v.p;
       c.A_log = l.A_log.p; c.dt_bias = l.dt_bias.p; c.head_norm = l.head_norm.p;
       c.scale = m.scale; c.unit_eps = m.unit_eps; c.eps = d.rms_norm_eps;
-      c.state = (float*)(kv->state + kv->state_off[l.state_index]);
-      c.ring = kv->state + kv->ring_off[l.state_index];
+      c.state = (float*)(kv->state + kv->state_off[run.state]);
+      c.ring = kv->state + kv->ring_off[run.state];
       c.scan = e->scan32; c.lds = e->scan_ld; c.gate = e->gate32; c.ldg = e->gate_ld;
       c.cat = e->cat; c.ldc = l.n_cat; c.ff = ff; c.act = act;
       const int cp = delta_chunk_pad(m.heads, m.dim, m.vdim, m.conv);
       if (cp > 0 && tb.maxlen >= DELTA_CHUNK_FROM && std::max((size_t)R * e->scan_ld, (size_t)R * m.heads * std::max(cp, DELTA_CHUNK)) < ((size_t)1 << 30)) {
         MI_TRY(grow(e, (void**)&e->dl_w, &e->dl_w_cap, (size_t)R * m.heads * cp * sizeof(float)));
         MI_TRY(grow(e, (void**)&e->dl_p, &e->dl_p_cap, (size_t)R * m.heads * DELTA_CHUNK * sizeof(float)));
-        MI_TRY(grow(e, (void**)&e->dl_k, &e->dl_k_cap, (size_t)t.nct * m.kv_heads * cp * DELTA_CHUNK * sizeof(float)));
-        MI_TRY(grow(e, (void**)&e->dl_f, &e->dl_f_cap, (size_t)t.nct * m.heads * DELTA_FAC * sizeof(float)));
-        c.wm = e->dl_w; c.pm = e->dl_p; c.kt = e->dl_k; c.fac = e->dl_f;
+        MI_TRY(grow(e, (void**)&e->dl_k, &e->dl_k_cap, (size_t)t.nct * (channel ? m.heads : m.kv_heads) * cp * DELTA_CHUNK * sizeof(float)));
+        MI_TRY(grow(e, (void**)&e->dl_f, &e->dl_f_cap, (size_t)t.nct * m.heads * (channel ? cp : DELTA_FAC) * sizeof(float)));
+        if (channel) MI_TRY(grow(e, (void**)&e->dl_q, &e->dl_q_cap, (size_t)R * m.heads * cp * sizeof(float)));
+        c.wm = e->dl_w; c.pm = e->dl_p; c.kt = e->dl_k; c.fac = e->dl_f; c.qm = e->dl_q;
       }
       Prof pr(e, "delta");
       MI_TRY(launch_delta(c, st));
     } else if (m.mixer == MI_MIXER_GQA) {
-      MI_TRY(run_gqa(e, kv, l, tb, rows, lens, n));
+      MI_TRY(run_gqa(e, kv, l, run, tb, rows, lens, n));
     } else {
       LatentCall c{};
-      const int li_src = e->list[l.src].lat_index;
+      int li_src = run.lat;                // (a layer that reads another's latents stands in a stack without loops: run = layer)
+      if (li_src < 0) li_src = e->runs[l.src].lat;
       c.t = t;
       c.s = AttnShape{1, 1, m.heads, 1, l.rp, act, kv->dtype, RND_NONE, kv->cap, nullptr, nullptr, 0, 0};
       kv_shape(kv, c.s);
@@ -734,14 +863,14 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
       MI_TRY(run_latent(e, kv, l, tb, rows, lens, n, c));
     }
     GemvCall co; co.x = e->cat; co.ldx = l.n_cat; co.act = act; co.epi = EPI_RESID; co.out32 = 1; co.resid = e->x32; co.ldo = e->wp;
-    if (post) { co.epi = EPI_STORE; co.resid = nullptr; co.out = e->y32; }
+    if (post || pre) { co.epi = EPI_STORE; co.resid = nullptr; co.out = e->y32; }
     MI_TRY(gemv_rows(e, l.out.f, co, R, es, sizeof(float), "gemv_out"));
     if (post) {
       PostNormCall pn{};
       pn.rows = R; pn.y = e->y32; pn.kind = d.norm_kind; pn.eps = d.rms_norm_eps; pn.norm = PostNormW{l.norm.p, l.norm_b.p, nstride};
       pn.width = d.hidden_size; pn.ld = e->wp; pn.x = e->x32; pn.h = e->hn; pn.act = act;
       const PostNormW last{e->list_final_norm.p, e->list_final_norm_b.p, nstride};
-      const bool end = li + 1 == d.num_layers;
+      const bool end = ri + 1 == n_runs;
       if (m.ff > 0) {
         const MoeCall mc = moe_call(e, l, R);
         const bool fused = route_fused(act, R, m.experts);
@@ -759,12 +888,25 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
       if (end) pn.next = last;
       Prof pr(e, m.ff > 0 ? "post_norm2" : "post_norm");
       MI_TRY(launch_post_norm(pn, st));
+    } else if (pre) {
+      int q = 0;
+      if (m.ff > 0) {
+        MI_TRY(stream_norm(l, 0, l.hc_in[1].p, RowNormW{l.norm2.p, nstride, d.rms_norm_eps}, false));
+        GemvCall cg; cg.x = e->hn; cg.ldx = e->wp; cg.act = act; cg.epi = EPI_SWIGLU; cg.out = e->cat; cg.ldo = l.ffp; cg.pair_offset = l.ffp;
+        MI_TRY(gemv_rows(e, l.gu.f, cg, R, es, es, "gemv_gate_up"));
+        GemvCall cd; cd.x = e->cat; cd.ldx = l.ffp; cd.act = act; cd.epi = EPI_STORE; cd.out32 = 1; cd.out = e->y32; cd.ldo = e->wp;
+        MI_TRY(gemv_rows(e, l.dn.f, cd, R, es, sizeof(float), "gemv_down"));
+        q = 1;
+      }
+      MI_TRY(stream_norm(l, q, in_of(ri + 1), norm_of(ri + 1), ri + 1 == n_runs));
     } else { Prof pr(e, "side");
       SideNormCall c{R, tok, e->side_embed, d.num_layers * d.side_dim, li * d.side_dim, d.vocab_size, l.side_gate, l.side_proj_t, l.side_proj_p,
-                     l.side_norm.p, d.rms_norm_eps, d.side_dim, d.hidden_size, e->wp, norm_of(li + 1), e->x32, e->hn, act};
+                     l.side_norm.p, d.rms_norm_eps, d.side_dim, d.hidden_size, e->wp, norm_of(ri + 1), e->x32, e->hn, act};
       MI_TRY(launch_side_norm(c, st)); }
     if (e->resid_out != nullptr) {
-      MI_HIP(hipMemcpy2DAsync(e->resid_out + (size_t)li * R * d.hidden_size, d.hidden_size * sizeof(float), e->x32, e->wp * sizeof(float),
+      const float* x = e->x32;
+      if (e->streams > 1) { MI_TRY(launch_stream_sum(e->x32, e->streams, R, e->wp, e->y32, st)); x = e->y32; }
+      MI_HIP(hipMemcpy2DAsync(e->resid_out + (size_t)ri * R * d.hidden_size, d.hidden_size * sizeof(float), x, e->wp * sizeof(float),
                               d.hidden_size * sizeof(float), R, hipMemcpyDeviceToHost, st));
       MI_HIP(hipStreamSynchronize(st));
     }
@@ -789,7 +931,7 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
     Prof pr(e, "logit_cap");
     MI_TRY(launch_logit_cap(e->logits, (size_t)n_out * d.vocab_size, d.logit_scale == 0.f ? 1.0f : d.logit_scale, d.logit_softcap, st));
   }
-  MI_TRY(launch_advance_segments(t, kv->d_off, st));
+  MI_TRY(launch_advance_segments(t, kv->d_off, tok, kv->d_prev, st));
   for (int i = 0; i < n; ++i) kv->h_off[rows[i]] += lens[i];
   return MI_OK;
 }
@@ -808,10 +950,17 @@ int mi_engine_create_layers(const mi_model_desc* desc, const mi_layer_desc* laye
   if (d.act_dtype != MI_F32 && d.act_dtype != MI_BF16 && d.act_dtype != MI_F16) return fail(MI_ERR_INVALID, "bad act_dtype");
   if (d.quant_bits != 0) return fail(MI_ERR_UNSUPPORTED, "layer-list models: no quantised weights");
   if (d.position != MI_POS_NONE && d.position != MI_POS_SINUSOIDAL) return fail(MI_ERR_UNSUPPORTED, "unknown position encoding");
-  if (d.block_form != MI_BLOCK_PARALLEL && d.block_form != MI_BLOCK_POST_NORM) return fail(MI_ERR_UNSUPPORTED, "unknown block form");
-  const bool post = d.block_form == MI_BLOCK_POST_NORM;
+  if (d.block_form != MI_BLOCK_PARALLEL && d.block_form != MI_BLOCK_POST_NORM && d.block_form != MI_BLOCK_PRE_NORM)
+    return fail(MI_ERR_UNSUPPORTED, "unknown block form");
+  const bool post = d.block_form == MI_BLOCK_POST_NORM, pre = d.block_form == MI_BLOCK_PRE_NORM;
   if (d.norm_kind != MI_NORM_VECTOR && d.norm_kind != MI_NORM_SCALAR && !(post && d.norm_kind == MI_NORM_LAYER)) return fail(MI_ERR_UNSUPPORTED, "unknown norm");
-  if (post && d.side_dim > 0) return fail(MI_ERR_UNSUPPORTED, "post-norm blocks: no per-layer token input");
+  if ((post || pre) && d.side_dim > 0) return fail(MI_ERR_UNSUPPORTED, "post- and pre-norm blocks: no per-layer token input");
+  if (d.streams < 0 || d.streams > MAX_STREAMS) return fail(MI_ERR_INVALID, "streams must be in [0, 16]");
+  if (d.streams > 0 && !pre) return fail(MI_ERR_UNSUPPORTED, "hyper-connections: pre-norm blocks only");
+  if (d.pair_buckets < 0 || (d.pair_buckets > 0 && (d.pair_mul_prev < 0 || d.pair_mul_prev >= d.pair_buckets || d.pair_mul_cur < 0 || d.pair_mul_cur >= d.pair_buckets)))
+    return fail(MI_ERR_INVALID, "pair embedding: multipliers must be in [0, buckets)");
+  if (d.loop_stop < 0 || (d.loop_stop > 0 && (d.loop_start < 0 || d.loop_start >= d.loop_stop || d.loop_stop > d.num_layers || d.loop_times < 0)))
+    return fail(MI_ERR_INVALID, "loop: not a range of the layers");
   int ndev = 0;
   if (hipGetDeviceCount(&ndev) != hipSuccess || ndev <= 0)
     return fail(MI_ERR_RUNTIME, "no HIP device available (this library has no CPU backend)");

@@ -1,14 +1,15 @@
-// gqa.hip -- grouped-query attention without rotation (layer-list models).  q and k are divided by their root mean square,
-// head h scores  softcap tanh(q.k scale / softcap) - slope_h (i - j)  over the keys j <= i of i's own chunk of positions, the
-// values are mixed with an earlier layer's of the same token before they are cached, and the output is multiplied element by
-// element with sigmoid(gate).
+// gqa.hip -- grouped-query attention (layer-list models).  q and k are divided by their root mean square and their first
+// coordinates rotated by the position, head h scores  softcap tanh(q.k scale / softcap) - slope_h (i - j)  over the keys j <= i of i's
+// own chunk of positions (or of a window behind i and the kept first tokens of the sequence), the denominator of the softmax also
+// contains exp(sink_h), the values are mixed with an earlier layer's of the same token before they are cached, and the output is
+// multiplied element by element with sigmoid(gate).  Each of these is a parameter that can be off.
 //
-//   gqa_pre        norms, value mix and append of every token of the longer segments (generic form: of all tokens)
+//   gqa_pre        norms, rotation, value mix and append of every token of the longer segments (generic form: of all tokens)
 //   gqa_generic    any size and dtype: one workgroup per (token, query head), float32 arithmetic
-//   gqa_decode     16-bit caches, one-token segments: norms, append, split-KV attention, combine and gate in ONE launch; the query
+//   gqa_decode     16-bit caches, one-token segments: norms, rotation, append, split-KV attention, combine and gate in ONE launch; the query
 //                  heads of a group are the columns of the MFMAs and share every key and value that is read
 //   gqa_prefill    16-bit caches, longer segments: flash attention over the paged cache, tiles of 64 or 128 queries of one head
-// Only the key blocks that a tile's chunks reach are walked.
+// Only the key blocks that a tile's chunks or windows reach are walked, and those of the kept tokens.
 #include <algorithm>
 #include <type_traits>
 
@@ -30,7 +31,56 @@ constexpr float LOG2E = 1.4426950408889634f;
 __device__ __forceinline__ size_t cache_at(const AttnShape& s, int row, int head, int key) {
   return s.btab ? kv_elem<true>(s, row, head, key) : kv_elem<false>(s, row, head, key);
 }
-__device__ __forceinline__ int chunk_start(int pos, int chunk) { return chunk > 0 ? pos / chunk * chunk : 0; }
+// the query at `pos` sees the keys [first_seen, pos] and [0, keep)
+__device__ __forceinline__ int first_seen(const GqaCall& c, int pos) {
+  return c.window > 0 ? max(0, pos - c.window + 1) : (c.chunk > 0 ? pos / c.chunk * c.chunk : 0);
+}
+
+// What the rotation of the N coordinates k .. k + N - 1 of a head needs besides themselves: their partners (as projected, and the
+// partners' norm weights), cosine and sine.  Coordinate j < rot / 2 goes with j + rot / 2.
+template <int N>
+struct Rot { float v[N], w[N], c[N], s[N]; };
+template <typename T, int N>
+__device__ __forceinline__ void load_rot(const GqaCall& c, const T* src, const float* w, int k, int pos, Rot<N>& r) {
+  const int half = c.rot >> 1;
+  const float2* tab = c.rot_tab + (size_t)pos * half;
+#pragma unroll
+  for (int i = 0; i < N; ++i) { r.v[i] = 0.f; r.w[i] = 0.f; r.c[i] = 1.f; r.s[i] = 0.f; }
+  if (k >= c.rot) return;
+  typedef T tv __attribute__((ext_vector_type(N)));
+  if (half % N == 0 && k % N == 0) {                 // (the N coordinates lie in one half)
+    const int p = k < half ? k + half : k - half, f = k < half ? k : k - half;
+    const bool aligned = ((uintptr_t)(src + p) & (N * sizeof(T) - 1)) == 0;
+    if (aligned) {
+      const tv x = *(const tv*)(src + p);
+#pragma unroll
+      for (int i = 0; i < N; ++i) r.v[i] = to_f32(x[i]);
+    } else {
+#pragma unroll
+      for (int i = 0; i < N; ++i) r.v[i] = to_f32(src[p + i]);
+    }
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const float2 cs = tab[f + i];
+      r.w[i] = w[p + i]; r.c[i] = cs.x; r.s[i] = k < half ? -cs.y : cs.y;
+    }
+    return;
+  }
+#pragma unroll
+  for (int i = 0; i < N; ++i) {
+    const int j = k + i;
+    if (j >= c.rot) continue;
+    const int p = j < half ? j + half : j - half;
+    const float2 cs = tab[j < half ? j : j - half];
+    r.v[i] = to_f32(src[p]); r.w[i] = w[p]; r.c[i] = cs.x; r.s[i] = j < half ? -cs.y : cs.y;
+  }
+}
+// v: the normed coordinates, rs: the head's reciprocal root mean square
+template <int N>
+__device__ __forceinline__ void rotate(const Rot<N>& r, float rs, float (&v)[N]) {
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = v[i] * r.c[i] + r.v[i] * rs * r.w[i] * r.s[i];
+}
 
 // ---- norms, value mix, append ----------------------------------------------------------------------------------------
 // grid R.  VEC: head sizes are multiples of 8 up to 128, 16 lanes per head; otherwise a wave per head.
@@ -63,6 +113,11 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
         if (k < n) {
 #pragma unroll
           for (int i = 0; i < 8; ++i) v[i] *= rs * w[k + i];
+          if (c.rot > 0) {
+            Rot<8> ro;
+            load_rot<T, 8>(c, src, w, k, at.pos, ro);
+            rotate<8>(ro, rs, v);
+          }
         }
       } else {
         const size_t fo = (size_t)r * c.G * c.vdim + hh * c.vdim + k;
@@ -96,8 +151,16 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
       }
       for (int k = lane; k < np; k += 64) {
         float v = k < n ? to_f32(src[k]) : 0.f;
-        if (kind < 2) { if (k < n) v *= rs * w[k]; }
-        else if (k < n) {
+        if (kind < 2) {
+          if (k < n) v *= rs * w[k];
+          if (k < c.rot) {
+            Rot<1> ro;
+            float one[1] = {v};
+            load_rot<T, 1>(c, src, w, k, at.pos, ro);
+            rotate<1>(ro, rs, one);
+            v = one[0];
+          }
+        } else if (k < n) {
           const size_t fo = (size_t)r * c.G * c.vdim + hh * c.vdim + k;
           if (c.v_first_out != nullptr) ((T*)c.v_first_out)[fo] = from_f32<T>(v);
           if (c.v_mix != nullptr) v = (1.0f - lam) * v + lam * to_f32(((const T*)c.v_first_in)[fo]);
@@ -109,30 +172,31 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
 }
 
 // ---- generic form ----------------------------------------------------------------------------------------------------
-// grid (R, H), 4 waves: wave w takes keys w, w + 4, .. of the token's chunk; NR key / value elements per lane
+// grid (R, H), 4 waves: wave w takes keys w, w + 4, .. of the kept and the other visible ones; NR key / value elements per lane
 template <typename T, int NR>
 __global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
   extern __shared__ float sm[];                      // [4][vdp] sums
   __shared__ float ml[8];
   const int r = blockIdx.x, h = blockIdx.y, g = h / (c.H / c.G), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const TokenAt at = token_at(c.t, r);
-  const int lo = chunk_start(at.pos, c.chunk);
+  const int lo = first_seen(c, at.pos), kept = min(c.keep, lo), n = kept + at.pos - lo + 1;      // visible keys, in order
+  auto key_at = [&](int i) { i = min(i, n - 1); return i < kept ? i : lo + i - kept; };
   const T* qp = (const T*)c.q + ((size_t)r * c.H + h) * c.kdp;
   const float slope = c.slopes[h];
   float q[NR], o[NR], m = -INFINITY, l = 0.f;
 #pragma unroll
   for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; q[i] = k < c.dim ? to_f32(qp[k]) : 0.f; o[i] = 0.f; }
   constexpr int U = NR <= 2 ? 4 : 2;                 // keys in flight
-  for (int key = lo + wave; key <= at.pos; key += 4 * U) {
+  for (int i0 = wave; i0 < n; i0 += 4 * U) {
     float x[U][NR], sc[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const T* p = (const T*)c.kcache + cache_at(c.sk, at.row, g, min(key + 4 * u, at.pos));
+      const T* p = (const T*)c.kcache + cache_at(c.sk, at.row, g, key_at(i0 + 4 * u));
       float a = 0.f;
 #pragma unroll
       for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; if (k < c.dim) a = fmaf(q[i], to_f32(p[k]), a); }
       sc[u] = a;
-      const T* pv = (const T*)c.vcache + cache_at(c.sv, at.row, g, min(key + 4 * u, at.pos));
+      const T* pv = (const T*)c.vcache + cache_at(c.sv, at.row, g, key_at(i0 + 4 * u));
 #pragma unroll
       for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; x[u][i] = k < c.vdim ? to_f32(pv[k]) : 0.f; }
     }
@@ -141,8 +205,8 @@ __global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
     for (int u = 0; u < U; ++u) {
       float s = wave_sum(sc[u]) * c.scale;
       if (c.softcap > 0.f) s = c.softcap * tanhf(s / c.softcap);
-      sc[u] = s - slope * (float)(at.pos - (key + 4 * u));
-      if (key + 4 * u <= at.pos) mx = fmaxf(mx, sc[u]);
+      sc[u] = s - slope * (float)(at.pos - key_at(i0 + 4 * u));
+      if (i0 + 4 * u < n) mx = fmaxf(mx, sc[u]);
     }
     const float corr = expf(m - mx);                 // (the first key of the loop is visible: mx is finite)
     m = mx; l *= corr;
@@ -150,7 +214,7 @@ __global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
     for (int i = 0; i < NR; ++i) o[i] *= corr;
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      const float p = key + 4 * u <= at.pos ? expf(sc[u] - m) : 0.f;
+      const float p = i0 + 4 * u < n ? expf(sc[u] - m) : 0.f;
       l += p;
 #pragma unroll
       for (int i = 0; i < NR; ++i) o[i] = fmaf(p, x[u][i], o[i]);
@@ -160,15 +224,16 @@ __global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
   for (int i = 0; i < NR; ++i) { const int k = lane + 64 * i; if (k < c.vdim) sm[wave * c.vdp + k] = o[i]; }
   if (lane == 0) { ml[wave] = m; ml[4 + wave] = l; }
   __syncthreads();
-  const float mx = fmaxf(fmaxf(ml[0], ml[1]), fmaxf(ml[2], ml[3]));
-  float w[4], lt = 0.f;
+  float mx = fmaxf(fmaxf(ml[0], ml[1]), fmaxf(ml[2], ml[3]));
+  if (c.sink != nullptr) mx = fmaxf(mx, c.sink[h]);
+  float w[4], lt = c.sink != nullptr ? expf(c.sink[h] - mx) : 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) { w[i] = expf(ml[i] - mx); lt += w[i] * ml[4 + i]; }
-  const T* gate = (const T*)c.proj + (size_t)r * c.ldp + c.o_g + h * c.vdim;
+  const T* gate = (const T*)c.proj + (size_t)r * c.ldp + max(c.o_g, 0) + h * c.vdim;
   T* cat = (T*)c.cat + (size_t)r * c.ldc + h * c.vdim;
   for (int k = threadIdx.x; k < c.vdim; k += 256) {
     const float v = (w[0] * sm[k] + w[1] * sm[c.vdp + k] + w[2] * sm[2 * c.vdp + k] + w[3] * sm[3 * c.vdp + k]) / lt;
-    cat[k] = from_f32<T>(v * sigmoid_f(to_f32(gate[k])));
+    cat[k] = from_f32<T>(c.o_g >= 0 ? v * sigmoid_f(to_f32(gate[k])) : v);
   }
 }
 
@@ -265,9 +330,12 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   const int split = blockIdx.x, kh = blockIdx.y / ht_n, ht = blockIdx.y % ht_n, m = blockIdx.z;
   const int seg = c.t.dec[m], row = c.t.row[seg], tok = c.t.tok0[seg], pos = c.t.off[row];
   const int h0 = kh * rep + ht * 16, nh = min(16, rep - ht * 16);
-  const int lo = max(chunk_start(pos, c.chunk), pos - key_reach(c, c.slopes[h0 + nh - 1] * LOG2E));     // cached keys [lo, pos) (the slopes fall)
-  const int blk0 = lo / KB, nblk = pos > lo ? (pos + KB - 1) / KB - blk0 : 0, per = (nblk + c.nsplit - 1) / c.nsplit;
-  const int b0 = blk0 + split * per, b1 = min(b0 + per, blk0 + nblk);
+  const int lo = max(first_seen(c, pos), pos - key_reach(c, c.slopes[h0 + nh - 1] * LOG2E));     // cached keys [lo, pos) (the slopes fall)
+  const int kept = min(c.keep, pos);                                                             // and [0, kept)
+  const int blk0 = lo / KB, nmain = pos > lo ? (pos + KB - 1) / KB - blk0 : 0;
+  const int nkept = nmain > 0 ? min((kept + KB - 1) / KB, blk0) : (kept + KB - 1) / KB, nblk = nkept + nmain;
+  const int per = (nblk + c.nsplit - 1) / c.nsplit, b0 = split * per, b1 = min(b0 + per, nblk);
+  auto block_of = [&](int i) { return i < nkept ? i : blk0 + i - nkept; };
   const T* kc = (const T*)c.kcache;
   const T* vc = (const T*)c.vcache;
   unsigned char* img = smem + wave * IMG;
@@ -295,6 +363,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
     const int hh = tid >> 4, l = tid & 15;
     constexpr int PL = KD / 16;                      // elements per lane: l PL ..
     float vq[PL], wq[PL], vk[PL], wk[PL];
+    Rot<PL> rq, rk;
     const bool key_lanes = own && tid < 16;
     load_upto<T, PL>(pr + c.o_q + (h0 + min(hh, nh - 1)) * c.dim, l * PL, c.dim, vq);
     load_upto<float, PL>(c.q_norm, l * PL, c.dim, wq);
@@ -302,17 +371,24 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
       load_upto<T, PL>(pr + c.o_k + kh * c.dim, l * PL, c.dim, vk);
       load_upto<float, PL>(c.k_norm, l * PL, c.dim, wk);
     }
-    if (b0 + wave < b1) { load_k(b0 + wave); load_v(b0 + wave); }
-    auto head = [&](const float (&v)[PL], const float (&w)[PL], bool there, T* dst) {
-      float ss = 0.f;
+    if (c.rot > 0) {
+      load_rot<T, PL>(c, pr + c.o_q + (h0 + min(hh, nh - 1)) * c.dim, c.q_norm, l * PL, pos, rq);
+      if (key_lanes) load_rot<T, PL>(c, pr + c.o_k + kh * c.dim, c.k_norm, l * PL, pos, rk);
+    }
+    if (b0 + wave < b1) { load_k(block_of(b0 + wave)); load_v(block_of(b0 + wave)); }
+    auto head = [&](const float (&v)[PL], const float (&w)[PL], const Rot<PL>& ro, bool there, T* dst) {
+      float ss = 0.f, x[PL];
 #pragma unroll
       for (int i = 0; i < PL; ++i) ss += v[i] * v[i];
       const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)c.dim + c.eps);
 #pragma unroll
-      for (int i = 0; i < PL; ++i) dst[l * PL + i] = from_f32<T>(there ? v[i] * rs * w[i] : 0.f);
+      for (int i = 0; i < PL; ++i) x[i] = v[i] * rs * w[i];
+      if (c.rot > 0) rotate<PL>(ro, rs, x);
+#pragma unroll
+      for (int i = 0; i < PL; ++i) dst[l * PL + i] = from_f32<T>(there ? x[i] : 0.f);
     };
-    head(vq, wq, hh < nh, qs + hh * LQ);
-    if (key_lanes) head(vk, wk, true, kn);
+    head(vq, wq, rq, hh < nh, qs + hh * LQ);
+    if (key_lanes) head(vk, wk, rk, true, kn);
     if (own && tid >= 64 && tid < 64 + VD) {
       const int k = tid - 64;
       float x = 0.f;
@@ -340,7 +416,8 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   for (int dt = 0; dt < DT; ++dt) acc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int tq4 = c16 >> 2, tp = c16 & 3;
 
-  for (int blk = b0 + wave; blk < b1; blk += 4) {
+  for (int it = b0 + wave; it < b1; it += 4) {
+    const int blk = block_of(it);
     f32x4 sc[2];
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
@@ -353,7 +430,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
       const int piece = i * 64 + lane, key = piece / (VD / 8), dc = piece % (VD / 8);
       *(u32x4*)(img + (size_t)(dc >> 1) * (KB * 32) + key * 32 + (dc & 1) * 16) = vr[i];
     }
-    if (blk + 4 < b1) { load_k(blk + 4); load_v(blk + 4); }
+    if (it + 4 < b1) { load_k(block_of(it + 4)); load_v(block_of(it + 4)); }
     float mx = -INFINITY;
     const float bias0 = fmaf(slope2, (float)(blk * KB + 4 * g4 - pos), ks.c0);
 #pragma unroll
@@ -362,7 +439,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
       for (int r = 0; r < 4; ++r) {
         const int key = blk * KB + 16 * t + 4 * g4 + r;
         const float s = score2<CAP>(ks, sc[t][r], fmaf(slope2, (float)(16 * t + r), bias0));
-        sc[t][r] = key >= lo && key < pos ? s : -INFINITY;
+        sc[t][r] = (key >= lo && key < pos) || key < kept ? s : -INFINITY;
         mx = fmaxf(mx, sc[t][r]);
       }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -421,7 +498,9 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   }
   __syncthreads();
   T* cat = (T*)c.cat + (size_t)tok * c.ldc;
-  const T* gate = pr + c.o_g;
+  const bool gated = c.o_g >= 0;
+  const T* gate = pr + max(c.o_g, 0);
+  auto sink_of = [&](int h, float mn) { return c.sink != nullptr ? __builtin_amdgcn_exp2f(c.sink[h] * LOG2E - mn) : 0.f; };
   float* pp0 = c.partial + (size_t)m * c.H * c.nsplit * (VD + 2);
   for (int idx = tid; idx < nh * VD; idx += 256) {
     const int hh = idx / VD, d = idx % VD;
@@ -437,7 +516,8 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
     }
     const int h = h0 + hh;
     if (c.nsplit == 1) {
-      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(to_f32(gate[h * c.vdim + d])));
+      L += sink_of(h, mn);
+      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(gated ? O / L * gate_f(to_f32(gate[h * c.vdim + d])) : O / L);
     } else {
       float* pp = pp0 + ((size_t)h * c.nsplit + split) * (VD + 2);
       __hip_atomic_store(&pp[2 + d], O, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -462,7 +542,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   for (int idx = tid; idx < nh * VD; idx += 256) {
     const int hh = idx / VD, d = idx % VD, h = h0 + hh;
     const float* pp = pp0 + (size_t)h * c.nsplit * (VD + 2);
-    const float gv = to_f32(gate[h * c.vdim + min(d, c.vdim - 1)]);
+    const float gv = gated ? to_f32(gate[h * c.vdim + min(d, c.vdim - 1)]) : 0.f;
     float mn = -1e30f, L = 0.f, O = 0.f;
     for (int i0 = 0; i0 < c.nsplit; i0 += 8) {       // eight splits' loads in flight, merged in split order
       float mv[8], lv[8], ov[8];
@@ -486,12 +566,13 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
           O = fmaf(ov[j], cw, O);
         }
     }
-    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(O / L * gate_f(gv));
+    L += sink_of(h, mn);
+    if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(gated ? O / L * gate_f(gv) : O / L);
   }
 }
 
 // grid (H, query tiles), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys from the
-// tile's last one downwards, two LDS buffers, the next block's global loads in flight during the current block's MFMAs.
+// tile's last one downwards (then the kept tokens' blocks), two LDS buffers, the next block's global loads in flight during the current block's MFMAs.
 // Downwards because of the distance bias: the running maximum is found in the first block and seldom moves.  It lags: a block's
 // weights are taken relative to the maximum of the blocks before it, and only a score more than 8 (a factor 256) above that makes
 // the wave find the new maximum and rescale -- no cross-lane step in most blocks.
@@ -509,8 +590,10 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
   const int row = c.t.row[seg], len = c.t.len[seg], off = c.t.off[row], tok0 = c.t.tok0[seg];
   const float slope2 = c.slopes[h] * LOG2E;
   const int nk = off + min(t0 + 64 * QG, len);       // keys any query of the tile may see: [first, nk)
-  const int first = max(chunk_start(off + t0, c.chunk), off + t0 - key_reach(c, slope2));
-  const int jlast = (nk - 1) / KB, jfirst = first / KB;
+  const int first = max(first_seen(c, off + t0), off + t0 - key_reach(c, slope2));
+  const int jlast = (nk - 1) / KB, jfirst = first / KB, nmain = jlast - jfirst + 1;
+  const int nkept = min((c.keep + KB - 1) / KB, jfirst), nblk = nmain + nkept;                   // blocks in front of jfirst that hold kept tokens
+  auto block_of = [&](int i) { i = min(i, nblk - 1); return i < nmain ? jlast - i : nblk - 1 - i; };
   const T* kc = (const T*)c.kcache;
   const T* vc = (const T*)c.vcache;
   auto kimg = [&](int b) { return smem + b * KIMG; };
@@ -519,7 +602,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
   // key block j of the cache: element of its first key (PG 0, 1); `page` is looked up one block ahead of its use
   const int32_t* btab = PG ? c.sk.btab + (size_t)row * c.sk.bt_stride : nullptr;
   int page = 0;
-  auto find_page = [&](int j) { if constexpr (PG == 1) page = __builtin_amdgcn_readfirstlane(btab[(max(j, jfirst) * KB) >> c.sk.bs_shift]); };
+  auto find_page = [&](int j) { if constexpr (PG == 1) page = __builtin_amdgcn_readfirstlane(btab[(j * KB) >> c.sk.bs_shift]); };
   auto block_at = [&](const AttnShape& s, int j) -> size_t {
     if constexpr (PG == 0) return (((size_t)row * s.Hkv + kh) * s.cap + (size_t)j * KB) * s.D;
     else return ((((size_t)page * s.Hkv + kh) << s.bs_shift) + (size_t)((j * KB) & ((1 << s.bs_shift) - 1))) * s.D;
@@ -567,13 +650,13 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
   };
   find_page(jlast);
   load_block(jlast);
-  find_page(jlast - 1);
+  find_page(block_of(1));
   u32x4 qf[QG][KK];
-  int tq[QG], lo[QG];                                // this lane's query of group u and the first key of its chunk
+  int tq[QG], lo[QG];                                // this lane's query of group u and the first key of its chunk or window
 #pragma unroll
   for (int u = 0; u < QG; ++u) {
     tq[u] = t0 + (wave * QG + u) * 16 + c16;
-    lo[u] = chunk_start(off + tq[u], c.chunk);
+    lo[u] = first_seen(c, off + tq[u]);
     const T* q = (const T*)c.q + ((size_t)(tok0 + min(tq[u], len - 1)) * c.H + h) * KD;
 #pragma unroll
     for (int kk = 0; kk < KK; ++kk) qf[u][kk] = *(const u32x4*)(q + 32 * kk + 8 * g4);
@@ -596,10 +679,10 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
     for (int dt = 0; dt < DT; ++dt) acc[u][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const int tq4 = c16 >> 2, tp = c16 & 3;
-  for (int j = jlast; j >= jfirst; --j) {
-    const int buf = (jlast - j) & 1;
-    load_block(max(j - 1, jfirst));               // straight-line (in front of the first block: that block again, not stored): a
-    find_page(j - 2);                                    // conditional load would make the compiler wait for all loads at the loop's head
+  for (int it = 0; it < nblk; ++it) {
+    const int j = block_of(it), buf = it & 1;
+    load_block(block_of(it + 1));                 // straight-line (behind the last block: that block again, not stored): a
+    find_page(block_of(it + 2));                         // conditional load would make the compiler wait for all loads at the loop's head
     f32x4 sc[QG][KT];
 #pragma unroll
     for (int t = 0; t < KT; ++t) {
@@ -639,14 +722,14 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) sc[u][t][r] = score2<CAP>(ks, sc[u][t][r], fmaf(slope2, (float)(16 * t + r), bias0 + ks.c0));
       }
-      // a block that reaches past the first query, or in front of the last query's chunk (uniform)
-      if (j * KB + KB - 1 > q0 || (c.chunk > 0 && j * KB < chunk_start(q0 + 15, c.chunk))) {
+      // a block that reaches past the first query, or in front of the last query's chunk or window (uniform)
+      if (j * KB + KB - 1 > q0 || j * KB < first_seen(c, q0 + 15)) {
 #pragma unroll
         for (int t = 0; t < KT; ++t)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int key = j * KB + 16 * t + 4 * g4 + r;
-            sc[u][t][r] = key <= q0 + c16 && key >= lo[u] ? sc[u][t][r] : -INFINITY;
+            sc[u][t][r] = key <= q0 + c16 && (key >= lo[u] || key < c.keep) ? sc[u][t][r] : -INFINITY;
           }
       }
       float mx = -INFINITY;
@@ -698,7 +781,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 #pragma unroll
         for (int u = 0; u < QG; ++u) acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
       }
-    if (j > jfirst) store_block(buf ^ 1);                // the other buffer: nobody reads it during this block
+    if (it + 1 < nblk) store_block(buf ^ 1);             // the other buffer: nobody reads it during this block
     __syncthreads();
   }
   // output: the gates of a query are fetched in one round trip
@@ -707,14 +790,16 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
     float l = l_run[u];
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
+    if (c.sink != nullptr) l += __builtin_amdgcn_exp2f(c.sink[h] * LOG2E - m_run[u]);
     const int tok = tok0 + min(tq[u], len - 1);
     const float inv = 1.0f / l;
-    const T* gate = (const T*)c.proj + (size_t)tok * c.ldp + c.o_g + h * c.vdim;
+    const bool gated = c.o_g >= 0;
+    const T* gate = (const T*)c.proj + (size_t)tok * c.ldp + max(c.o_g, 0) + h * c.vdim;
     T* o = (T*)c.cat + (size_t)tok * c.ldc + h * c.vdim;
     if (c.vdim % 4 == 0) {
       uint2 gt[DT];
 #pragma unroll
-      for (int dt = 0; dt < DT; ++dt) gt[dt] = *(const uint2*)(gate + min(16 * dt + 4 * g4, c.vdim - 4));
+      for (int dt = 0; dt < DT; ++dt) gt[dt] = gated ? *(const uint2*)(gate + min(16 * dt + 4 * g4, c.vdim - 4)) : uint2{0, 0};
       if (tq[u] >= len) continue;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
@@ -722,7 +807,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
         const T* ge = (const T*)&gt[dt];
         T v[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) v[r] = (T)(acc[u][dt][r] * inv * gate_f(to_f32(ge[r])));
+        for (int r = 0; r < 4; ++r) v[r] = (T)(acc[u][dt][r] * inv * (gated ? gate_f(to_f32(ge[r])) : 1.0f));
         if (k < c.vdim) *(uint2*)(o + k) = __builtin_bit_cast(uint2, v);
       }
     } else if (tq[u] < len) {
@@ -731,7 +816,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int k = 16 * dt + 4 * g4 + r;
-          if (k < c.vdim) o[k] = (T)(acc[u][dt][r] * inv * gate_f(to_f32(gate[k])));
+          if (k < c.vdim) o[k] = (T)(acc[u][dt][r] * inv * (gated ? gate_f(to_f32(gate[k])) : 1.0f));
         }
     }
   }
@@ -806,6 +891,8 @@ int fast_at(const GqaCall& c, hipStream_t st) {
 int check_call(const GqaCall& c) {
   if (c.G < 1 || c.H % c.G != 0 || c.sk.D != c.kdp || c.sv.D != c.vdp || c.sk.Hkv != c.G || c.sv.Hkv != c.G || c.kdp < c.dim || c.vdp < c.vdim)
     return fail(MI_ERR_INVALID, "gqa: cache shape does not match the layer");
+  if (c.rot < 0 || c.rot % 2 != 0 || c.rot > c.dim || (c.rot > 0 && c.rot_tab == nullptr)) return fail(MI_ERR_INVALID, "gqa: rotation does not fit the head size");
+  if (c.window < 0 || c.keep < 0 || (c.window > 0 && c.chunk > 0) || (c.window == 0 && c.keep > 0)) return fail(MI_ERR_INVALID, "gqa: bad mask");
   return MI_OK;
 }
 

@@ -26,8 +26,12 @@ struct SegTables {               // device tables of one call (engine_layers.hip
 
 struct RowNormW { const float* w; int stride; float eps; };     // stride 1: a weight per coordinate, 0: one number for all
 
-// x = table[token] (+ sinusoidal position), h = norm(x) (norm.w null: h = x) in the activation dtype; columns [width, ld) are
-// zero (layer_rows.hip)
+// x = scale table[token] (+ sinusoidal position) (+ a row of the table of token pairs), h = norm(x) (norm.w null: h = x) in the
+// activation dtype; columns [width, ld) are zero.  With several streams every one of them is x, and h = norm(sum_s in[s] x).
+// (layer_rows.hip)
+struct PairEmbed { const void* table; int buckets, mul_prev, mul_cur; const int32_t* prev; };   // table [buckets + 1][width] or null; prev
+                                 // [cache rows]: a row's last token before this call.  Row (prev mul_prev + token mul_cur) mod buckets,
+                                 // the last one for the first token of a sequence
 struct EmbedPosCall {
   SegTables t;
   const int32_t* tokens;
@@ -35,8 +39,11 @@ struct EmbedPosCall {
   const double* freq;            // [ceil(width / 2)] or null: no positions
   int vocab, width, ld;
   RowNormW norm;
-  float* x; void* h;
+  float* x; void* h;             // x [R][max(1, streams)][ld]
   int act;
+  float scale;
+  PairEmbed pair;
+  int streams; const float* in;  // streams 0: one plain stream, in is null
 };
 int launch_embed_pos(const EmbedPosCall& c, hipStream_t st);
 
@@ -58,18 +65,43 @@ struct SideNormCall {
 bool side_mfma_supported(int act, int dim, int ld);
 int launch_side_norm(const SideNormCall& c, hipStream_t st);
 
-int launch_advance_segments(const SegTables& t, int32_t* off, hipStream_t st);    // off[row of each segment] += its length
+// off[row of each segment] += its length; prev (or null): the row's last token
+int launch_advance_segments(const SegTables& t, int32_t* off, const int32_t* tokens, int32_t* prev, hipStream_t st);
+
+// Residual update of a pre-norm block and the norm in front of what follows.  One stream (streams 0): x += mult y, h = norm(x).
+// Several: x_t <- sum_s mix[s][t] x_s + mult out[t] y from the old ones, h = norm(sum_s in[s] x_s); in null: h = norm(sum_s x_s).
+struct StreamNormCall {
+  int rows;
+  const float* y;                // [rows][ld] a sublayer's output
+  int streams;
+  const float* mix; const float* out; const float* in;
+  float mult;
+  RowNormW norm;
+  int width, ld;
+  float* x; void* h;             // x [rows][max(1, streams)][ld]
+  int store;                     // 0: the streams are not needed any more
+  int act;
+};
+constexpr int MAX_STREAMS = 16;
+int launch_stream_norm(const StreamNormCall& c, hipStream_t st);
+int launch_stream_sum(const float* x, int streams, int rows, int ld, float* out, hipStream_t st);     // out [rows][ld]
+// tab [positions][dims / 2]: cosine and sine of p base^(-2i / dims) (angles in double precision)
+int launch_rotation_table(float2* tab, int positions, int dims, double base, hipStream_t st);
 
 struct PolyNormArgs { int ff, in_off, out_off; const float* coef; float eps; };     // ff = 0: none
 
-// Gated delta rule (delta.hip).  Channels of the convolutions, their ring and the scan buffer: [q: G d | k: G d | v: H e]
+// Gated delta rule (delta.hip).  Channels of the convolutions, their ring and the scan buffer: [q: G d | k: G d | v: H e], in the scan
+// buffer of a rule with a decay per channel also [decays: H d]
 struct DeltaCall {
   SegTables t;
   int H, G, d, e, taps;
   const void* proj; int ldp;     // [R][ldp] outputs of the fused input projection
-  int o_q, o_k, o_v, o_g, o_b, o_a;
+  int o_q, o_k, o_v, o_b;
+  const void* ap; int ldap, o_a; // [R][ldap] what the decays are made of: one per value head, or (channel) one per value head and key channel
+  const void* gp; int ldgp, o_g; // [R][ldgp] output gates, [H e]
+  int channel, gate_act;         // gate_act: MI_GATE_SILU or MI_GATE_SIGMOID
   const float* conv_q; const float* conv_k; const float* conv_v;    // [channels][taps]
-  const float* A_log; const float* dt_bias; const float* head_norm;
+  const float* A_log; const float* dt_bias; const float* head_norm;       // dt_bias [H] or (channel) [H d]
   float scale, unit_eps, eps;
   float* state;                  // [cache row][H][d][e]
   void* ring;                    // [cache row][taps][channels]: the inputs of position p at slot p mod taps
@@ -77,6 +109,8 @@ struct DeltaCall {
   float* gate; int ldg;          // [R][ldg] four numbers per value head: decay, step size, k . q (token by token)
   float* wm; float* pm;          // chunked form: [R][H][padded d], [R][H][DELTA_CHUNK]; null: token by token
   float* kt; float* fac;         // [chunks][G][padded d][DELTA_CHUNK] unit keys transposed, [chunks][H][DELTA_FAC]
+  float* qm;                     // channel: [R][H][padded d] unit queries with their decay from the chunk's start; then kt is [chunks][H]..
+                                 // (keys with their decay to the chunk's end) and fac [chunks][H][padded d] (the whole chunk's decay)
   void* cat; int ldc;            // [R][ldc] mixer output from column 0
   PolyNormArgs ff;
   int act;
@@ -114,20 +148,24 @@ int launch_latent_gather(const LatentCall& c, void* dst, hipStream_t st);   // c
 int launch_latent_prefill(const LatentCall& c, hipStream_t st);        // segments of two tokens and more
 constexpr int LATENT_GT = 64;    // keys per gather tile
 
-// Grouped-query attention without rotation (gqa.hip): q and k divided by their root mean square, scores
-//   softcap tanh(q.k scale / softcap) - slope_h (i - j),  j <= i in i's own chunk of positions,
-// values mixed with an earlier layer's of the same token, the output times sigmoid(gate) element by element.
+// Grouped-query attention (gqa.hip): q and k divided by their root mean square and rotated, scores
+//   softcap tanh(q.k scale / softcap) - slope_h (i - j),  j <= i in i's own chunk of positions, or in i's window, or kept,
+// exp(sink_h) in the denominator, values mixed with an earlier layer's of the same token, the output times sigmoid(gate) element by
+// element.  Every mechanism can be off.
 // K and V arenas of the layer: [place][G][..][kdp] / [vdp] as AttnShape sk / sv address them.
 struct GqaCall {
   SegTables t;
   AttnShape sk, sv;              // cache addressing of the keys (D = kdp) and of the values (D = vdp)
   int H, G, dim, vdim, kdp, vdp;
   const void* proj; int ldp;     // [R][ldp] outputs of the fused input projection
-  int o_q, o_k, o_v, o_g;
+  int o_q, o_k, o_v, o_g;        // o_g < 0: no gate
   const float* q_norm; const float* k_norm; float eps;
+  int rot; const float2* rot_tab;          // rotated coordinates (0: none), [position][rot / 2] cosine and sine
   float scale, softcap;          // softcap 0: none
   const float* slopes;           // [H]
+  const float* sink;             // [H], or null
   int chunk;                     // 0: causal only
+  int window, keep;              // window 0: no window (keep is 0 then, and chunk is 0 where window is not)
   const float* v_mix;            // weight of v_first, or null
   const void* v_first_in;        // [R][G vdim] values of the first mixing layer (v_mix non-null)
   void* v_first_out;             // this layer IS the first mixing layer: its values go here; or null

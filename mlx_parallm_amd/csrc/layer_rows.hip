@@ -1,7 +1,8 @@
 // layer_rows.hip -- row-wise steps of layer-list models: embedding + positions + first norm, per-layer token input + the norm
-// in front of the next layer.  The residual stream is float32; the normed rows that feed the matrix products are in the
-// activation dtype.
+// in front of the next layer, residual update of post- and pre-norm blocks (the latter with several streams).  The residual stream
+// is float32; the normed rows that feed the matrix products are in the activation dtype.
 #include <algorithm>
+#include <cmath>
 #include <type_traits>
 
 #include "layer_rows.h"
@@ -15,17 +16,32 @@ using namespace rows;
 template <typename T, int NT>
 __global__ __launch_bounds__(NT) void embed_pos_kernel(EmbedPosCall c) {
   __shared__ float red[NT / 64];
-  const int r = blockIdx.x;
+  const int r = blockIdx.x, streams = max(c.streams, 1);
   const int tok = min(max(c.tokens[r], 0), c.vocab - 1);
-  const int pos = token_at(c.t, r).pos;
+  const TokenAt at = token_at(c.t, r);
+  const int pos = at.pos;
   const T* src = (const T*)c.table + (size_t)tok * c.width;
-  float* x = c.x + (size_t)r * c.ld;
+  const T* pair = nullptr;
+  if (c.pair.table != nullptr) {
+    int row = c.pair.buckets;
+    if (pos > 0) {
+      const int before = min(max(at.t > 0 ? c.tokens[r - 1] : c.pair.prev[at.row], 0), c.vocab - 1);
+      row = (int)(((uint64_t)before * (uint64_t)c.pair.mul_prev + (uint64_t)tok * (uint64_t)c.pair.mul_cur) % (uint64_t)c.pair.buckets);
+    }
+    pair = (const T*)c.pair.table + (size_t)row * c.width;
+  }
+  float fin = (float)streams;                        // what is read of the streams is fin x
+  if (c.in != nullptr) {
+    fin = 0.f;
+    for (int s = 0; s < streams; ++s) fin += c.in[s];
+  }
+  float* x = c.x + (size_t)r * streams * c.ld;
   float ss[1] = {0.f};
   for (int k = 2 * threadIdx.x; k < c.ld; k += 2 * NT) {        // (ld is even)
     float2 v = {0.f, 0.f};
     if (k < c.width) {
-      v.x = to_f32(src[k]);
-      if (k + 1 < c.width) v.y = to_f32(src[k + 1]);
+      v.x = to_f32(src[k]) * c.scale;
+      if (k + 1 < c.width) v.y = to_f32(src[k + 1]) * c.scale;
       if (c.freq != nullptr) {
         // the angle is reduced in double precision, the functions taken in single
         const double a = (double)pos * c.freq[k >> 1];
@@ -33,9 +49,13 @@ __global__ __launch_bounds__(NT) void embed_pos_kernel(EmbedPosCall c) {
         v.x += sinf(f);
         if (k + 1 < c.width) v.y += cosf(f);
       }
+      if (pair != nullptr) {
+        v.x += to_f32(pair[k]);
+        if (k + 1 < c.width) v.y += to_f32(pair[k + 1]);
+      }
       ss[0] += v.x * v.x + v.y * v.y;
     }
-    *(float2*)(x + k) = v;
+    for (int s = 0; s < streams; ++s) *(float2*)(x + (size_t)s * c.ld + k) = v;
   }
   T* h = (T*)c.h + (size_t)r * c.ld;
   if (c.norm.w == nullptr) {
@@ -45,7 +65,7 @@ __global__ __launch_bounds__(NT) void embed_pos_kernel(EmbedPosCall c) {
     return;
   }
   block_sum<NT, 1>(ss, red);
-  const float rs = 1.0f / sqrtf(ss[0] / (float)c.width + c.norm.eps);
+  const float rs = fin / sqrtf(ss[0] * fin * fin / (float)c.width + c.norm.eps);
   for (int k = 2 * threadIdx.x; k < c.ld; k += 2 * NT)          // (each thread reads what it wrote)
 #pragma unroll
     for (int j = k; j < k + 2; ++j)
@@ -529,9 +549,103 @@ __global__ __launch_bounds__(256) void logit_cap_kernel(float* z, size_t n, floa
   }
 }
 
-__global__ void advance_segments_kernel(SegTables t, int32_t* off) {
+__global__ void advance_segments_kernel(SegTables t, int32_t* off, const int32_t* tokens, int32_t* prev) {
   const int i = blockIdx.x * 256 + threadIdx.x;
-  if (i < t.n) off[t.row[i]] += t.len[i];            // (distinct rows)
+  if (i >= t.n) return;
+  off[t.row[i]] += t.len[i];                         // (distinct rows)
+  if (prev != nullptr) prev[t.row[i]] = tokens[t.tok0[i] + t.len[i] - 1];
+}
+
+// one workgroup per row; NT threads x 4 NQ columns.  S: number of streams, 0: c.streams of them (at most MAX_STREAMS)
+template <typename T, int NT, int NQ, int S>
+__global__ __launch_bounds__(NT) void stream_norm_kernel(StreamNormCall c) {
+  constexpr int MS = S > 0 ? S : MAX_STREAMS;
+  __shared__ float red[NT / 64];
+  const int r = blockIdx.x, tid = threadIdx.x, n4 = c.ld / 4, ns = S > 0 ? S : c.streams;
+  float* xg = c.x + (size_t)r * ns * c.ld;
+  f32x4 u[NQ];
+  float ss[1] = {0.f};
+#pragma unroll
+  for (int q = 0; q < NQ; ++q) {
+    const int i = q * NT + tid;
+    u[q] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (i >= n4) continue;
+    f32x4 x[MS];
+#pragma unroll
+    for (int s = 0; s < MS; ++s) if (s < ns) x[s] = ((const f32x4*)(xg + (size_t)s * c.ld))[i];
+    const f32x4 y = ((const f32x4*)(c.y + (size_t)r * c.ld))[i] * c.mult;
+#pragma unroll
+    for (int t = 0; t < MS; ++t) {
+      if (t >= ns) continue;
+      f32x4 v;
+      if (c.mix != nullptr) {
+        v = y * c.out[t];
+#pragma unroll
+        for (int s = 0; s < MS; ++s) if (s < ns) v += x[s] * c.mix[s * ns + t];
+      } else v = x[t] + y;
+      if (c.store) ((f32x4*)(xg + (size_t)t * c.ld))[i] = v;
+      u[q] += c.in != nullptr ? v * c.in[t] : v;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) if (4 * i + j < c.width) ss[0] += u[q][j] * u[q][j];
+  }
+  block_sum<NT, 1>(ss, red);
+  const float rs = 1.0f / sqrtf(ss[0] / (float)c.width + c.norm.eps);
+  T* h = (T*)c.h + (size_t)r * c.ld;
+#pragma unroll
+  for (int q = 0; q < NQ; ++q) {
+    const int i = q * NT + tid;
+    if (i >= n4) continue;
+    T o[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) { const int k = 4 * i + j; o[j] = from_f32<T>(k < c.width ? u[q][j] * rs * c.norm.w[k * c.norm.stride] : 0.f); }
+    if constexpr (sizeof(T) == 2) *(uint2*)(h + 4 * i) = __builtin_bit_cast(uint2, o);
+    else *(f32x4*)(h + 4 * i) = __builtin_bit_cast(f32x4, o);
+  }
+}
+
+template <typename T, int S>
+int stream_norm_s(const StreamNormCall& c, hipStream_t st) {
+#define SN(NT, NQ) do { hipLaunchKernelGGL((stream_norm_kernel<T, NT, NQ, S>), dim3(c.rows), dim3(NT), 0, st, c); MI_HIP(hipGetLastError()); return MI_OK; } while (0)
+  if (c.rows < 256) {                                  // few rows: more threads for each
+    if (c.ld <= 1024) SN(256, 1);
+    if (c.ld <= 4096) SN(1024, 1);
+    if (c.ld <= 8192) SN(1024, 2);
+    if (c.ld <= 16384) SN(1024, 4);
+  }
+  if (c.ld <= 1024) SN(256, 1);
+  if (c.ld <= 2048) SN(256, 2);
+  if (c.ld <= 4096) SN(512, 2);
+  if (c.ld <= 8192) SN(1024, 2);
+  if (c.ld <= 16384) SN(1024, 4);
+#undef SN
+  return fail(MI_ERR_UNSUPPORTED, "stream_norm: rows of more than 16384 columns");
+}
+template <typename T>
+int stream_norm_at(const StreamNormCall& c, hipStream_t st) {
+  switch (c.streams) {
+    case 0: case 1: return stream_norm_s<T, 1>(c, st);
+    case 2: return stream_norm_s<T, 2>(c, st);
+    case 3: return stream_norm_s<T, 3>(c, st);
+    case 4: return stream_norm_s<T, 4>(c, st);
+    default: return stream_norm_s<T, 0>(c, st);
+  }
+}
+
+__global__ __launch_bounds__(256) void stream_sum_kernel(const float* x, int streams, int rows, int ld, float* out) {
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < (size_t)rows * ld; i += (size_t)gridDim.x * 256) {
+    const size_t r = i / ld, k = i % ld;
+    float v = 0.f;
+    for (int s = 0; s < streams; ++s) v += x[(r * streams + s) * ld + k];
+    out[i] = v;
+  }
+}
+
+__global__ __launch_bounds__(256) void rotation_table_kernel(float2* tab, int positions, int half, double step) {
+  for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < (size_t)positions * half; i += (size_t)gridDim.x * 256) {
+    const double a = (double)(i / half) * pow(2.0, step * (double)(i % half));
+    tab[i] = float2{(float)cos(a), (float)sin(a)};
+  }
 }
 
 template <typename E>
@@ -589,8 +703,34 @@ int launch_logit_cap(float* logits, size_t n, float scale, float softcap, hipStr
   return MI_OK;
 }
 
-int launch_advance_segments(const SegTables& t, int32_t* off, hipStream_t st) {
-  hipLaunchKernelGGL(advance_segments_kernel, dim3((t.n + 255) / 256), dim3(256), 0, st, t, off);
+int launch_advance_segments(const SegTables& t, int32_t* off, const int32_t* tokens, int32_t* prev, hipStream_t st) {
+  hipLaunchKernelGGL(advance_segments_kernel, dim3((t.n + 255) / 256), dim3(256), 0, st, t, off, tokens, prev);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_stream_norm(const StreamNormCall& c, hipStream_t st) {
+  if (c.ld % 8 != 0 || c.streams < 0 || c.streams > MAX_STREAMS || c.norm.w == nullptr || (c.mix == nullptr) != (c.out == nullptr) ||
+      (c.streams > 1 && c.mix == nullptr))
+    return fail(MI_ERR_INVALID, "stream_norm: bad call");
+  switch (c.act) {
+    case MI_F32: return stream_norm_at<float>(c, st);
+    case MI_BF16: return stream_norm_at<bf16>(c, st);
+    case MI_F16: return stream_norm_at<f16>(c, st);
+  }
+  return fail(MI_ERR_INVALID, "stream_norm: bad dtype");
+}
+
+int launch_stream_sum(const float* x, int streams, int rows, int ld, float* out, hipStream_t st) {
+  hipLaunchKernelGGL(stream_sum_kernel, dim3((unsigned)std::min<size_t>(((size_t)rows * ld + 255) / 256, 4096)), dim3(256), 0, st, x, streams, rows, ld, out);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_rotation_table(float2* tab, int positions, int dims, double base, hipStream_t st) {
+  const size_t n = (size_t)positions * (dims / 2);
+  hipLaunchKernelGGL(rotation_table_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 8192)), dim3(256), 0, st, tab, positions, dims / 2,
+                     -2.0 / dims * std::log2(base));
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -15,7 +15,7 @@ import numpy as np
 
 from . import _lib as L
 
-LAYER_LIST_MODELS = ("runevik", "dolurax")     # described layer by layer (models/<name>.py: layer_list)
+LAYER_LIST_MODELS = ("runevik", "dolurax", "temetar")     # described layer by layer (models/<name>.py: layer_list)
 _DT_NAMES = {"float32": L.MI_F32, "bfloat16": L.MI_BF16, "float16": L.MI_F16}
 
 
@@ -295,8 +295,16 @@ class Engine:
                 if x.mixer == L.MI_MIXER_LATENT:
                     return (x.kv_rank + 63) // 64 * 64 if x.kv_from < 0 else 0
                 return x.kv_heads * (head(x.dim) + head(x.vdim)) if x.mixer == L.MI_MIXER_GQA else 0
-            return max(1, sum(map(elements, self.layer_descs)) * block_tokens * esz)
+            return max(1, sum(elements(self.layer_descs[i]) for i in self.layer_runs()) * block_tokens * esz)
         return 2 * d.num_layers * d.num_kv_heads * block_tokens * d.head_dim * esz
+
+    def layer_runs(self) -> list:
+        """Layer-list models: the layers in the order in which they run (a looped layer once per pass; each run has a cache or
+        state of its own)."""
+        d, n = self.desc, len(self.layer_descs)
+        if d.loop_stop <= 0:
+            return list(range(n))
+        return list(range(d.loop_start)) + list(range(d.loop_start, d.loop_stop)) * d.loop_times + list(range(d.loop_stop, n))
 
     # -- loading
     def set_tensor(self, name: str, tensor) -> None:
@@ -449,9 +457,9 @@ class Engine:
         return out
 
     def capture_residual(self, tokens: int) -> np.ndarray:
-        """Layer-list models: the array (layers, tokens, width) that the next passes of ``tokens`` tokens fill with the
-        residual stream after every layer; ``capture_residual(0)`` switches off."""
-        self._resid = np.zeros((self.desc.num_layers, tokens, self.desc.hidden_size), np.float32) if tokens else None
+        """Layer-list models: the array (layer runs, tokens, width) that the next passes of ``tokens`` tokens fill with
+        the residual stream after every layer (the sum of the streams, if there are several); ``capture_residual(0)`` switches off."""
+        self._resid = np.zeros((len(self.layer_runs()), tokens, self.desc.hidden_size), np.float32) if tokens else None
         ptr = self._resid.ctypes.data_as(C.POINTER(C.c_float)) if tokens else None
         L.check(L.lib().mi_debug_residual(self._h, ptr, self._resid.size if tokens else 0))
         return self._resid

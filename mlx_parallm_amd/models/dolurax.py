@@ -53,7 +53,7 @@ def layer_list(config: dict):
         m, mlp = layer["mixer"], layer.get("mlp")
         d = dict(mixer=L.MI_MIXER_GQA, heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
                  kv_from=-1, scale=float(m["scale"]), softcap=float(m.get("softcap") or 0.0), slope_exp=SLOPE_EXP,
-                 chunk=int((m.get("mask") or {}).get("size") or 0), v_mix=int(bool(m.get("v_mix"))), act=L.MI_ACT_SWIGLU)
+                 chunk=int((m.get("mask") or {}).get("size") or 0), v_mix=int(bool(m.get("v_mix"))), out_gate=L.MI_GATE_SIGMOID, act=L.MI_ACT_SWIGLU)
         if mlp:
             r = mlp["router"]
             g = r.get("groups") or {"count": 1, "keep": 1}

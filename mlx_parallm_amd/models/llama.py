@@ -65,6 +65,11 @@ class Model:
 
     _ARCH = "llama"
 
+    @classmethod
+    def complete_config(cls, config: dict, shapes: Dict[str, Tuple[int, ...]]) -> dict:
+        """The configuration with what only the tensors' shapes tell (nothing, for most designs)."""
+        return config
+
     def __init__(self, args: ModelArgs, *, config: Optional[dict] = None, device: int = 0,
                  dtype: str = "bfloat16", max_positions: Optional[int] = None):
         from ..engine import Engine

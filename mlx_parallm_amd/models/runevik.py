@@ -56,7 +56,7 @@ def layer_list(config: dict):
                  ff=int(mlp["ff"]) if mlp else 0, act=L.MI_ACT_POLYNORM)
         if layer["type"] == "delta":
             d.update(mixer=L.MI_MIXER_DELTA, kv_heads=int(m["kv_heads"]), conv=int(m["conv"]), scale=float(m["dim"]) ** -0.5,
-                     unit_eps=UNIT_EPS)
+                     unit_eps=UNIT_EPS, out_gate=L.MI_GATE_SILU)
         else:
             d.update(mixer=L.MI_MIXER_LATENT, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]))
             if m.get("kv_from") is not None:

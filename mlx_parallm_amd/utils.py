@@ -425,6 +425,7 @@ def load_model(model_path: Path, lazy: bool = False, model_config: dict = {}, *,
         weights = replicate_checkpoint(weights if reader else None, src=weights_from_rank, device=dev,
                                        stats=replicate_stats)
     model_class, model_args_class = _get_classes(config=config)
+    config = model_class.complete_config(config, {k: tuple(v.shape) for k, v in weights.items()})
     model_args = model_args_class.from_dict(config)
     stored = _checkpoint_dtype(weights)
     if dtype is not None and dtype != stored:
