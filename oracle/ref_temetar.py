@@ -213,14 +213,14 @@ def random_model(cfg: dict, seed: int = 0, decay_rank: int = 5, gate_rank: int =
         p, m, mlp = f"l{i}.", layer["mixer"], layer.get("mlp")
         for sub in (1, 2) if mlp else (1,):
             w[p + f"norm{sub}"] = bf(0.2 * rng.standard_normal(W))
-            w[p + f"hc{sub}.in"] = bf((1.0 + 0.5 * rng.standard_normal(S)) / S)
-            w[p + f"hc{sub}.out"] = bf(1.0 + 0.5 * rng.standard_normal(S))
-            w[p + f"hc{sub}.mix"] = bf(0.8 * np.eye(S) + 0.25 * rng.standard_normal((S, S)) / np.sqrt(S))
+            w[p + f"hc{sub}.in"] = bf((1.0 + 0.3 * rng.standard_normal(S)) / S)
+            w[p + f"hc{sub}.out"] = bf(0.6 + 0.3 * rng.standard_normal(S))
+            w[p + f"hc{sub}.mix"] = bf(0.9 * np.eye(S) + 0.1 * rng.standard_normal((S, S)))
         if layer["type"] == "channel_delta":
             H, d, qk, vv = m["heads"], m["dim"], m["kv_heads"] * m["dim"], m["heads"] * m["vdim"]
             for t, c in (("q", qk), ("k", qk), ("v", vv)):
                 lin(p + "mix." + t, c, W)
-                w[p + f"mix.{t}.conv"] = bf(rng.standard_normal((c, m["conv"])) / np.sqrt(m["conv"]))
+                w[p + f"mix.{t}.conv"] = bf(rng.standard_normal((c, m["conv"])) * 0.7 / np.sqrt(m["conv"]) + 0.7 * (np.arange(m["conv"]) == m["conv"] - 1))
             lin(p + "mix.b", H, W)
             w[p + "mix.A_log"] = bf(np.log(rng.uniform(0.05, 1.5, H)))
             w[p + "mix.dt_bias"] = bf(rng.uniform(-4.0, 0.5, H * d))
@@ -233,8 +233,8 @@ def random_model(cfg: dict, seed: int = 0, decay_rank: int = 5, gate_rank: int =
         else:
             for t, c in (("q", m["heads"] * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])):
                 lin(p + "mix." + t, c, W)
-            w[p + "mix.q.norm"] = bf(1.5 * (1.0 + 0.2 * rng.standard_normal(m["dim"])))
-            w[p + "mix.k.norm"] = bf(1.5 * (1.0 + 0.2 * rng.standard_normal(m["dim"])))
+            w[p + "mix.q.norm"] = bf(1.0 + 0.2 * rng.standard_normal(m["dim"]))
+            w[p + "mix.k.norm"] = bf(1.0 + 0.2 * rng.standard_normal(m["dim"]))
             w[p + "mix.sink"] = bf(1.0 + rng.standard_normal(m["heads"]))
             lin(p + "mix.o", W, m["heads"] * m["vdim"])
         if mlp:

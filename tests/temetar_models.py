@@ -27,7 +27,7 @@ CONFIGS = {
     "odd": config(100, 333, [attn(6, 2, 20, 36, 37, 3, 12, ff=72), delta(6, 3, 20, 24, 3), attn(5, 5, 24, 12, 64, 0, 10),
                              delta(5, 5, 18, 9, 2, 50), attn(3, 1, 33, 30, 25, 7, 22, ff=130)], 3, (1, 4, 2), (61, 1000, 77), 2.5, 0.6, 3e-6),
     # head sizes of the matrix-core kernels, two head tiles, more key channels than a chunk has tokens
-    "wide": config(256, 512, [attn(34, 2, 128, 64, 96, 4, 64, 0.09, 320), delta(4, 2, 128, 64, 4, 192), attn(8, 4, 64, 128, 130, 1, 32, 0.125),
+    "wide": config(256, 512, [attn(34, 2, 128, 64, 90, 5, 64, 0.09, 320), delta(4, 2, 128, 64, 4, 192), attn(8, 4, 64, 128, 130, 1, 32, 0.125),
                               delta(3, 3, 64, 128, 5), attn(4, 1, 32, 128, 70, 65, 8, 0.2, 64)], 4, (0, 2, 3)),
     # everything is one
     "ones": config(64, 96, [attn(1, 1, 2, 1, 1, 1, 2, 1.0, 1), delta(1, 1, 1, 1, 1, 1), attn(1, 1, 2, 1, 1, 0, 2, 1.0), attn(2, 1, 2, 1, 3, 1, 2, 1.0)],
