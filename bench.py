@@ -301,7 +301,7 @@ def parse_args(argv=None):
                          "96, the row limit of its weight-streaming kernel)")
     ap.add_argument("--no-other-configs", action="store_true",
                     help="N = 1, default workload only: skip the short legs of BASELINE configs 3 / 4 / 5 (`other_configs` of the line)")
-    ap.add_argument("--design", default=None, choices=["runevik", "dolurax"],
+    ap.add_argument("--design", default=None, choices=["runevik", "dolurax", "temetar"],
                     help="instead of the headline workload: prefill and decode of this layer-list design beside a llama stack of "
                          "equal size (random weights), one JSON line with every leg and its kernel times")
     ap.add_argument("--design-sizes", default="1024x8,2048x8,4096x4", help="--design: comma-separated WIDTHxLAYERS")
@@ -449,6 +449,16 @@ def design_configs(design, width, layers):
         run = {"model_type": "dolurax", "architecture": "Dolurax", "width": width, "vocab": vocab, "norm": {"eps": 1e-5},
                "layers": [{"type": "attention", "mixer": mixer, "mlp": mlp}] * layers, "logit_scale": 0.25, "logit_softcap": 30.0}
         return run, llama_like(width, layers, heads, vocab)
+    if design == "temetar":
+        att = {"type": "attention", "mlp": {"ff": 3 * width, "kind": "dense"},
+               "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "mask": {"size": 1024, "keep_first": 8},
+                         "rot": {"base": 10000.0, "dims": 64}, "scale": 128 ** -0.5}}
+        rec = {"type": "channel_delta", "mlp": {"ff": 5 * width // 2, "kind": "dense"},
+               "mixer": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": 128, "gate_rank": 128}}
+        run = {"model_type": "temetar", "architecture": "Temetar", "width": width, "vocab": vocab, "layers": [att, rec] * (layers // 2),
+               "norm": {"eps": 1e-5}, "streams": 4, "residual_mult": 1.0, "loop": None,
+               "embedding": {"scale": 1.0, "bigram": {"buckets": 8191, "mul_prev": 127, "mul_cur": 31}}}
+        return run, llama_like(width, layers, heads, vocab)
     one = []
     for i in range(layers):
         if i % 4 == 3:
@@ -488,6 +498,44 @@ def dolurax_specs(cfg):
             yield p + f"mlp.{e}.down", (W, ff)
     yield "final.norm", (W,)
     yield "final.norm.b", (W,)
+    yield "head", (V, W)
+
+
+def temetar_specs(cfg):
+    W, V, S = cfg["width"], cfg["vocab"], cfg["streams"]
+    yield "embed", (V, W)
+    yield "bigram", (cfg["embedding"]["bigram"]["buckets"] + 1, W)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]["ff"]
+        vv = m["heads"] * m["vdim"]
+        for q in (1, 2):
+            yield p + f"norm{q}", (W,)
+            yield p + f"hc{q}.in", (S,)
+            yield p + f"hc{q}.out", (S,)
+            yield p + f"hc{q}.mix", (S, S)
+        if layer["type"] == "channel_delta":
+            qk = m["kv_heads"] * m["dim"]
+            for t, n in (("q", qk), ("k", qk), ("v", vv)):
+                yield p + "mix." + t, (n, W)
+                yield p + f"mix.{t}.conv", (n, m["conv"])
+            yield p + "mix.b", (m["heads"], W)
+            yield p + "mix.A_log", (m["heads"],)
+            yield p + "mix.dt_bias", (m["heads"] * m["dim"],)
+            yield p + "mix.norm", (m["vdim"],)
+            for t, rank, n in (("a", m["decay_rank"], m["heads"] * m["dim"]), ("g", m["gate_rank"], vv)):
+                yield p + f"mix.{t}1", (rank, W)
+                yield p + f"mix.{t}2", (n, rank)
+        else:
+            for t, n in (("q", m["heads"] * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])):
+                yield p + "mix." + t, (n, W)
+            yield p + "mix.q.norm", (m["dim"],)
+            yield p + "mix.k.norm", (m["dim"],)
+            yield p + "mix.sink", (m["heads"],)
+        yield p + "mix.o", (W, vv)
+        yield p + "mlp.gate", (ff, W)
+        yield p + "mlp.up", (ff, W)
+        yield p + "mlp.down", (W, ff)
+    yield "final.norm", (W,)
     yield "head", (V, W)
 
 
@@ -540,12 +588,15 @@ def design_engine(cfg, seed, max_positions):
         params = sum(int(__import__("math").prod(sh)) for _n, sh, _k in tensor_specs(cfg))
         return eng, params
     gen = torch.Generator(device="cuda")
-    for i, (name, shape) in enumerate({"runevik": runevik_specs, "dolurax": dolurax_specs}[cfg["model_type"]](cfg)):
+    for i, (name, shape) in enumerate({"runevik": runevik_specs, "dolurax": dolurax_specs, "temetar": temetar_specs}[cfg["model_type"]](cfg)):
         gen.manual_seed(seed * 1000003 + i)
         if len(shape) == 2:
             t = torch.randn(shape, generator=gen, device="cuda") * (0.02 if "conv" not in name else 0.5)
         else:
-            t = torch.full(shape, 0.5 if name.endswith(("act", "vmix")) else (0.0 if name.endswith(".b") and "norm" in name else 1.0), device="cuda")
+            zero = name.endswith(".b") and "norm" in name or cfg["model_type"] == "temetar" and name.endswith(("norm1", "norm2", "final.norm"))
+            t = torch.full(shape, 0.5 if name.endswith(("act", "vmix")) else (0.0 if zero else 1.0), device="cuda")
+        if ".hc" in name:            # every stream is read and written alike and kept
+            t = {"in": torch.full(shape, 1.0 / shape[0]), "out": torch.ones(shape), "mix": torch.eye(shape[0])}[name.rsplit(".", 1)[1]]
         eng.set_tensor(name, t.to(torch.bfloat16))
         params += t.numel()
     torch.cuda.synchronize()
@@ -563,6 +614,7 @@ def design_leg(args):
     legs = []
     fams = {"runevik": ["gemv_in", "gemv_out", "delta", "latent_pre", "latent_decode", "latent_gather", "latent_kv", "latent_prefill", "side", "embed", "gemv_head", "sample"],
             "dolurax": ["gemv_in", "gqa_pre", "gqa_decode", "gqa_prefill", "gemv_out", "post_norm", "moe_route", "moe_plan", "moe_up", "moe_down", "post_norm2", "embed", "gemv_head", "logit_cap", "sample"],
+            "temetar": ["gemv_in", "gemv_low", "delta", "gqa_pre", "gqa_decode", "gqa_prefill", "gemv_out", "stream_norm", "gemv_gate_up", "gemv_down", "embed", "gemv_head", "sample"],
             "llama": ["gemv_qkv", "attn", "gemv_o", "gemv_gate_up", "gemv_down", "rope_append", "embed", "gemv_head", "sample"]}
     for width, layers in [tuple(map(int, x.split("x"))) for x in args.design_sizes.split(",")]:
         for name, cfg in zip((args.design, "llama"), design_configs(args.design, width, layers)):
