@@ -67,6 +67,36 @@ __device__ __forceinline__ float out_gate(const DeltaCall& c, int r, int i) {
   return c.gate_act == MI_GATE_SIGMOID ? sigmoid_f(z) : silu_f(z);
 }
 
+// The outer low-rank maps of one token and value head by a workgroup of NT threads: decays[d] and gates[e] from the inner
+// projections in the token's row `pr`.  P neighbouring threads share an output.
+template <typename T, int NT>
+__device__ __forceinline__ void low_rank_rows(const DeltaCall& c, const T* pr, int h, float* decays, float* gates) {
+  const int tid = threadIdx.x, n = c.d + c.e;
+  int P = 1;
+  while (P < 8 && 2 * P * n <= NT) P *= 2;
+  for (int o0 = 0; o0 < n; o0 += NT / P) {
+    const int o = o0 + tid / P, p = tid % P;
+    const bool isa = o < c.d, on = o < n;
+    const T* w = isa ? (const T*)c.low_a + (size_t)(h * c.d + o) * c.ld_a : (const T*)c.low_g + (size_t)(h * c.e + min(o, n - 1) - c.d) * c.ld_gt;
+    const T* x = pr + (isa ? c.in_a : c.in_g);
+    const int len = isa ? c.ld_a : c.ld_gt;
+    float s = 0.f;
+#pragma unroll 8
+    for (int k = 8 * p; k < len; k += 8 * P) {
+      float a[8], b[8];
+      load8f<T>(w + k, a);
+      load8f<T>(x + k, b);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) s = fmaf(a[i], b[i], s);
+    }
+    for (int m = 1; m < P; m *= 2) s += __shfl_xor(s, m, 64);
+    if (on && p == 0) {
+      if (isa) decays[o] = decay_of(c, h, h * c.d + o, s);
+      else gates[o - c.d] = c.gate_act == MI_GATE_SIGMOID ? sigmoid_f(s) : silu_f(s);
+    }
+  }
+}
+
 template <int VEC> struct Vec;
 template <> struct Vec<1> { float v[1]; };
 template <> struct alignas(16) Vec<4> { float v[4]; };
@@ -78,7 +108,7 @@ template <typename T, int VEC, int MAXR, bool CHAN>
 __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
   __shared__ float red[DNT / 64 * 3];
   __shared__ Vec<VEC> part[2][DNT];
-  __shared__ float ks[512], qs[512], gs[CHAN ? 512 : 1];
+  __shared__ float ks[512], qs[512], gs[CHAN ? 512 : 1], og[CHAN ? DNT * VEC : 1];
   __shared__ float vs[DNT * VEC];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int seg = c.t.dec[blockIdx.x], r = c.t.tok0[seg], row = c.t.row[seg], pos = c.t.off[row];
@@ -121,7 +151,11 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
   }
   const T* ar = (const T*)c.ap + (size_t)r * c.ldap + c.o_a;
   if constexpr (CHAN) {
-    for (int i = tid; i < d; i += DNT) gs[i] = decay_of(c, h, h * d + i, to_f32(ar[h * d + i]));
+    if (c.low_a != nullptr) low_rank_rows<T, DNT>(c, pr, h, gs, og);
+    else {
+      for (int i = tid; i < d; i += DNT) gs[i] = decay_of(c, h, h * d + i, to_f32(ar[h * d + i]));
+      for (int i = tid; i < e; i += DNT) og[i] = out_gate<T>(c, r, h * e + i);
+    }
   }
   __syncthreads();
   float n3[3] = {0.f, 0.f, 0.f};
@@ -206,7 +240,9 @@ __global__ __launch_bounds__(DNT) void delta_decode_kernel(DeltaCall c) {
 #pragma unroll
     for (int j = 0; j < VEC; ++j) {
       const int k = col * VEC + j;
-      cat[h * e + k] = from_f32<T>(o.v[j] * rs * c.head_norm[k] * out_gate<T>(c, r, h * e + k));
+      float gate;
+      if constexpr (CHAN) gate = og[k]; else gate = out_gate<T>(c, r, h * e + k);
+      cat[h * e + k] = from_f32<T>(o.v[j] * rs * c.head_norm[k] * gate);
     }
   }
   (void)lane; (void)wave;
@@ -591,18 +627,20 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_kernel(DeltaCall c) {
   }
 }
 
-// ---- a decay per channel: grid (chunks, H), 8 waves ----------------------------------------------------------------------
+// ---- a decay per channel: grid (chunks, H), NW waves ---------------------------------------------------------------------
 // T = (I + A)^-1 in place of A by the first four waves (all waves of the workgroup call this): block (i, j) of T ends up at block (j, i)
 __device__ __forceinline__ void invert_chunk(float* am, int LA, int wave, int c16, int g4) {
   f32x4 tb[4];
   const int o = 16 * wave;
   if (wave < 4) {
-    float tc[16];
+    float tc[16], ac[16];                             // column c16 of the diagonal block, of T's and of A's
+#pragma unroll
+    for (int i = 0; i < 16; ++i) ac[i] = -am[(o + i) * LA + o + c16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float v = i == c16 ? 1.f : 0.f;
 #pragma unroll
-      for (int l = 0; l < i; ++l) v = fmaf(-am[(o + i) * LA + o + l], tc[l], v);
+      for (int l = 0; l < i; ++l) v = fmaf(lane_value(ac[i], l), tc[l], v);
       tc[i] = v;
     }
     f32x4 t;
@@ -634,16 +672,44 @@ __device__ __forceinline__ void invert_chunk(float* am, int LA, int wave, int c1
   __syncthreads();
 }
 
-template <typename T, int DP>
-__global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c) {
-  constexpr int LK = DP + 4, LA = CH + 4, NS = DP / 16;
+// sums over the four lane groups of v[0 .. 15]: lane (c16, g4) gets those of v[4 g4 .. 4 g4 + 3].  A swap of lane halves brings both
+// addends of two values' sums into place.
+__device__ __forceinline__ f32x4 group_sums(const float (&v)[16]) {
+  auto bits = [](float x) { return __builtin_bit_cast(uint32_t, x); };
+  auto sum = [](uint32_t x, uint32_t y) { return __builtin_bit_cast(float, x) + __builtin_bit_cast(float, y); };
+  // (a bit cast straight from an element of the returned vector would take the first one)
+  float h[8];                                         // lanes below 32: v[r], the others: v[8 + r]
+#pragma unroll
+  for (int r = 0; r < 8; ++r) {
+    const auto x = __builtin_amdgcn_permlane32_swap(bits(v[r]), bits(v[8 + r]), false, false);
+    h[r] = sum(x[0], x[1]);
+  }
+  f32x4 o;                                            // odd groups take the upper half of the eight
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const auto x = __builtin_amdgcn_permlane16_swap(bits(h[r]), bits(h[4 + r]), false, false);
+    o[r] = sum(x[0], x[1]);
+  }
+  return o;
+}
+
+// exp(-ea softplus(z)) on the hardware's exponential and logarithm: what counts is the absolute error of the exponent
+__device__ __forceinline__ float decay_fast(float ea, float z) {
+  constexpr float LOG2E = 1.4426950408889634f;
+  const float sp2 = fmaxf(z, 0.f) * LOG2E + __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(z) * LOG2E));
+  return __builtin_amdgcn_exp2f(-ea * sp2);
+}
+
+template <typename T, int DP, int NW>
+__global__ __launch_bounds__(64 * NW) void delta_chunk_channel_kernel(DeltaCall c) {
+  constexpr int NT = 64 * NW, LK = DP + 4, LA = CH + 4, NS = DP / 16, NB = NW / 4;      // NB: waves per diagonal block
   extern __shared__ __attribute__((aligned(16))) float csm[];
-  float* ks = csm;                                    // [CH][LK] unit keys
+  float* ks = csm;                                    // [CH][LK] unit keys; from step 3 on times the decay from their block's start
   float* qs = ks + CH * LK;                           // unit queries; from step 3 on times the decay from their block's start
-  float* gs = qs + CH * LK;                           // decays of the tokens; from step 3 on the decay from the block's start to the token
-  float* kr = gs + CH * LK;                           // step 2: partial sums; from step 3 on the keys times the decay to their block's end
-  float* am = kr + CH * LK;                           // [CH][LA] as in delta_chunk_kernel
+  float* gs = qs + CH * LK;                           // decays of the tokens; from step 3 on the unit keys times the decay to their block's end
+  float* am = gs + CH * LK;                           // [CH][LA] as in delta_chunk_kernel
   float* tot = am + CH * LA;                          // [4][DP] a block's whole decay
+  float* part = tot + 4 * DP;                         // [NB - 1][4][2][256] partial sums of the diagonal blocks
   __shared__ float be[CH];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
   const int h = blockIdx.y, seg = c.t.ctile[2 * blockIdx.x], t0 = c.t.ctile[2 * blockIdx.x + 1];
@@ -653,15 +719,23 @@ __global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c
   const float* kb = qb + gd;
   float* vb = c.scan + (size_t)r0 * c.lds + 2 * gd + (size_t)h * e;
 
-  // 1. unit keys and queries (eight threads per token), decays; tokens beyond the end: zero vectors, decay one
+  // 1. unit keys and queries (PT threads per token), decays; tokens beyond the end: zero vectors, decay one
   {
-    const int t = tid >> 3, p = tid & 7;
-    constexpr int NV = (DP + 31) / 32;
+    constexpr int PT = NT / CH, NV = (DP + 4 * PT - 1) / (4 * PT), NG = (CH * DP / 4 + NT - 1) / NT;
+    const T* ar = (const T*)c.ap + (size_t)r0 * c.ldap + c.o_a + h * d;
+    float4 av[NG], bv[NG];
+#pragma unroll
+    for (int i = 0; i < NG; ++i) {                    // (four channels of a token; d is a multiple of four)
+      const int x = min(i * NT + tid, CH * DP / 4 - 1), tt = min(x / (DP / 4), n - 1), ch = min(x % (DP / 4) * 4, d - 4);
+      av[i] = load4f<T>(ar + (size_t)tt * c.ldap + ch);
+      bv[i] = *(const float4*)(c.dt_bias + h * d + ch);
+    }
+    const int t = tid / PT, p = tid % PT;
     float sk = 0.f, sq = 0.f;
     f32x4 kv[NV], qv[NV];
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      const int k = 32 * i + 4 * p;
+      const int k = 4 * (PT * i + p);
       kv[i] = qv[i] = f32x4{0.f, 0.f, 0.f, 0.f};
       if (t < n && k < d) {
         kv[i] = *(const f32x4*)(kb + (size_t)t * c.lds + k);
@@ -671,95 +745,100 @@ __global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c
       }
     }
 #pragma unroll
-    for (int s = 1; s < 8; s *= 2) { sk += __shfl_xor(sk, s, 64); sq += __shfl_xor(sq, s, 64); }
+    for (int s = 1; s < PT; s *= 2) { sk += __shfl_xor(sk, s, 64); sq += __shfl_xor(sq, s, 64); }
     const float ik = 1.0f / sqrtf(sk + c.unit_eps), iq = c.scale / sqrtf(sq + c.unit_eps);
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
-      *(f32x4*)(ks + t * LK + 32 * i + 4 * p) = kv[i] * ik;
-      *(f32x4*)(qs + t * LK + 32 * i + 4 * p) = qv[i] * iq;
+      const int k = 4 * (PT * i + p);
+      if (k >= DP) continue;
+      *(f32x4*)(ks + t * LK + k) = kv[i] * ik;
+      *(f32x4*)(qs + t * LK + k) = qv[i] * iq;
     }
-    const T* ar = (const T*)c.ap + (size_t)r0 * c.ldap + c.o_a + h * d;
     const float ea = expf(c.A_log[h]);
-    for (int i = tid; i < CH * DP; i += 512) {
-      const int tt = i / DP, ch = i % DP;
-      float g = 1.f;
-      if (tt < n && ch < d) g = expf(-ea * softplus_f(to_f32(ar[(size_t)tt * c.ldap + ch]) + c.dt_bias[h * d + ch]));
-      gs[tt * LK + ch] = g;
+#pragma unroll
+    for (int i = 0; i < NG; ++i) {
+      const int x = i * NT + tid, tt = x / (DP / 4), ch = x % (DP / 4) * 4;
+      if (x >= CH * DP / 4) continue;
+      const bool on = tt < n && ch < d;
+      *(f32x4*)(gs + tt * LK + ch) = on ? f32x4{decay_fast(ea, av[i].x + bv[i].x), decay_fast(ea, av[i].y + bv[i].y), decay_fast(ea, av[i].z + bv[i].z),
+                                                decay_fast(ea, av[i].w + bv[i].w)} : f32x4{1.f, 1.f, 1.f, 1.f};
     }
     if (tid < CH) be[tid] = tid < n ? sigmoid_f(to_f32(((const T*)c.proj)[(size_t)(r0 + tid) * c.ldp + c.o_b + h])) : 0.f;
   }
   __syncthreads();
 
-  // 2. the blocks on the diagonal: wave w has block w mod 4 and every second 16-channel slice, lane (c16, g4) column c16 and four
+  // 2. the blocks on the diagonal: wave w has block w mod 4 and every NB-th 16-channel slice, lane (c16, g4) column c16 and four
   // channels of a slice.  p runs down the column: k_j at token j, times a token's decay from there on (above the diagonal zero).
-  float sa[16], sp[16];
+  const int blk = wave & 3;
+  f32x4 da, dp;                                       // rows 4 g4 .. 4 g4 + 3 of column c16
   {
-    const int b = wave & 3;
+    float sa[16], sp[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) sa[i] = sp[i] = 0.f;
-    for (int s = wave >> 2; s < NS; s += 2) {
+    for (int s = wave >> 2; s < NS; s += NB) {
       const int k = 16 * s + 4 * g4;
-      const f32x4 kj = *(const f32x4*)(ks + (16 * b + c16) * LK + k);
+      const f32x4 kj = *(const f32x4*)(ks + (16 * blk + c16) * LK + k);
       f32x4 p = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < 16; ++i) {
-        const int at = (16 * b + i) * LK + k;
+        const int at = (16 * blk + i) * LK + k;
         const f32x4 g = *(const f32x4*)(gs + at), ki = *(const f32x4*)(ks + at), qi = *(const f32x4*)(qs + at);
         p *= g;
         if (i == c16) p = kj;
 #pragma unroll
         for (int j = 0; j < 4; ++j) { sa[i] = fmaf(p[j], ki[j], sa[i]); sp[i] = fmaf(p[j], qi[j], sp[i]); }
+        if (i % 4 == 3) asm volatile("" ::: "memory");
       }
     }
-#pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      sa[i] += __shfl_xor(sa[i], 16, 64); sa[i] += __shfl_xor(sa[i], 32, 64);
-      sp[i] += __shfl_xor(sp[i], 16, 64); sp[i] += __shfl_xor(sp[i], 32, 64);
-    }
-    if (wave >= 4 && g4 == 0) {
-#pragma unroll
-      for (int i = 0; i < 16; ++i) { kr[(b * 32 + i) * 16 + c16] = sa[i]; kr[(b * 32 + 16 + i) * 16 + c16] = sp[i]; }
+    da = group_sums(sa);
+    dp = group_sums(sp);
+    if (wave >= 4) {
+      float* o = part + ((wave >> 2) - 1) * 2048 + blk * 512 + 4 * lane;
+      *(f32x4*)o = da;
+      *(f32x4*)(o + 256) = dp;
     }
   }
   __syncthreads();
-  if (wave < 4) {                                     // lane (c16, g4): rows 4 g4 .. 4 g4 + 3 of column c16
+  if (wave < 4) {
+    for (int w = 0; w < NB - 1; ++w) {
+      const float* o = part + w * 2048 + blk * 512 + 4 * lane;
+      da += *(const f32x4*)o;
+      dp += *(const f32x4*)(o + 256);
+    }
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      if (i / 4 != g4) continue;
-      const float a = sa[i] + kr[(wave * 32 + i) * 16 + c16], p = sp[i] + kr[(wave * 32 + 16 + i) * 16 + c16];
-      const int row = 16 * wave + i, col = 16 * wave + c16;
-      am[row * LA + col] = i > c16 ? be[row] * a : 0.f;
-      if (row < n) c.pm[((size_t)(r0 + row) * c.H + h) * CH + col] = i >= c16 ? p : 0.f;
+    for (int r = 0; r < 4; ++r) {
+      const int i = 4 * g4 + r, row = 16 * wave + i, col = 16 * wave + c16;
+      am[row * LA + col] = i > c16 ? be[row] * da[r] : 0.f;
+      if (row < n) c.pm[((size_t)(r0 + row) * c.H + h) * CH + col] = i >= c16 ? dp[r] : 0.f;
     }
   }
-  __syncthreads();
 
   // 3. decays inside the blocks: a thread per channel and block
-  if (tid < 4 * DP) {
-    const int b = tid / DP, ch = tid % DP, at = 16 * b * LK + ch;
-    float g[16], suf = 1.f, pre = 1.f;
+  for (int x = tid; x < 4 * DP; x += NT) {
+    const int b = x / DP, ch = x % DP, at = 16 * b * LK + ch;
+    float g[16], k[16], suf = 1.f, pre = 1.f;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) g[i] = gs[at + i * LK];
+    for (int i = 0; i < 16; ++i) { g[i] = gs[at + i * LK]; k[i] = ks[at + i * LK]; }
 #pragma unroll
-    for (int i = 15; i >= 0; --i) { kr[at + i * LK] = ks[at + i * LK] * suf; suf *= g[i]; }
+    for (int i = 15; i >= 0; --i) { gs[at + i * LK] = k[i] * suf; suf *= g[i]; }
 #pragma unroll
-    for (int i = 0; i < 16; ++i) { pre *= g[i]; gs[at + i * LK] = pre; qs[at + i * LK] *= pre; }
+    for (int i = 0; i < 16; ++i) { pre *= g[i]; ks[at + i * LK] = k[i] * pre; qs[at + i * LK] *= pre; }
     tot[b * DP + ch] = suf;
   }
   __syncthreads();
 
   // 4. the six tiles below the diagonal, of A and of P
-  for (int job = wave; job < 12; job += 8) {
+  for (int job = wave; job < 12; job += NW) {
     const bool isq = job & 1;
     const int pr = job >> 1, ti = pr < 1 ? 1 : (pr < 3 ? 2 : 3), tj = pr - ti * (ti - 1) / 2;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    const float* left = (isq ? qs : ks) + (16 * ti + c16) * LK + 4 * g4;
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
-      const int k = 16 * s + 4 * g4, at = (16 * ti + c16) * LK + k;
-      const f32x4 a = isq ? *(const f32x4*)(qs + at) : *(const f32x4*)(ks + at) * *(const f32x4*)(gs + at);
-      f32x4 b = *(const f32x4*)(kr + (16 * tj + c16) * LK + k);
+      const int k = 16 * s + 4 * g4;
+      f32x4 b = *(const f32x4*)(gs + (16 * tj + c16) * LK + k);
       for (int m = tj + 1; m < ti; ++m) b *= *(const f32x4*)(tot + m * DP + k);
-      acc = mfma_slice(a, b, acc);
+      acc = mfma_slice(*(const f32x4*)(left + 16 * s), b, acc);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
@@ -769,7 +848,7 @@ __global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c
     }
   }
   // what delta_carry reads besides: queries from the chunk's start, keys to the chunk's end (transposed), the chunk's decay
-  for (int i = tid; i < CH * (DP / 4); i += 512) {
+  for (int i = tid; i < CH * (DP / 4); i += NT) {
     const int t = i / (DP / 4), k = i % (DP / 4) * 4;
     if (t >= n) break;
     f32x4 q = *(const f32x4*)(qs + t * LK + k);
@@ -777,11 +856,11 @@ __global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c
     *(f32x4*)(c.qm + ((size_t)(r0 + t) * c.H + h) * DP + k) = q;
   }
   float* kt = c.kt + ((size_t)blockIdx.x * c.H + h) * DP * CH;
-  for (int i = tid; i < DP * (CH / 4); i += 512) {
+  for (int i = tid; i < DP * (CH / 4); i += NT) {
     const int k = i / (CH / 4), t = i % (CH / 4) * 4;
     float f = 1.f;
     for (int m = t / 16 + 1; m < 4; ++m) f *= tot[m * DP + k];
-    *(f32x4*)(kt + (size_t)k * CH + t) = f32x4{kr[t * LK + k], kr[(t + 1) * LK + k], kr[(t + 2) * LK + k], kr[(t + 3) * LK + k]} * f;
+    *(f32x4*)(kt + (size_t)k * CH + t) = f32x4{gs[t * LK + k], gs[(t + 1) * LK + k], gs[(t + 2) * LK + k], gs[(t + 3) * LK + k]} * f;
   }
   if (tid < DP) c.fac[((size_t)blockIdx.x * c.H + h) * DP + tid] = tot[tid] * tot[DP + tid] * tot[2 * DP + tid] * tot[3 * DP + tid];
   __syncthreads();
@@ -789,51 +868,50 @@ __global__ __launch_bounds__(512, 2) void delta_chunk_channel_kernel(DeltaCall c
   // 5. T = (I + A)^-1, W = T diag(beta) (K with the decay from the chunk's start), U = T diag(beta) V
   invert_chunk(am, LA, wave, c16, g4);
   auto t_block = [&](int i, int l) { return *(const f32x4*)(am + (16 * l + c16) * LA + 16 * i + 4 * g4); };
-  for (int ct = wave; ct < NS; ct += 8) {
-    const int col = 16 * ct + c16;
-    f32x4 acc[4];
+  auto apply = [&](f32x4 (&acc)[4], const f32x4 (&b)[4]) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    float start = 1.f;
 #pragma unroll
     for (int l = 0; l < 4; ++l) {
-      f32x4 b;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) { const int t = 16 * l + 4 * g4 + j; b[j] = ks[t * LK + col] * gs[t * LK + col] * start * be[t]; }
-      start *= tot[l * DP + col];
-#pragma unroll
-      for (int i = l; i < 4; ++i) acc[i] = mfma_slice(t_block(i, l), b, acc[i]);
+      for (int i = l; i < 4; ++i) acc[i] = mfma_slice(t_block(i, l), b[l], acc[i]);
+      asm volatile("" ::: "memory");
     }
+  };
+  auto put = [&](float* out, uint32_t ld, const f32x4 (&acc)[4]) {       // (a workgroup's outputs stay below 4 GiB)
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int t = 16 * i + 4 * g4 + r;
-        if (t < n) c.wm[((size_t)(r0 + t) * c.H + h) * DP + col] = acc[i][r];
+        const uint32_t t = 16 * i + 4 * g4 + r;
+        if ((int)t < n) *(float*)((char*)out + t * ld * 4u) = acc[i][r];
       }
+  };
+  for (int ct = wave; ct < NS; ct += NW) {
+    const int col = 16 * ct + c16;
+    f32x4 acc[4], b[4];
+    float start = 1.f;
+#pragma unroll
+    for (int l = 0; l < 4; ++l) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { const int t = 16 * l + 4 * g4 + j; b[l][j] = ks[t * LK + col] * start * be[t]; }
+      start *= tot[l * DP + col];
+    }
+    apply(acc, b);
+    put(c.wm + ((size_t)r0 * c.H + h) * DP + col, c.H * DP, acc);
   }
-  for (int ct = wave; ct * 16 < e; ct += 8) {
+  for (int ct = (wave + NW - NS % NW) % NW; ct * 16 < e; ct += NW) {       // (beginning with the waves that had no column of W)
     const int col = min(16 * ct + c16, e - 1);
     f32x4 acc[4], b[4];
 #pragma unroll
-    for (int l = 0; l < 4; ++l) {
-      acc[l] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int j = 0; j < 4; ++j) { const int t = 16 * l + 4 * g4 + j; b[l][j] = vb[(size_t)min(t, n - 1) * c.lds + col] * be[t]; }
-    }
-#pragma unroll
     for (int l = 0; l < 4; ++l)
 #pragma unroll
-      for (int i = l; i < 4; ++i) acc[i] = mfma_slice(t_block(i, l), b[l], acc[i]);
-    if (16 * ct + c16 < e) {                          // (U replaces v: this wave alone reads and writes these columns)
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int t = 16 * i + 4 * g4 + r;
-          if (t < n) vb[(size_t)t * c.lds + col] = acc[i][r];
-        }
-    }
+      for (int j = 0; j < 4; ++j) {
+        const int t = 16 * l + 4 * g4 + j;
+        b[l][j] = *(const float*)((const char*)(vb + col) + (uint32_t)min(t, n - 1) * (uint32_t)c.lds * 4u) * be[t];
+      }
+    apply(acc, b);
+    if (16 * ct + c16 < e) put(vb + col, c.lds, acc);  // (U replaces v: this wave alone reads and writes these columns)
   }
 }
 
@@ -1078,9 +1156,10 @@ template <typename T, int DP>
 int chunked_dp(const DeltaCall& c, hipStream_t st) {
   const dim3 carry_grid(c.H, (c.e + 15) / 16, c.t.nc);
   if (c.channel) {
-    const int lds = (4 * CH * (DP + 4) + CH * (CH + 4) + 4 * DP) * (int)sizeof(float);
-    MI_HIP(hipFuncSetAttribute((const void*)delta_chunk_channel_kernel<T, DP>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
-    hipLaunchKernelGGL((delta_chunk_channel_kernel<T, DP>), dim3(c.t.nct, c.H), dim3(512), lds, st, c);
+    constexpr int NW = DP > 64 ? 16 : 8;               // (one workgroup of 16 waves per CU, or two of 8)
+    const int lds = (3 * CH * (DP + 4) + CH * (CH + 4) + 4 * DP + (NW / 4 - 1) * 2048) * (int)sizeof(float);
+    MI_HIP(hipFuncSetAttribute((const void*)delta_chunk_channel_kernel<T, DP, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+    hipLaunchKernelGGL((delta_chunk_channel_kernel<T, DP, NW>), dim3(c.t.nct, c.H), dim3(64 * NW), lds, st, c);
     MI_HIP(hipGetLastError());
     hipLaunchKernelGGL((delta_carry_kernel<T, DP, true>), carry_grid, dim3(512), 0, st, c);
   } else {

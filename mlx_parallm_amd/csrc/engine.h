@@ -66,7 +66,8 @@ struct ListLayer {
   // low-rank maps: the inner projections (decay | gate) lie side by side in `in`'s output from o_lr, the outer ones are one matrix
   // over both (block-diagonal); o_a / o_g then count in a row of its output
   PackedLinear lr;
-  int o_lr = -1;
+  int o_lr = -1, o_lrg = -1;     // (o_lrg: the gate's)
+  void* low_a = nullptr; void* low_g = nullptr;      // the outer maps row-major (one-token segments), stride a multiple of 8
   // latent attention
   Vec32 c_norm;
   PackedLinear ukv;              // [heads x kdp key rows | heads x vdp value rows] over the latent (padded per head)

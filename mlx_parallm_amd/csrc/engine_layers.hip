@@ -188,6 +188,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
         if (rank == 0) return;
         const int at = part_below(l.in, p + "mix." + name + "1", rank, 64);
         if (l.o_lr < 0) l.o_lr = at;
+        l.o_lrg = at;
         out_at = part(l.lr, p + "mix." + name + "2", l.lr.N, at - l.o_lr, rows, rank);
         l.lr.N += up(rows, 16);
         l.lr.K = at - l.o_lr + up(rank, 64);
@@ -561,6 +562,14 @@ int layers_set_tensor(mi_engine* e, const std::string& name, const void* data, c
   MI_TRY(try_packed(e->list_head, found));
   for (auto& l : e->list)
     for (PackedLinear* L : {&l.in, &l.lr, &l.out, &l.gu, &l.dn, &l.sgu, &l.sdn}) MI_TRY(try_packed(*L, found));
+  for (int i = 0; i < d.num_layers && found; ++i) {    // (the outer low-rank maps are kept row-major as well)
+    ListLayer& l = e->list[i];
+    const mi_layer_desc& m = l.d;
+    const std::string p = "l" + std::to_string(i) + ".mix.";
+    if (!(m.mixer == MI_MIXER_DELTA && m.decay_rank > 0 && m.gate_rank > 0)) continue;
+    if (name == p + "a2") MI_TRY(put_raw(e, l.low_a, m.heads * m.dim, m.decay_rank, up(m.decay_rank, 8), data, on_device));
+    if (name == p + "g2") MI_TRY(put_raw(e, l.low_g, m.heads * m.vdim, m.gate_rank, up(m.gate_rank, 8), data, on_device));
+  }
   if (found) return MI_OK;
   const int W = d.hidden_size;
   if (name == "embed") {
@@ -680,7 +689,7 @@ void layers_free(mi_engine* e) {
   each_vec(e, [](Vec32& v) { hipFree(v.p); v.p = nullptr; });
   for (auto& l : e->list) {
     for (PackedLinear* L : {&l.in, &l.lr, &l.out, &l.ukv, &l.gu, &l.dn, &l.sgu, &l.sdn}) free_packed(*L);
-    hipFree(l.slopes); hipFree(l.router);
+    hipFree(l.slopes); hipFree(l.router); hipFree(l.low_a); hipFree(l.low_g);
     hipFree(l.uk); hipFree(l.uv); hipFree(l.uk_t); hipFree(l.uv_p); hipFree(l.side_gate); hipFree(l.side_proj_t); hipFree(l.side_proj_p);
   }
   free_packed(e->list_head);
@@ -815,7 +824,7 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
     const PolyNormArgs ff{post || pre ? 0 : m.ff, l.o_up, l.o_ff, l.act.p, d.rms_norm_eps};
     if (m.mixer == MI_MIXER_DELTA) {
       const bool channel = m.decay_rank > 0;
-      if (l.lr.N > 0) {
+      if (l.lr.N > 0 && (l.low_a == nullptr || t.nc > 0)) {
         GemvCall cl; cl.x = (const char*)e->proj + (size_t)l.o_lr * es; cl.ldx = l.in.N; cl.act = act; cl.epi = EPI_STORE; cl.out = e->low; cl.ldo = l.lr.N;
         MI_TRY(gemv_rows(e, l.lr.f, cl, R, es, es, "gemv_low"));
       }
@@ -826,6 +835,7 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
       c.ap = channel ? e->low : e->proj; c.ldap = channel ? l.lr.N : l.in.N;
       c.gp = m.gate_rank > 0 ? e->low : e->proj; c.ldgp = m.gate_rank > 0 ? l.lr.N : l.in.N;
       c.channel = channel; c.gate_act = m.out_gate;
+      c.low_a = l.low_a; c.low_g = l.low_g; c.ld_a = up(m.decay_rank, 8); c.ld_gt = up(m.gate_rank, 8); c.in_a = l.o_lr; c.in_g = l.o_lrg;
       c.conv_q = l.conv_q.p; c.conv_k = l.conv_k.p; c.conv_v = l.conv_v.p;
       c.A_log = l.A_log.p; c.dt_bias = l.dt_bias.p; c.head_norm = l.head_norm.p;
       c.scale = m.scale; c.unit_eps = m.unit_eps; c.eps = d.rms_norm_eps;

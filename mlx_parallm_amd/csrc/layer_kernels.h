@@ -100,6 +100,9 @@ struct DeltaCall {
   const void* ap; int ldap, o_a; // [R][ldap] what the decays are made of: one per value head, or (channel) one per value head and key channel
   const void* gp; int ldgp, o_g; // [R][ldgp] output gates, [H e]
   int channel, gate_act;         // gate_act: MI_GATE_SILU or MI_GATE_SIGMOID
+  // one-token segments make both from the inner projections themselves (null: from ap, gp): outer maps [H d][ld_a], [H e][ld_gt] (strides
+  // padded with zeros to a multiple of 8), the inner projections' places in a row of proj
+  const void* low_a; const void* low_g; int ld_a, ld_gt, in_a, in_g;
   const float* conv_q; const float* conv_k; const float* conv_v;    // [channels][taps]
   const float* A_log; const float* dt_bias; const float* head_norm;       // dt_bias [H] or (channel) [H d]
   float scale, unit_eps, eps;
