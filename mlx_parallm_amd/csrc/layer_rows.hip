@@ -609,6 +609,7 @@ int stream_norm_s(const StreamNormCall& c, hipStream_t st) {
 #define SN(NT, NQ) do { hipLaunchKernelGGL((stream_norm_kernel<T, NT, NQ, S>), dim3(c.rows), dim3(NT), 0, st, c); MI_HIP(hipGetLastError()); return MI_OK; } while (0)
   if (c.rows < 256) {                                  // few rows: more threads for each
     if (c.ld <= 1024) SN(256, 1);
+    if (c.ld <= 2048) SN(512, 1);
     if (c.ld <= 4096) SN(1024, 1);
     if (c.ld <= 8192) SN(1024, 2);
     if (c.ld <= 16384) SN(1024, 4);
