@@ -83,8 +83,8 @@ __device__ __forceinline__ void rotate(const Rot<N>& r, float rs, float (&v)[N])
 }
 
 // ---- norms, value mix, append ----------------------------------------------------------------------------------------
-// grid R.  VEC: head sizes are multiples of 8 up to 128, 16 lanes per head; otherwise a wave per head.
-template <typename T, bool VEC>
+// grid R.  VEC: head sizes are multiples of 8 up to 128 (rotated coordinates of 16), 16 lanes per head; otherwise a wave per head.
+template <typename T, bool VEC, bool ROT>
 __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const TokenAt at = token_at(c.t, r);
@@ -113,10 +113,17 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
         if (k < n) {
 #pragma unroll
           for (int i = 0; i < 8; ++i) v[i] *= rs * w[k + i];
-          if (c.rot > 0) {
-            Rot<8> ro;
-            load_rot<T, 8>(c, src, w, k, at.pos, ro);
-            rotate<8>(ro, rs, v);
+        }
+        if constexpr (ROT) {                                    // (rot a multiple of 16: the partners are another lane's eight, normed)
+          const int half = c.rot >> 1;
+          const bool on = k < c.rot, low = k < half;
+          const int with = on ? (low ? lane + half / 8 : lane - half / 8) : lane;
+          const float2* tab = c.rot_tab + (size_t)at.pos * half + (on ? (low ? k : k - half) : 0);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            const float u = __shfl(v[i], with, 64);
+            const float2 cs = tab[i];
+            if (on) v[i] = v[i] * cs.x + (low ? -u : u) * cs.y;
           }
         }
       } else {
@@ -153,7 +160,7 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
         float v = k < n ? to_f32(src[k]) : 0.f;
         if (kind < 2) {
           if (k < n) v *= rs * w[k];
-          if (k < c.rot) {
+          if (ROT && k < c.rot) {
             Rot<1> ro;
             float one[1] = {v};
             load_rot<T, 1>(c, src, w, k, at.pos, ro);
@@ -824,9 +831,10 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 
 template <typename T>
 int pre_at(const GqaCall& c, hipStream_t st) {
-  if (c.dim % 8 == 0 && c.vdim % 8 == 0 && c.kdp <= 128 && c.vdp <= 128)
-    hipLaunchKernelGGL((gqa_pre_kernel<T, true>), dim3(c.t.R), dim3(256), 0, st, c);
-  else hipLaunchKernelGGL((gqa_pre_kernel<T, false>), dim3(c.t.R), dim3(256), 0, st, c);
+  const bool vec = c.dim % 8 == 0 && c.vdim % 8 == 0 && c.kdp <= 128 && c.vdp <= 128 && c.rot % 16 == 0;
+  auto go = [&](auto k) { hipLaunchKernelGGL(k, dim3(c.t.R), dim3(256), 0, st, c); };
+  if (c.rot > 0) { if (vec) go(gqa_pre_kernel<T, true, true>); else go(gqa_pre_kernel<T, false, true>); }
+  else { if (vec) go(gqa_pre_kernel<T, true, false>); else go(gqa_pre_kernel<T, false, false>); }
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
