@@ -438,7 +438,8 @@ def mixed_leg(engine, cfg, args, sample, dist, world):
 
 
 # ---- --design NAME: a layer-list design beside a llama stack of equal width, depth, vocabulary and parameter count (dolurax: of
-# ---- as many parameters per token: four experts of width / 2 and a shared one of width against one layer of 3 x width) ----
+# ---- as many parameters per token: four experts of width / 2 and a shared one of width against one layer of 3 x width; temetar: every
+# ---- second layer recurrent, four residual streams, every layer runs once) ----
 def design_configs(design, width, layers):
     heads, vocab = width // 128, 32000
     if design == "dolurax":

@@ -26,6 +26,7 @@
 // delta_scan (token by token; columns of S are independent, so a wave owns four columns and keeps them in registers, 16 lanes
 // per column).  Both end in delta_out.
 #include <algorithm>
+#include <type_traits>
 
 #include "layer_rows.h"
 
@@ -1137,6 +1138,66 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaCall c) {
   if (c.ff.ff > 0) polynorm_row<T, 256>(c.ff, pr + c.ff.in_off, cat + c.ff.out_off, red);
 }
 
+// ---- outer low-rank maps --------------------------------------------------------------------------------------------
+// grid (ceil(N / 256), ceil(rows / 64)), 4 waves: a wave keeps the 64 rows of x in registers and takes every fourth 16-column tile.
+// The matrix is the left operand, so a lane ends up with four neighbouring outputs of one row.
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef _Float16 f16x8 __attribute__((ext_vector_type(8)));
+template <typename T>
+__device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
+  if constexpr (std::is_same<T, bf16>::value)
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
+  else
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(f16x8, a), __builtin_bit_cast(f16x8, b), c, 0, 0, 0);
+}
+template <typename T, int KS>
+__global__ __launch_bounds__(256) void low_rank_kernel(LowRankCall c) {
+  constexpr int RT = 4, CT = 4;                       // row tiles, column tiles per wave
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int r0 = blockIdx.y * 64, nt = c.W.N / 16, kb = c.W.K / 32;
+  int part = -1;
+  u32x4 x[RT][KS];
+#pragma unroll
+  for (int i = 0; i < CT; ++i) {
+    const int ct = blockIdx.x * 16 + i * 4 + wave;
+    if (ct >= nt) break;
+    const int p = ct * 16 >= c.split ? 1 : 0;
+    const u32x4* w = (const u32x4*)c.W.w + ((size_t)ct * kb + p * KS) * 64 + lane;
+    u32x4 a[KS];
+#pragma unroll
+    for (int s = 0; s < KS; ++s) a[s] = w[s * 64];
+    if (p != part) {                                  // (the workgroup's first tile, and where the two halves meet)
+      part = p;
+#pragma unroll
+      for (int t = 0; t < RT; ++t) {
+        const T* src = (const T*)c.x + (size_t)min(r0 + 16 * t + c16, c.rows - 1) * c.ldx + p * c.k + 8 * g4;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) x[t][s] = *(const u32x4*)(src + 32 * s);
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < RT; ++t) {
+      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < KS; ++s) acc = mfma16<T>(a[s], x[t][s], acc);
+      const int r = r0 + 16 * t + c16;
+      const T o[4] = {from_f32<T>(acc[0]), from_f32<T>(acc[1]), from_f32<T>(acc[2]), from_f32<T>(acc[3])};
+      if (r < c.rows) *(uint2*)((T*)c.out + (size_t)r * c.ldo + 16 * ct + 4 * g4) = __builtin_bit_cast(uint2, o);
+    }
+  }
+}
+
+template <typename T>
+int low_rank_at(const LowRankCall& c, hipStream_t st) {
+  const dim3 grid((c.W.N + 255) / 256, (c.rows + 63) / 64);
+#define GO(KS) hipLaunchKernelGGL((low_rank_kernel<T, KS>), grid, dim3(256), 0, st, c)
+  switch (c.k) { case 64: GO(2); break; case 128: GO(4); break; case 192: GO(6); break; default: GO(8); break; }
+#undef GO
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
 template <typename T>
 int scanned_at(const DeltaCall& c, hipStream_t st) {
   hipLaunchKernelGGL(delta_prep_kernel<T>, dim3(c.t.R), dim3(256), 0, st, c);
@@ -1219,6 +1280,16 @@ int delta_chunk_pad(int H, int d, int e, int taps) {
 }
 
 bool delta_supported(int d, int e) { return d >= 1 && d <= 512 && e >= 1 && (e <= DNT || (e % 4 == 0 && e <= 4 * DNT)); }
+
+bool low_rank_supported(const LowRankCall& c) {
+  const bool kind = (c.W.wk == WK_BF16 && c.act == MI_BF16) || (c.W.wk == WK_F16 && c.act == MI_F16);
+  return kind && c.W.layout == 1 && c.k >= 64 && c.k <= 256 && c.k % 64 == 0 && c.W.K == 2 * c.k && c.split % 16 == 0 && c.W.N % 16 == 0 &&
+         c.ldx % 8 == 0 && c.ldo % 4 == 0 && c.rows > 0 && c.rows <= 65535 * 64;
+}
+int launch_low_rank(const LowRankCall& c, hipStream_t st) {
+  if (!low_rank_supported(c)) return fail(MI_ERR_INVALID, "low_rank: shape or layout not supported");
+  return c.act == MI_BF16 ? low_rank_at<bf16>(c, st) : low_rank_at<f16>(c, st);
+}
 
 int launch_delta(const DeltaCall& c, hipStream_t st) {
   if (!delta_supported(c.d, c.e) || c.taps < 1 || c.H % c.G != 0) return fail(MI_ERR_UNSUPPORTED, "delta: head sizes not supported");

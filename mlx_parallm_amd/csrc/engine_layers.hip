@@ -825,8 +825,15 @@ int forward_segments(mi_engine* e, mi_kv* kv, const int32_t* rows, const int32_t
     if (m.mixer == MI_MIXER_DELTA) {
       const bool channel = m.decay_rank > 0;
       if (l.lr.N > 0 && (l.low_a == nullptr || t.nc > 0)) {
-        GemvCall cl; cl.x = (const char*)e->proj + (size_t)l.o_lr * es; cl.ldx = l.in.N; cl.act = act; cl.epi = EPI_STORE; cl.out = e->low; cl.ldo = l.lr.N;
-        MI_TRY(gemv_rows(e, l.lr.f, cl, R, es, es, "gemv_low"));
+        const char* x = (const char*)e->proj + (size_t)l.o_lr * es;
+        const LowRankCall lc{l.lr.f.W, l.o_g, up(m.decay_rank, 64), x, l.in.N, R, e->low, l.lr.N, act};
+        if (R >= 256 && m.decay_rank > 0 && up(m.gate_rank, 64) == lc.k && low_rank_supported(lc)) {
+          Prof pr(e, "gemv_low");
+          MI_TRY(launch_low_rank(lc, st));
+        } else {
+          GemvCall cl; cl.x = x; cl.ldx = l.in.N; cl.act = act; cl.epi = EPI_STORE; cl.out = e->low; cl.ldo = l.lr.N;
+          MI_TRY(gemv_rows(e, l.lr.f, cl, R, es, es, "gemv_low"));
+        }
       }
       DeltaCall c{};
       c.t = t; c.H = m.heads; c.G = m.kv_heads; c.d = m.dim; c.e = m.vdim; c.taps = m.conv;

@@ -122,6 +122,12 @@ int launch_delta(const DeltaCall& c, hipStream_t st);
 bool delta_supported(int d, int e);
 int delta_chunk_pad(int H, int d, int e, int taps);     // padded head size of the chunked form, 0 = not supported
 
+// The outer low-rank maps of many rows (delta.hip): out[r][0 .. n) = W x[r], where rows [0, split) of W use the columns [0, k) of x and
+// W, the rows behind them the next k (W is block-diagonal).  16-bit, tile-major W, split a multiple of 16.
+struct LowRankCall { LinearW W; int split, k; const void* x; int ldx, rows; void* out; int ldo, act; };
+bool low_rank_supported(const LowRankCall& c);
+int launch_low_rank(const LowRankCall& c, hipStream_t st);
+
 // Latent attention (latent.hip): the cache holds one latent per token, [token][rp]; keys and values are maps of it
 struct LatentCall {
   SegTables t;

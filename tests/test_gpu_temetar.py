@@ -172,6 +172,15 @@ def test_each_delta_form_alone(bank, name, dtype):
     check_portions(m, t, R.forward(cfg, w, t), dtype, ([140], [64, 64, 12], [65, 1, 63, 2, 9], [24, 23, 25, 2, 66], [2] * 70, [1] * 140))
 
 
+@pytest.mark.parametrize("dtype", ["bfloat16", "float16"])
+@pytest.mark.parametrize("ranks", [(5, 7), (100, 128), (70, 190), (130, 192), (256, 250), (300, 270)])
+def test_low_rank_maps_of_many_rows(bank, ranks, dtype):
+    """Inner sizes of every form of the kernel for many rows, unequal ones and larger ones, beside one-token segments."""
+    cfg, w, m = bank(f"ranks_{ranks}", dtype, config(72, 96, [delta(3, 1, 20, 36, 3), delta(5, 5, 36, 17, 2)], 2, None, None), ranks=ranks)
+    t = tokens(cfg, 340, 12)
+    check_portions(m, t, R.forward(cfg, w, t), dtype, ([340], [260, 1, 1, 78]), 64)
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("decay", ["none", "strong", "extreme", "mixed", "steps"])
 def test_ends_of_the_decays_range(bank, decay, dtype):
