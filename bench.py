@@ -458,7 +458,7 @@ def design_configs(design, width, layers):
                "mixer": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4, "decay_rank": 128, "gate_rank": 128}}
         run = {"model_type": "temetar", "architecture": "Temetar", "width": width, "vocab": vocab, "layers": [att, rec] * (layers // 2),
                "norm": {"eps": 1e-5}, "streams": 4, "residual_mult": 1.0, "loop": None,
-               "embedding": {"scale": 1.0, "bigram": {"buckets": 8191, "mul_prev": 127, "mul_cur": 31}}}
+               "embedding": {"scale": 1.0, "bigram": {"buckets": 8191, "mul_prev": 401, "mul_cur": 31}}}
         return run, llama_like(width, layers, heads, vocab)
     one = []
     for i in range(layers):
