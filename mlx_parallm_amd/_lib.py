@@ -152,12 +152,12 @@ SIGNATURES = {
 _lib = None
 
 
-def build(verbose: bool = False) -> Path:
-    """Compile the HIP sources in-tree (``make`` in mlx_parallm_amd/csrc) for gfx950."""
+def build(verbose: bool = False, force: bool = False) -> Path:
+    """Compile the HIP sources in-tree (``make`` in mlx_parallm_amd/csrc) for gfx950; ``force``: all of them."""
     env = dict(os.environ)
     env.setdefault("HIPCC", "/opt/rocm/bin/hipcc")
     jobs = str(min(int(os.environ.get("MAX_JOBS") or 8), 16, max(2, os.cpu_count() or 2)))
-    res = subprocess.run(["make", "-C", str(CSRC), "-j", jobs], env=env, capture_output=True, text=True)
+    res = subprocess.run(["make", "-C", str(CSRC), "-j", jobs] + (["-B"] if force else []), env=env, capture_output=True, text=True)
     if verbose or res.returncode != 0:
         print(res.stdout[-4000:])
         print(res.stderr[-8000:])
