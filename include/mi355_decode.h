@@ -35,7 +35,7 @@ extern "C" {
  * `struct_size`, which the caller sets to sizeof() of ITS definition -- a binding generated from another version of this
  * header (a shorter mi_sample_params would make the library read pointers past its end) is refused with MI_ERR_INVALID
  * by mi_engine_create / mi_decode_sample / mi_step_enqueue(_rows) / mi_score_tokens instead of being read. */
-#define MI_ABI_VERSION 5
+#define MI_ABI_VERSION 6
 
 #define MI_OK 0
 #define MI_ERR_INVALID (-1)
@@ -61,25 +61,39 @@ extern "C" {
 #define MI_BLOCK_POST_NORM 1 /* x += norm1(mixer(x)), then x += norm2(ff(x)); nothing in front of mixer and ff */
 #define MI_BLOCK_PRE_NORM 2 /* x += m mixer(norm1(x)), then x += m ff(norm2(x)); with `streams` copies of x (hyper-connections): a sublayer
                              * reads u = sum_s in[s] x_s and writes x_t <- sum_s mix[s][t] x_s + m out[t] y, per layer and sublayer */
+#define MI_BLOCK_SANDWICH 3 /* x += norm1b(mixer(norm1(x))), then x += norm2b(ff(norm2(x))) */
 #define MI_NORM_VECTOR 0    /* RMS norm, a weight per coordinate */
 #define MI_NORM_SCALAR 1    /* RMS norm, one weight for all coordinates */
 #define MI_NORM_LAYER 2     /* layer norm (mean taken off), weight and bias per coordinate; MI_BLOCK_POST_NORM only */
 /* mixers */
 #define MI_MIXER_DELTA 0    /* gated delta rule with short convolutions (recurrent state per cache row); the decay is one number per
                              * head, or one per head and key channel through a low-rank map (decay_rank) */
-#define MI_MIXER_LATENT 1   /* latent attention without positions (the cache holds one latent per token) */
-#define MI_MIXER_GQA 2      /* grouped-query attention with normed q / k (post- and pre-norm blocks).  Each of: rotation, soft cap,
+#define MI_MIXER_LATENT 1   /* latent attention (the cache holds one latent per token).  Each of: a rotated part of queries and keys (the
+                             * keys' is one for all heads and lies beside the latent in the cache), queries through a latent of their
+                             * own, sigmoid gate per head */
+#define MI_MIXER_GQA 2      /* grouped-query attention with normed q / k (post-, pre-norm and sandwich blocks).  Each of: rotation, soft cap,
                              * distance bias, chunks of positions or a sliding window with kept first tokens, sink, values mixed with
-                             * an earlier layer's, sigmoid gate on the output */
+                             * an earlier layer's, keys and values of an earlier layer, sigmoid gate on the output */
+#define MI_MIXER_LIGHTNING 3 /* linear attention, S <- decay_h S + k v^T, o = S^T q (recurrent state per cache row); q, k, v through silu, the
+                             * concatenated heads through one RMS norm and a sigmoid gate */
 /* feed-forward kinds and activations */
 #define MI_FF_DENSE 0
-#define MI_FF_MOE 1         /* routed experts and at most one shared expert (MI_BLOCK_POST_NORM) */
+#define MI_FF_MOE 1         /* routed experts and at most one shared expert (MI_BLOCK_POST_NORM, MI_BLOCK_SANDWICH) */
 #define MI_ACT_POLYNORM 0   /* a N(z) + b N(z^2) + c N(z^3) + e, N = division by the root mean square over the row */
 #define MI_ACT_SWIGLU 1     /* silu(gate) * up */
-/* gate on a mixer's output, element by element */
+#define MI_ACT_GEGLU 2      /* gelu(gate) * up, gelu in its tanh form */
+#define MI_ACT_CLAMPED 3    /* g sigmoid(1.702 g) (u + 1), g = min(gate, act_limit), u = up clamped to [-act_limit, act_limit] */
+/* gate on a mixer's output: element by element, or one number per head */
 #define MI_GATE_NONE 0
 #define MI_GATE_SILU 1
 #define MI_GATE_SIGMOID 2
+#define MI_GATE_SIGMOID_HEAD 3
+/* norm of a query or key head: RMS norm with weights in front of the rotation, or without weights behind it */
+#define MI_QK_NORM_FIRST 0
+#define MI_QK_NORM_LAST 1
+/* partners of a rotation: coordinate i and i + rot_dims / 2, or 2i and 2i + 1 */
+#define MI_ROT_HALVES 0
+#define MI_ROT_PAIRS 1
 
 /* KV-cache element type selector for mi_kv_create */
 #define MI_KV_MODEL (-1) /* BatchedKVCache semantics: KV in the model dtype (models/base.py:66-85) */
@@ -138,7 +152,7 @@ typedef struct mi_layer_desc {
   int32_t vdim;              /* value size per head */
   int32_t conv;              /* delta: taps of the short convolutions (>= 1) */
   int32_t kv_rank;           /* latent: size of the latent */
-  int32_t kv_from;           /* latent: earlier layer whose latents are read, -1 = this layer's own */
+  int32_t kv_from;           /* latent, gqa: earlier layer whose latents / keys and values are read, -1 = this layer's own */
   float scale;               /* latent, gqa: score scale; delta: factor on the unit query */
   float unit_eps;            /* delta: eps of the unit vectors x / sqrt(sum x^2 + eps) */
   int32_t ff;                /* feed-forward width (of one expert for MI_FF_MOE), 0 = none */
@@ -148,23 +162,37 @@ typedef struct mi_layer_desc {
   float slope_exp;           /* distance bias -2^(-slope_exp (h + 1) / heads) (i - j) of head h, 0 = none */
   int32_t chunk;             /* i sees j <= i only if i / chunk = j / chunk (positions of the sequence), 0 = causal only */
   int32_t v_mix;             /* 1: v = (1 - w) v + w v_first, v_first = the values of the first such layer (which mixes nothing) */
-  /* mixture of experts: softmax router, `top` experts among the `keep` best of `groups` equal groups, weights normalised */
+  /* mixture of experts: `top` experts among the `keep` best of `groups` equal groups, weights = softmax over the chosen logits */
   int32_t ff_kind;           /* MI_FF_* */
   int32_t experts;
   int32_t top;
   int32_t groups;
   int32_t keep;
   int32_t shared_ff;         /* width of the shared expert, 0 = none */
-  int32_t out_gate;          /* delta, gqa: MI_GATE_* */
+  int32_t out_gate;          /* delta, gqa, latent: MI_GATE_* */
+  /* gqa, latent */
+  int32_t rot_dims;          /* gqa: the first rot_dims (even) coordinates of a query or key head are rotated; latent: size of the rotated part */
+  float rot_base;            /* by position * rot_base^(-2i / rot_dims) for pair i; rot_dims = 0: none */
   /* gqa */
-  int32_t rot_dims;          /* the first rot_dims (even) coordinates of a query or key head are rotated, coordinate i with i + rot_dims / 2 */
-  float rot_base;            /* by position * rot_base^(-2i / rot_dims); rot_dims = 0: none */
   int32_t window;            /* i sees j <= i only if i - j < window or j < keep_first; 0 = all (not together with chunk) */
   int32_t keep_first;
   int32_t sink;              /* 1: the softmax denominator has the term exp(sink_h) as well */
   /* delta */
   int32_t decay_rank;        /* > 0: one decay per head and key channel, a = W_a2 (W_a1 h) with this inner size; 0: one per head, a = W_a h */
   int32_t gate_rank;         /* > 0: gate = W_g2 (W_g1 h) with this inner size; 0: W_g h */
+  /* gqa, latent: pairs of the rotation, and its frequencies f_i stretched to a longer context (YaRN): rot_factor > 0: f_i / rot_factor where
+   * a pair turns less than rot_slow times within rot_original tokens, f_i where it turns more than rot_fast times, a ramp over i in
+   * between; cosines and sines times 0.1 ln(rot_factor) + 1.  rot_factor = 0: f_i as it is */
+  int32_t rot_pairs;         /* MI_ROT_* */
+  float rot_factor;
+  float rot_original;
+  float rot_fast;
+  float rot_slow;
+  int32_t qk_norm;           /* gqa: MI_QK_NORM_* */
+  int32_t q_rank;            /* latent: > 0: q = W_uq rms(W_dq h) with this inner size; 0: W_q h */
+  float act_limit;           /* MI_ACT_CLAMPED */
+  int32_t router_bias;       /* 1: the router has a bias ("router.b") */
+  const double* decay;       /* lightning: [heads], each in [0, 1]; read during the call only */
 } mi_layer_desc;
 
 /* arguments of the `sample` closure (utils.py:345-364) + top_p_sampling (sample_utils.py:3-38) */

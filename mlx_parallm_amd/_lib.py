@@ -18,14 +18,16 @@ MI_F32, MI_BF16, MI_F16, MI_U32 = 0, 1, 2, 3
 MI_KV_MODEL = -1
 MI_ARCH_LLAMA, MI_ARCH_QWEN3, MI_ARCH_LAYERS = 0, 1, 2
 MI_POS_NONE, MI_POS_SINUSOIDAL = 0, 1
-MI_BLOCK_PARALLEL, MI_BLOCK_POST_NORM, MI_BLOCK_PRE_NORM = 0, 1, 2
+MI_BLOCK_PARALLEL, MI_BLOCK_POST_NORM, MI_BLOCK_PRE_NORM, MI_BLOCK_SANDWICH = 0, 1, 2, 3
 MI_NORM_VECTOR, MI_NORM_SCALAR, MI_NORM_LAYER = 0, 1, 2
-MI_MIXER_DELTA, MI_MIXER_LATENT, MI_MIXER_GQA = 0, 1, 2
+MI_MIXER_DELTA, MI_MIXER_LATENT, MI_MIXER_GQA, MI_MIXER_LIGHTNING = 0, 1, 2, 3
 MI_FF_DENSE, MI_FF_MOE = 0, 1
-MI_ACT_POLYNORM, MI_ACT_SWIGLU = 0, 1
-MI_GATE_NONE, MI_GATE_SILU, MI_GATE_SIGMOID = 0, 1, 2
+MI_ACT_POLYNORM, MI_ACT_SWIGLU, MI_ACT_GEGLU, MI_ACT_CLAMPED = 0, 1, 2, 3
+MI_GATE_NONE, MI_GATE_SILU, MI_GATE_SIGMOID, MI_GATE_SIGMOID_HEAD = 0, 1, 2, 3
+MI_QK_NORM_FIRST, MI_QK_NORM_LAST = 0, 1
+MI_ROT_HALVES, MI_ROT_PAIRS = 0, 1
 MI_MAX_TOP_LOGPROBS = 20
-MI_ABI_VERSION = 5
+MI_ABI_VERSION = 6
 WK = {"f32": 0, "bf16": 1, "f16": 2, "q4_f32": 3, "q4_bf16": 4, "q4_f16": 5, "q8_f32": 6, "q8_bf16": 7, "q8_f16": 8}
 RND_NONE, RND_BF16, RND_F16 = 0, 1, 2
 PRO_NONE, PRO_NORM = 0, 1
@@ -59,6 +61,9 @@ class LayerDesc(C.Structure):
         ("experts", C.c_int32), ("top", C.c_int32), ("groups", C.c_int32), ("keep", C.c_int32), ("shared_ff", C.c_int32),
         ("out_gate", C.c_int32), ("rot_dims", C.c_int32), ("rot_base", C.c_float), ("window", C.c_int32), ("keep_first", C.c_int32),
         ("sink", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32),
+        ("rot_pairs", C.c_int32), ("rot_factor", C.c_float), ("rot_original", C.c_float), ("rot_fast", C.c_float), ("rot_slow", C.c_float),
+        ("qk_norm", C.c_int32), ("q_rank", C.c_int32), ("act_limit", C.c_float), ("router_bias", C.c_int32),
+        ("decay", C.POINTER(C.c_double)),
     ]
 
 

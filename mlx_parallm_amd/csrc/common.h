@@ -2,6 +2,7 @@
 #pragma once
 #include <hip/hip_runtime.h>
 #include <stdint.h>
+#include <cmath>
 #include <string>
 
 #include "../../include/mi355_decode.h"
@@ -126,6 +127,27 @@ __device__ __forceinline__ float wave_max(float v) {
   for (int o = 32; o > 0; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
   return v;
 }
+
+// Gated linear unit of a feed-forward, gate g and up u:  t sigma(t (a + b t^2)) (v + add),  t = min(g, lim), v = u clamped to [-lim, lim].
+// kind GLU_SILU: a = 1 (silu(g) u); GLU_GELU: gelu in its tanh form, z (1 + tanh(c (z + 0.044715 z^3))) / 2 = z sigma(2 c (z + ..)),
+// c = sqrt(2 / pi); GLU_CLAMP: a = 1.702, both clamped, add = 1.
+enum : int { GLU_SILU = 0, GLU_GELU = 1, GLU_CLAMP = 2 };
+struct Glu { int kind = GLU_SILU; float a = 1.f, b = 0.f, lim = INFINITY, add = 0.f; };
+__device__ __forceinline__ float glu_f(const Glu& c, float g, float u) {
+  const float t = fminf(g, c.lim), v = fminf(fmaxf(u, -c.lim), c.lim);
+  return t / (1.0f + expf(-t * fmaf(c.b * t, t, c.a))) * (v + c.add);
+}
+// the same on a 16-bit model's accumulators: silu rounds every operation to AT, the others the result alone
+template <typename AT>
+__device__ __forceinline__ AT glu16(const Glu& c, float g, float u) {
+  if (c.kind != GLU_SILU) return (AT)glu_f(c, g, u);
+  const float gt = (float)(AT)g, up = (float)(AT)u;
+  const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
+  const float sl = (float)(AT)(gt * sig);
+  return (AT)(sl * up);
+}
+// an output column in front of `silu_cols` of a plain store goes through silu (projections that are used only that way)
+__device__ __forceinline__ float silu_col(int silu_cols, int n, float y) { return n < silu_cols ? y / (1.0f + expf(-y)) : y; }
 
 // weight kinds for the generic kernels
 enum : int {

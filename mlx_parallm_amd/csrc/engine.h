@@ -70,6 +70,9 @@ struct ListLayer {
   void* low_a = nullptr; void* low_g = nullptr;      // the outer maps row-major (one-token segments), stride a multiple of 8
   // latent attention
   Vec32 c_norm;
+  PackedLinear uq;               // queries from their latent
+  Vec32 dq_norm;
+  int o_qc = -1, qr = 0, cp = 0; // the queries' latent in a row of `in`'s output, its padded size; place of the rotated key part in a cached row
   PackedLinear ukv;              // [heads x kdp key rows | heads x vdp value rows] over the latent (padded per head)
   void* uk = nullptr; void* uv = nullptr;    // the two maps as loaded, [heads * dim][kv_rank] / [heads * vdim][kv_rank]
   void* uk_t = nullptr;          // [heads][latent (padded)][kdp]: the key map transposed, for queries absorbed into the latent space
@@ -81,14 +84,19 @@ struct ListLayer {
   void* side_gate = nullptr; void* side_proj_t = nullptr; void* side_proj_p = nullptr;   // [dim][width], transposed [dim][width], padded [width][dim]
   bool side_gate_seen = false, side_proj_seen = false;
   Vec32 side_norm;
-  // grouped-query attention
+  // grouped-query attention (q_norm, k_norm: ones where the norm has no weights)
   Vec32 q_norm, k_norm, vmix, sink;
   const float2* rot_tab = nullptr;   // owned by the engine (mi_engine::rot_tabs)
   float* slopes = nullptr;       // [heads] distance bias
   bool v_first = false;          // the first layer whose values are mixed: the later ones read its values
   bool gqa_fast = false;         // matrix-core forms
-  // `norm` is in front of a parallel block and of a pre-norm mixer, behind a post-norm one; norm2 the feed-forward's
-  Vec32 norm_b, norm2, norm2_b;
+  float rot_gain = 1.f;
+  // lightning attention (its norm: head_norm)
+  float* decay = nullptr; float* log2_decay = nullptr;      // [heads]
+  int sd = 0;                    // row stride of the state
+  // `norm` is in front of a parallel block and of a pre-norm or sandwich mixer, behind a post-norm one; norm2 the feed-forward's; norm_out,
+  // norm2_out: behind the sublayers of a sandwich block
+  Vec32 norm_b, norm2, norm2_b, norm_out, norm2_out;
   // hyper-connections of the two sublayers: weights of the streams in what is read, [from][to], of the output in the streams
   Vec32 hc_in[2], hc_mix[2], hc_out[2];
   // SwiGLU feed-forward: gate | up and down matrices (gu, dn); mixture of experts: all routed experts' stacked, the shared expert's
@@ -96,6 +104,8 @@ struct ListLayer {
   int ffp = 0, sffp = 0;         // padded widths
   void* router = nullptr;        // [experts][padded width] row-major
   bool router_seen = false;
+  Vec32 router_b;
+  Glu glu;                       // the feed-forward's unit
 };
 
 // One pass through a layer: what it keeps between calls is its own, also where a layer runs more than once
@@ -183,12 +193,17 @@ struct mi_engine {
   std::vector<ListLayer> list;
   std::vector<LayerRun> runs;    // the layers in the order in which they run
   int n_arena = 0, n_state = 0;
-  struct RotTab { int dims; float base; float2* p; };
-  std::vector<RotTab> rot_tabs;  // one per (rotated coordinates, base)
+  struct RotTab { int dims; float base, factor, original, fast, slow, gain; float2* p; };
+  std::vector<RotTab> rot_tabs;  // one per rotation
   int streams = 1;               // copies of the residual stream
   void* pair_embed = nullptr; bool pair_embed_seen = false;   // [pair_buckets + 1][width]
   void* low = nullptr;           // [rows][max N of `lr`]
   float* dl_q = nullptr; size_t dl_q_cap = 0;                 // channel form: queries with their decays
+  void* qc = nullptr; void* qfull = nullptr;                  // latent attention: [rows][max qr] queries' latents, [rows][max uq.N] queries
+  bool any_light = false, any_latent = false;
+  int latent_qt = 128;           // queries per tile of the latent attention's longer portions, at most
+  float* light_ws = nullptr; size_t light_ws_cap = 0;         // lightning attention: matrices of the chunks
+  int* light_ctr = nullptr; size_t light_ctr_cap = 0;         // arrival tickets of its one-token form (zero between launches)
   PackedLinear list_head;
   Vec32 list_final_norm, list_final_norm_b;
   float* y32 = nullptr;          // [rows][wp] a sublayer's output in front of its norm / of the residual update
@@ -261,7 +276,7 @@ struct mi_kv {
   std::vector<KvArena> arenas;
   char* state = nullptr;
   size_t list_bytes = 0, state_bytes = 0;
-  std::vector<size_t> state_off, ring_off;   // bytes: [row][heads][dim][vdim] float32, [row][taps][channels] model dtype
+  std::vector<size_t> state_off, ring_off;   // bytes: [row][heads][dim][vdim] float32 (lightning: [row][heads][vdim][sd]), [row][taps][channels] model dtype
   int32_t* d_prev = nullptr;     // [row] last token (inside `state`; a model whose embedding looks at the previous token)
 };
 

@@ -56,6 +56,7 @@ struct GemmParams {
                                     // every (x part, W part) pair once.
   int out32;                        // outputs / residual stream are float32 (PagedKVCache mode), no 16-bit rounding
   int epi; void* out; int ldo; void* resid; int pair_offset;
+  Glu glu; int silu_cols;
   // 128 x 128 tile only: K split over gridDim.z workgroups when the (M, N) grid alone leaves most CUs idle (a prompt of a
   // few hundred tokens against N = 4096: 32 x 2..8 blocks); slice z leaves its float32 partial tile in ws[z][M][N] and
   // splitk_epilogue_kernel adds the slices in order and applies the epilogue
@@ -67,6 +68,7 @@ struct GemmParams {
 
 // the epilogues in float32 storage (PagedKVCache mode after layer 0: every op produces a float32 array)
 __device__ __forceinline__ void epi32_swiglu(const GemmParams& p, int m, int n, float gt, float up) {
+  if (p.glu.kind != GLU_SILU) { ((float*)p.out)[(size_t)m * p.ldo + n] = glu_f(p.glu, gt, up); return; }
   const float sig = 1.0f / (1.0f + expf(-gt));
   const float sl = gt * sig;
   ((float*)p.out)[(size_t)m * p.ldo + n] = sl * up;
@@ -77,8 +79,6 @@ __device__ __forceinline__ void epi32_plain(const GemmParams& p, int m, int n, f
 }
 
 // grid: (n blocks, m blocks).  SWIGLU: a block covers 64 gate columns + the 64 matching up columns.
-__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.0f + expf(-g)) * u; }
-
 // grouped form: the matrix and the rows of tile bm of the device-resident table; false: no such tile, or no columns from n0 on
 template <typename AT, bool SWIGLU>
 __device__ __forceinline__ bool group_of_tile(GemmParams& p, int bm, int n0, int& place0) {
@@ -233,12 +233,9 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
         for (int j = 0; j < 2; ++j) {
           const int n = bn * 64 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
-          if constexpr (GROUPED) { out[(size_t)m * p.ldo + n] = (AT)silu_mul(acc[mt][j][r], acc[mt][j + 2][r]); continue; }
+          if constexpr (GROUPED) { out[(size_t)m * p.ldo + n] = (AT)glu_f(p.glu, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
-          const float gt = (float)(AT)acc[mt][j][r], up = (float)(AT)acc[mt][j + 2][r];
-          const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-          const float sl = (float)(AT)(gt * sig);
-          out[(size_t)m * p.ldo + n] = (AT)(sl * up);
+          out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, acc[mt][j][r], acc[mt][j + 2][r]);
         }
       } else {
 #pragma unroll
@@ -246,7 +243,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
           const int n = bn * BN + wn * 64 + nt * 16 + c16;
           if (n >= p.N) continue;
           if (p.out32) { epi32_plain(p, m, n, acc[mt][nt][r]); continue; }
-          const float y = (float)(AT)acc[mt][nt][r];
+          const float y = (float)(AT)silu_col(p.silu_cols, n, acc[mt][nt][r]);
           if (p.epi == EPI_STORE) out[(size_t)m * p.ldo + n] = (AT)y;
           else {
             AT* h = (AT*)p.resid;
@@ -270,7 +267,7 @@ __global__ __launch_bounds__(256) void splitk_epilogue_kernel(GemmParams p) {
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     if (p.out32) { epi32_plain(p, m, n + j, a[j]); continue; }
-    const float y = (float)(AT)a[j];
+    const float y = (float)(AT)silu_col(p.silu_cols, n + j, a[j]);
     if (p.epi == EPI_STORE) ((AT*)p.out)[(size_t)m * p.ldo + n + j] = (AT)y;
     else { AT* h = (AT*)p.resid; h[(size_t)m * p.ldo + n + j] = (AT)((float)h[(size_t)m * p.ldo + n + j] + y); }
   }
@@ -280,7 +277,8 @@ constexpr int BM2 = 256, BN2 = 256;
 
 // the epilogue of the 256 x 256 tiles (2 x 4 waves, 128 x 64 per wave): lane (c16, g) holds C[m = 4g + r][n = c16] of
 // every 16 x 16 tile
-template <typename AT, bool SWIGLU>
+// SILU: a plain store with silu_cols (common.h)
+template <typename AT, bool SWIGLU, bool SILU = false>
 __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&acc)[8][4], int m0, int bn, int wm, int wn, int c16, int g) {
   AT* out = (AT*)p.out;
 #pragma unroll
@@ -295,10 +293,7 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
           const int n = bn * 128 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
-          const float gt = (float)(AT)acc[mt][j][r], up = (float)(AT)acc[mt][j + 2][r];
-          const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-          const float sl = (float)(AT)(gt * sig);
-          out[(size_t)m * p.ldo + n] = (AT)(sl * up);
+          out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, acc[mt][j][r], acc[mt][j + 2][r]);
         }
       } else {
 #pragma unroll
@@ -306,7 +301,7 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
           const int n = bn * BN2 + wn * 64 + nt * 16 + c16;
           if (n >= p.N) continue;
           if (p.out32) { epi32_plain(p, m, n, acc[mt][nt][r]); continue; }
-          const float y = (float)(AT)acc[mt][nt][r];
+          const float y = (float)(AT)(SILU ? silu_col(p.silu_cols, n, acc[mt][nt][r]) : acc[mt][nt][r]);
           if (p.epi == EPI_STORE) out[(size_t)m * p.ldo + n] = (AT)y;
           else {
             AT* h = (AT*)p.resid;
@@ -335,7 +330,7 @@ __device__ __forceinline__ void tile256_epilogue_rows(const GemmParams& p, f32x4
         const f32x4 (&a)[4] = acc[hf * 4 + mt];
         if constexpr (SWIGLU) {
 #pragma unroll
-          for (int j = 0; j < 2; ++j) row[j * 16] = (AT)silu_mul(a[j][r], a[j + 2][r]);
+          for (int j = 0; j < 2; ++j) row[j * 16] = (AT)glu_f(p.glu, a[j][r], a[j + 2][r]);
         } else {
 #pragma unroll
           for (int nt = 0; nt < 4; ++nt) row[nt * 16] = (AT)a[nt][r];
@@ -569,7 +564,8 @@ __global__ __launch_bounds__(512) void gemm_tile256_kernel(GemmParams p) {
       return;
     }
   }
-  tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  if (!SWIGLU && p.silu_cols > bn * BN2) tile256_epilogue<AT, SWIGLU, !SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
 }
 
 
@@ -788,7 +784,8 @@ __global__ __launch_bounds__(512) void gemm_dma256_kernel(GemmParams p) {
   if constexpr (GROUPED) {
     __syncthreads();
     tile256_epilogue_rows<AT, SWIGLU>(p, acc, smem2, bn, wave, lane, place0);
-  } else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  } else if (!SWIGLU && p.silu_cols > bn * BN2) tile256_epilogue<AT, SWIGLU, !SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
 }
 
 
@@ -935,17 +932,14 @@ __global__ __launch_bounds__(512) void gemm_tile256_m32_kernel(GemmParams p) {
         const int n = bn * 128 + wn * 32 + c32;
         if (n >= p.pair_offset) continue;
         if (p.out32) { epi32_swiglu(p, m, n, acc[mt][0][r], acc[mt][1][r]); continue; }
-        const float gt = (float)(AT)acc[mt][0][r], up = (float)(AT)acc[mt][1][r];
-        const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-        const float sl = (float)(AT)(gt * sig);
-        out[(size_t)m * p.ldo + n] = (AT)(sl * up);
+        out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, acc[mt][0][r], acc[mt][1][r]);
       } else {
 #pragma unroll
         for (int nt = 0; nt < 2; ++nt) {
           const int n = bn * BN2 + wn * 64 + nt * 32 + c32;
           if (n >= p.N) continue;
           if (p.out32) { epi32_plain(p, m, n, acc[mt][nt][r]); continue; }
-          const float y = (float)(AT)acc[mt][nt][r];
+          const float y = (float)(AT)silu_col(p.silu_cols, n, acc[mt][nt][r]);
           if (p.epi == EPI_STORE) out[(size_t)m * p.ldo + n] = (AT)y;
           else {
             AT* hh = (AT*)p.resid;
@@ -1236,6 +1230,7 @@ int launch_gemm_prefill(const LinearW& W, const GemvCall& c, size_t rows, hipStr
   }
   if (c.out32) p.out32 = 1;
   p.epi = c.epi; p.out = c.out; p.ldo = c.ldo; p.resid = c.resid; p.pair_offset = c.pair_offset;
+  p.glu = c.glu; p.silu_cols = c.silu_cols;
   const bool sw = c.epi == EPI_SWIGLU;
   const int ncols = sw ? c.pair_offset : W.N;
   static const bool small_only = getenv("MI_GEMM_TILE128") != nullptr;        // A/B: always the 128 x 128 kernel
@@ -1344,7 +1339,7 @@ int launch_gemm_grouped(const GroupedGemm& g, hipStream_t st) {
   GemmParams p{};
   p.ksplit = 1;
   p.x = g.x; p.ldx = g.ldx; p.w = g.W.w; p.N = g.rows; p.K = p.ka = p.kw = g.W.K;
-  p.epi = EPI_STORE; p.out = g.out; p.ldo = g.ldo;
+  p.epi = EPI_STORE; p.out = g.out; p.ldo = g.ldo; p.glu = g.glu;
   p.tiles = g.tiles; p.x_rows = g.x_rows; p.out_rows = g.out_rows; p.groups = g.groups;
   p.w_last = g.last.w; p.N_last = last ? g.last.N : 0; p.K_last = last ? g.last.K : 0;
   const int cols = std::max(g.rows, p.N_last) / (g.swiglu ? 2 : 1);

@@ -624,7 +624,7 @@ bool gemm_q4_supported(const LinearW& W, const GemvCall& c, size_t rows) {
   if (!q4 || (int)rows < min_rows || rows > 128 || c.ldx % 8 != 0) return false;
   const int n = c.epi == EPI_SWIGLU ? c.pair_offset : W.N;
   if (n % 16 != 0) return false;
-  if (c.epi == EPI_SWIGLU_GU8) return false;
+  if (c.epi == EPI_SWIGLU_GU8 || c.glu.kind != GLU_SILU || c.silu_cols > 0) return false;
   // wide matrices only (gate|up, lm_head: >= 1024 tiles), unless a plan is forced (tests, A/B): see q4_plan
   // ... and, behind MI_Q4_NARROW=1 (A/B), the narrow matrix that has an RMSNorm in front (q|k|v), where the preparation pass
   // replaces the norm launch: measured on the config-5 shard 7301 / 7309 tok/s against 7345 / 7342 without (same box,

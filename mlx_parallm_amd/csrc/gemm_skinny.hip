@@ -63,6 +63,7 @@ struct SkinnyParams {
   const void* x; int ldx; int M;
   const void* w; int N, K;
   int epi; void* out; int ldo; void* resid; int pair_offset;
+  Glu glu; int silu_cols;
   int out32;                       // GemvCall::out32 (16-bit activations only)
   // RMSNorm hand-over between two launches of the 16-row instantiation (see "norm hand-over" in the kernel):
   float* sq_out;                   // producer (residual epilogue): [tile groups][sq_ld] sums of h^2 over the group's 128 columns
@@ -757,12 +758,14 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
         const float rsm = dn ? rs_row[ml] : 1.0f;
         y0 *= rsm;
         if constexpr (SWIGLU) {
-          const float gt = round_rt(y0, p.rnd), up = round_rt(acc[NA - 1][mt][r] * rsm, p.rnd);
+          const float up0 = acc[NA - 1][mt][r] * rsm;
+          if (p.glu.kind != GLU_SILU) { o32[(size_t)m * p.ldo + n] = round_rt(glu_f(p.glu, y0, up0), p.rnd); continue; }
+          const float gt = round_rt(y0, p.rnd), up = round_rt(up0, p.rnd);
           const float sig = round_rt(1.0f / (1.0f + expf(-gt)), p.rnd);
           const float sl = round_rt(gt * sig, p.rnd);
           o32[(size_t)m * p.ldo + n] = round_rt(sl * up, p.rnd);
         } else {
-          float y = round_rt(y0, p.rnd);
+          float y = round_rt(silu_col(p.silu_cols, n, y0), p.rnd);
           if (p.lora_t != nullptr) {             // LoRALinear in this mode: y + T(scale (x A) B), the term in float32 (App. A.6)
 #pragma unroll
             for (int sl = 0; sl < 2; ++sl) {
@@ -792,10 +795,7 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
         continue;
       }
       if constexpr (SWIGLU) {
-        const float gt = (float)(AT)y0, up = (float)(AT)acc[NA - 1][mt][r];
-        const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-        const float sl = (float)(AT)(gt * sig);
-        out[(size_t)m * p.ldo + n] = (AT)(sl * up);
+        out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, y0, acc[NA - 1][mt][r]);
       } else {
         if (p.out32) {                             // float32 outputs / residual stream, nothing rounded
           if (p.epi == EPI_RESID) {
@@ -805,7 +805,7 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
           } else ((float*)p.out)[(size_t)m * p.ldo + n] = y0;
           continue;
         }
-        float y = (float)(AT)y0;
+        float y = (float)(AT)silu_col(p.silu_cols, n, y0);
         if (p.lora_t != nullptr) {
 #pragma unroll
           for (int sl = 0; sl < 2; ++sl) {
@@ -1104,6 +1104,7 @@ int launch_gemm_skinny(const LinearW& W, const GemvCall& c, size_t rows, hipStre
   if (p.kx != W.K && (2 * p.kx != W.K || p.kx % SK_KC != 0)) return fail(MI_ERR_INVALID, "gemm_skinny: a [hi | lo] matrix has 2 kx columns, kx a multiple of 256");
   p.out32 = c.out32 && c.act != MI_F32;
   p.epi = c.epi; p.out = c.out; p.ldo = c.ldo; p.resid = c.resid; p.pair_offset = c.epi == EPI_SWIGLU ? c.pair_offset : 0;
+  p.glu = c.glu; p.silu_cols = c.silu_cols;
   const bool nh = (pl.mt == 1 || (pl.mt == 2 && !wk_is_quant(W.wk))) && c.act != MI_F32;
   p.sq_out = (nh && c.epi == EPI_RESID) ? c.sq_out : nullptr;
   p.sq_in = (nh && c.pro == PRO_NORM) ? c.sq_in : nullptr; p.sq_parts = c.sq_parts;

@@ -180,6 +180,7 @@ MfmaParams make_params(const LinearW& W, const GemvCall& c) {
   p.x = c.x; p.ldx = c.ldx; p.M = c.M; p.pro = c.pro; p.norm_w = c.norm_w; p.eps = c.eps;
   p.w = W.w; p.scales = W.scales; p.biases = W.biases; p.N = (c.epi == EPI_SWIGLU) ? c.pair_offset : W.N; p.K = W.K;
   p.epi = c.epi; p.out = c.out; p.ldo = c.ldo; p.resid = c.resid; p.pair_offset = c.pair_offset;
+  p.glu = c.glu; p.silu_cols = c.silu_cols;
   // activation chunk held in LDS as fragments: whole K up to 6144 (M <= 8) / 4096 (M <= 16),
   // else chunks of 4096 (a multiple of every batch span and of the int4 block; 8192 was measured: no gain)
   const int kc_max = c.M <= 8 ? 6144 : 4096;

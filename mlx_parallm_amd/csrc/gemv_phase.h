@@ -20,6 +20,7 @@ struct MfmaParams {
   const void* w; const void* scales; const void* biases;
   int N, K;
   int epi; void* out; int ldo; void* resid; int pair_offset;
+  Glu glu; int silu_cols;
   int layout;       // always 1 here: tile-major (16 rows x 32 k blocks of 1 KiB, repack.hip)
   int kc;       // K elements staged in LDS per chunk
   int out32;    // GemvCall::out32
@@ -417,20 +418,14 @@ struct Phase {
         if (m < p.M) {
           AT* out = (AT*)p.out;
           if constexpr (SWIGLU) {
-            const float gt = (float)(AT)y0, up = (float)(AT)y1;
-            const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-            const float sl = (float)(AT)(gt * sig);
-            store_elem<AT>(&out[(size_t)m * p.ldo + n], (AT)(sl * up), WT);
+            store_elem<AT>(&out[(size_t)m * p.ldo + n], glu16<AT>(p.glu, y0, y1), WT);
           } else if (p.epi == EPI_SWIGLU_GU8) {
             // row-interleaved gate|up tile: columns 0..7 are gate, 8..15 the matching up rows (same reduction order as above)
             if ((el & 15) < 8) {
               float yu = 0.f;
 #pragma unroll
               for (int ww = 0; ww < NW; ++ww) yu += red[((ww * NA + 0) * 64 + el + 8) * 4 + r];
-              const float gt = (float)(AT)y0, up = (float)(AT)yu;
-              const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
-              const float sl = (float)(AT)(gt * sig);
-              store_elem<AT>(&out[(size_t)m * p.ldo + (n >> 4) * 8 + (el & 15)], (AT)(sl * up), WT);
+              store_elem<AT>(&out[(size_t)m * p.ldo + (n >> 4) * 8 + (el & 15)], glu16<AT>(p.glu, y0, yu), WT);
             }
           } else {
             if (p.out32) {                         // float32 outputs / residual stream, nothing rounded
@@ -442,7 +437,7 @@ struct Phase {
               }
               continue;
             }
-            float y = (float)(AT)y0;
+            float y = (float)(AT)silu_col(p.silu_cols, n, y0);
             if (p.lora_t != nullptr) {
 #pragma unroll
               for (int sl = 0; sl < 2; ++sl) {

@@ -34,6 +34,7 @@ struct GemvParams {
   const void* w; const void* scales; const void* biases;
   int N, K, group, layout;
   int epi; void* out; int ldo; void* resid; int pair_offset;
+  Glu glu; int silu_cols;
   int out32;                   // GemvCall::out32
   int npairs;
   // LoRA
@@ -232,6 +233,7 @@ __global__ __launch_bounds__(NTHR) void gemv_v1_kernel(GemvParams p) {
     AT* out = (AT*)p.out;
     if (p.epi == EPI_SWIGLU) {
       // nn.silu(gate) * up, every op rounded to the activation dtype (llama.py:165)
+      if (p.glu.kind != GLU_SILU) { out[(size_t)m * p.ldo + rows[a][0]] = store_act<AT>(glu_f(p.glu, mine[0], mine[1]), p.rnd); continue; }
       const float g = to_f32(store_act<AT>(mine[0], p.rnd));
       const float u = to_f32(store_act<AT>(mine[1], p.rnd));
       const float sig = to_f32(store_act<AT>(1.0f / (1.0f + expf(-g)), p.rnd));
@@ -248,7 +250,7 @@ __global__ __launch_bounds__(NTHR) void gemv_v1_kernel(GemvParams p) {
         else ((float*)p.out)[(size_t)m * p.ldo + n] = mine[r];
         continue;
       }
-      float y = to_f32(store_act<AT>(mine[r], p.rnd));
+      float y = to_f32(store_act<AT>(silu_col(p.silu_cols, n, mine[r]), p.rnd));
       // LoRALinear: y + (scale * ((x A) B)).astype(x.dtype)
       if (p.lora_t != nullptr) {
 #pragma unroll
@@ -431,6 +433,7 @@ GemvParams make_params(const LinearW& W, const GemvCall& c) {
   p.x = c.x; p.ldx = c.ldx; p.M = c.M; p.rnd = c.rnd; p.pro = c.pro; p.norm_w = c.norm_w; p.eps = c.eps;
   p.w = W.w; p.scales = W.scales; p.biases = W.biases; p.N = W.N; p.K = W.K; p.group = W.group; p.layout = W.layout;
   p.epi = c.epi; p.out = c.out; p.ldo = c.ldo; p.resid = c.resid; p.pair_offset = c.pair_offset;
+  p.glu = c.glu; p.silu_cols = c.silu_cols;
   p.out32 = c.out32;
   p.npairs = (c.epi == EPI_SWIGLU) ? c.pair_offset : (W.N + 1) / 2;
   p.lora_t = c.lora_t; p.lora_t_ld = c.lora_t_ld;

@@ -1,8 +1,11 @@
 // gqa.hip -- grouped-query attention (layer-list models).  q and k are divided by their root mean square and their first
-// coordinates rotated by the position, head h scores  softcap tanh(q.k scale / softcap) - slope_h (i - j)  over the keys j <= i of i's
+// coordinates rotated by the position (or first rotated and then divided), head h scores  softcap tanh(q.k scale / softcap) - slope_h (i - j)  over the keys j <= i of i's
 // own chunk of positions (or of a window behind i and the kept first tokens of the sequence), the denominator of the softmax also
 // contains exp(sink_h), the values are mixed with an earlier layer's of the same token before they are cached, and the output is
-// multiplied element by element with sigmoid(gate).  Each of these is a parameter that can be off.
+// multiplied with sigmoid(gate), element by element or head by head.  Keys and values may be an earlier layer's: then nothing is
+// appended.  Each of these is a parameter that can be off.
+// A rotation keeps the length of a pair up to the table's gain, so the mean square behind it is that of the plain coordinates with the
+// rotated ones weighted by the gain squared (rot_gain2): both orders of norm and rotation run as norm, then rotation.
 //
 //   gqa_pre        norms, rotation, value mix and append of every token of the longer segments (generic form: of all tokens)
 //   gqa_generic    any size and dtype: one workgroup per (token, query head), float32 arithmetic
@@ -36,8 +39,13 @@ __device__ __forceinline__ int first_seen(const GqaCall& c, int pos) {
   return c.window > 0 ? max(0, pos - c.window + 1) : (c.chunk > 0 ? pos / c.chunk * c.chunk : 0);
 }
 
+// weight of coordinate k in the mean square
+__device__ __forceinline__ float square_weight(const GqaCall& c, int k) { return k < c.rot ? c.rot_gain2 : 1.f; }
+// where head h's gates begin, and the one of its element d
+__device__ __forceinline__ int gate_at(const GqaCall& c, int h, int d) { return c.gate_head ? h : h * c.vdim + d; }
+
 // What the rotation of the N coordinates k .. k + N - 1 of a head needs besides themselves: their partners (as projected, and the
-// partners' norm weights), cosine and sine.  Coordinate j < rot / 2 goes with j + rot / 2.
+// partners' norm weights), cosine and sine.
 template <int N>
 struct Rot { float v[N], w[N], c[N], s[N]; };
 template <typename T, int N>
@@ -48,6 +56,17 @@ __device__ __forceinline__ void load_rot(const GqaCall& c, const T* src, const f
   for (int i = 0; i < N; ++i) { r.v[i] = 0.f; r.w[i] = 0.f; r.c[i] = 1.f; r.s[i] = 0.f; }
   if (k >= c.rot) return;
   typedef T tv __attribute__((ext_vector_type(N)));
+  if (c.pairs) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int j = k + i;
+      if (j >= c.rot) continue;
+      const RotAt a = rot_at(j, c.rot, 1);
+      const float2 cs = tab[a.f];
+      r.v[i] = to_f32(src[a.partner]); r.w[i] = w[a.partner]; r.c[i] = cs.x; r.s[i] = a.sign * cs.y;
+    }
+    return;
+  }
   if (half % N == 0 && k % N == 0) {                 // (the N coordinates lie in one half)
     const int p = k < half ? k + half : k - half, f = k < half ? k : k - half;
     const bool aligned = ((uintptr_t)(src + p) & (N * sizeof(T) - 1)) == 0;
@@ -70,9 +89,9 @@ __device__ __forceinline__ void load_rot(const GqaCall& c, const T* src, const f
   for (int i = 0; i < N; ++i) {
     const int j = k + i;
     if (j >= c.rot) continue;
-    const int p = j < half ? j + half : j - half;
-    const float2 cs = tab[j < half ? j : j - half];
-    r.v[i] = to_f32(src[p]); r.w[i] = w[p]; r.c[i] = cs.x; r.s[i] = j < half ? -cs.y : cs.y;
+    const RotAt a = rot_at(j, c.rot, 0);
+    const float2 cs = tab[a.f];
+    r.v[i] = to_f32(src[a.partner]); r.w[i] = w[a.partner]; r.c[i] = cs.x; r.s[i] = a.sign * cs.y;
   }
 }
 // v: the normed coordinates, rs: the head's reciprocal root mean square
@@ -83,7 +102,7 @@ __device__ __forceinline__ void rotate(const Rot<N>& r, float rs, float (&v)[N])
 }
 
 // ---- norms, value mix, append ----------------------------------------------------------------------------------------
-// grid R.  VEC: head sizes are multiples of 8 up to 128 (rotated coordinates of 16), 16 lanes per head; otherwise a wave per head.
+// grid R.  VEC: head sizes are multiples of 8 up to 128 (coordinates rotated in halves: of 16), 16 lanes per head; otherwise a wave per head.
 template <typename T, bool VEC, bool ROT>
 __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
   const int r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -91,7 +110,7 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
   if (!c.all_tokens && c.t.len[at.seg] == 1) return;           // (gqa_decode does its own)
   const T* pr = (const T*)c.proj + (size_t)r * c.ldp;
   const float lam = c.v_mix != nullptr ? *c.v_mix : 0.f;
-  const int nh = c.H + 2 * c.G;
+  const int nh = c.H + (c.shared ? 0 : 2 * c.G);
   if constexpr (VEC) {
     const int g = lane >> 4, l = lane & 15;
     for (int h0 = wave * 4; h0 < nh; h0 += 16) {
@@ -107,14 +126,25 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
       if (kind < 2) {
         float ss = 0.f;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
+        for (int i = 0; i < 8; ++i) ss += v[i] * v[i] * square_weight(c, k + i);
         const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)n + c.eps);
         const float* w = kind == 0 ? c.q_norm : c.k_norm;
         if (k < n) {
 #pragma unroll
           for (int i = 0; i < 8; ++i) v[i] *= rs * w[k + i];
         }
-        if constexpr (ROT) {                                    // (rot a multiple of 16: the partners are another lane's eight, normed)
+        if (ROT && c.pairs) {                                   // (the partners are this lane's)
+          const float2* tab = c.rot_tab + (size_t)at.pos * (c.rot >> 1);
+          float u[8];
+#pragma unroll
+          for (int i = 0; i < 8; ++i) u[i] = v[i];
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            if (k + i >= c.rot) continue;
+            const float2 cs = tab[(k + i) >> 1];
+            v[i] = u[i] * cs.x + ((i & 1) ? u[i ^ 1] : -u[i ^ 1]) * cs.y;
+          }
+        } else if constexpr (ROT) {                             // (rot a multiple of 16: the partners are another lane's eight, normed)
           const int half = c.rot >> 1;
           const bool on = k < c.rot, low = k < half;
           const int with = on ? (low ? lane + half / 8 : lane - half / 8) : lane;
@@ -153,7 +183,7 @@ __global__ __launch_bounds__(256) void gqa_pre_kernel(GqaCall c) {
       const float* w = kind == 0 ? c.q_norm : c.k_norm;
       if (kind < 2) {
         float ss = 0.f;
-        for (int k = lane; k < n; k += 64) { const float v = to_f32(src[k]); ss += v * v; }
+        for (int k = lane; k < n; k += 64) { const float v = to_f32(src[k]); ss += v * v * square_weight(c, k); }
         rs = 1.0f / sqrtf(wave_sum(ss) / (float)n + c.eps);
       }
       for (int k = lane; k < np; k += 64) {
@@ -236,11 +266,11 @@ __global__ __launch_bounds__(256) void gqa_generic_kernel(GqaCall c) {
   float w[4], lt = c.sink != nullptr ? expf(c.sink[h] - mx) : 0.f;
 #pragma unroll
   for (int i = 0; i < 4; ++i) { w[i] = expf(ml[i] - mx); lt += w[i] * ml[4 + i]; }
-  const T* gate = (const T*)c.proj + (size_t)r * c.ldp + max(c.o_g, 0) + h * c.vdim;
+  const T* gate = (const T*)c.proj + (size_t)r * c.ldp + max(c.o_g, 0);
   T* cat = (T*)c.cat + (size_t)r * c.ldc + h * c.vdim;
   for (int k = threadIdx.x; k < c.vdim; k += 256) {
     const float v = (w[0] * sm[k] + w[1] * sm[c.vdp + k] + w[2] * sm[2 * c.vdp + k] + w[3] * sm[3 * c.vdp + k]) / lt;
-    cat[k] = from_f32<T>(c.o_g >= 0 ? v * sigmoid_f(to_f32(gate[k])) : v);
+    cat[k] = from_f32<T>(c.o_g >= 0 ? v * sigmoid_f(to_f32(gate[gate_at(c, h, k)])) : v);
   }
 }
 
@@ -321,7 +351,8 @@ __device__ __forceinline__ void load_upto(const T* p, int k, int n, float (&v)[N
 }
 
 // grid (nsplit, G x head tiles, nd), 4 waves; a wave walks its 32-key blocks on its own, the next block's loads in flight during
-// the current one.  The token's own key and value are added by the last split from LDS, which also appends them.
+// the current one.  The token's own key and value are added by the last split from LDS, which also appends them (shared: they are in
+// the cache already).
 template <typename T, int KD, int VD, bool PAGED, bool CAP>
 __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   constexpr int KK = KD / 32, DT = VD / 16, KB = 32, IMG = KB * VD * 2, NV = KB * VD / 8 / 64, LQ = KD + 8;
@@ -337,9 +368,10 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   const int split = blockIdx.x, kh = blockIdx.y / ht_n, ht = blockIdx.y % ht_n, m = blockIdx.z;
   const int seg = c.t.dec[m], row = c.t.row[seg], tok = c.t.tok0[seg], pos = c.t.off[row];
   const int h0 = kh * rep + ht * 16, nh = min(16, rep - ht * 16);
-  const int lo = max(first_seen(c, pos), pos - key_reach(c, c.slopes[h0 + nh - 1] * LOG2E));     // cached keys [lo, pos) (the slopes fall)
+  const int end = pos + (c.shared ? 1 : 0);
+  const int lo = max(first_seen(c, pos), pos - key_reach(c, c.slopes[h0 + nh - 1] * LOG2E));     // cached keys [lo, end) (the slopes fall)
   const int kept = min(c.keep, pos);                                                             // and [0, kept)
-  const int blk0 = lo / KB, nmain = pos > lo ? (pos + KB - 1) / KB - blk0 : 0;
+  const int blk0 = lo / KB, nmain = end > lo ? (end + KB - 1) / KB - blk0 : 0;
   const int nkept = nmain > 0 ? min((kept + KB - 1) / KB, blk0) : (kept + KB - 1) / KB, nblk = nkept + nmain;
   const int per = (nblk + c.nsplit - 1) / c.nsplit, b0 = split * per, b1 = min(b0 + per, nblk);
   auto block_of = [&](int i) { return i < nkept ? i : blk0 + i - nkept; };
@@ -350,7 +382,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   auto load_k = [&](int blk) {
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
-      const T* p = kc + kv_elem<PAGED>(c.sk, row, kh, max(0, min(blk * KB + 16 * t + c16, pos - 1))) + 8 * g4;
+      const T* p = kc + kv_elem<PAGED>(c.sk, row, kh, max(0, min(blk * KB + 16 * t + c16, end - 1))) + 8 * g4;
 #pragma unroll
       for (int kk = 0; kk < KK; ++kk) kf[t][kk] = *(const u32x4*)(p + 32 * kk);
     }
@@ -359,13 +391,13 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
       const int piece = i * 64 + lane;
-      vr[i] = *(const u32x4*)(vc + kv_elem<PAGED>(c.sv, row, kh, max(0, min(blk * KB + piece / (VD / 8), pos - 1))) + 8 * (piece % (VD / 8)));
+      vr[i] = *(const u32x4*)(vc + kv_elem<PAGED>(c.sv, row, kh, max(0, min(blk * KB + piece / (VD / 8), end - 1))) + 8 * (piece % (VD / 8)));
     }
   };
 
   // queries (and, in the last split, the token's own key and value): 16 lanes per head.  Their loads go first: memory answers in order
   const T* pr = (const T*)c.proj + (size_t)tok * c.ldp;
-  const bool own = split == c.nsplit - 1;
+  const bool own = split == c.nsplit - 1 && !c.shared;
   {
     const int hh = tid >> 4, l = tid & 15;
     constexpr int PL = KD / 16;                      // elements per lane: l PL ..
@@ -386,7 +418,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
     auto head = [&](const float (&v)[PL], const float (&w)[PL], const Rot<PL>& ro, bool there, T* dst) {
       float ss = 0.f, x[PL];
 #pragma unroll
-      for (int i = 0; i < PL; ++i) ss += v[i] * v[i];
+      for (int i = 0; i < PL; ++i) ss += v[i] * v[i] * square_weight(c, l * PL + i);
       const float rs = 1.0f / sqrtf(row16_sum(ss) / (float)c.dim + c.eps);
 #pragma unroll
       for (int i = 0; i < PL; ++i) x[i] = v[i] * rs * w[i];
@@ -446,7 +478,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
       for (int r = 0; r < 4; ++r) {
         const int key = blk * KB + 16 * t + 4 * g4 + r;
         const float s = score2<CAP>(ks, sc[t][r], fmaf(slope2, (float)(16 * t + r), bias0));
-        sc[t][r] = (key >= lo && key < pos) || key < kept ? s : -INFINITY;
+        sc[t][r] = (key >= lo && key < end) || key < kept ? s : -INFINITY;
         mx = fmaxf(mx, sc[t][r]);
       }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
@@ -524,7 +556,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
     const int h = h0 + hh;
     if (c.nsplit == 1) {
       L += sink_of(h, mn);
-      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(gated ? O / L * gate_f(to_f32(gate[h * c.vdim + d])) : O / L);
+      if (d < c.vdim) cat[h * c.vdim + d] = from_f32<T>(gated ? O / L * gate_f(to_f32(gate[gate_at(c, h, d)])) : O / L);
     } else {
       float* pp = pp0 + ((size_t)h * c.nsplit + split) * (VD + 2);
       __hip_atomic_store(&pp[2 + d], O, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -549,7 +581,7 @@ __global__ __launch_bounds__(256, 1) void gqa_decode_kernel(GqaCall c) {
   for (int idx = tid; idx < nh * VD; idx += 256) {
     const int hh = idx / VD, d = idx % VD, h = h0 + hh;
     const float* pp = pp0 + (size_t)h * c.nsplit * (VD + 2);
-    const float gv = gated ? to_f32(gate[h * c.vdim + min(d, c.vdim - 1)]) : 0.f;
+    const float gv = gated ? to_f32(gate[gate_at(c, h, min(d, c.vdim - 1))]) : 0.f;
     float mn = -1e30f, L = 0.f, O = 0.f;
     for (int i0 = 0; i0 < c.nsplit; i0 += 8) {       // eight splits' loads in flight, merged in split order
       float mv[8], lv[8], ov[8];
@@ -799,9 +831,10 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
     l += __shfl_xor(l, 32, 64);
     if (c.sink != nullptr) l += __builtin_amdgcn_exp2f(c.sink[h] * LOG2E - m_run[u]);
     const int tok = tok0 + min(tq[u], len - 1);
-    const float inv = 1.0f / l;
-    const bool gated = c.o_g >= 0;
-    const T* gate = (const T*)c.proj + (size_t)tok * c.ldp + max(c.o_g, 0) + h * c.vdim;
+    const bool gated = c.o_g >= 0 && !c.gate_head;
+    const T* gates = (const T*)c.proj + (size_t)tok * c.ldp + max(c.o_g, 0);
+    const T* gate = gates + (c.gate_head ? 0 : h * c.vdim);
+    const float inv = (c.o_g >= 0 && c.gate_head ? gate_f(to_f32(gates[h])) : 1.0f) / l;
     T* o = (T*)c.cat + (size_t)tok * c.ldc + h * c.vdim;
     if (c.vdim % 4 == 0) {
       uint2 gt[DT];
@@ -831,7 +864,7 @@ __global__ __launch_bounds__(256, 2) void gqa_prefill_kernel(GqaCall c) {
 
 template <typename T>
 int pre_at(const GqaCall& c, hipStream_t st) {
-  const bool vec = c.dim % 8 == 0 && c.vdim % 8 == 0 && c.kdp <= 128 && c.vdp <= 128 && c.rot % 16 == 0;
+  const bool vec = c.dim % 8 == 0 && c.vdim % 8 == 0 && c.kdp <= 128 && c.vdp <= 128 && (c.pairs || c.rot % 16 == 0);
   auto go = [&](auto k) { hipLaunchKernelGGL(k, dim3(c.t.R), dim3(256), 0, st, c); };
   if (c.rot > 0) { if (vec) go(gqa_pre_kernel<T, true, true>); else go(gqa_pre_kernel<T, false, true>); }
   else { if (vec) go(gqa_pre_kernel<T, true, false>); else go(gqa_pre_kernel<T, false, false>); }
@@ -900,6 +933,7 @@ int check_call(const GqaCall& c) {
   if (c.G < 1 || c.H % c.G != 0 || c.sk.D != c.kdp || c.sv.D != c.vdp || c.sk.Hkv != c.G || c.sv.Hkv != c.G || c.kdp < c.dim || c.vdp < c.vdim)
     return fail(MI_ERR_INVALID, "gqa: cache shape does not match the layer");
   if (c.rot < 0 || c.rot % 2 != 0 || c.rot > c.dim || (c.rot > 0 && c.rot_tab == nullptr)) return fail(MI_ERR_INVALID, "gqa: rotation does not fit the head size");
+  if (c.shared && (c.v_mix != nullptr || c.v_first_out != nullptr)) return fail(MI_ERR_INVALID, "gqa: mixed values need a layer's own");
   if (c.window < 0 || c.keep < 0 || (c.window > 0 && c.chunk > 0) || (c.window == 0 && c.keep > 0)) return fail(MI_ERR_INVALID, "gqa: bad mask");
   return MI_OK;
 }

@@ -26,7 +26,7 @@ enum : int {
   EPI_STORE = 0,      // out[m][n] = T(acc)
   EPI_STORE_F32 = 1,  // out_f32[m][n] = float(T(acc))            (logits for the sampler)
   EPI_RESID = 2,      // resid[m][n] = T(resid[m][n] + T(acc))     (h = x + r, llama.py:188,190)
-  EPI_SWIGLU = 3,     // out[m][n] = T(T(silu(g)) * u), g/u = rows n, n+pair_offset (llama.py:165)
+  EPI_SWIGLU = 3,     // out[m][n] = T(T(silu(g)) * u), g/u = rows n, n+pair_offset (llama.py:165); or another unit (GemvCall::glu)
   EPI_SWIGLU_GU8 = 4, // the same on the row-interleaved copy of a gate|up matrix (tile t = gate rows 8t..8t+7, then up rows
                       // 8t..8t+7; launch_gate_up_interleave): a PLAIN one-stream GEMV over 2 x pair_offset rows whose
                       // epilogue pairs columns j and j + 8 of every tile -- gemv_mfma only (decode steps of <= 16 rows)
@@ -51,6 +51,8 @@ struct GemvCall {
   int force_v1 = 0;
   int out32 = 0;                  // 16-bit activations, EPI_STORE / EPI_RESID: out / resid are float32 and the accumulator is stored (added)
                                   // unrounded -- a residual stream kept in 32 bits, logits of the layer-list models
+  Glu glu;                        // EPI_SWIGLU: the unit (common.h); everything but silu is one float32 expression, rounded once
+  int silu_cols = 0;              // EPI_STORE in the activation dtype: columns [0, silu_cols) are stored as silu(acc), rounded once
   int kx = 0;                     // > 0: W is a [hi | lo] matrix of 2 kx columns (an f16 model in the float32-activation mode): the
                                   // activations have kx columns and are walked twice (k mod kx); 0: W.K columns
   // RMSNorm hand-over between two launches of gemm_skinny.hip's 16-row instantiation: a residual epilogue leaves
@@ -96,8 +98,9 @@ struct GroupedGemm {
   void* out; int ldo; const int32_t* out_rows;
   const int32_t* tiles; int max_tiles;
   int tile;                   // 128 or 256 places per tile: the 128 x 128 kernel, or the 256 x 256 LDS-DMA kernel
-  bool swiglu;                // rows = gate rows, then as many up rows: out = silu(gate) * up, in float32 before the store
+  bool swiglu;                // rows = gate rows, then as many up rows: out = glu(gate, up), in float32 before the store
   int act;
+  Glu glu;
 };
 int launch_gemm_grouped(const GroupedGemm& g, hipStream_t st);
 // float32 activations (PagedKVCache mode) in front of launch_gemm_prefill: rows of [hi | mid | lo] bf16, 3 K wide, with the

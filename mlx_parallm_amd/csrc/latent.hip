@@ -1,5 +1,8 @@
-// latent.hip -- latent attention without positions (layer-list models): the cache holds one latent c per token, head h's keys
-// and values are W_uk c and W_uv c, scores (q . k) * scale, ordinary causal softmax, the head's output times sigmoid(gate).
+// latent.hip -- latent attention (layer-list models): the cache holds one latent c per token, head h's keys and values are W_uk c and
+// W_uv c, scores (q . k) * scale, ordinary causal softmax, the head's output times sigmoid(gate) (or no gate).
+// With a rotated part every query head has `rot` more coordinates, turned by the position; the keys' are one vector per token for all
+// heads, turned and cached behind the latent.  A score is then ([W_uk^T q | q_rot] . [c | k_rot]) * scale: the latent space has more
+// coordinates, which only the scores look at.  Where keys are materialised, [W_uk | 1] hands the rotated part through.
 //
 //   generic form     any size and dtype: the query goes into the latent space (W_uk^T q), scores and the weighted sum are taken
 //                    over the latents, W_uv is applied to the sum.  One workgroup per (token, head), float32 arithmetic.
@@ -24,38 +27,70 @@ __device__ __forceinline__ size_t lat_at(const AttnShape& s, int row, int key) {
   return s.btab ? kv_elem<true>(s, row, 0, key) : kv_elem<false>(s, row, 0, key);
 }
 
-// grid R: c = rms(W_dkv h) * w appended to the cache; the feed-forward activation of the row
+// coordinate j of a rotated part at position pos, x: the part as projected
+template <typename T>
+__device__ __forceinline__ float rotated(const LatentCall& c, const T* x, int j, int pos) {
+  const RotAt a = rot_at(j, c.rot, c.pairs);
+  const float2 cs = c.rot_tab[(size_t)pos * (c.rot >> 1) + a.f];
+  return to_f32(x[j]) * cs.x + a.sign * to_f32(x[a.partner]) * cs.y;
+}
+
+// grid (R, parts): c = rms(W_dkv h) * w and the rotated key part appended to the cache; the feed-forward activation of the row; the
+// latent of the queries
+enum : int { PRE_CACHE, PRE_FF, PRE_QUERY };
+__host__ __device__ inline int pre_parts(const LatentCall& c) { return (c.o_c >= 0 ? 1 : 0) + (c.ff.ff > 0 ? 1 : 0) + (c.q_rank > 0 ? 1 : 0); }
+__device__ __forceinline__ int pre_part(const LatentCall& c, int i) {
+  if (c.o_c >= 0 && i-- == 0) return PRE_CACHE;
+  if (c.ff.ff > 0 && i-- == 0) return PRE_FF;
+  return PRE_QUERY;
+}
 template <typename T>
 __global__ __launch_bounds__(256) void latent_pre_kernel(LatentCall c) {
   __shared__ float red[12];
-  const int r = blockIdx.x;
+  const int r = blockIdx.x, part = pre_part(c, blockIdx.y);
   const T* pr = (const T*)c.proj + (size_t)r * c.ldp;
-  if (blockIdx.y == 1 || c.o_c < 0) {
-    if (c.ff.ff > 0) polynorm_row<T, 256>(c.ff, pr + c.ff.in_off, (T*)c.cat + (size_t)r * c.ldc + c.ff.out_off, red);
+  if (part == PRE_FF) {
+    polynorm_row<T, 256>(c.ff, pr + c.ff.in_off, (T*)c.cat + (size_t)r * c.ldc + c.ff.out_off, red);
     return;
   }
+  const bool cache = part == PRE_CACHE;
   const TokenAt at = token_at(c.t, r);
+  const int n = cache ? c.rank : c.q_rank, np = cache ? c.rp : c.ldqc;
+  const T* src = pr + (cache ? c.o_c : c.o_qc);
+  const float* w = cache ? c.c_norm : c.q_norm;
+  T* dst = cache ? (T*)c.cache + lat_at(c.s, at.row, at.pos) : (T*)c.qc + (size_t)r * c.ldqc;
   float ss[1] = {0.f};
-  for (int i = threadIdx.x; i < c.rank; i += 256) { const float v = to_f32(pr[c.o_c + i]); ss[0] += v * v; }
+  for (int i = threadIdx.x; i < n; i += 256) { const float v = to_f32(src[i]); ss[0] += v * v; }
   block_sum<256, 1>(ss, red);
-  const float rs = 1.0f / sqrtf(ss[0] / (float)c.rank + c.eps);
-  T* dst = (T*)c.cache + lat_at(c.s, at.row, at.pos);
-  for (int i = threadIdx.x; i < c.rp; i += 256)
-    dst[i] = i < c.rank ? from_f32<T>(to_f32(pr[c.o_c + i]) * rs * c.c_norm[i]) : from_f32<T>(0.f);
+  const float rs = 1.0f / sqrtf(ss[0] / (float)n + c.eps);
+  for (int i = threadIdx.x; i < np; i += 256) {
+    float v = 0.f;
+    if (i < n) v = to_f32(src[i]) * rs * w[i];
+    else if (cache && i >= c.cp && i < c.cp + c.rot) v = rotated<T>(c, src + n, i - c.cp, at.pos);
+    dst[i] = from_f32<T>(v);
+  }
+}
+
+// gate of token r and head h
+template <typename T>
+__device__ __forceinline__ float head_gate(const LatentCall& c, int r, int h) {
+  return c.o_g >= 0 ? sigmoid_f(to_f32(((const T*)c.proj)[(size_t)r * c.ldp + c.o_g + h])) : 1.f;
 }
 
 // ---- generic form --------------------------------------------------------------------------------------------------
-// grid (R, H): lq[r][h][:] = W_uk^T q
+// grid (R, H): lq[r][h][:] = [W_uk^T q | rotated part]
 template <typename T>
 __global__ __launch_bounds__(256) void latent_absorb_generic_kernel(LatentCall c) {
   const int r = blockIdx.x, h = blockIdx.y;
-  const T* q = (const T*)c.proj + (size_t)r * c.ldp + c.o_q + h * c.dim;
+  const T* q = (const T*)c.q + (size_t)r * c.ldq + h * (c.dim + c.rot);
   const T* uk = (const T*)c.uk + (size_t)h * c.dim * c.rank;
+  const int pos = c.rot > 0 ? token_at(c.t, r).pos : 0;
   float* out = (float*)c.lq + ((size_t)r * c.H + h) * c.rp;
   for (int k = threadIdx.x; k < c.rp; k += 256) {
     float a = 0.f;
     if (k < c.rank)
       for (int j = 0; j < c.dim; ++j) a = fmaf(to_f32(q[j]), to_f32(uk[(size_t)j * c.rank + k]), a);
+    else if (k >= c.cp && k < c.cp + c.rot) a = rotated<T>(c, q + c.dim, k - c.cp, pos);
     out[k] = a;
   }
 }
@@ -113,7 +148,7 @@ __global__ __launch_bounds__(256) void latent_attn_generic_kernel(LatentCall c) 
   for (int k = threadIdx.x; k < c.rp; k += 256)
     sm[k] = (w[0] * sm[k] + w[1] * sm[c.rp + k] + w[2] * sm[2 * c.rp + k] + w[3] * sm[3 * c.rp + k]) / lt;
   __syncthreads();
-  const float gate = sigmoid_f(to_f32(((const T*)c.proj)[(size_t)r * c.ldp + c.o_g + h]));
+  const float gate = head_gate<T>(c, r, h);
   const T* uv = (const T*)c.uv + (size_t)h * c.vdim * c.rank;
   T* cat = (T*)c.cat + (size_t)r * c.ldc + h * c.vdim;
   for (int j = wave; j < c.vdim; j += 4) {
@@ -151,7 +186,7 @@ int generic_at(const LatentCall& c, hipStream_t st) {
 
 template <typename T>
 static int pre_at(const LatentCall& c, hipStream_t st) {
-  const int parts = (c.o_c >= 0 ? 1 : 0) + (c.ff.ff > 0 ? 1 : 0);
+  const int parts = pre_parts(c);
   if (parts == 0) return MI_OK;
   hipLaunchKernelGGL(latent_pre_kernel<T>, dim3(c.t.R, parts), dim3(256), 0, st, c);
   MI_HIP(hipGetLastError());
@@ -202,16 +237,39 @@ __device__ __forceinline__ u32x4 load8_upto(const T* p, int k, int n) {
   return __builtin_bit_cast(u32x4, v);
 }
 
-// one-token segments: lq[m][h] = W_uk^T q as a 16-bit pair hi + lo.  grid (H, rp / 64, ceil(nd / 16)); a wave owns 16 latent columns
+// elements [k, k + 8) of query head qh [dim | rot] with the rotated part turned, zeros beyond
+template <typename T>
+__device__ __forceinline__ u32x4 query8(const LatentCall& c, const T* qh, int k, int pos) {
+  const u32x4 x = load8_upto<T>(qh, k, c.dim + c.rot);
+  if (c.rot == 0 || k + 8 <= c.dim || k >= c.dim + c.rot) return x;
+  T v[8];
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int j = k + i - c.dim;
+    v[i] = ((const T*)&x)[i];
+    if (j >= 0 && j < c.rot) v[i] = from_f32<T>(rotated<T>(c, qh + c.dim, j, pos));
+  }
+  return __builtin_bit_cast(u32x4, v);
+}
+
+// one-token segments: lq[m][h] = [W_uk^T q | rotated part] as a 16-bit pair hi + lo.  grid (H, rp / 64, ceil(nd / 16)); a wave owns 16
+// columns (cp is a multiple of 16)
 template <typename T>
 __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentCall c) {
   const int h = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c16 = lane & 15, g4 = lane >> 4;
   const int r0 = blockIdx.y * 64 + wave * 16, m0 = blockIdx.z * 16;
   const int m = min(m0 + c16, c.t.nd - 1);
-  const T* q = (const T*)c.proj + (size_t)c.t.tok0[c.t.dec[m]] * c.ldp + c.o_q + h * c.dim;
+  const T* q = (const T*)c.q + (size_t)c.t.tok0[c.t.dec[m]] * c.ldq + h * (c.dim + c.rot);
   const T* w = (const T*)c.uk_t + ((size_t)h * c.rp + r0 + c16) * c.kdp;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < c.kdp; k += 32)
+  if (c.rot > 0 && r0 >= c.cp) {
+    const int j = r0 + c16 - c.cp;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int seg = c.t.dec[min(m0 + 4 * g4 + r, c.t.nd - 1)];
+      if (j < c.rot) acc[r] = rotated<T>(c, (const T*)c.q + (size_t)c.t.tok0[seg] * c.ldq + h * (c.dim + c.rot) + c.dim, j, c.t.off[c.t.row[seg]]);
+    }
+  } else for (int k = 0; k < c.dim; k += 32)           // (kdp is a multiple of 32 and at least dim)
     acc = mfma16<T>(load8_upto<T>(q, k + 8 * g4, c.dim), *(const u32x4*)(w + k + 8 * g4), acc);
   T* out = (T*)c.lq;                                 // [m][h][hi | lo][rp]
 #pragma unroll
@@ -347,9 +405,9 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(LatentCall c) {
   }
 }
 
-// merge the splits: c.merged[m][h] = the weighted sum of the latents as a 16-bit pair hi + lo.  grid (H, nd), four latent elements per thread (rp <= 512)
+// merge the splits: c.merged[m][h] = the weighted sum of the latents as a 16-bit pair hi + lo.  grid (H, nd), four latent elements per thread (rp <= 768)
 template <typename T>
-__global__ __launch_bounds__(128) void latent_merge_kernel(LatentCall c) {
+__global__ __launch_bounds__(192) void latent_merge_kernel(LatentCall c) {
   const int h = blockIdx.x, m = blockIdx.y, ns = c.nsplit, lp = c.rp + LAT_PART_PAD, lane = threadIdx.x & 63, k = threadIdx.x * 4;
   const float* p = c.partial + ((size_t)m * ((c.H + 15) / 16 * 16) + h) * ns * lp;
   // lane s holds the weight of split s (at most 32 of them)
@@ -387,7 +445,7 @@ __global__ __launch_bounds__(64) void latent_uv_kernel(LatentCall c) {
   const T* x = (const T*)c.merged + ((size_t)(m0 + min(c16, nm - 1)) * c.H + h) * 2 * c.rp + 8 * g4;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int k = 0; k < 16; ++k)
+  for (int k = 0; k < 18; ++k)
     if (k < nk) {
       const u32x4 b = *(const u32x4*)(w + 32 * k);
       acc = mfma16<T>(*(const u32x4*)(x + 32 * k), b, acc);
@@ -400,7 +458,7 @@ __global__ __launch_bounds__(64) void latent_uv_kernel(LatentCall c) {
     const int m = 4 * g4 + r;
     if (m >= nm) continue;
     const int tok = c.t.tok0[c.t.dec[m0 + m]];
-    const float gate = sigmoid_f(to_f32(((const T*)c.proj)[(size_t)tok * c.ldp + c.o_g + h]));
+    const float gate = head_gate<T>(c, tok, h);
     ((T*)c.cat)[(size_t)tok * c.ldc + h * c.vdim + col] = from_f32<T>(acc[r] * gate);
   }
 }
@@ -465,9 +523,10 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
 #pragma unroll
   for (int u = 0; u < QG; ++u) {
     tq[u] = t0 + (wave * QG + u) * 16 + c16;
-    const T* q = (const T*)c.proj + (size_t)(tok0 + min(tq[u], len - 1)) * c.ldp + c.o_q + h * c.dim;
+    const int tc = min(tq[u], len - 1);
+    const T* q = (const T*)c.q + (size_t)(tok0 + tc) * c.ldq + h * (c.dim + c.rot);
 #pragma unroll
-    for (int kk = 0; kk < KK; ++kk) qf[u][kk] = load8_upto<T>(q, 32 * kk + 8 * g4, c.dim);
+    for (int kk = 0; kk < KK; ++kk) qf[u][kk] = query8<T>(c, q, 32 * kk + 8 * g4, off + tc);
   }
   store_block(0);
 #pragma unroll
@@ -566,7 +625,7 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
     l += __shfl_xor(l, 32, 64);
     if (tq[u] >= len) continue;
     const int tok = tok0 + tq[u];
-    const float f = sigmoid_f(to_f32(((const T*)c.proj)[(size_t)tok * c.ldp + c.o_g + h])) / l;
+    const float f = head_gate<T>(c, tok, h) / l;
     T* o = (T*)c.cat + (size_t)tok * c.ldc + h * c.vdim;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
@@ -611,9 +670,10 @@ int decode_at(const LatentCall& c, hipStream_t st) {
       case 6: MI_TRY((decode_nk<T, 6>(c, st))); break;
       case 7: MI_TRY((decode_nk<T, 7>(c, st))); break;
       case 8: MI_TRY((decode_nk<T, 8>(c, st))); break;
+      case 9: MI_TRY((decode_nk<T, 9>(c, st))); break;
       default: return fail(MI_ERR_UNSUPPORTED, "latent_decode: latent size");
     }
-    hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(c.H, c.t.nd), dim3(128), 0, st, c);
+    hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(c.H, c.t.nd), dim3(c.rp <= 512 ? 128 : 192), 0, st, c);
     MI_HIP(hipGetLastError());
     hipLaunchKernelGGL(latent_uv_kernel<T>, dim3((c.vdim + 15) / 16, c.H, (c.t.nd + 15) / 16), dim3(64), 0, st, c);
     MI_HIP(hipGetLastError());
@@ -630,7 +690,11 @@ int prefill_kv(const LatentCall& c, hipStream_t st) {
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
-  return c.t.qt == 128 ? go(latent_prefill_kernel<T, KD, VD, 2>) : go(latent_prefill_kernel<T, KD, VD, 1>);
+  if constexpr (KD <= 128) {
+    if (c.t.qt == 128) return go(latent_prefill_kernel<T, KD, VD, 2>);
+  }
+  if (c.t.qt != 64) return fail(MI_ERR_INVALID, "latent_prefill: tile size");
+  return go(latent_prefill_kernel<T, KD, VD, 1>);
 }
 
 template <typename T>
@@ -641,6 +705,7 @@ int prefill_at(const LatentCall& c, hipStream_t st) {
       case 32: V(32);
       case 64: V(64);
       case 128: V(128);
+      case 192: V(192);
     }
 #undef V
   }
@@ -659,8 +724,10 @@ int gather_at(const LatentCall& c, void* dst, hipStream_t st) {
 }  // namespace
 
 int latent_pad(int n) { return n <= 32 ? 32 : (n <= 64 ? 64 : (n <= 128 ? 128 : 0)); }
+int latent_tile(int kdp) { return kdp <= 128 ? 128 : 64; }
+int latent_key_pad(int n) { return n > 128 && n <= 192 ? 192 : latent_pad(n); }
 bool latent_mfma_supported(int act, int dim, int vdim, int rp) {
-  return (act == MI_BF16 || act == MI_F16) && latent_pad(dim) > 0 && latent_pad(vdim) > 0 && rp % 64 == 0 && rp <= 512;
+  return (act == MI_BF16 || act == MI_F16) && latent_key_pad(dim) > 0 && latent_pad(vdim) > 0 && rp % 64 == 0 && rp <= 576;
 }
 int launch_latent_decode(const LatentCall& c, hipStream_t st) {
   if (c.nsplit < 1 || c.nsplit > 32 || c.partial == nullptr) return fail(MI_ERR_INVALID, "latent_decode: bad split configuration");

@@ -85,8 +85,8 @@ struct StreamNormCall {
 constexpr int MAX_STREAMS = 16;
 int launch_stream_norm(const StreamNormCall& c, hipStream_t st);
 int launch_stream_sum(const float* x, int streams, int rows, int ld, float* out, hipStream_t st);     // out [rows][ld]
-// tab [positions][dims / 2]: cosine and sine of p base^(-2i / dims) (angles in double precision)
-int launch_rotation_table(float2* tab, int positions, int dims, double base, hipStream_t st);
+// tab [positions][pairs]: gain times cosine and sine of p freq[i] (angles in double precision); freq [pairs] on the device
+int launch_rotation_table(float2* tab, int positions, int pairs, const double* freq, double gain, hipStream_t st);
 
 struct PolyNormArgs { int ff, in_off, out_off; const float* coef; float eps; };     // ff = 0: none
 
@@ -128,13 +128,18 @@ struct LowRankCall { LinearW W; int split, k; const void* x; int ldx, rows; void
 bool low_rank_supported(const LowRankCall& c);
 int launch_low_rank(const LowRankCall& c, hipStream_t st);
 
-// Latent attention (latent.hip): the cache holds one latent per token, [token][rp]; keys and values are maps of it
+// Latent attention (latent.hip): the cache holds one latent per token, [token][rp]; keys and values are maps of it.  With a rotated part
+// (rot > 0) a token's row is [latent | padding to cp | rotated key part, one for all heads | padding], a query head [dim | rot], and a
+// score the sum of both products.
 struct LatentCall {
   SegTables t;
   AttnShape s;                   // cache addressing: Hkv = 1, D = rp, cap / btab as usual
   int H, dim, vdim, rank, rp, kdp, vdp;
+  int rot, cp, pairs; const float2* rot_tab;       // size of the rotated part (0: none), its place in a cached row, MI_ROT_*, [position][rot / 2]
   const void* proj; int ldp;
-  int o_q, o_g, o_c;             // o_c < 0: the latents are another layer's, nothing is appended
+  int o_g, o_c;                  // o_g < 0: no gate; o_c < 0: the latents are another layer's, nothing is appended
+  const void* q; int ldq;        // [R][ldq] queries, head h's dim + rot from element h (dim + rot) on
+  int q_rank, ldqc; const float* q_norm; void* qc; int o_qc;      // q_rank > 0: latent_pre leaves rms(proj from o_qc on) * q_norm in qc [R][ldqc]
   const float* c_norm; float eps;
   void* cache;                   // the arena of the layer the latents belong to
   const void* uk; const void* uv;          // [H * dim][rank], [H * vdim][rank]
@@ -148,19 +153,21 @@ struct LatentCall {
   PolyNormArgs ff;
   int act;
 };
-int launch_latent_pre(const LatentCall& c, hipStream_t st);            // append the latents, feed-forward activation
+int launch_latent_pre(const LatentCall& c, hipStream_t st);            // append the latents, feed-forward activation, the queries' latent
 int launch_latent_generic(const LatentCall& c, hipStream_t st);        // any size and dtype, all tokens
-bool latent_mfma_supported(int act, int dim, int vdim, int rp);
-int latent_pad(int n);                                                 // padded head size of the prefill kernel, 0 = none
+int latent_tile(int kdp);                                              // queries per tile at most
+bool latent_mfma_supported(int act, int dim, int vdim, int rp);        // dim: with the rotated part
+int latent_pad(int n);                                                 // padded value head size of the prefill kernel, 0 = none
+int latent_key_pad(int n);                                             // of a key head (with its rotated part)
 int launch_latent_decode(const LatentCall& c, hipStream_t st);         // one-token segments
 int launch_latent_gather(const LatentCall& c, void* dst, hipStream_t st);   // cached + new latents of the chunks, contiguous
 int launch_latent_prefill(const LatentCall& c, hipStream_t st);        // segments of two tokens and more
 constexpr int LATENT_GT = 64;    // keys per gather tile
 
-// Grouped-query attention (gqa.hip): q and k divided by their root mean square and rotated, scores
+// Grouped-query attention (gqa.hip): q and k divided by their root mean square and rotated (or in the other order), scores
 //   softcap tanh(q.k scale / softcap) - slope_h (i - j),  j <= i in i's own chunk of positions, or in i's window, or kept,
-// exp(sink_h) in the denominator, values mixed with an earlier layer's of the same token, the output times sigmoid(gate) element by
-// element.  Every mechanism can be off.
+// exp(sink_h) in the denominator, values mixed with an earlier layer's of the same token, the output times sigmoid(gate), element by
+// element or one number per head.  Every mechanism can be off.
 // K and V arenas of the layer: [place][G][..][kdp] / [vdp] as AttnShape sk / sv address them.
 struct GqaCall {
   SegTables t;
@@ -168,8 +175,11 @@ struct GqaCall {
   int H, G, dim, vdim, kdp, vdp;
   const void* proj; int ldp;     // [R][ldp] outputs of the fused input projection
   int o_q, o_k, o_v, o_g;        // o_g < 0: no gate
+  int gate_head;                 // 1: one gate per head
+  int shared;                    // 1: keys and values are another layer's, whose cache holds this call's tokens already
   const float* q_norm; const float* k_norm; float eps;
-  int rot; const float2* rot_tab;          // rotated coordinates (0: none), [position][rot / 2] cosine and sine
+  int rot, pairs; const float2* rot_tab;   // rotated coordinates (0: none), MI_ROT_*, [position][rot / 2] cosine and sine
+  float rot_gain2;               // weight of a rotated coordinate in the mean square: 1, or (norm behind the rotation) the table's gain squared
   float scale, softcap;          // softcap 0: none
   const float* slopes;           // [H]
   const float* sink;             // [H], or null
@@ -196,9 +206,10 @@ inline int gqa_head_tiles(int H, int G) { return (H / G + 15) / 16; }
 
 // Norm of a sublayer's output + residual update + operand of what follows (layer_rows.hip):
 //   x += norm(y) ;  h = next.w ? norm'(x) : x            kind: MI_NORM_*
-// y comes from `y` or is the weighted sum of the experts' outputs; `router` non-null: the routing of the row as well.
+// y comes from `y` or is the weighted sum of the experts' outputs; `router` non-null: the routing of the row as well (by x, or by h as
+// stored where next.w is set).
 struct PostNormW { const float* w; const float* b; int stride; };     // b: layer norm only
-struct RouteArgs { int experts, top, groups, keep; };
+struct RouteArgs { int experts, top, groups, keep; const float* bias; };      // bias [experts] or null
 struct PostNormCall {
   int rows;
   const float* y;                // [rows][ld], or null: parts
@@ -223,7 +234,7 @@ constexpr int MOE_STREAM_ROWS = 64;      // calls of up to so many tokens stream
 struct MoeCall {
   int R, width, ld;              // ld: padded width
   RouteArgs r;
-  const float* x;                // [R][ld] residual stream (router)
+  const float* x;                // [R][ld] residual stream (router), or null: the router reads h
   const void* h;                 // [R][ld] the same in the activation dtype
   const void* router;            // [experts][ld]
   int32_t* ids; float* wts;      // [R][top]
@@ -236,6 +247,7 @@ struct MoeCall {
   int32_t* counts;               // [experts] slots per expert, [R][top] a slot's place among its expert's: left by launch_route, whose
                                  // caller clears the counts first (launch_post_norm: `clear`)
   int act;
+  Glu glu;                       // the experts' unit
 };
 size_t moe_plan_ints(int R, const RouteArgs& r, int shared);
 inline size_t moe_count_ints(int R, const RouteArgs& r) { return (size_t)r.experts + (size_t)R * r.top; }
@@ -243,8 +255,30 @@ bool moe_mfma_supported(const MoeCall& c);
 int launch_route(const MoeCall& c, hipStream_t st);         // many rows of 16-bit models (few: launch_post_norm)
 bool route_fused(int act, int rows, int experts);           // launch_post_norm does the routing
 int launch_moe_plan(const MoeCall& c, hipStream_t st);      // many rows: order of the slots (nothing otherwise)
-int launch_moe_up(const MoeCall& c, hipStream_t st);        // mid[slot] = silu(W_gate h) * W_up h
+int launch_moe_up(const MoeCall& c, hipStream_t st);        // mid[slot] = glu(W_gate h, W_up h)
 int launch_moe_down(const MoeCall& c, hipStream_t st);      // out[slot] = W_down mid[slot]
+
+// Linear attention with a fixed decay per head (lightning.hip): S <- decay S + k v^T, o = S^T q, out = rms(o of all heads) * norm *
+// sigmoid(gate).  q, k and v have been through silu.  The state is kept transposed: [value column][key channel].
+constexpr int LIGHT_QT = 64;     // queries per tile; a chunk is a multiple of it
+struct LightCall {
+  SegTables t;
+  int H, d, e;
+  const void* proj; int ldp, o_q, o_k, o_v, o_g;
+  const float* decay;            // [H]
+  const float* log2_decay;       // [H], -1e4 for a decay of zero
+  const float* norm; float eps;  // [H e]
+  float* state; int sd;          // [cache row][H][e][sd], sd = d rounded up to 4
+  float* o; int ldo;             // [R][ldo] outputs of the heads
+  int* tickets;                  // [nd] zero between launches
+  float* ws;                     // [chunks][H][padded e][padded d]: what a chunk adds to the state, then the state in front of it; null: token by token
+  const int32_t* ctile; const int32_t* cbase; int nct, chunk;      // chunks of the longer segments: segment, first token; [n] a segment's first; their length
+  void* cat; int ldc;
+  int act;
+};
+bool light_supported(int d, int e);
+size_t light_ws_floats(int act, int H, int d, int e);       // per chunk, 0 = token by token only
+int launch_lightning(const LightCall& c, hipStream_t st);
 
 // dst[b * db + i * di + j * dj] = src[b * sb + i * si + j * sj] for an [nb][ni][nj] box of es-byte elements
 struct PlaceCall { const void* src; void* dst; int nb, ni, nj, es; size_t sb, si, sj, db, di, dj; };

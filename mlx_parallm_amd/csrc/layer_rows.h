@@ -46,6 +46,15 @@ __device__ __forceinline__ TokenAt token_at(const SegTables& s, int r) {
   return a;
 }
 
+// Rotated coordinate j of `dims`: its partner, the pair's number, and the sign of  partner * sine  (j's own value times the cosine is
+// added).  Partners are dims / 2 apart, or neighbours (pairs).
+struct RotAt { int partner, f; float sign; };
+__device__ __forceinline__ RotAt rot_at(int j, int dims, int pairs) {
+  if (pairs) return RotAt{j ^ 1, j >> 1, (j & 1) ? 1.f : -1.f};
+  const int half = dims >> 1;
+  return j < half ? RotAt{j + half, j, -1.f} : RotAt{j - half, j - half, 1.f};
+}
+
 // eight / four consecutive elements as float32 (16- / 8-byte aligned)
 template <typename T>
 __device__ __forceinline__ void load8f(const T* p, float (&o)[8]) {

@@ -387,7 +387,7 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
   if (c.clear != nullptr && r == 0)
     for (int i = tid; i < c.n_clear; i += NT) c.clear[i] = 0;
   // the first router rows of this wave (columns below 512 PRE) are on their way while the norm runs
-  constexpr int JB = 2, PRE = ROUTE && sizeof(T) == 2 ? 4 : 0;
+  constexpr int JB = 2, PRE = ROUTE && sizeof(T) == 2 && NQ < 4 ? 4 : 0;
   const int lane = tid & 63, wave = tid >> 6;
   u32x4 wpre[JB][PRE > 0 ? PRE : 1];
   if constexpr (PRE > 0) {
@@ -454,7 +454,6 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
     const int i = q * NT + tid;
     if (i >= n4) continue;
     ((f32x4*)xg)[i] = x[q];
-    if constexpr (ROUTE) ((f32x4*)smem)[i] = x[q];
   }
   if (c.next.w != nullptr) normed(x, c.next);
   T* h = (T*)c.h + (size_t)r * c.ld;
@@ -465,6 +464,7 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
     T o[4] = {from_f32<T>(x[q][0]), from_f32<T>(x[q][1]), from_f32<T>(x[q][2]), from_f32<T>(x[q][3])};
     if constexpr (sizeof(T) == 2) *(uint2*)(h + 4 * i) = __builtin_bit_cast(uint2, o);
     else *(f32x4*)(h + 4 * i) = x[q];
+    if constexpr (ROUTE) ((f32x4*)smem)[i] = c.next.w != nullptr ? f32x4{to_f32(o[0]), to_f32(o[1]), to_f32(o[2]), to_f32(o[3])} : x[q];
   }
   if constexpr (ROUTE) {
     float* z = smem + c.ld;
@@ -508,7 +508,7 @@ __global__ __launch_bounds__(NT) void post_norm_kernel(PostNormCall c) {
 #pragma unroll
       for (int j = 0; j < JB; ++j) {
         const float v = wave_sum(acc[j]);
-        if (lane == 0 && e0 + j < c.r.experts) z[e0 + j] = v;
+        if (lane == 0 && e0 + j < c.r.experts) z[e0 + j] = c.r.bias != nullptr ? v + c.r.bias[e0 + j] : v;
       }
     }
     __syncthreads();
@@ -642,10 +642,10 @@ __global__ __launch_bounds__(256) void stream_sum_kernel(const float* x, int str
   }
 }
 
-__global__ __launch_bounds__(256) void rotation_table_kernel(float2* tab, int positions, int half, double step) {
+__global__ __launch_bounds__(256) void rotation_table_kernel(float2* tab, int positions, int half, const double* freq, double gain) {
   for (size_t i = (size_t)blockIdx.x * 256 + threadIdx.x; i < (size_t)positions * half; i += (size_t)gridDim.x * 256) {
-    const double a = (double)(i / half) * pow(2.0, step * (double)(i % half));
-    tab[i] = float2{(float)cos(a), (float)sin(a)};
+    const double a = (double)(i / half) * freq[i % half];
+    tab[i] = float2{(float)(gain * cos(a)), (float)(gain * sin(a))};
   }
 }
 
@@ -728,10 +728,9 @@ int launch_stream_sum(const float* x, int streams, int rows, int ld, float* out,
   return MI_OK;
 }
 
-int launch_rotation_table(float2* tab, int positions, int dims, double base, hipStream_t st) {
-  const size_t n = (size_t)positions * (dims / 2);
-  hipLaunchKernelGGL(rotation_table_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 8192)), dim3(256), 0, st, tab, positions, dims / 2,
-                     -2.0 / dims * std::log2(base));
+int launch_rotation_table(float2* tab, int positions, int pairs, const double* freq, double gain, hipStream_t st) {
+  const size_t n = (size_t)positions * pairs;
+  hipLaunchKernelGGL(rotation_table_kernel, dim3((unsigned)std::min<size_t>((n + 255) / 256, 8192)), dim3(256), 0, st, tab, positions, pairs, freq, gain);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

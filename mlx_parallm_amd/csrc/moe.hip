@@ -1,8 +1,8 @@
 // moe.hip -- mixture of experts (layer-list models): a softmax router picks `top` experts per token among the `keep` best of
-// `groups` equal groups; an expert is W_down (silu(W_gate h) * W_up h); the shared expert takes all tokens.  The weighted sum
+// `groups` equal groups; an expert is W_down glu(W_gate h, W_up h) (common.h: Glu); the shared expert takes all tokens.  The weighted sum
 // over a token's slots is taken by the row kernel behind (layer_rows.hip: post_norm_kernel).
 //
-//   route       many rows: router logits on the matrix cores (x as hi + lo, so they keep 32-bit accuracy), softmax, groups, choice
+//   route       many rows: router logits on the matrix cores (x as hi + lo, so they keep 32-bit accuracy, or h), softmax, groups, choice
 //               (few rows and float32: inside post_norm_kernel)
 //   plan        many rows: slots sorted by expert, table of tiles, for the grouped tile GEMM (gemm_prefill.hip)
 //   stream      up to MOE_STREAM_ROWS tokens: one workgroup per (expert, strip of weight rows) collects the expert's slots and
@@ -33,23 +33,26 @@ __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
 }
 
 // ---- router of many rows: 16 rows per workgroup, RTW waves split K ---------------------------------------------------------
-template <typename T, int NE, int RTW>                 // NE: 16-expert tiles
+template <typename T, int NE, int RTW, bool H16>       // NE: 16-expert tiles; H16: the rows are h
 __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
   extern __shared__ __attribute__((aligned(16))) float sm[];      // partial tiles [RTW][NE][64][4]; then logits [16][16 NE], per wave weights | marks, choices
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
   const int r0 = blockIdx.x * 16, nr = min(16, c.R - r0), E = c.r.experts;
-  const float* x = c.x + (size_t)(r0 + min(c16, nr - 1)) * c.ld + 8 * g4;
+  const size_t row = (size_t)(r0 + min(c16, nr - 1)) * c.ld + 8 * g4;
+  const float* x = H16 ? nullptr : c.x + row;
+  const T* xh = (const T*)c.h + row;
   f32x4 acc[NE];
 #pragma unroll
   for (int t = 0; t < NE; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
   constexpr int KU = NE <= 2 ? 4 : (NE <= 4 ? 2 : 1);               // k steps whose loads are in flight together
   for (int k0 = wave * 32; k0 < c.ld; k0 += KU * RTW * 32) {
-    float v[KU][8];
-    u32x4 b[KU][NE];
+    float v[H16 ? 1 : KU][8];
+    u32x4 vh[H16 ? KU : 1], b[KU][NE];
 #pragma unroll
     for (int u = 0; u < KU; ++u) {
       const int k = min(k0 + u * RTW * 32, c.ld - 32);               // (steps beyond the row: loaded, not used)
-      load8f<float>(x + k, v[u]);
+      if constexpr (H16) vh[u] = *(const u32x4*)(xh + k);
+      else load8f<float>(x + k, v[u]);
 #pragma unroll
       for (int t = 0; t < NE; ++t) b[u][t] = *(const u32x4*)((const T*)c.router + (size_t)min(t * 16 + c16, E - 1) * c.ld + k + 8 * g4);
     }
@@ -57,14 +60,19 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
 #pragma unroll
     for (int u = 0; u < KU; ++u)
       if (k0 + u * RTW * 32 < c.ld) {
-        T hi[8], lo[8];
+        if constexpr (H16) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) { hi[i] = (T)v[u][i]; lo[i] = (T)(v[u][i] - (float)hi[i]); }
-        const u32x4 ah = __builtin_bit_cast(u32x4, hi), al = __builtin_bit_cast(u32x4, lo);
+          for (int t = 0; t < NE; ++t) acc[t] = mfma16<T>(vh[u], b[u][t], acc[t]);
+        } else {
+          T hi[8], lo[8];
 #pragma unroll
-        for (int t = 0; t < NE; ++t) {
-          acc[t] = mfma16<T>(ah, b[u][t], acc[t]);
-          acc[t] = mfma16<T>(al, b[u][t], acc[t]);
+          for (int i = 0; i < 8; ++i) { hi[i] = (T)v[u][i]; lo[i] = (T)(v[u][i] - (float)hi[i]); }
+          const u32x4 ah = __builtin_bit_cast(u32x4, hi), al = __builtin_bit_cast(u32x4, lo);
+#pragma unroll
+          for (int t = 0; t < NE; ++t) {
+            acc[t] = mfma16<T>(ah, b[u][t], acc[t]);
+            acc[t] = mfma16<T>(al, b[u][t], acc[t]);
+          }
         }
       }
   }
@@ -80,7 +88,7 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
     float s = 0.f;
 #pragma unroll
     for (int w = 0; w < RTW; ++w) s += sm[((w * NE + (e >> 4)) * 64 + (m >> 2) * 16 + (e & 15)) * 4 + (m & 3)];
-    z[i] = s;
+    z[i] = c.r.bias != nullptr ? s + c.r.bias[min(e, E - 1)] : s;
   }
   __syncthreads();
 #pragma unroll
@@ -105,8 +113,8 @@ __global__ __launch_bounds__(RTW * 64) void route_kernel(MoeCall c) {
   for (int i = 0; i < NI; ++i) { const int idx = i * RTW * 64 + tid; if (idx < nr * top) c.counts[E + (size_t)r0 * top + idx] = cnt[sel[idx]] + at[i]; }
 }
 
-template <typename T>
-int route_at(const MoeCall& c, hipStream_t st) {
+template <typename T, bool H16>
+int route_rows(const MoeCall& c, hipStream_t st) {
   const int ne = (c.r.experts + 15) / 16;
   auto go = [&](auto k, int NE, int RTW) -> int {
     const size_t part = (size_t)RTW * NE * 1024,
@@ -117,12 +125,14 @@ int route_at(const MoeCall& c, hipStream_t st) {
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
-  if (ne <= 1) return go(route_kernel<T, 1, 16>, 1, 16);
-  if (ne <= 2) return go(route_kernel<T, 2, 16>, 2, 16);
-  if (ne <= 4) return go(route_kernel<T, 4, 16>, 4, 16);
-  if (ne <= 8) return go(route_kernel<T, 8, 16>, 8, 16);
-  return go(route_kernel<T, 16, 8>, 16, 8);                  // (route_fused: at most ROUTE_MFMA_EXPERTS)
+  if (ne <= 1) return go(route_kernel<T, 1, 16, H16>, 1, 16);
+  if (ne <= 2) return go(route_kernel<T, 2, 16, H16>, 2, 16);
+  if (ne <= 4) return go(route_kernel<T, 4, 16, H16>, 4, 16);
+  if (ne <= 8) return go(route_kernel<T, 8, 16, H16>, 8, 16);
+  return go(route_kernel<T, 16, 8, H16>, 16, 8);             // (route_fused: at most ROUTE_MFMA_EXPERTS)
 }
+template <typename T>
+int route_at(const MoeCall& c, hipStream_t st) { return c.x != nullptr ? route_rows<T, false>(c, st) : route_rows<T, true>(c, st); }
 constexpr int ROUTE_MFMA_EXPERTS = 256;
 
 // ---- plan: the slots sorted by expert, and the tile table ------------------------------------------------------------------
@@ -261,7 +271,7 @@ __device__ __forceinline__ f32x4 strip_sum(const float* red, int t, int m) {
   return s;
 }
 
-// grid (strips, experts + shared): mid[slot] = silu(W_gate h) * W_up h.  A strip: one gate tile and its up tile
+// grid (strips, experts + shared): mid[slot] = glu(W_gate h, W_up h).  A strip: one gate tile and its up tile
 template <typename T, int MT>
 __global__ __launch_bounds__(256) void moe_stream_up_kernel(MoeCall c) {
   __shared__ int list[MOE_STREAM_ROWS];
@@ -289,7 +299,7 @@ __global__ __launch_bounds__(256) void moe_stream_up_kernel(MoeCall c) {
       if (i < n) {
         T o[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) o[r] = from_f32<T>(silu_f(g[r]) * u[r]);
+        for (int r = 0; r < 4; ++r) o[r] = from_f32<T>(glu_f(c.glu, g[r], u[r]));
         *(uint2*)((T*)c.mid + (size_t)list[i] * c.lda + strip * 16 + 4 * g4) = __builtin_bit_cast(uint2, o);
       }
     }
@@ -366,7 +376,7 @@ __global__ __launch_bounds__(256) void moe_generic_kernel(MoeCall c) {
   for (int i = wave; i < 64 && r0 + i < rows; i += 4) {
     const int row = r0 + i;
     float v = dot(row);
-    if constexpr (UP) v = silu_f(v) * dot(ffp + row);
+    if constexpr (UP) v = glu_f(c.glu, v, dot(ffp + row));
     if (lane == 0) {
       if constexpr (UP) ((T*)c.mid)[(size_t)slot * c.lda + row] = from_f32<T>(v);
       else ((T*)c.out)[(size_t)slot * c.ld + row] = from_f32<T>(v);
@@ -431,7 +441,7 @@ int experts_at(const MoeCall& c, hipStream_t st) {
   const int32_t* slot = c.plan + 8 + 4 * max_tiles;
   const int32_t* token = slot + n + (shared ? c.R : 0);
   GroupedGemm g{};
-  g.tiles = c.plan; g.max_tiles = max_tiles; g.tile = tile; g.groups = c.r.experts; g.act = c.act; g.swiglu = UP;
+  g.tiles = c.plan; g.max_tiles = max_tiles; g.tile = tile; g.groups = c.r.experts; g.act = c.act; g.swiglu = UP; g.glu = c.glu;
   if (UP) {
     g.x = c.h; g.ldx = c.ld; g.x_rows = token; g.out = c.mid; g.ldo = c.lda;
     g.W = c.gu; g.rows = 2 * c.ffp; g.last = shared ? c.sgu : LinearW{};

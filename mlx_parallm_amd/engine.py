@@ -15,7 +15,7 @@ import numpy as np
 
 from . import _lib as L
 
-LAYER_LIST_MODELS = ("runevik", "dolurax", "temetar")     # described layer by layer (models/<name>.py: layer_list)
+LAYER_LIST_MODELS = ("runevik", "dolurax", "temetar", "beronex")     # described layer by layer (models/<name>.py: layer_list)
 _DT_NAMES = {"float32": L.MI_F32, "bfloat16": L.MI_BF16, "float16": L.MI_F16}
 
 
@@ -271,7 +271,7 @@ class Engine:
         for one, f in zip(arr, layers):
             one.struct_size = C.sizeof(L.LayerDesc)
             for k, v in f.items():
-                setattr(one, k, v)
+                setattr(one, k, (C.c_double * len(v))(*v) if isinstance(v, (list, tuple)) else v)
         self.desc, self.layer_descs = d, arr
         self.config = dict(config)
         self.model_type = model_type
@@ -292,9 +292,11 @@ class Engine:
                 return next((p for p in (32, 64, 128) if n <= p), (n + 31) // 32 * 32)
 
             def elements(x):                     # one latent per token (padded to 64), or the keys and values of every head
-                if x.mixer == L.MI_MIXER_LATENT:
-                    return (x.kv_rank + 63) // 64 * 64 if x.kv_from < 0 else 0
-                return x.kv_heads * (head(x.dim) + head(x.vdim)) if x.mixer == L.MI_MIXER_GQA else 0
+                if x.mixer not in (L.MI_MIXER_LATENT, L.MI_MIXER_GQA) or x.kv_from >= 0:
+                    return 0
+                if x.mixer == L.MI_MIXER_LATENT:     # (and the rotated key part beside it)
+                    return ((x.kv_rank + 15) // 16 * 16 + x.rot_dims + 63) // 64 * 64
+                return x.kv_heads * (head(x.dim) + head(x.vdim))
             return max(1, sum(elements(self.layer_descs[i]) for i in self.layer_runs()) * block_tokens * esz)
         return 2 * d.num_layers * d.num_kv_heads * block_tokens * d.head_dim * esz
 

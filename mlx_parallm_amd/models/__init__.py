@@ -1,1 +1,1 @@
-"""Model families on the hot path: llama (incl. mistral), qwen3, runevik, dolurax and temetar (``utils._get_classes``)."""
+"""Model families on the hot path: llama (incl. mistral), qwen3, runevik, dolurax, temetar and beronex (``utils._get_classes``)."""

@@ -58,7 +58,7 @@ def layer_list(config: dict):
             d.update(mixer=L.MI_MIXER_DELTA, kv_heads=int(m["kv_heads"]), conv=int(m["conv"]), scale=float(m["dim"]) ** -0.5,
                      unit_eps=UNIT_EPS, out_gate=L.MI_GATE_SILU)
         else:
-            d.update(mixer=L.MI_MIXER_LATENT, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]))
+            d.update(mixer=L.MI_MIXER_LATENT, kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), out_gate=L.MI_GATE_SIGMOID_HEAD)
             if m.get("kv_from") is not None:
                 d["kv_from"] = int(m["kv_from"])
         layers.append(d)
