@@ -301,7 +301,7 @@ def parse_args(argv=None):
                          "96, the row limit of its weight-streaming kernel)")
     ap.add_argument("--no-other-configs", action="store_true",
                     help="N = 1, default workload only: skip the short legs of BASELINE configs 3 / 4 / 5 (`other_configs` of the line)")
-    ap.add_argument("--design", default=None, choices=["runevik", "dolurax", "temetar"],
+    ap.add_argument("--design", default=None, choices=["runevik", "dolurax", "temetar", "beronex"],
                     help="instead of the headline workload: prefill and decode of this layer-list design beside a llama stack of "
                          "equal size (random weights), one JSON line with every leg and its kernel times")
     ap.add_argument("--design-sizes", default="1024x8,2048x8,4096x4", help="--design: comma-separated WIDTHxLAYERS")
@@ -439,7 +439,8 @@ def mixed_leg(engine, cfg, args, sample, dist, world):
 
 # ---- --design NAME: a layer-list design beside a llama stack of equal width, depth, vocabulary and parameter count (dolurax: of
 # ---- as many parameters per token: four experts of width / 2 and a shared one of width against one layer of 3 x width; temetar: every
-# ---- second layer recurrent, four residual streams, every layer runs once) ----
+# ---- second layer recurrent, four residual streams, every layer runs once; beronex: latent, windowed and lightning attention in turn, the
+# ---- second windowed layer of four on the first one's keys and values, experts of width / 2 behind the windowed ones) ----
 def design_configs(design, width, layers):
     heads, vocab = width // 128, 32000
     if design == "dolurax":
@@ -459,6 +460,20 @@ def design_configs(design, width, layers):
         run = {"model_type": "temetar", "architecture": "Temetar", "width": width, "vocab": vocab, "layers": [att, rec] * (layers // 2),
                "norm": {"eps": 1e-5}, "streams": 4, "residual_mult": 1.0, "loop": None,
                "embedding": {"scale": 1.0, "bigram": {"buckets": 8191, "mul_prev": 401, "mul_cur": 31}}}
+        return run, llama_like(width, layers, heads, vocab)
+    if design == "beronex":
+        yarn = {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+        dense = {"kind": "dense", "ff": 3 * width}
+        moe = {"kind": "moe", "expert": {"ff": width // 2, "limit": 7.0}, "router": {"experts": 32, "top": 4}}
+        lat = {"type": "latent_attention", "mlp": dense,
+               "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": min(1536, width // 2), "kv_rank": min(512, width // 4),
+                         "scale": 192 ** -0.5, "rot": {"base": 10000.0, "dims": 64, "scaling": yarn}}}
+        att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024},
+               "rot": {"base": 10000.0, "dims": 128, "scaling": yarn}}
+        rec = {"type": "lightning", "mlp": dense, "mixer": {"heads": heads, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** -(3 + 6 * h / heads) for h in range(heads)]}}
+        run = {"model_type": "beronex", "architecture": "Beronex", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0},
+               "layers": [x for i in range(0, layers, 4) for x in (lat, {"type": "attention", "mixer": att, "mlp": moe}, rec,
+                                                                   {"type": "attention", "mixer": {**att, "kv_from": i + 1}, "mlp": moe})]}
         return run, llama_like(width, layers, heads, vocab)
     one = []
     for i in range(layers):
@@ -540,6 +555,41 @@ def temetar_specs(cfg):
     yield "head", (V, W)
 
 
+def beronex_specs(cfg):
+    W, V = cfg["width"], cfg["vocab"]
+    yield "embed", (V, W)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, mlp = f"l{i}.", layer["mixer"], layer["mlp"]
+        H, vv = m["heads"], m["heads"] * m["vdim"]
+        for t in ("norm1", "norm1b", "norm2", "norm2b"):
+            yield p + t, (W,)
+        if layer["type"] == "latent_attention":
+            for t, n, k in (("dq", m["q_rank"], W), ("uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"]), ("dkv", m["kv_rank"] + m["rot_dim"], W),
+                            ("uk", H * m["dim"], m["kv_rank"]), ("uv", vv, m["kv_rank"])):
+                yield p + "mix." + t, (n, k)
+            yield p + "mix.dq.norm", (m["q_rank"],)
+            yield p + "mix.dkv.norm", (m["kv_rank"],)
+        elif layer["type"] == "attention":
+            own = () if m.get("kv_from") is not None else (("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"]))
+            for t, n in (("q", H * m["dim"]), *own, ("g", H)):
+                yield p + "mix." + t, (n, W)
+        else:
+            for t, n in (("q", H * m["dim"]), ("k", H * m["dim"]), ("v", vv), ("g", vv)):
+                yield p + "mix." + t, (n, W)
+            yield p + "mix.norm", (vv,)
+        yield p + "mix.o", (W, vv)
+        units = [("", mlp["ff"])] if mlp["kind"] == "dense" else [(f"e{e}.", mlp["expert"]["ff"]) for e in range(mlp["router"]["experts"])]
+        if mlp["kind"] == "moe":
+            yield p + "mlp.router", (mlp["router"]["experts"], W)
+            yield p + "mlp.router.b", (mlp["router"]["experts"],)
+        for e, ff in units:
+            yield p + f"mlp.{e}gate", (ff, W)
+            yield p + f"mlp.{e}up", (ff, W)
+            yield p + f"mlp.{e}down", (W, ff)
+    yield "final.norm", (W,)
+    yield "head", (V, W)
+
+
 def runevik_specs(cfg):
     W, V, side = cfg["width"], cfg["vocab"], cfg["token_side"]["dim"]
     yield "embed", (V, W)
@@ -589,12 +639,12 @@ def design_engine(cfg, seed, max_positions):
         params = sum(int(__import__("math").prod(sh)) for _n, sh, _k in tensor_specs(cfg))
         return eng, params
     gen = torch.Generator(device="cuda")
-    for i, (name, shape) in enumerate({"runevik": runevik_specs, "dolurax": dolurax_specs, "temetar": temetar_specs}[cfg["model_type"]](cfg)):
+    for i, (name, shape) in enumerate({"runevik": runevik_specs, "dolurax": dolurax_specs, "temetar": temetar_specs, "beronex": beronex_specs}[cfg["model_type"]](cfg)):
         gen.manual_seed(seed * 1000003 + i)
         if len(shape) == 2:
             t = torch.randn(shape, generator=gen, device="cuda") * (0.02 if "conv" not in name else 0.5)
         else:
-            zero = name.endswith(".b") and "norm" in name or cfg["model_type"] == "temetar" and name.endswith(("norm1", "norm2", "final.norm"))
+            zero = name.endswith(".b") and ("norm" in name or "router" in name) or cfg["model_type"] == "temetar" and name.endswith(("norm1", "norm2", "final.norm"))
             t = torch.full(shape, 0.5 if name.endswith(("act", "vmix")) else (0.0 if zero else 1.0), device="cuda")
         if ".hc" in name:            # every stream is read and written alike and kept
             t = {"in": torch.full(shape, 1.0 / shape[0]), "out": torch.ones(shape), "mix": torch.eye(shape[0])}[name.rsplit(".", 1)[1]]
@@ -616,6 +666,8 @@ def design_leg(args):
     fams = {"runevik": ["gemv_in", "gemv_out", "delta", "latent_pre", "latent_decode", "latent_gather", "latent_kv", "latent_prefill", "side", "embed", "gemv_head", "sample"],
             "dolurax": ["gemv_in", "gqa_pre", "gqa_decode", "gqa_prefill", "gemv_out", "post_norm", "moe_route", "moe_plan", "moe_up", "moe_down", "post_norm2", "embed", "gemv_head", "logit_cap", "sample"],
             "temetar": ["gemv_in", "gemv_low", "delta", "gqa_pre", "gqa_decode", "gqa_prefill", "gemv_out", "stream_norm", "gemv_gate_up", "gemv_down", "embed", "gemv_head", "sample"],
+            "beronex": ["gemv_in", "latent_pre", "latent_uq", "latent_decode", "latent_gather", "latent_kv", "latent_prefill", "gqa_pre", "gqa_decode", "gqa_prefill", "lightning",
+                        "gemv_out", "post_norm", "moe_route", "moe_plan", "moe_up", "moe_down", "post_norm2", "gemv_gate_up", "gemv_down", "embed", "gemv_head", "sample"],
             "llama": ["gemv_qkv", "attn", "gemv_o", "gemv_gate_up", "gemv_down", "rope_append", "embed", "gemv_head", "sample"]}
     for width, layers in [tuple(map(int, x.split("x"))) for x in args.design_sizes.split(",")]:
         for name, cfg in zip((args.design, "llama"), design_configs(args.design, width, layers)):
