@@ -302,7 +302,7 @@ int init_layers(mi_engine* e, const mi_layer_desc* layers) {
       }
       if (mfma16 && m.scale > 0.f && latent_mfma_supported(d.act_dtype, qd, m.vdim, l.rp)) {
         l.kdp = latent_key_pad(qd); l.vdp = latent_pad(m.vdim);
-        e->latent_qt = std::min(e->latent_qt, latent_tile(l.kdp));
+        e->latent_qt = std::min(e->latent_qt, latent_tile(l.kdp, l.vdp));
         l.ukv.K = l.rp; l.ukv.N = m.heads * (l.kdp + l.vdp);
       }
     } else if (m.mixer == MI_MIXER_GQA) {

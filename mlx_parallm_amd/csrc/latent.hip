@@ -35,39 +35,78 @@ __device__ __forceinline__ float rotated(const LatentCall& c, const T* x, int j,
   return to_f32(x[j]) * cs.x + a.sign * to_f32(x[a.partner]) * cs.y;
 }
 
-// grid (R, parts): c = rms(W_dkv h) * w and the rotated key part appended to the cache; the feed-forward activation of the row; the
-// latent of the queries
+// grid (rows / RPW, parts): c = rms(W_dkv h) * w and the rotated key part appended to the cache; the feed-forward activation of the row;
+// the latent of the queries.  A wave takes a row of a norm; the feed-forward needs the whole workgroup (RPW = 1: the norms' other
+// waves are idle).
 enum : int { PRE_CACHE, PRE_FF, PRE_QUERY };
-__host__ __device__ inline int pre_parts(const LatentCall& c) { return (c.o_c >= 0 ? 1 : 0) + (c.ff.ff > 0 ? 1 : 0) + (c.q_rank > 0 ? 1 : 0); }
+inline int pre_parts(const LatentCall& c) { return (c.o_c >= 0 ? 1 : 0) + (c.ff.ff > 0 ? 1 : 0) + (c.q_rank > 0 ? 1 : 0); }
 __device__ __forceinline__ int pre_part(const LatentCall& c, int i) {
   if (c.o_c >= 0 && i-- == 0) return PRE_CACHE;
   if (c.ff.ff > 0 && i-- == 0) return PRE_FF;
   return PRE_QUERY;
 }
-template <typename T>
+template <typename T, int RPW>
 __global__ __launch_bounds__(256) void latent_pre_kernel(LatentCall c) {
   __shared__ float red[12];
-  const int r = blockIdx.x, part = pre_part(c, blockIdx.y);
-  const T* pr = (const T*)c.proj + (size_t)r * c.ldp;
-  if (part == PRE_FF) {
-    polynorm_row<T, 256>(c.ff, pr + c.ff.in_off, (T*)c.cat + (size_t)r * c.ldc + c.ff.out_off, red);
-    return;
+  const int part = pre_part(c, blockIdx.y), lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  if constexpr (RPW == 1) {
+    if (part == PRE_FF) {
+      const int r = blockIdx.x;
+      polynorm_row<T, 256>(c.ff, (const T*)c.proj + (size_t)r * c.ldp + c.ff.in_off, (T*)c.cat + (size_t)r * c.ldc + c.ff.out_off, red);
+      return;
+    }
   }
+  const int r = __builtin_amdgcn_readfirstlane(blockIdx.x * RPW + wave);
+  if (wave >= RPW || r >= c.t.R) return;
   const bool cache = part == PRE_CACHE;
-  const TokenAt at = token_at(c.t, r);
   const int n = cache ? c.rank : c.q_rank, np = cache ? c.rp : c.ldqc;
-  const T* src = pr + (cache ? c.o_c : c.o_qc);
+  const T* src = (const T*)c.proj + (size_t)r * c.ldp + (cache ? c.o_c : c.o_qc);       // (parts of a projected row begin at multiples of 16)
   const float* w = cache ? c.c_norm : c.q_norm;
+  const TokenAt at = token_at(c.t, r);
   T* dst = cache ? (T*)c.cache + lat_at(c.s, at.row, at.pos) : (T*)c.qc + (size_t)r * c.ldqc;
-  float ss[1] = {0.f};
-  for (int i = threadIdx.x; i < n; i += 256) { const float v = to_f32(src[i]); ss[0] += v * v; }
-  block_sum<256, 1>(ss, red);
-  const float rs = 1.0f / sqrtf(ss[0] / (float)n + c.eps);
-  for (int i = threadIdx.x; i < np; i += 256) {
-    float v = 0.f;
-    if (i < n) v = to_f32(src[i]) * rs * w[i];
-    else if (cache && i >= c.cp && i < c.cp + c.rot) v = rotated<T>(c, src + n, i - c.cp, at.pos);
-    dst[i] = from_f32<T>(v);
+  // pieces of eight: [0, n) the norm's, [cp, cp + rot) the rotated key part, zeros between and behind (cp is a multiple of 16)
+  auto in_rot = [&](int k) { return cache && k >= c.cp && k < c.cp + c.rot; };
+  auto load = [&](int k, float (&x)[8], float (&g)[8]) {
+    if (k + 8 <= n) {
+      load8f<T>(src + k, x);
+      load8f<float>(w + k, g);
+      return;
+    }
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      x[i] = g[i] = 0.f;
+      if (k + i < n) { x[i] = to_f32(src[k + i]); g[i] = w[k + i]; }
+      else if (in_rot(k) && k + i < c.cp + c.rot) g[i] = rotated<T>(c, src + n, k + i - c.cp, at.pos);       // (x = 0: not the norm's)
+    }
+  };
+  constexpr int KEEP = 2;                              // pieces per lane that stay in registers
+  float x[KEEP][8], g[KEEP][8], ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < KEEP; ++p) load(8 * (lane + 64 * p), x[p], g[p]);
+#pragma unroll
+  for (int p = 0; p < KEEP; ++p)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += x[p][i] * x[p][i];
+  for (int k = 8 * (lane + 64 * KEEP); k < n; k += 512) {
+    float y[8], z[8];
+    load(k, y, z);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) ss += y[i] * y[i];
+  }
+  const float rs = 1.0f / sqrtf(wave_sum(ss) / (float)n + c.eps);
+  auto put = [&](int k, float (&y)[8], const float (&z)[8]) {
+    if (k >= np) return;
+    const bool rot = in_rot(k);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) y[i] = rot ? z[i] : y[i] * rs * z[i];
+    store8f<T>(dst + k, y);
+  };
+#pragma unroll
+  for (int p = 0; p < KEEP; ++p) put(8 * (lane + 64 * p), x[p], g[p]);
+  for (int k = 8 * (lane + 64 * KEEP); k < np; k += 512) {
+    float y[8], z[8];
+    load(k, y, z);
+    put(k, y, z);
   }
 }
 
@@ -188,7 +227,8 @@ template <typename T>
 static int pre_at(const LatentCall& c, hipStream_t st) {
   const int parts = pre_parts(c);
   if (parts == 0) return MI_OK;
-  hipLaunchKernelGGL(latent_pre_kernel<T>, dim3(c.t.R, parts), dim3(256), 0, st, c);
+  if (c.ff.ff > 0) hipLaunchKernelGGL((latent_pre_kernel<T, 1>), dim3(c.t.R, parts), dim3(256), 0, st, c);
+  else hipLaunchKernelGGL((latent_pre_kernel<T, 4>), dim3((c.t.R + 3) / 4, parts), dim3(256), 0, st, c);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -217,11 +257,12 @@ __device__ __forceinline__ f32x4 mfma16(u32x4 a, u32x4 b, f32x4 c) {
 // two float32 values as hi + lo pairs of 16-bit values (float32 weights / queries as two exact-ish MFMA operands)
 template <typename T>
 __device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
-  const T ha = (T)a, hb = (T)b;
-  T h[2] = {ha, hb};
-  T l[2] = {(T)(a - (float)ha), (T)(b - (float)hb)};
+  typedef float f32x2 __attribute__((ext_vector_type(2)));
+  typedef T tx2 __attribute__((ext_vector_type(2)));
+  const tx2 h = __builtin_convertvector((f32x2{a, b}), tx2);
+  const f32x2 back = __builtin_convertvector(h, f32x2);
   hi = __builtin_bit_cast(uint32_t, h);
-  lo = __builtin_bit_cast(uint32_t, l);
+  lo = __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2{a - back[0], b - back[1]}), tx2));
 }
 
 // elements [k, k + 8) of a vector of n, zeros beyond n
@@ -436,21 +477,27 @@ __global__ __launch_bounds__(192) void latent_merge_kernel(LatentCall c) {
 }
 
 // W_uv and the gate.  grid (ceil(vdim / 16), H, ceil(nd / 16)), one wave of 16 tokens and 16 output columns
-template <typename T>
+template <typename T, int NK>
 __global__ __launch_bounds__(64) void latent_uv_kernel(LatentCall c) {
   const int lane = threadIdx.x, c16 = lane & 15, g4 = lane >> 4;
-  const int h = blockIdx.y, m0 = blockIdx.z * 16, nm = min(16, c.t.nd - m0), nk = c.rp / 32;
+  const int h = blockIdx.y, m0 = blockIdx.z * 16, nm = min(16, c.t.nd - m0);
   const int col = blockIdx.x * 16 + c16;
   const T* w = (const T*)c.uv_p + ((size_t)h * c.vdim + min(col, c.vdim - 1)) * c.rp + 8 * g4;
   const T* x = (const T*)c.merged + ((size_t)(m0 + min(c16, nm - 1)) * c.H + h) * 2 * c.rp + 8 * g4;
   f32x4 acc = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
+  u32x4 b[2 * NK], xh[2 * NK], xl[2 * NK];            // (all loads in one round trip)
 #pragma unroll
-  for (int k = 0; k < 18; ++k)
-    if (k < nk) {
-      const u32x4 b = *(const u32x4*)(w + 32 * k);
-      acc = mfma16<T>(*(const u32x4*)(x + 32 * k), b, acc);
-      acc1 = mfma16<T>(*(const u32x4*)(x + c.rp + 32 * k), b, acc1);
-    }
+  for (int k = 0; k < 2 * NK; ++k) {
+    b[k] = *(const u32x4*)(w + 32 * k);
+    xh[k] = *(const u32x4*)(x + 32 * k);
+    xl[k] = *(const u32x4*)(x + c.rp + 32 * k);
+  }
+  __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+  for (int k = 0; k < 2 * NK; ++k) {
+    acc = mfma16<T>(xh[k], b[k], acc);
+    acc1 = mfma16<T>(xl[k], b[k], acc1);
+  }
   acc += acc1;
   if (col >= c.vdim) return;
 #pragma unroll
@@ -475,12 +522,17 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(LatentCall c, T* dst
   }
 }
 
-// grid (query tiles, H), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys, two LDS
-// buffers, the next block's global loads in flight during the current block's MFMAs
+// grid (query tiles, H), 4 waves of 16 QG queries each; all waves share the head's keys and values: blocks of 64 keys from the
+// diagonal downwards, two LDS buffers, the next block's global loads in flight during the current block's MFMAs.  The running maximum
+// lags: weights are taken relative to that of the blocks before, and only a score more than 8 (a factor 256) above it makes the wave
+// find the new one and rescale -- no cross-lane step in most blocks.
+// LDS images, XOR-ed so that the 16-byte writes of consecutive lanes hit different banks:
+//   K [16-key tile][piece of eight][key ^ piece] x 16 B     V [32 keys][16-value tile dt][key ^ (dt & 7)] x 32 B
 template <typename T, int KD, int VD, int QG>
 __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
   constexpr int KB = 64, KK = KD / 32, DT = VD / 16, KT = KB / 16, KIMG = KB * KD * 2, VIMG = KB * VD * 2;
   constexpr int NKP = KB * KD / 8 / 256, NVP = KB * VD / 8 / 256;      // 16-byte pieces per thread
+  constexpr float UNSET = -1e30f, LAG = 8.0f;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];  // K[2], V[2]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
   const int seg = c.t.tile[2 * blockIdx.x], t0 = c.t.tile[2 * blockIdx.x + 1], h = blockIdx.y;
@@ -493,31 +545,34 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
   auto vimg = [&](int b) { return smem + 2 * KIMG + b * VIMG; };
 
   u32x4 kreg[NKP], vreg[NVP];
-  auto load_block = [&](int j) {
+  auto load_block = [&](int j) {                     // (keys beyond nk are read as the last one)
+    const T* kb = kp + (size_t)j * KB * c.ldkv;
+    const T* vb = vp + (size_t)j * KB * c.ldkv;
+    const int top = min(nk - 1 - j * KB, KB - 1);
 #pragma unroll
     for (int i = 0; i < NKP; ++i) {
       const int piece = i * 256 + tid;
-      kreg[i] = *(const u32x4*)(kp + (size_t)min(j * KB + piece / (KD / 8), nk - 1) * c.ldkv + 8 * (piece % (KD / 8)));
+      kreg[i] = *(const u32x4*)(kb + (uint32_t)min(piece / (KD / 8), top) * (uint32_t)c.ldkv + 8 * (piece % (KD / 8)));
     }
 #pragma unroll
     for (int i = 0; i < NVP; ++i) {
       const int piece = i * 256 + tid;
-      vreg[i] = *(const u32x4*)(vp + (size_t)min(j * KB + piece / (VD / 8), nk - 1) * c.ldkv + 8 * (piece % (VD / 8)));
+      vreg[i] = *(const u32x4*)(vb + (uint32_t)min(piece / (VD / 8), top) * (uint32_t)c.ldkv + 8 * (piece % (VD / 8)));
     }
   };
   auto store_block = [&](int buf) {
 #pragma unroll
     for (int i = 0; i < NKP; ++i) {
       const int piece = i * 256 + tid, key = piece / (KD / 8), dc = piece % (KD / 8);
-      *(u32x4*)(kimg(buf) + ((((key >> 4) * KK + (dc >> 2)) * 4 + (dc & 3)) * 16 + (key & 15)) * 16) = kreg[i];
+      *(u32x4*)(kimg(buf) + (((key >> 4) * KK * 4 + dc) * 16 + ((key ^ dc) & 15)) * 16) = kreg[i];
     }
 #pragma unroll
     for (int i = 0; i < NVP; ++i) {
       const int piece = i * 256 + tid, key = piece / (VD / 8), dc = piece % (VD / 8);
-      *(u32x4*)(vimg(buf) + (size_t)((key >> 5) * DT + (dc >> 1)) * (32 * 32) + (key & 31) * 32 + (dc & 1) * 16) = vreg[i];
+      *(u32x4*)(vimg(buf) + (size_t)((key >> 5) * DT + (dc >> 1)) * (32 * 32) + ((key & 31) ^ ((dc >> 1) & 7)) * 32 + (dc & 1) * 16) = vreg[i];
     }
   };
-  load_block(0);
+  load_block(nb - 1);
   u32x4 qf[QG][KK];
   int tq[QG];
 #pragma unroll
@@ -534,19 +589,19 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
 #pragma unroll
     for (int kk = 0; kk < KK; ++kk) asm volatile("" :: "v"(qf[u][kk]));      // (loaded from here on: no wait carried round the loop)
   __syncthreads();
-  const float sc2 = c.scale * LOG2E;
+  const float sc2 = c.scale * LOG2E;                   // (positive)
   float m_run[QG], l_run[QG];
   f32x4 acc[QG][DT];
 #pragma unroll
   for (int u = 0; u < QG; ++u) {
-    m_run[u] = -1e30f; l_run[u] = 0.f;
+    m_run[u] = UNSET; l_run[u] = 0.f;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) acc[u][dt] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const int tq4 = c16 >> 2, tp = c16 & 3;
-  for (int j = 0; j < nb; ++j) {
-    const int buf = j & 1;
-    if (j + 1 < nb) load_block(j + 1);
+  for (int it = 0; it < nb; ++it) {
+    const int j = nb - 1 - it, buf = it & 1;
+    load_block(max(j - 1, 0));                         // straight-line (behind the last block: that one again, not stored)
     f32x4 sc[QG][KT];
 #pragma unroll
     for (int t = 0; t < KT; ++t) {
@@ -554,7 +609,7 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
       for (int u = 0; u < QG; ++u) sc[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < KK; ++kk) {
-        const u32x4 kf = *(const u32x4*)(kimg(buf) + (((t * KK + kk) * 4 + g4) * 16 + c16) * 16);
+        const u32x4 kf = *(const u32x4*)(kimg(buf) + (((t * KK + kk) * 4 + g4) * 16 + (c16 ^ ((4 * kk + g4) & 15))) * 16);
 #pragma unroll
         for (int u = 0; u < QG; ++u) sc[u][t] = mfma16<T>(kf, qf[u][kk], sc[u][t]);
       }
@@ -563,26 +618,35 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
 #pragma unroll
     for (int u = 0; u < QG; ++u) {
       const int q0 = off + t0 + (wave * QG + u) * 16;    // position of the group's first query
-      float mx = -INFINITY;
+      const float ref = m_run[u] == UNSET ? 0.f : m_run[u];
+#pragma unroll
+      for (int t = 0; t < KT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) sc[u][t][r] = fmaf(sc[u][t][r], sc2, -ref);          // relative to the running maximum
       if (j * KB + KB - 1 > q0) {                        // a block that reaches past it (uniform)
 #pragma unroll
         for (int t = 0; t < KT; ++t)
 #pragma unroll
           for (int r = 0; r < 4; ++r) sc[u][t][r] = j * KB + 16 * t + 4 * g4 + r <= q0 + c16 ? sc[u][t][r] : -INFINITY;
       }
+      float mx = -INFINITY;
 #pragma unroll
       for (int t = 0; t < KT; ++t)
 #pragma unroll
         for (int r = 0; r < 4; ++r) mx = fmaxf(mx, sc[u][t][r]);
-      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m_run[u], mx * sc2);        // (scale > 0)
-      if (__builtin_amdgcn_ballot_w64(mn != m_run[u]) != 0) {
-        const float corr = __builtin_amdgcn_exp2f(m_run[u] - mn);
+      if (__builtin_amdgcn_ballot_w64(mx > LAG || m_run[u] == UNSET) != 0) {
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        const float mn = fmaxf(m_run[u], ref + mx);                    // (UNSET while the query has seen no key)
+        const float corr = __builtin_amdgcn_exp2f(m_run[u] - mn), d = (mn == UNSET ? 0.f : mn) - ref;
         m_run[u] = mn;
         l_run[u] *= corr;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt) acc[u][dt] *= corr;
+#pragma unroll
+        for (int t = 0; t < KT; ++t)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sc[u][t][r] -= d;
       }
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf) {
@@ -591,7 +655,7 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
         for (int t = 0; t < 2; ++t) {
           float p[4];
 #pragma unroll
-          for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(fmaf(sc[u][2 * hf + t][r], sc2, -mn)); l_run[u] += p[r]; }
+          for (int r = 0; r < 4; ++r) { p[r] = __builtin_amdgcn_exp2f(sc[u][2 * hf + t][r]); l_run[u] += p[r]; }
           split2<T>(p[0], p[1], ph[2 * t], pw[2 * t]);
           split2<T>(p[2], p[3], ph[2 * t + 1], pw[2 * t + 1]);
         }
@@ -603,19 +667,18 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(LatentCall c) {
     for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
-        const unsigned char* a0 = vimg(buf) + (size_t)(hf * DT + dt) * (32 * 32) + (4 * g4 + tq4) * 32 + tp * 8;
+        const unsigned char* a0 = vimg(buf) + (size_t)(hf * DT + dt) * (32 * 32) + ((4 * g4 + tq4) ^ (dt & 7)) * 32 + tp * 8;
         const s16x4 v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)a0);
         const s16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) s16x4*)(a0 + 16 * 32));
         const uint32_t* w0 = (const uint32_t*)&v0;
         const uint32_t* w1 = (const uint32_t*)&v1;
         const u32x4 vf = {w0[0], w0[1], w1[0], w1[1]};
 #pragma unroll
-        for (int u = 0; u < QG; ++u) {
-          acc[u][dt] = mfma16<T>(vf, pf[u][hf], acc[u][dt]);
-          acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
-        }
+        for (int u = 0; u < QG; ++u) acc[u][dt] = mfma16<T>(vf, pf[u][hf], acc[u][dt]);
+#pragma unroll
+        for (int u = 0; u < QG; ++u) acc[u][dt] = mfma16<T>(vf, pl[u][hf], acc[u][dt]);
       }
-    if (j + 1 < nb) store_block(buf ^ 1);                // the other buffer: nobody reads it during this block
+    if (it + 1 < nb) store_block(buf ^ 1);               // the other buffer: nobody reads it during this block
     __syncthreads();
   }
 #pragma unroll
@@ -653,7 +716,13 @@ int decode_nk(const LatentCall& c, hipStream_t st) {
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
-  return c.s.btab ? go(latent_decode_kernel<T, NK, true>) : go(latent_decode_kernel<T, NK, false>);
+  if (c.s.btab) MI_TRY(go(latent_decode_kernel<T, NK, true>));
+  else MI_TRY(go(latent_decode_kernel<T, NK, false>));
+  hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(c.H, c.t.nd), dim3(c.rp <= 512 ? 128 : 192), 0, st, c);
+  MI_HIP(hipGetLastError());
+  hipLaunchKernelGGL((latent_uv_kernel<T, NK>), dim3((c.vdim + 15) / 16, c.H, (c.t.nd + 15) / 16), dim3(64), 0, st, c);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
 }
 
 template <typename T>
@@ -662,22 +731,17 @@ int decode_at(const LatentCall& c, hipStream_t st) {
     hipLaunchKernelGGL(latent_absorb_kernel<T>, dim3(c.H, c.rp / 64, (c.t.nd + 15) / 16), dim3(256), 0, st, c);
     MI_HIP(hipGetLastError());
     switch (c.rp / 64) {
-      case 1: MI_TRY((decode_nk<T, 1>(c, st))); break;
-      case 2: MI_TRY((decode_nk<T, 2>(c, st))); break;
-      case 3: MI_TRY((decode_nk<T, 3>(c, st))); break;
-      case 4: MI_TRY((decode_nk<T, 4>(c, st))); break;
-      case 5: MI_TRY((decode_nk<T, 5>(c, st))); break;
-      case 6: MI_TRY((decode_nk<T, 6>(c, st))); break;
-      case 7: MI_TRY((decode_nk<T, 7>(c, st))); break;
-      case 8: MI_TRY((decode_nk<T, 8>(c, st))); break;
-      case 9: MI_TRY((decode_nk<T, 9>(c, st))); break;
-      default: return fail(MI_ERR_UNSUPPORTED, "latent_decode: latent size");
+      case 1: return decode_nk<T, 1>(c, st);
+      case 2: return decode_nk<T, 2>(c, st);
+      case 3: return decode_nk<T, 3>(c, st);
+      case 4: return decode_nk<T, 4>(c, st);
+      case 5: return decode_nk<T, 5>(c, st);
+      case 6: return decode_nk<T, 6>(c, st);
+      case 7: return decode_nk<T, 7>(c, st);
+      case 8: return decode_nk<T, 8>(c, st);
+      case 9: return decode_nk<T, 9>(c, st);
     }
-    hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(c.H, c.t.nd), dim3(c.rp <= 512 ? 128 : 192), 0, st, c);
-    MI_HIP(hipGetLastError());
-    hipLaunchKernelGGL(latent_uv_kernel<T>, dim3((c.vdim + 15) / 16, c.H, (c.t.nd + 15) / 16), dim3(64), 0, st, c);
-    MI_HIP(hipGetLastError());
-    return MI_OK;
+    return fail(MI_ERR_UNSUPPORTED, "latent_decode: latent size");
   } else return fail(MI_ERR_UNSUPPORTED, "latent_decode: 16-bit caches only");
 }
 
@@ -690,7 +754,7 @@ int prefill_kv(const LatentCall& c, hipStream_t st) {
     MI_HIP(hipGetLastError());
     return MI_OK;
   };
-  if constexpr (KD <= 128) {
+  if constexpr (KD + VD < 256) {                       // (larger heads do not fit the registers)
     if (c.t.qt == 128) return go(latent_prefill_kernel<T, KD, VD, 2>);
   }
   if (c.t.qt != 64) return fail(MI_ERR_INVALID, "latent_prefill: tile size");
@@ -724,7 +788,7 @@ int gather_at(const LatentCall& c, void* dst, hipStream_t st) {
 }  // namespace
 
 int latent_pad(int n) { return n <= 32 ? 32 : (n <= 64 ? 64 : (n <= 128 ? 128 : 0)); }
-int latent_tile(int kdp) { return kdp <= 128 ? 128 : 64; }
+int latent_tile(int kdp, int vdp) { return kdp + vdp < 256 ? 128 : 64; }
 int latent_key_pad(int n) { return n > 128 && n <= 192 ? 192 : latent_pad(n); }
 bool latent_mfma_supported(int act, int dim, int vdim, int rp) {
   return (act == MI_BF16 || act == MI_F16) && latent_key_pad(dim) > 0 && latent_pad(vdim) > 0 && rp % 64 == 0 && rp <= 576;

@@ -155,7 +155,7 @@ struct LatentCall {
 };
 int launch_latent_pre(const LatentCall& c, hipStream_t st);            // append the latents, feed-forward activation, the queries' latent
 int launch_latent_generic(const LatentCall& c, hipStream_t st);        // any size and dtype, all tokens
-int latent_tile(int kdp);                                              // queries per tile at most
+int latent_tile(int kdp, int vdp);                                            // queries per tile at most
 bool latent_mfma_supported(int act, int dim, int vdim, int rp);        // dim: with the rotated part
 int latent_pad(int n);                                                 // padded value head size of the prefill kernel, 0 = none
 int latent_key_pad(int n);                                             // of a key head (with its rotated part)

@@ -81,23 +81,59 @@ __device__ __forceinline__ float lanes_sum(float v) {
   }
 }
 
-// norm over all heads and gate of token r by NT threads; o(k): output k of the token
-template <typename T, int NT, typename F>
+// norm over all heads and gate of token r by NT threads; o(k): output k of the token.  NQ > 0: four consecutive outputs per thread and
+// round, NQ rounds, in registers (n a multiple of four); 0: any n
+template <typename T, int NT, int NQ, typename F>
 __device__ __forceinline__ void norm_and_gate(const LightCall& c, int r, float* red, F o) {
   const int n = c.H * c.e;
+  if constexpr (NQ > 0) {
+    const T* gate = (const T*)c.proj + (size_t)r * c.ldp + c.o_g;
+    f32x4 v[NQ], w[NQ];
+    float4 z[NQ];
+    float ss[1] = {0.f};
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {                     // (one round trip)
+      const int k = min(4 * (q * NT + (int)threadIdx.x), n - 4);
+      v[q] = o(k);
+      w[q] = *(const f32x4*)(c.norm + k);
+      z[q] = load4f<T>(gate + k);
+    }
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+      if (4 * (q * NT + (int)threadIdx.x) >= n) continue;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss[0] += v[q][j] * v[q][j];
+    }
+    block_sum<NT, 1>(ss, red);
+    const float rs = 1.0f / sqrtf(ss[0] / (float)n + c.eps);
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+      const int k = 4 * (q * NT + (int)threadIdx.x);
+      if (k >= n) continue;
+      const float g[4] = {z[q].x, z[q].y, z[q].z, z[q].w};
+      T out[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) out[j] = from_f32<T>(v[q][j] * rs * w[q][j] * sigmoid_f(g[j]));
+      T* dst = (T*)c.cat + (size_t)r * c.ldc + k;
+      if constexpr (sizeof(T) == 2) *(uint2*)dst = __builtin_bit_cast(uint2, out);
+      else *(f32x4*)dst = f32x4{(float)out[0], (float)out[1], (float)out[2], (float)out[3]};
+    }
+    return;
+  }
   float ss[1] = {0.f};
-  for (int k = threadIdx.x; k < n; k += NT) { const float v = o(k); ss[0] += v * v; }
+  for (int k = threadIdx.x; k < n; k += NT) { const float v = o(k)[0]; ss[0] += v * v; }
   block_sum<NT, 1>(ss, red);
   const float rs = 1.0f / sqrtf(ss[0] / (float)n + c.eps);
   const T* gate = (const T*)c.proj + (size_t)r * c.ldp + c.o_g;
   T* cat = (T*)c.cat + (size_t)r * c.ldc;
-  for (int k = threadIdx.x; k < n; k += NT) cat[k] = from_f32<T>(o(k) * rs * c.norm[k] * sigmoid_f(to_f32(gate[k])));
+  for (int k = threadIdx.x; k < n; k += NT) cat[k] = from_f32<T>(o(k)[0] * rs * c.norm[k] * sigmoid_f(to_f32(gate[k])));
 }
 
 // ---- one-token segments --------------------------------------------------------------------------------------------------
 // grid (nd, H, strips of DE value columns), 4 waves.  L lanes share a column, NV pieces of four key channels each (4 L NV >= d).
+// NQ: of norm_and_gate.  The new state is stored behind the ticket, so nobody waits for it.
 constexpr int DE = 32;
-template <typename T, int L, int NV>
+template <typename T, int L, int NV, int NQ>
 __global__ __launch_bounds__(256) void light_decode_kernel(LightCall c) {
   constexpr int CPW = 64 / L, STEP = 4 * CPW, NI = (DE + STEP - 1) / STEP;      // columns per wave and step, steps
   __shared__ float red[4];
@@ -140,7 +176,6 @@ __global__ __launch_bounds__(256) void light_decode_kernel(LightCall c) {
         s[i][v][j] = fmaf(kk[v][j], vv, g * s[i][v][j]);
         a = fmaf(s[i][v][j], q[v][j], a);
       }
-      if (on && k < c.sd) *(f32x4*)(S + (size_t)col * c.sd + k) = s[i][v];
     }
     a = lanes_sum<L>(a);
     if (on && sl == 0) __hip_atomic_store(&o[col], a, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
@@ -153,10 +188,24 @@ __global__ __launch_bounds__(256) void light_decode_kernel(LightCall c) {
     last_sh = ticket == (int)(gridDim.y * gridDim.z) - 1;
     if (last_sh) __hip_atomic_store(&c.tickets[blockIdx.x], 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
+#pragma unroll
+  for (int i = 0; i < NI; ++i) {
+    const int in = i * STEP + cw, col = e0 + in;
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+      const int k = 4 * (sl + v * L);
+      if (in < DE && col < c.e && k < c.sd) *(f32x4*)(S + (size_t)col * c.sd + k) = s[i][v];
+    }
+  }
   __syncthreads();
   if (!last_sh) return;
   const float* all = c.o + (size_t)r * c.ldo;
-  norm_and_gate<T, 256>(c, r, red, [&](int k) { return __hip_atomic_load(&all[k], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); });
+  norm_and_gate<T, 256, NQ>(c, r, red, [&](int k) {
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < (NQ > 0 ? 4 : 1); ++j) v[j] = __hip_atomic_load(&all[k + j], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    return v;
+  });
 }
 
 // ---- token by token ------------------------------------------------------------------------------------------------------
@@ -191,13 +240,16 @@ __global__ __launch_bounds__(256) void light_scan_kernel(LightCall c) {
     if (sl + 16 * i < c.sd) S[sl + 16 * i] = s[i];
 }
 
-template <typename T>
+template <typename T, int NQ>
 __global__ __launch_bounds__(256) void light_norm_kernel(LightCall c) {
   __shared__ float red[4];
   const int r = blockIdx.x;
   if (c.t.len[c.t.tok_seg[r]] < 2) return;
   const float* o = c.o + (size_t)r * c.ldo;
-  norm_and_gate<T, 256>(c, r, red, [&](int k) { return o[k]; });
+  norm_and_gate<T, 256, NQ>(c, r, red, [&](int k) {
+    if constexpr (NQ > 0) return *(const f32x4*)(o + k);
+    else return f32x4{o[k], 0.f, 0.f, 0.f};
+  });
 }
 
 // ---- chunks --------------------------------------------------------------------------------------------------------------
@@ -219,7 +271,7 @@ __device__ __forceinline__ u32x4 tread(const unsigned char* img, int hf, int ct,
 
 // grid (H, chunks), 4 waves: wave (wd, we) has every WD-th 16-channel tile of the keys and every WE-th 16-column tile of the values
 template <typename T, int DP, int EP>
-__global__ __launch_bounds__(256) void light_chunk_kernel(LightCall c) {
+__global__ __launch_bounds__(256, 3) void light_chunk_kernel(LightCall c) {
   constexpr int KB = 64, WD = DP >= 64 ? 4 : 2, WE = 4 / WD, ND = DP / 16 / WD, NE = EP / 16 / WE;
   constexpr int NKP = (KB * DP / 8 + 255) / 256, NVP = (KB * EP / 8 + 255) / 256;          // 16-byte pieces per thread
   __shared__ __attribute__((aligned(16))) unsigned char khi[KB * DP * 2], klo[KB * DP * 2], vim[KB * EP * 2];
@@ -327,7 +379,7 @@ __global__ __launch_bounds__(256) void light_carry_kernel(LightCall c) {
 // grid (H, chunks x chunk / LIGHT_QT), 4 waves of 16 queries each.  The products are laid out as in the attention kernels:
 // rows = keys / state columns / output columns, columns = queries.
 template <typename T, int DP, int EP>
-__global__ __launch_bounds__(256) void light_out_kernel(LightCall c) {
+__global__ __launch_bounds__(256, 4) void light_out_kernel(LightCall c) {
   constexpr int KB = 64, KK = DP / 32, ET = EP / 16, SB = EP < 64 ? EP : 64;               // SB: state columns staged at a time
   constexpr int NKP = (KB * DP / 8 + 255) / 256, NVP = (KB * EP / 8 + 255) / 256, NSP = (SB * DP / 8 + 255) / 256;
   constexpr int AIMG = KB * DP * 2, BIMG = KB * (EP > DP ? EP : DP) * 2;
@@ -489,9 +541,13 @@ int scan_at(const LightCall& c, hipStream_t st) {
 
 template <typename T>
 int light_at(const LightCall& c, hipStream_t st) {
+  // rounds of four outputs per thread of the norm, 0: element by element
+  const int n = c.H * c.e, nq = n % 4 == 0 && n <= 8 * 1024 && c.ldo % 4 == 0 && c.ldc % 4 == 0 ? (n + 1023) / 1024 : 0;
   if (c.t.nd > 0) {
     const dim3 grid(c.t.nd, c.H, (c.e + DE - 1) / DE), block(256);
-#define GO(L, NV) hipLaunchKernelGGL((light_decode_kernel<T, L, NV>), grid, block, 0, st, c)
+#define GO(L, NV) do { if (nq == 0) hipLaunchKernelGGL((light_decode_kernel<T, L, NV, 0>), grid, block, 0, st, c); \
+    else if (nq <= 2) hipLaunchKernelGGL((light_decode_kernel<T, L, NV, 2>), grid, block, 0, st, c); \
+    else hipLaunchKernelGGL((light_decode_kernel<T, L, NV, 8>), grid, block, 0, st, c); } while (0)
     if (c.d <= 16) GO(4, 1); else if (c.d <= 32) GO(8, 1); else if (c.d <= 64) GO(16, 1); else if (c.d <= 128) GO(32, 1);
     else if (c.d <= 256) GO(64, 1); else GO(64, 2);
 #undef GO
@@ -500,7 +556,9 @@ int light_at(const LightCall& c, hipStream_t st) {
   if (c.t.nc > 0) {
     if (c.ws != nullptr) MI_TRY(chunks_at<T>(c, st));
     else MI_TRY(scan_at<T>(c, st));
-    hipLaunchKernelGGL(light_norm_kernel<T>, dim3(c.t.R), dim3(256), 0, st, c);
+#define GO(NQ) hipLaunchKernelGGL((light_norm_kernel<T, NQ>), dim3(c.t.R), dim3(256), 0, st, c)
+    if (nq == 0) GO(0); else if (nq <= 1) GO(1); else if (nq <= 2) GO(2); else if (nq <= 4) GO(4); else GO(8);
+#undef GO
     MI_HIP(hipGetLastError());
   }
   return MI_OK;
