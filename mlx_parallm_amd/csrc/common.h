@@ -139,13 +139,14 @@ __device__ __forceinline__ float glu_f(const Glu& c, float g, float u) {
 }
 // the same on a 16-bit model's accumulators: silu rounds every operation to AT, the others the result alone
 template <typename AT>
-__device__ __forceinline__ AT glu16(const Glu& c, float g, float u) {
-  if (c.kind != GLU_SILU) return (AT)glu_f(c, g, u);
+__device__ __forceinline__ AT silu16(float g, float u) {
   const float gt = (float)(AT)g, up = (float)(AT)u;
   const float sig = (float)(AT)(1.0f / (1.0f + expf(-gt)));
   const float sl = (float)(AT)(gt * sig);
   return (AT)(sl * up);
 }
+template <typename AT>
+__device__ __forceinline__ AT glu16(const Glu& c, float g, float u) { return c.kind != GLU_SILU ? (AT)glu_f(c, g, u) : silu16<AT>(g, u); }
 // an output column in front of `silu_cols` of a plain store goes through silu (projections that are used only that way)
 __device__ __forceinline__ float silu_col(int silu_cols, int n, float y) { return n < silu_cols ? y / (1.0f + expf(-y)) : y; }
 

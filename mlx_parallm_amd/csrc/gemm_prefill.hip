@@ -78,6 +78,8 @@ __device__ __forceinline__ void epi32_plain(const GemmParams& p, int m, int n, f
   else { float* h = (float*)p.resid; h[(size_t)m * p.ldo + n] = h[(size_t)m * p.ldo + n] + y; }
 }
 
+__device__ __forceinline__ float silu_mul(float g, float u) { return g / (1.0f + expf(-g)) * u; }
+
 // grid: (n blocks, m blocks).  SWIGLU: a block covers 64 gate columns + the 64 matching up columns.
 // grouped form: the matrix and the rows of tile bm of the device-resident table; false: no such tile, or no columns from n0 on
 template <typename AT, bool SWIGLU>
@@ -220,7 +222,10 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
   }
 
   // ---- epilogue: lane (c16, g) holds C[m = 4g + r][n = c16] of every 16 x 16 tile
+  // (var: another unit than silu, or a plain store with silu columns -- asked once, not per element)
   AT* out = (AT*)p.out;
+  auto store = [&](auto var) {
+    constexpr bool VAR = decltype(var)::value;
 #pragma unroll
   for (int mt = 0; mt < 4; ++mt)
 #pragma unroll
@@ -233,9 +238,9 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
         for (int j = 0; j < 2; ++j) {
           const int n = bn * 64 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
-          if constexpr (GROUPED) { out[(size_t)m * p.ldo + n] = (AT)glu_f(p.glu, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
+          if constexpr (GROUPED) { out[(size_t)m * p.ldo + n] = (AT)(VAR ? glu_f(p.glu, acc[mt][j][r], acc[mt][j + 2][r]) : silu_mul(acc[mt][j][r], acc[mt][j + 2][r])); continue; }
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
-          out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, acc[mt][j][r], acc[mt][j + 2][r]);
+          out[(size_t)m * p.ldo + n] = (VAR ? (AT)glu_f(p.glu, acc[mt][j][r], acc[mt][j + 2][r]) : silu16<AT>(acc[mt][j][r], acc[mt][j + 2][r]));
         }
       } else {
 #pragma unroll
@@ -243,7 +248,7 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
           const int n = bn * BN + wn * 64 + nt * 16 + c16;
           if (n >= p.N) continue;
           if (p.out32) { epi32_plain(p, m, n, acc[mt][nt][r]); continue; }
-          const float y = (float)(AT)silu_col(p.silu_cols, n, acc[mt][nt][r]);
+          const float y = (float)(AT)(VAR ? silu_col(p.silu_cols, n, acc[mt][nt][r]) : acc[mt][nt][r]);
           if (p.epi == EPI_STORE) out[(size_t)m * p.ldo + n] = (AT)y;
           else {
             AT* h = (AT*)p.resid;
@@ -252,6 +257,10 @@ __global__ __launch_bounds__(256) void gemm_tile_kernel(GemmParams p) {
         }
       }
     }
+  };
+  if constexpr (GROUPED && !SWIGLU) store(std::false_type{});
+  else if (SWIGLU ? p.glu.kind != GLU_SILU : p.silu_cols > bn * BN) store(std::true_type{});
+  else store(std::false_type{});
 }
 
 // the K slices of gemm_tile_kernel, added in slice order, + the epilogue (EPI_STORE / EPI_RESID); 4 columns per thread
@@ -274,11 +283,13 @@ __global__ __launch_bounds__(256) void splitk_epilogue_kernel(GemmParams p) {
 }
 
 constexpr int BM2 = 256, BN2 = 256;
+template <bool SWIGLU>
+__device__ __forceinline__ bool epilogue_varies(const GemmParams& p, int bn) { return SWIGLU ? p.glu.kind != GLU_SILU : p.silu_cols > bn * BN2; }
 
 // the epilogue of the 256 x 256 tiles (2 x 4 waves, 128 x 64 per wave): lane (c16, g) holds C[m = 4g + r][n = c16] of
 // every 16 x 16 tile
-// SILU: a plain store with silu_cols (common.h)
-template <typename AT, bool SWIGLU, bool SILU = false>
+// VAR: another unit than silu, or a plain store with silu columns (common.h)
+template <typename AT, bool SWIGLU, bool VAR>
 __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&acc)[8][4], int m0, int bn, int wm, int wn, int c16, int g) {
   AT* out = (AT*)p.out;
 #pragma unroll
@@ -293,7 +304,7 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
           const int n = bn * 128 + wn * 32 + j * 16 + c16;
           if (n >= p.pair_offset) continue;
           if (p.out32) { epi32_swiglu(p, m, n, acc[mt][j][r], acc[mt][j + 2][r]); continue; }
-          out[(size_t)m * p.ldo + n] = glu16<AT>(p.glu, acc[mt][j][r], acc[mt][j + 2][r]);
+          out[(size_t)m * p.ldo + n] = VAR ? (AT)glu_f(p.glu, acc[mt][j][r], acc[mt][j + 2][r]) : silu16<AT>(acc[mt][j][r], acc[mt][j + 2][r]);
         }
       } else {
 #pragma unroll
@@ -301,7 +312,7 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
           const int n = bn * BN2 + wn * 64 + nt * 16 + c16;
           if (n >= p.N) continue;
           if (p.out32) { epi32_plain(p, m, n, acc[mt][nt][r]); continue; }
-          const float y = (float)(AT)(SILU ? silu_col(p.silu_cols, n, acc[mt][nt][r]) : acc[mt][nt][r]);
+          const float y = (float)(AT)(VAR ? silu_col(p.silu_cols, n, acc[mt][nt][r]) : acc[mt][nt][r]);
           if (p.epi == EPI_STORE) out[(size_t)m * p.ldo + n] = (AT)y;
           else {
             AT* h = (AT*)p.resid;
@@ -314,7 +325,7 @@ __device__ __forceinline__ void tile256_epilogue(const GemmParams& p, f32x4 (&ac
 
 // Grouped form: whole rows.  A wave's tile goes through its own strip of LDS, 64 rows at a time, and leaves it as 16-byte pieces of
 // rows (out_rows may scatter them): 16 stores per wave instead of 128.  The LDS must be free (every DMA landed, every read done).
-template <typename AT, bool SWIGLU>
+template <typename AT, bool SWIGLU, bool VAR>
 __device__ __forceinline__ void tile256_epilogue_rows(const GemmParams& p, f32x4 (&acc)[8][4], unsigned char* lds, int bn, int wave, int lane, int place0) {
   constexpr int WC = SWIGLU ? 32 : 64, LDW = WC + 8, NP = WC / 8;
   const int wm = wave >> 2, wn = wave & 3, c16 = lane & 15, g = lane >> 4;
@@ -330,7 +341,7 @@ __device__ __forceinline__ void tile256_epilogue_rows(const GemmParams& p, f32x4
         const f32x4 (&a)[4] = acc[hf * 4 + mt];
         if constexpr (SWIGLU) {
 #pragma unroll
-          for (int j = 0; j < 2; ++j) row[j * 16] = (AT)glu_f(p.glu, a[j][r], a[j + 2][r]);
+          for (int j = 0; j < 2; ++j) row[j * 16] = (AT)(VAR ? glu_f(p.glu, a[j][r], a[j + 2][r]) : silu_mul(a[j][r], a[j + 2][r]));
         } else {
 #pragma unroll
           for (int nt = 0; nt < 4; ++nt) row[nt * 16] = (AT)a[nt][r];
@@ -564,8 +575,8 @@ __global__ __launch_bounds__(512) void gemm_tile256_kernel(GemmParams p) {
       return;
     }
   }
-  if (!SWIGLU && p.silu_cols > bn * BN2) tile256_epilogue<AT, SWIGLU, !SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
-  else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+  if (epilogue_varies<SWIGLU>(p, bn)) tile256_epilogue<AT, SWIGLU, true>(p, acc, m0, bn, wm, wn, c16, g);
+  else tile256_epilogue<AT, SWIGLU, false>(p, acc, m0, bn, wm, wn, c16, g);
 }
 
 
@@ -783,9 +794,10 @@ __global__ __launch_bounds__(512) void gemm_dma256_kernel(GemmParams p) {
   }
   if constexpr (GROUPED) {
     __syncthreads();
-    tile256_epilogue_rows<AT, SWIGLU>(p, acc, smem2, bn, wave, lane, place0);
-  } else if (!SWIGLU && p.silu_cols > bn * BN2) tile256_epilogue<AT, SWIGLU, !SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
-  else tile256_epilogue<AT, SWIGLU>(p, acc, m0, bn, wm, wn, c16, g);
+    if (SWIGLU && p.glu.kind != GLU_SILU) tile256_epilogue_rows<AT, SWIGLU, SWIGLU>(p, acc, smem2, bn, wave, lane, place0);
+    else tile256_epilogue_rows<AT, SWIGLU, false>(p, acc, smem2, bn, wave, lane, place0);
+  } else if (epilogue_varies<SWIGLU>(p, bn)) tile256_epilogue<AT, SWIGLU, true>(p, acc, m0, bn, wm, wn, c16, g);
+  else tile256_epilogue<AT, SWIGLU, false>(p, acc, m0, bn, wm, wn, c16, g);
 }
 
 

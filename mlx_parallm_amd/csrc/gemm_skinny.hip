@@ -724,6 +724,14 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
   // ================= epilogue: lane (c16, g) holds y[16 mt + 4 g + r][16 tile + c16]
   const int n = tile * 16 + c16;
   AT* out = (AT*)p.out;
+  if constexpr (!SWIGLU && !X32) {
+    if (p.silu_cols > 0) {                         // (asked once, not per element)
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[0][mt][r] = silu_col(p.silu_cols, n, acc[0][mt][r]);
+    }
+  }
   float hsq[NH ? MT * 4 : 1];
 #pragma unroll
   for (int i = 0; i < (NH ? MT * 4 : 1); ++i) hsq[i] = 0.f;
@@ -758,14 +766,12 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
         const float rsm = dn ? rs_row[ml] : 1.0f;
         y0 *= rsm;
         if constexpr (SWIGLU) {
-          const float up0 = acc[NA - 1][mt][r] * rsm;
-          if (p.glu.kind != GLU_SILU) { o32[(size_t)m * p.ldo + n] = round_rt(glu_f(p.glu, y0, up0), p.rnd); continue; }
-          const float gt = round_rt(y0, p.rnd), up = round_rt(up0, p.rnd);
+          const float gt = round_rt(y0, p.rnd), up = round_rt(acc[NA - 1][mt][r] * rsm, p.rnd);
           const float sig = round_rt(1.0f / (1.0f + expf(-gt)), p.rnd);
           const float sl = round_rt(gt * sig, p.rnd);
           o32[(size_t)m * p.ldo + n] = round_rt(sl * up, p.rnd);
         } else {
-          float y = round_rt(silu_col(p.silu_cols, n, y0), p.rnd);
+          float y = round_rt(y0, p.rnd);
           if (p.lora_t != nullptr) {             // LoRALinear in this mode: y + T(scale (x A) B), the term in float32 (App. A.6)
 #pragma unroll
             for (int sl = 0; sl < 2; ++sl) {
@@ -805,7 +811,7 @@ __global__ __launch_bounds__(SK_NW * 64, (QB == 4 || (QB == 8 && MT >= 3) || MT 
           } else ((float*)p.out)[(size_t)m * p.ldo + n] = y0;
           continue;
         }
-        float y = (float)(AT)silu_col(p.silu_cols, n, y0);
+        float y = (float)(AT)y0;
         if (p.lora_t != nullptr) {
 #pragma unroll
           for (int sl = 0; sl < 2; ++sl) {
@@ -997,6 +1003,7 @@ static int skinny_min_rows() {
 }
 
 bool gemm_skinny_supported(const LinearW& W, const GemvCall& c, size_t rows) {
+  if (c.act == MI_F32 && (c.glu.kind != GLU_SILU || c.silu_cols > 0)) return false;
   if (c.force_v1 || W.layout != 1) return false;
   // float32 activations on 16-bit dense weights (PagedKVCache mode): the 16-row instantiation with x split three ways
   if (c.act == MI_F32) {
